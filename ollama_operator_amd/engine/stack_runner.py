@@ -216,9 +216,10 @@ class StackRunner(Runner):
         self.kc, self.vc, self.states = [], [], []
         for li, _ps, _first in self.runs:
             m = cfg.layers[li].mixer
-            if cfg.block == BLOCK_SANDWICH:  # K/V pools, and one state row per slot: [second mixer's matrix | input window]
-                self.kc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.dim, **tt))
-                self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt))
+            if cfg.block == BLOCK_SANDWICH or cfg.canon_both:  # K/V pools of attention, and one state row per slot: [the mixers'
+                attn = m.kind == MIX_ATTENTION                 # state | input windows]
+                self.kc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.dim, **tt) if attn else None)
+                self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt) if attn else None)
                 ns = cfg.run_state_floats(li)
                 self.states.append(torch.zeros(max_seqs, ns, **f32) if ns else None)
             elif m.kind == MIX_ATTENTION and m.score_talk:  # one K row per token: every key/value head's key side by side

@@ -442,7 +442,7 @@ class StackWeights:
                 self.layers.append(self._load_sandwich_layer(st, p, spec))
                 continue
             if cfg.block == BLOCK_PRENORM:
-                self.layers.append(self._load_prenorm_layer(p, spec))
+                self.layers.append(self._load_prenorm_layer(st, p, spec))
                 continue
             L: dict = dict(norm_w=vec(get(p + "norm1", (E,))), norm_b=vec(get(p + "norm1.b", (E,))))
             if cfg.block == BLOCK_POSTNORM:
@@ -488,7 +488,8 @@ class StackWeights:
             self.final_w, self.final_b = vec(get("final.norm", (E,))), None
         else:
             self.final_w, self.final_b = vec(get("final.norm", (E,))), vec(get("final.norm.b", (E,)))
-        self.head = mat(get("head", (V, E)))
+        # (a design without a head of its own reads the logits off the embedding table)
+        self.head = self.embed if cfg.tied_head else mat(get("head", (V, E)))
         self.local = dict(E=E, V=V)
 
     def _load_postnorm_layer(self, L: dict, p: str, spec) -> None:
@@ -521,12 +522,7 @@ class StackWeights:
             L["i_b"], L["f_b"] = vec(get(p + "mix.i.b", (H,))), vec(get(p + "mix.f.b", (H,)))
             L["mnorm"] = vec(get(p + "mix.norm", (H * Dv,)))
         elif m.kind == MIX_MAMBA2:
-            inner, GN, ch = H * Dv, m.groups * m.state, m.conv_channels
-            parts = [get(p + "mix.in", (2 * inner + 2 * GN + H, E))]
-            off = dict(g=0, conv=inner, dt=2 * inner + 2 * GN)      # z | x B C | dt
-            L["conv_w"], L["conv_b"] = vec(get(p + "mix.conv", (ch, m.conv))), vec(get(p + "mix.conv.b", (ch,)))
-            L["dt_bias"], L["a_log"], L["d_skip"] = (vec(get(p + "mix." + k, (H,))) for k in ("dt_bias", "A_log", "D"))
-            L["mnorm"] = vec(get(p + "mix.norm", (inner,)))
+            parts, off = self._load_mamba2(L, p, m)
         else:
             raise ValueError("this block style has no mixer of that kind")
         L["w_in"] = mat(*parts)
@@ -556,6 +552,33 @@ class StackWeights:
             dn.append(get(q + "down", (E, F)))
         L["w_gu"] = mat(*gu).view(X, 2 * F, E)
         L["w_down"] = mat(*dn).view(X, E, F)
+
+    def _load_mamba2(self, L: dict, p: str, m) -> tuple[list, dict]:
+        """The state-space mixer's own tensors into L; its input projection and the columns in it: z | x B C | dt."""
+        get, vec, E, H = self._get, self._vec, self.cfg.n_embd, m.heads
+        inner, GN, ch = m.n_out, m.groups * m.state, m.conv_channels
+        L["conv_w"], L["conv_b"] = vec(get(p + "mix.conv", (ch, m.conv))), vec(get(p + "mix.conv.b", (ch,)))
+        L["dt_bias"], L["a_log"], L["d_skip"] = (vec(get(p + "mix." + k, (H,))) for k in ("dt_bias", "A_log", "D"))
+        L["mnorm"] = vec(get(p + "mix.norm", (inner,)))
+        return [get(p + "mix.in", (2 * inner + 2 * GN + H, E))], dict(g=0, conv=inner, dt=2 * inner + 2 * GN)
+
+    def _load_delta(self, L: dict, st, b: str, r, parts: list, off: dict) -> None:
+        """A gated delta rule's tensors into L, its input matrices onto the stack `parts` (q | k | v, which pass one
+        convolution and sit side by side, then the write strengths and the first factors of the two low-rank maps)."""
+        get, mat, vec, E = self._get, self._mat, self._vec, self.cfg.n_embd
+        nq, nk, nv = r.kv_heads * r.dim, r.kv_heads * r.dim, r.n_out
+        r.decay_rank, r.gate_rank = (int(st.shape(b + k)[0]) if st.has(b + k) else 0 for k in ("a1", "g1"))
+        n = sum(t.shape[0] for t in parts)
+        for key, name, rows in (("rq", "q", nq), ("rk", "k", nk), ("rv", "v", nv), ("rb", "b", r.heads),
+                                ("a1", "a1", r.decay_rank), ("g1", "g1", r.gate_rank)):
+            parts.append(get(b + name, (rows, E)))
+            off[key] = n
+            n += rows
+        L["conv_w"] = vec(torch.cat([get(b + k + ".conv", (rows, r.conv)).to(torch.float32)
+                                     for k, rows in (("q", nq), ("k", nk), ("v", nv))], 0))
+        L["a2"], L["g2"] = mat(get(b + "a2", (r.n_q, r.decay_rank))), mat(get(b + "g2", (nv, r.gate_rank)))
+        L["a_log"], L["dt_bias"] = vec(get(b + "A_log", (r.heads,))), vec(get(b + "dt_bias", (r.n_q,)))
+        L["gnorm"] = vec(get(b + "norm", (r.vdim,)))
 
     def _load_sandwich_layer(self, st, p: str, spec) -> dict:
         """A layer with scalar-weight RMS norms around both sublayers. The matrices that read the mixer's input are
@@ -620,14 +643,17 @@ class StackWeights:
             L["w_dense_down"] = mat(get(p + "mlp.down", (E, f.ff)))
         return L
 
-    def _load_prenorm_layer(self, p: str, spec) -> dict:
+    def _load_prenorm_layer(self, st, p: str, spec) -> dict:
         """A layer with RMS norms (weight vectors) on the inputs of both sublayers. The mixer's matrices that read its
         normed input are one stack `w_in` (attention q | k | v | [gate]; latent attention q | dkv | gate), the
         feed-forward's are a second stack `w_ff` (gate | up of the dense one, or the router) because it reads the
         updated stream. Constants that are functions of the weights alone are worked out here in float32: the
         differential attention's lambda, and the score-mixing matrix with the heads' factors folded in
-        (M[h][g] = talk[h][g] * temp[g]). Rotary frequencies are float64."""
-        from ..models.config import FF_GLU, GATE_ELEMENT, MIX_LATENT, rotary_inv_freq
+        (M[h][g] = talk[h][g] * temp[g]), the heads' distance slopes. Rotary frequencies are float64. A second mixer
+        beside the attention adds its matrices to the stack `w_in`, and its output projection sits beside the
+        attention's in `w_o` (the layer's result is one product over both mixers' outputs, whose scales are applied
+        to the outputs); the inner sizes of its low-rank maps come from the tensors' shapes."""
+        from ..models.config import FF_GLU, GATE_HEAD, GATE_NONE, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, rotary_inv_freq
         get, mat, vec = self._get, self._mat, self._vec
         cfg, dev = self.cfg, self.device
         E, m, f = cfg.n_embd, spec.mixer, spec.mlp
@@ -642,12 +668,23 @@ class StackWeights:
             L["w_uvT"] = mat(get(p + "mix.uv", (H * Dv, C)).view(H, Dv, C).transpose(1, 2).reshape(H * C, Dv))
             L["w_ukT"] = mat(get(p + "mix.uk", (H * D, C)).view(H, D, C).transpose(1, 2).reshape(H * C, D))
             L["w_uv"] = mat(get(p + "mix.uv", (H * Dv, C)))
+        elif m.kind == MIX_MAMBA2:
+            parts, off = self._load_mamba2(L, p, m)
+        elif m.kind == MIX_LINEAR:
+            parts = [get(p + "mix.q", (H * D, E)), get(p + "mix.k", (H * D, E)), get(p + "mix.v", (H * Dv, E)),
+                     get(p + "mix.g", (H * Dv, E))]
+            off = dict(q=0, k=H * D, v=2 * H * D, g=2 * H * D + H * Dv)
+            L["decay"] = torch.tensor(m.decay, dtype=torch.float32, device=dev)
+            L["mnorm"] = vec(get(p + "mix.norm", (H * Dv,)))
         else:
-            parts = [get(p + "mix.q", (m.n_q, E)), get(p + "mix.k", (m.n_k, E)), get(p + "mix.v", (m.n_v, E))]
+            a = p + ("mix.left." if m.right is not None else "mix.")
+            parts = [get(a + "q", (m.n_q, E)), get(a + "k", (m.n_k, E)), get(a + "v", (m.n_v, E))]
             off = dict(q=0, k=m.n_q, v=m.n_q + m.n_k)
-            if m.gate == GATE_ELEMENT:
-                parts.append(get(p + "mix.g", (m.n_out, E)))
+            if m.gate != GATE_NONE:
+                parts.append(get(a + "g", (H if m.gate == GATE_HEAD else m.n_out, E)))
                 off["g"] = m.n_q + m.n_k + m.n_v
+            if m.alibi:
+                L["slopes"] = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)], dtype=torch.float32, device=dev)
             if m.maps == 2:
                 lq1, lk1, lq2, lk2 = (get(p + "mix." + k, (D,)).to(torch.float32) for k in ("lq1", "lk1", "lq2", "lk2"))
                 L["lam"] = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum()) + torch.tensor(m.diff, dtype=torch.float32))
@@ -657,12 +694,20 @@ class StackWeights:
                 L["talk"] = (talk * temp[None, :]).reshape(-1).contiguous().to(dev)
         L["inv_freq64"] = (torch.tensor(rotary_inv_freq(m.rot_dims, m.rot_base, m.rot_scaling), dtype=torch.float64, device=dev)
                            if m.rot_dims else None)
+        if m.right is not None:
+            self._load_delta(L, st, p + "mix.right.", m.right, parts, off)
+            L["w_o"] = mat(torch.cat([get(p + "mix.left.o", (E, m.n_out)), get(p + "mix.right.o", (E, m.right.n_out))], 1))
+        else:
+            L["w_o"] = mat(get(p + "mix.o", (E, m.n_out)))
         L["w_in"] = mat(*parts)
         L["off"], L["n_in"], L["n_ff"] = off, sum(t.shape[0] for t in parts), 0
-        L["w_o"] = mat(get(p + "mix.o", (E, m.n_out)))
+        if cfg.canon_both:
+            L["canon"] = vec(get(p + "canon1", (E, cfg.canon_taps)))
         if f is None:
             return L
         L["norm2_w"] = vec(get(p + "norm2", (E,)))
+        if cfg.canon_both:
+            L["canon2"] = vec(get(p + "canon2", (E, cfg.canon_taps)))
         if f.kind == FF_GLU:
             L["w_ff"], L["n_ff"] = mat(get(p + "mlp.gate", (f.ff, E)), get(p + "mlp.up", (f.ff, E))), 2 * f.ff
             L["w_dense_down"] = mat(get(p + "mlp.down", (E, f.ff)))
@@ -681,7 +726,7 @@ class StackWeights:
 
     @property
     def nbytes(self) -> int:
-        n = self.embed.numel() + self.head.numel() + (self.loop_in.numel() if self.loop_in is not None else 0)
+        n = self.embed.numel() + (0 if self.head is self.embed else self.head.numel()) + (self.loop_in.numel() if self.loop_in is not None else 0)
         for L in self.layers:
             n += sum(v.numel() for v in L.values() if isinstance(v, torch.Tensor) and v.dtype == self.dtype)
         return n * (2 if self.dtype == torch.bfloat16 else 4)

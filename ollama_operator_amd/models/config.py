@@ -250,20 +250,29 @@ MIX_LATENT = 2      # softmax attention whose keys and values come from one cach
 MIX_MLSTM = 3       # matrix memory with exponential input / forget gates and a running stabiliser
 MIX_MAMBA2 = 4      # selective state space layer (scalar decay per head) behind a short causal convolution
 MIX_GLA = 5         # gated linear attention: a state matrix whose rows (key channels) decay by a per-token vector
-STATE_MIXERS = (MIX_RETENTION, MIX_MLSTM, MIX_MAMBA2, MIX_GLA)   # mixers that own a per-sequence state slot
+MIX_LINEAR = 6      # linear attention with one constant decay per head, activated queries, keys and values and one norm
+                    # over all heads
+MIX_DELTA = 7       # gated delta rule: rows of the state decay by a per-token vector, a write takes off what the state
+                    # already answers to its key
+STATE_MIXERS = (MIX_RETENTION, MIX_MLSTM, MIX_MAMBA2, MIX_GLA, MIX_LINEAR, MIX_DELTA)   # mixers that own a per-sequence state slot
 
 BLOCK_PARALLEL = 0  # x <- x + m (mixer(LN(x)) + ff(LN(x))): one norm, both sublayers read it
 BLOCK_POSTNORM = 1  # x <- x + LN1(mixer(x)), then x <- x + LN2(ff(x)): the norm sits on the sublayer's output
 BLOCK_SANDWICH = 2  # x <- x + s1 N1b(mixer(conv_in(N1(x)))), then x <- x + s2 N2b(ff(N2(x))): scalar-weight RMS norms
                     # before and after each sublayer, per-channel scales on the results, a short causal convolution
                     # added to the mixer's input
-BLOCK_PRENORM = 3   # x <- x + mixer(N1(x)), then x <- x + ff(N2(x)): RMS norms with a weight vector on the sublayers' inputs
+BLOCK_PRENORM = 3   # x <- x + mixer(N1(x)), then x <- x + ff(N2(x)): RMS norms with a weight vector on the sublayers' inputs,
+                    # optionally with a short causal convolution added to what each sublayer reads
+CANON_FUSED_ROWS = 8  # a carried input window is a ring over positions with this many rows to spare, so that one launch
+                      # may read the old inputs and write the new ones of up to this many rows
 
 FF_MOE = 0          # routed experts (+ shared expert)
 FF_DENSE = 1        # W_down act(W_up h), act = relu(z)^2
 FF_GLU = 2          # W_down (act(W_gate h) * (W_up h)), act = the tanh form of gelu
 ACT_GELU_TANH = 0   # activation of a gated dense feed-forward (FF_GLU)
 ACT_RELU = 1
+ACT_SILU = 2             # (experts) silu(gate) * up
+ACT_CLAMPED_GLU = 3      # (experts) g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(1.702 g) (u + 1)
 ROUTE_TOPK_SOFTMAX = 0   # top-k of (logits + bias), softmax over the chosen logits
 ROUTE_SCORE_GROUPS = 1   # softmax over all outputs; choice by score + correction inside the best expert groups;
                          # weights = the chosen scores; trailing outputs may be identity experts
@@ -346,12 +355,16 @@ class MixerSpec:
     # gated linear attention
     tau: float = 1.0            # decay = sigmoid(z)^(1 / tau)
     decay_rank: int = 0         # inner size of the low-rank map that gives z (read from the tensor's shape)
+    gate_rank: int = 0          # delta rule: inner size of the low-rank map behind the output gate (from the tensor's shape)
     # a second mixer that reads the same input; the layer's result is left_scale * this + right_scale * right
     right: "MixerSpec | None" = None
     left_scale: float = 1.0
     right_scale: float = 1.0
     # attention options of the pre-norm block's mixers
     window: int = 0             # > 0: position i sees only j with 0 <= i - j < window
+    chunk: int = 0              # > 0: position i sees only j <= i of its own block of `chunk` positions (counted from 0)
+    alibi: bool = False         # score of head h loses 2^(-8 (h + 1) / heads) * (i - j)
+    v_unit: bool = False        # each head's value is divided by its root mean square
     maps: int = 1               # 2: differential attention, every head holds two query / key maps [map 1 | map 2] over the
                                 # same values; o = a1 - lambda a2, unit RMS per head, times (1 - diff)
     diff: float = 0.0           # lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff (learned vectors of size dim)
@@ -381,7 +394,9 @@ class MixerSpec:
         return self.n_out + (self.right.n_out if self.right is not None else 0)
 
     @property
-    def conv_channels(self) -> int:   # mamba2: x | B | C pass the convolution
+    def conv_channels(self) -> int:   # mamba2: x | B | C pass the convolution; delta rule: q | k | v
+        if self.kind == MIX_DELTA:
+            return 2 * self.kv_heads * self.dim + self.heads * self.vdim
         return self.heads * self.vdim + 2 * self.groups * self.state
 
     @property
@@ -391,7 +406,9 @@ class MixerSpec:
     @property
     def state_floats(self) -> int:
         """float32 words of the per-sequence state of one run of this mixer."""
-        if self.kind in (MIX_RETENTION, MIX_GLA):
+        if self.kind == MIX_DELTA:      # S [H][dim][vdim] | the convolution's last inputs (q | k | v)
+            return self.heads * self.dim * self.vdim + (self.conv - 1) * self.conv_channels
+        if self.kind in (MIX_RETENTION, MIX_GLA, MIX_LINEAR):
             return self.heads * self.dim * self.vdim
         if self.kind == MIX_MLSTM:      # S [H][dim][vdim] | n [H][dim] | m [H]
             return self.heads * (self.dim * self.vdim + self.dim + 1)
@@ -413,7 +430,11 @@ class MoESpec:
     group_keep: int = 1         # only experts of the best group_keep groups can be chosen
     shared_gate: bool = True    # the shared expert sits behind a scalar sigmoid gate
     act: int = ACT_GELU_TANH    # FF_GLU: the gate's activation
-    route_scale: float = 1.0    # ROUTE_SIGMOID_GROUPS: factor on the normalised weights
+    route_scale: float = 1.0    # ROUTE_SIGMOID_GROUPS: factor on the weights
+    route_norm: bool = True     # ROUTE_SIGMOID_GROUPS: the chosen scores are divided by their sum
+    expert_act: int = ACT_SILU
+    limit: float = 0.0          # ACT_CLAMPED_GLU
+    scale_input: bool = False   # a chosen expert's weight multiplies its input instead of its output
 
     @property
     def n_router(self) -> int:
@@ -441,8 +462,10 @@ class StackConfig:
     block: int = BLOCK_PARALLEL
     embed_scale: float = 1.0
     logit_scale: float = 1.0    # logits = head x * logit_scale
-    canon_taps: int = 1         # sandwich block: taps of the convolution added to the mixer's input (the last one is
-                                # the current token's; with 1 nothing is carried between tokens)
+    canon_taps: int = 1         # taps of the convolution added to the mixer's input (sandwich block, and pre-norm block with
+                                # canon_both; the last one is the current token's, with 1 nothing is carried)
+    tied_head: bool = False     # logits = embedding table x (no head matrix)
+    canon_both: bool = False    # pre-norm block: the inputs of both sublayers pass such a convolution
     ctx_len: int = 1 << 20      # the design has no positional table: bounded by the cache pool only
     bos_id: int = 0
     eos_id: int = -1            # no tokenizer ships with these models: generation never stops on a token
@@ -473,12 +496,20 @@ class StackConfig:
 
     def run_state_floats(self, li: int) -> int:
         """float32 words of the per-sequence state of one run of layer li: the mixer's (and its second mixer's) state
-        matrix, then, in a sandwich block, the last canon_taps - 1 inputs of the input convolution."""
+        matrix, then the input convolutions' windows: in a sandwich block the mixer's last canon_taps - 1 inputs, in a
+        pre-norm block with canon_both a ring of inputs for each sublayer."""
         m = self.layers[li].mixer
         n = m.state_floats + (m.right.state_floats if m.right is not None else 0)
         if self.block == BLOCK_SANDWICH:
             n += (self.canon_taps - 1) * self.n_embd
+        elif self.canon_both:
+            n += self.canon_ring * self.n_embd * (2 if self.layers[li].mlp is not None else 1)
         return n
+
+    @property
+    def canon_ring(self) -> int:
+        """Rows of a pre-norm block's carried input window: inputs of position p sit in row p % canon_ring."""
+        return self.canon_taps - 1 + CANON_FUSED_ROWS if self.canon_both and self.canon_taps > 1 else 0
 
     def to_dict(self) -> dict:
         return asdict(self)
@@ -853,7 +884,96 @@ class StackConfig:
             c["loop"] = dict(start=self.loop_start, stop=self.loop_stop, times=self.loop_times)
         return c
 
+    # -- config.json of the Rogisun design
+    @classmethod
+    def from_rogisun(cls, c: dict) -> "StackConfig":
+        def bad(msg):
+            raise UnsupportedArchitecture("Rogisun: " + msg)
+
+        layers = []
+        for ent in c["layers"]:
+            m, t = ent["mixer"], ent["type"]
+            if t == "lightning":
+                mx = MixerSpec(kind=MIX_LINEAR, heads=int(m["heads"]), kv_heads=int(m["heads"]), dim=int(m["dim"]),
+                               vdim=int(m.get("vdim", m["dim"])), decay=tuple(float(d) for d in m["decay"]), gate=GATE_ELEMENT)
+                if len(mx.decay) != mx.heads or not all(0.0 <= d <= 1.0 for d in mx.decay):
+                    bad("lightning: one decay in 0..1 per head expected")
+            elif t == "mamba2":
+                mx = MixerSpec(kind=MIX_MAMBA2, heads=int(m["heads"]), kv_heads=int(m.get("groups", 1)), dim=int(m["state"]),
+                               vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m.get("groups", 1)), conv=int(m["conv"]),
+                               norm_groups=int(m.get("norm_groups", 1)))
+                if mx.groups <= 0 or mx.heads % mx.groups:
+                    bad("heads must be a multiple of groups")
+                if mx.norm_groups <= 0 or (mx.heads * mx.vdim) % mx.norm_groups:
+                    bad("heads * vdim must be a multiple of norm_groups")
+            elif t == "parallel":
+                a, r = m["left"], m["right"]
+                mx = MixerSpec(kind=MIX_ATTENTION, heads=int(a["heads"]), kv_heads=int(a.get("kv_heads", a["heads"])),
+                               dim=int(a["dim"]), vdim=int(a.get("vdim", a["dim"])), scale=float(a["scale"]),
+                               chunk=int(a["mask"]["size"]), alibi=True, v_unit=True, gate=GATE_HEAD,
+                               left_scale=float(m["left_scale"]), right_scale=float(m["right_scale"]))
+                mx.right = MixerSpec(kind=MIX_DELTA, heads=int(r["heads"]), kv_heads=int(r.get("kv_heads", r["heads"])),
+                                     dim=int(r["dim"]), vdim=int(r.get("vdim", r["dim"])), conv=int(r["conv"]))
+                if mx.chunk <= 0:
+                    bad("mask.size must be positive")
+                for z in (mx, mx.right):
+                    if min(z.heads, z.kv_heads, z.dim, z.vdim) <= 0 or z.heads % z.kv_heads:
+                        bad("heads must be a positive multiple of kv_heads")
+                if mx.right.conv < 1:
+                    bad("conv must be at least 1")
+            else:
+                raise UnsupportedArchitecture(f"unknown mixer type {t!r}")
+            if min(mx.heads, mx.dim, mx.vdim) <= 0 or mx.conv < 1:
+                bad("mixer sizes must be positive")
+            mlp = None
+            f = ent.get("mlp")
+            if f:
+                if f.get("kind", "moe") != "moe":
+                    raise UnsupportedArchitecture(f"unknown feed-forward kind {f.get('kind')!r}")
+                r = f["router"]
+                mlp = MoESpec(kind=FF_MOE, route=ROUTE_SIGMOID_GROUPS, experts=int(r["experts"]), top=int(r["top"]),
+                              ff=int(f["expert"]["ff"]), shared_gate=False, route_norm=False, expert_act=ACT_CLAMPED_GLU,
+                              limit=float(f["expert"]["limit"]), scale_input=True)
+                if not 0 < mlp.top <= mlp.experts or mlp.ff <= 0:
+                    bad("router: top must be in 1..experts")
+                if mlp.limit <= 0:
+                    bad("expert.limit must be positive")
+            layers.append(LayerSpec(mixer=mx, mlp=mlp))
+        taps = int((c.get("canon") or {}).get("taps", 1))
+        if taps < 1:
+            bad("canon.taps must be at least 1")
+        return cls(arch="rogisun", n_vocab=int(c["vocab"]), n_embd=int(c["width"]), layers=layers,
+                   norm_eps=float(c["norm"]["eps"]), block=BLOCK_PRENORM, canon_taps=taps, canon_both=True, tied_head=True,
+                   name=str(c.get("name", "")))
+
+    def to_rogisun(self) -> dict:
+        """The config.json this configuration is read from (random-init fixtures, tests)."""
+        out = []
+        for s in self.layers:
+            m = s.mixer
+            if m.kind == MIX_LINEAR:
+                ent = dict(type="lightning", mixer=dict(heads=m.heads, dim=m.dim, vdim=m.vdim, decay=list(m.decay)))
+            elif m.kind == MIX_MAMBA2:
+                ent = dict(type="mamba2", mixer=dict(heads=m.heads, vdim=m.vdim, state=m.state, groups=m.groups, conv=m.conv,
+                                                     norm_groups=m.norm_groups))
+            elif m.kind == MIX_ATTENTION and m.right is not None and m.right.kind == MIX_DELTA:
+                r = m.right
+                ent = dict(type="parallel", mixer=dict(
+                    left=dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, scale=m.scale, mask=dict(size=m.chunk)),
+                    right=dict(heads=r.heads, kv_heads=r.kv_heads, dim=r.dim, vdim=r.vdim, conv=r.conv),
+                    left_scale=m.left_scale, right_scale=m.right_scale))
+            else:
+                raise UnsupportedArchitecture("Rogisun has no mixer of this kind")
+            f = s.mlp
+            ent["mlp"] = None if f is None else dict(kind="moe", expert=dict(ff=f.ff, limit=f.limit),
+                                                     router=dict(experts=f.experts, top=f.top))
+            out.append(ent)
+        return dict(architecture="Rogisun", vocab=self.n_vocab, width=self.n_embd, layers=out, norm=dict(eps=self.norm_eps),
+                    canon=dict(taps=self.canon_taps))
+
     def to_config_json(self) -> dict:
+        if self.arch == "rogisun":
+            return self.to_rogisun()
         if self.arch == "dekalorn":
             return self.to_dekalorn()
         if self.arch == "suvunex":
@@ -862,7 +982,7 @@ class StackConfig:
 
 
 STACK_ARCHS = {"Bizulix": StackConfig.from_bizulix, "Norevik": StackConfig.from_norevik, "Suvunex": StackConfig.from_suvunex,
-               "Dekalorn": StackConfig.from_dekalorn}
+               "Dekalorn": StackConfig.from_dekalorn, "Rogisun": StackConfig.from_rogisun}
 
 
 def is_stack_model(path: str) -> bool:

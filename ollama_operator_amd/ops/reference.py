@@ -487,20 +487,64 @@ def stack_rms_norm(x, w, eps):
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w
 
 
-def stack_attention_window(q, kc, vc, block_table, q_seq, q_len, bs, scale, window, k_off, v_head):
+def stack_canon_ring(hn, w, ring, pos, q_seq):
+    """hn [B, E] + causal per-channel convolution over each sequence's rows (w [E, taps], the last tap is the current
+    token's), continued from `ring` [slots, R, E], where the input of position p sits in row p % R; the rows' inputs
+    are written there in place. Nothing precedes position 0."""
+    K, R = w.shape[1], ring.shape[1]
+    out = hn.clone()
+    for b in range(hn.shape[0]):
+        st, p = ring[int(q_seq[b])], int(pos[b])
+        if K > 1:
+            st[p % R] = hn[b]
+        for back in range(K):
+            if back <= p:
+                out[b] += w[:, K - 1 - back] * (st[(p - back) % R] if back else hn[b])
+    return out
+
+
+def stack_delta_rule(q, k, v, decay, beta, S, q_seq):
+    """Per row: S [slots, H, D, Dv] <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q. q, k [B, G, D]
+    with head h using head h // (H / G), v [B, H, Dv], decay [B, H, D], beta [B, H]. Returns float32 [B, H, Dv]."""
+    B, H, _ = v.shape
+    out = torch.empty_like(v)
+    hg = torch.arange(H, device=v.device) // (H // k.shape[1])
+    for r in range(B):
+        St, kr = S[int(q_seq[r])], k[r][hg]
+        St.mul_(decay[r][:, :, None])
+        u = beta[r][:, None] * (v[r] - torch.einsum("hdv,hd->hv", St, kr))
+        St.add_(kr[:, :, None] * u[:, None, :])
+        out[r] = torch.einsum("hdv,hd->hv", St, q[r][hg])
+    return out
+
+
+def stack_expert_mid(gu, ff, act, limit, w=None):
+    """A routed expert's hidden activation from its gate | up products; w: the routing weight on the expert's input."""
+    if w is not None:
+        gu = gu * w
+    if act == 3:  # ACT_CLAMPED_GLU
+        g, u = torch.clamp(gu[:ff], max=limit), torch.clamp(gu[ff:], min=-limit, max=limit)
+        return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+    return F.silu(gu[:ff]) * gu[ff:]
+
+
+def stack_attention_window(q, kc, vc, block_table, q_seq, q_len, bs, scale, window, k_off, v_head, chunk=0, slopes=None):
     """q [B, Hq, D] float32. kc [blocks, Gk, bs, Wk]: query head h reads D elements at k_off[h] of the rows of key
     head h // (Hq // Gk); vc [blocks, Gv, bs, Dv]: it meets the values of head v_head[h]. Row b sees the keys
-    max(0, q_len[b] - window) .. q_len[b] - 1 of its sequence (window 0: all). Returns float32 [B, Hq, Dv]."""
+    max(0, q_len[b] - window) .. q_len[b] - 1 of its sequence (window 0: all), with `chunk` those of its own block of
+    `chunk` positions; slopes [Hq]: a score loses slope * distance. Returns float32 [B, Hq, Dv]."""
     B, Hq, D = q.shape
     Gk = kc.shape[1]
     out = torch.empty(B, Hq, vc.shape[-1], dtype=torch.float32, device=q.device)
     for b in range(B):
         n = int(q_len[b])
-        t = torch.arange(max(0, n - window) if window else 0, n, device=q.device)
+        t = torch.arange((n - 1) // chunk * chunk if chunk else max(0, n - window) if window else 0, n, device=q.device)
         bt = block_table[int(q_seq[b])].long()
         kk, vv = kc[bt[t // bs], :, t % bs].float(), vc[bt[t // bs], :, t % bs].float()   # [n, G, W]
         for h in range(Hq):
             s = (kk[:, h // (Hq // Gk), k_off[h]:k_off[h] + D] @ q[b, h]) * scale
+            if slopes is not None:
+                s = s - slopes[h] * (n - 1 - t)
             out[b, h] = torch.softmax(s, 0) @ vv[:, v_head[h]]
     return out
 
@@ -525,10 +569,10 @@ def stack_rotate_fold(q, k, pos, inv_freq, mix, groups):
     return qf.reshape(B, H, G * D), k
 
 
-def stack_route_sigmoid(z, top, group_count, group_keep, scale):
+def stack_route_sigmoid(z, top, group_count, group_keep, scale, norm=True):
     """Router logits [B, X] -> sigmoid scores; a group of neighbours ranks by the sum of its two largest scores and
-    only the best `group_keep` groups stay; the `top` largest scores among them (ties: the lower index), divided by
-    their sum (+ 1e-20), times `scale`. Returns expert ids [B, top] int32 and weights [B, top]."""
+    only the best `group_keep` groups stay; the `top` largest scores among them (ties: the lower index), with `norm`
+    divided by their sum (+ 1e-20), times `scale`. Returns expert ids [B, top] int32 and weights [B, top]."""
     s = torch.sigmoid(z)
     choice = s
     if group_count > 1:
@@ -539,7 +583,7 @@ def stack_route_sigmoid(z, top, group_count, group_keep, scale):
         choice = s.masked_fill(~ok.repeat_interleave(per, dim=1), -1.0)
     ids = torch.topk(choice, top, dim=-1).indices
     wt = torch.gather(s, 1, ids)
-    return ids.to(torch.int32), wt / (wt.sum(-1, keepdim=True) + 1e-20) * scale
+    return ids.to(torch.int32), (wt / (wt.sum(-1, keepdim=True) + 1e-20) if norm else wt) * scale
 
 
 class TorchStackExecutor:
@@ -652,19 +696,7 @@ class TorchStackExecutor:
             a = stack_group_rms(o.reshape(B, n_out), H, L["mnorm"], cfg.norm_eps, proj[:, off["g"]:off["g"] + n_out])
         else:
             assert m.kind == MIX_MAMBA2
-            st = r.states[ri]
-            N, G, ch = m.state, m.groups, m.conv_channels
-            nS = H * N * Dv
-            S, cst = st[:, :nS].view(-1, H, N, Dv), st[:, nS:].view(st.shape[0], m.conv - 1, ch)
-            xbc = stack_conv_silu(proj[:, off["conv"]:off["conv"] + ch], L["conv_w"].view(ch, m.conv), L["conv_b"], cst, qseq)
-            xs = xbc[:, :n_out].view(B, H, Dv)
-            Bm = xbc[:, n_out:n_out + G * N].view(B, G, N)
-            Cm = xbc[:, n_out + G * N:].view(B, G, N)
-            dt = F.softplus(proj[:, off["dt"]:off["dt"] + H] + L["dt_bias"])
-            ga = torch.exp(-torch.exp(L["a_log"]) * dt)
-            y = stack_gated_scan(Cm, Bm, xs, ga, dt, S, qseq, kv_group=H // G) + L["d_skip"][None, :, None] * xs
-            y = y.reshape(B, n_out) * F.silu(proj[:, off["g"]:off["g"] + n_out])
-            a = stack_group_rms(y, m.norm_groups, L["mnorm"], cfg.norm_eps)
+            a = self._mamba2(L, m, proj, r.states[ri], qseq)
         r.abuf[:B, :n_out] = a.to(T)
         r.ybuf[:B] = stack_matmul(r.abuf[:B, :n_out], L["w_o"])
         stack_post_norm_add(x, r.ybuf[:B], L["norm_w"], L["norm_b"], cfg.norm_eps)
@@ -698,10 +730,52 @@ class TorchStackExecutor:
         r.ybuf[:B] = y
         stack_post_norm_add(x, r.ybuf[:B], L["norm2_w"], L["norm2_b"], cfg.norm_eps, idw)
 
+    def _mamba2(self, L, m, proj, st, qseq):
+        """The state-space mixer up to its output projection; st [slots, state | the convolution's window]."""
+        B, H, Dv, N, G, ch, n_out, off = proj.shape[0], m.heads, m.vdim, m.state, m.groups, m.conv_channels, m.n_out, L["off"]
+        nS = H * N * Dv
+        S = st[:, :nS].view(-1, H, N, Dv)
+        cst = st[:, nS:nS + (m.conv - 1) * ch].view(st.shape[0], m.conv - 1, ch)
+        xbc = stack_conv_silu(proj[:, off["conv"]:off["conv"] + ch], L["conv_w"].view(ch, m.conv), L["conv_b"], cst, qseq)
+        xs = xbc[:, :n_out].view(B, H, Dv)
+        Bm = xbc[:, n_out:n_out + G * N].view(B, G, N)
+        Cm = xbc[:, n_out + G * N:].view(B, G, N)
+        dt = F.softplus(proj[:, off["dt"]:off["dt"] + H] + L["dt_bias"])
+        ga = torch.exp(-torch.exp(L["a_log"]) * dt)
+        y = stack_gated_scan(Cm, Bm, xs, ga, dt, S, qseq, kv_group=H // G) + L["d_skip"][None, :, None] * xs
+        y = y.reshape(B, n_out) * F.silu(proj[:, off["g"]:off["g"] + n_out])
+        return stack_group_rms(y, m.norm_groups, L["mnorm"], self.r.cfg.norm_eps)
+
+    def _linear(self, L, m, proj, st, qseq):
+        """Linear attention with constant decays and activated q, k, v, up to its output projection; st [slots, state]."""
+        B, H, D, Dv, off = proj.shape[0], m.heads, m.dim, m.vdim, L["off"]
+        q = F.silu(proj[:, off["q"]:off["q"] + H * D]).view(B, H, D)
+        k = F.silu(proj[:, off["k"]:off["k"] + H * D]).view(B, H, D)
+        v = F.silu(proj[:, off["v"]:off["v"] + H * Dv]).view(B, H, Dv)
+        S = st[:, :H * D * Dv].view(-1, H, D, Dv)
+        o = stack_gated_scan(q, k, v, L["decay"].expand(B, H), torch.ones(B, H), S, qseq)
+        return stack_group_rms(o.reshape(B, m.n_out), 1, L["mnorm"], self.r.cfg.norm_eps, proj[:, off["g"]:off["g"] + m.n_out])
+
+    def _delta(self, L, m, proj, st, qseq):
+        """The gated delta rule up to its output projection; st [slots, state | the convolution's window]."""
+        B, H, G, D, Dv, ch, off = proj.shape[0], m.heads, m.kv_heads, m.dim, m.vdim, m.conv_channels, L["off"]
+        nS, nq, eps = H * D * Dv, G * D, self.r.cfg.norm_eps
+        S = st[:, :nS].view(-1, H, D, Dv)
+        cst = st[:, nS:nS + (m.conv - 1) * ch].view(st.shape[0], m.conv - 1, ch)
+        x = stack_conv_silu(proj[:, off["rq"]:off["rq"] + ch], L["conv_w"].view(ch, m.conv), torch.zeros(ch), cst, qseq)
+        unit = lambda t: t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)  # noqa: E731
+        q, k = unit(x[:, :nq].view(B, G, D)) * float(D) ** -0.5, unit(x[:, nq:2 * nq].view(B, G, D))
+        v = x[:, 2 * nq:].view(B, H, Dv)
+        z = proj[:, off["a1"]:off["a1"] + m.decay_rank] @ L["a2"].float().T + L["dt_bias"]
+        decay = torch.exp(-torch.exp(L["a_log"])[None, :, None] * F.softplus(z).view(B, H, D))
+        o = stack_delta_rule(q, k, v, decay, torch.sigmoid(proj[:, off["rb"]:off["rb"] + H]), S, qseq)
+        o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * L["gnorm"]).reshape(B, H * Dv)
+        return o * torch.sigmoid(proj[:, off["g1"]:off["g1"] + m.gate_rank] @ L["g2"].float().T)
+
     def layer_run_prenorm(self, ri: int, B: int):
-        """x <- x + mixer(N1(x)), then x <- x + ff(N2(x)), N an RMS norm with a weight vector; a pass of a repeated span
-        opens with x <- W_in [x; x0]."""
-        from ..models.config import FF_GLU, MIX_LATENT
+        """x <- x + mixer(N1(x)), then x <- x + ff(N2(x)), N an RMS norm with a weight vector, optionally with a causal
+        convolution added to its result; a pass of a repeated span opens with x <- W_in [x; x0]."""
+        from ..models.config import FF_GLU, GATE_HEAD, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2
         r = self.r
         w, cfg, T = r.w, r.cfg, r.w.dtype
         li, _ps, opens = r.runs[ri]
@@ -715,10 +789,24 @@ class TorchStackExecutor:
         pos, qseq, qlen, bs = r.d_pos[:B], r.d_qseq[:B], r.d_qlen[:B], r.block_size
         slot = r.d_slot[:B].long()
         blk, o = slot // bs, slot % bs
-        r.hbuf[:B] = stack_rms_norm(x, L["norm_w"], eps).to(T)
+        E, taps, ring, st = x.shape[1], cfg.canon_taps, cfg.canon_ring, r.states[ri]
+        at = cfg.run_state_floats(li) - ring * E * (0 if not cfg.canon_both else 2 if f is not None else 1)
+
+        def canon(h, key, which):  # the sublayer's input convolution; its carried window is a ring behind the mixer's state
+            if not cfg.canon_both:
+                return h
+            win = (st[:, at + which * ring * E:at + (which + 1) * ring * E].view(-1, ring, E) if ring
+                   else torch.zeros(r.max_seqs, 1, E))
+            return stack_canon_ring(h, L[key].view(E, taps), win, pos, qseq)
+
+        r.hbuf[:B] = canon(stack_rms_norm(x, L["norm_w"], eps), "canon", 0).to(T)
         proj = stack_matmul(r.hbuf[:B], L["w_in"])
         r.proj[:B, :proj.shape[1]] = proj
-        if m.kind == MIX_LATENT:
+        if m.kind == MIX_MAMBA2:
+            a = self._mamba2(L, m, proj, st, qseq)
+        elif m.kind == MIX_LINEAR:
+            a = self._linear(L, m, proj, st, qseq)
+        elif m.kind == MIX_LATENT:
             C = m.kv_rank
             qa = stack_latent_prepare(proj, off, m, dict(L, inv_freq=L["inv_freq64"]), pos, r.d_slot[:B], r.kc[ri], bs, eps)
             lat = stack_latent_attention(qa, r.kc[ri], C, r.d_block_table, qseq, qlen, bs, m.scale,
@@ -729,23 +817,37 @@ class TorchStackExecutor:
         else:
             q = proj[:, off["q"]:off["q"] + m.n_q]
             k = proj[:, off["k"]:off["k"] + m.n_k]
-            r.vc[ri][blk, :, o] = proj[:, off["v"]:off["v"] + m.n_v].view(B, G, Dv).to(T)
+            v = proj[:, off["v"]:off["v"] + m.n_v].view(B, G, Dv)
+            if m.v_unit:
+                v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+            r.vc[ri][blk, :, o] = v.to(T)
             if m.maps == 2:  # two maps per head: the K pool's rows hold [map 1 | map 2] of a key/value head
                 r.kc[ri][blk, :, o] = k.view(B, G, 2 * D).to(T)
                 a2 = stack_attention_window(q.view(B, 2 * H, D), r.kc[ri], r.vc[ri], r.d_block_table, qseq, qlen, bs, m.scale,
                                             m.window, [(h % 2) * D for h in range(2 * H)], [h // 2 // (H // G) for h in range(2 * H)])
                 a = stack_diff_combine(a2.view(B, H, 2, Dv), L["lam"], m.diff, eps, proj[:, off["g"]:off["g"] + n_out])
+            elif not m.score_talk:
+                r.kc[ri][blk, :, o] = k.view(B, G, D).to(T)
+                a = stack_attention_window(q.view(B, H, D), r.kc[ri], r.vc[ri], r.d_block_table, qseq, qlen, bs, m.scale, m.window,
+                                           [0] * H, [h // (H // G) for h in range(H)], m.chunk, L.get("slopes"))
+                if m.gate == GATE_HEAD:
+                    a = a * torch.sigmoid(proj[:, off["g"]:off["g"] + H])[:, :, None]
+                a = a.reshape(B, n_out)
+                if m.right is not None:  # both mixers' outputs side by side, scaled, before one output projection
+                    ns = m.state_floats
+                    a = torch.cat([m.left_scale * a, m.right_scale * self._delta(L, m.right, proj, st[:, ns:], qseq)], 1)
             else:            # mixed scores: one K row per token holds every key/value head's key side by side
                 qf, kr = stack_rotate_fold(q.view(B, H, D), k.view(B, G, D), pos, L["inv_freq64"], L["talk"].view(H, H), H // G)
                 r.cbuf[:B, :H * G * D] = qf.reshape(B, H * G * D)
                 r.kc[ri][blk, 0, o] = kr.reshape(B, G * D).to(T)
                 a = stack_attention_window(qf, r.kc[ri], r.vc[ri], r.d_block_table, qseq, qlen, bs, m.scale, m.window,
                                            [0] * H, [h // (H // G) for h in range(H)]).reshape(B, n_out)
-        r.abuf[:B, :n_out] = a.to(T)
-        x += stack_matmul(r.abuf[:B, :n_out], L["w_o"])
+        n_all = m.n_out_all
+        r.abuf[:B, :n_all] = a.to(T)
+        x += stack_matmul(r.abuf[:B, :n_all], L["w_o"])
         if f is None:
             return
-        r.hbuf[:B] = stack_rms_norm(x, L["norm2_w"], eps).to(T)
+        r.hbuf[:B] = canon(stack_rms_norm(x, L["norm2_w"], eps), "canon2", 1).to(T)
         h = r.hbuf[:B]
         proj = stack_matmul(h, L["w_ff"])
         r.proj[:B, :proj.shape[1]] = proj
@@ -753,15 +855,15 @@ class TorchStackExecutor:
             r.hmid[:B, :f.ff] = (torch.relu(proj[:, :f.ff]) * proj[:, f.ff:2 * f.ff]).to(T)
             x += stack_matmul(r.hmid[:B, :f.ff], L["w_dense_down"])
             return
-        ids, wt = stack_route_sigmoid(proj[:, :f.experts], f.top, f.group_count, f.group_keep, f.route_scale)
+        ids, wt = stack_route_sigmoid(proj[:, :f.experts], f.top, f.group_count, f.group_keep, f.route_scale, f.route_norm)
         r.eids[:B, :f.top], r.ew[:B, :f.top] = ids, wt
         y = torch.zeros_like(x)
         for b in range(B):
             for j in range(f.top):
                 e = int(ids[b, j])
                 gu = stack_matmul(h[b:b + 1], L["w_gu"][e])[0]
-                mid = (F.silu(gu[:f.ff]) * gu[f.ff:]).to(T)
-                y[b] += wt[b, j] * stack_matmul(mid[None], L["w_down"][e])[0]
+                mid = stack_expert_mid(gu, f.ff, f.expert_act, f.limit, wt[b, j] if f.scale_input else None).to(T)
+                y[b] += (1.0 if f.scale_input else wt[b, j]) * stack_matmul(mid[None], L["w_down"][e])[0]
         x += y
 
     def layer_run_sandwich(self, ri: int, B: int):
