@@ -71,6 +71,8 @@ PYBIND11_MODULE(_stack, m) {
         e.cfg.embed_scale = getf(c, "embed_scale", 1.f);
         e.cfg.logit_scale = getf(c, "logit_scale", 1.f);
         e.cfg.canon_taps = geti(c, "canon_taps", 1);
+        e.cfg.canon_both = geti(c, "canon_both");
+        e.cfg.canon_ring = geti(c, "canon_ring");
       })
       .def("set_globals", [](StackExecutor& e, py::dict d) {
         e.embed_w = Pp<const void>(ptr(d, "embed"));
@@ -184,6 +186,20 @@ PYBIND11_MODULE(_stack, m) {
         L.gate = geti(d, "gate");
         L.score_talk = geti(d, "score_talk");
         L.route_scale = getf(d, "route_scale", 1.f);
+        L.chunk = geti(d, "chunk");
+        L.v_unit = geti(d, "v_unit");
+        L.slopes = Pp<const float>(ptr(d, "slopes"));
+        L.canon2 = Pp<const float>(ptr(d, "canon2"));
+        L.route_raw = geti(d, "route_raw");
+        L.expert_act = geti(d, "expert_act");
+        L.scale_input = geti(d, "scale_input");
+        L.limit = getf(d, "limit");
+        L.r_delta = geti(d, "r_delta");
+        L.r_kv_heads = geti(d, "r_kv_heads");
+        L.r_grank = geti(d, "r_grank");
+        L.off_rb = geti(d, "off_rb");
+        L.off_g1 = geti(d, "off_g1");
+        L.g2 = Pp<const void>(ptr(d, "g2"));
         if (L.qtemp_every <= 0) throw std::runtime_error("q_temp.every must be positive");
       })
       .def("set_runs", [](StackExecutor& e, std::vector<py::dict> runs) {
@@ -247,6 +263,15 @@ PYBIND11_MODULE(_stack, m) {
         w.hn = Pp<float>(ptr(d, "hn"));
         w.y2 = Pp<float>(ptr(d, "y2"));
         w.lna = w.coef;
+        w.dl_lg = Pp<float>(ptr(d, "dl_lg"));
+        w.ld_dl_lg = geti(d, "ld_dl_lg");
+        w.dl_gate = Pp<float>(ptr(d, "dl_gate"));
+        w.ld_dl_gate = geti(d, "ld_dl_gate");
+        w.dl_W = Pp<float>(ptr(d, "dl_W"));
+        w.dl_Kd = Pp<float>(ptr(d, "dl_Kd"));
+        w.dl_u = Pp<float>(ptr(d, "dl_u"));
+        w.dl_Bm = Pp<float>(ptr(d, "dl_Bm"));
+        w.dl_heads = geti(d, "dl_heads");
       })
       .def("set_inputs", [](StackExecutor& e, py::dict d) {
         StackInputs& in = e.in;

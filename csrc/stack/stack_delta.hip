@@ -1,0 +1,551 @@
+// Gated delta rule (interface: stack_ops.h): per head a float32 state S (D x Dv) whose rows (key channels) decay by a
+// per-token vector g; a write takes off what the state already answers to its key:
+//   S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t.
+// q, k and v come through one short causal convolution with silu; q and k are unit vectors per head (q also times
+// D^(-1/2)); g = exp(-exp(A_log) softplus(z)) with z from a low-rank map, the output gate from another one.
+//   delta_prepare_kernel  convolution, silu, unit vectors, log decays and the output gate of every row
+//   delta_walk_kernel     token by token, the state in registers (decode steps, and sizes the chunks do not take)
+//   delta_wy / scan / out prompt portions in chunks (see there)
+// Everything but the matrix operands is float32. Wave = 64 lanes.
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+#include <algorithm>
+
+#include "stack_device.h"
+#include "stack_ops.h"
+
+namespace omx {
+namespace stack {
+
+constexpr int DELTA_MAX = 256;       // key and value size of a head
+constexpr int DELTA_MAX_RANK = 1024;  // both low-rank maps together
+__device__ __forceinline__ float delta_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+// ------------------------------------------------------------------------------------------------ preparation
+// Grid (groups of RB rows, low-rank blocks then convolution blocks). A low-rank block takes 256 outputs (decay
+// channels, then gate channels): the rows' first factors sit in LDS, a thread reads its row of the second factor once
+// for all RB rows. A convolution block takes four head units (G query heads, G key heads, H value heads), one per
+// wave, four channels per lane. Inputs from before the step's first row of the sequence come from its carried window
+// (oldest first); a sequence with one row in the step advances its window here, the others in conv_window.
+template <typename T, int RB>
+__global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepRows R, int nlow) {
+  extern __shared__ float lds[];
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int r0 = blockIdx.x * RB, nr = min(RB, R.B - r0);
+  const int HD = P.H * P.D, HV = P.H * P.Dv, ra = P.rank_a, rg = P.rank_g;
+  if ((int)blockIdx.y < nlow) {
+    for (int i = tid; i < RB * (ra + rg); i += 256) {
+      const int r = i / (ra + rg), c = i % (ra + rg);
+      lds[i] = r < nr ? P.proj[(long long)(r0 + r) * P.ld + (c < ra ? P.off_a1 + c : P.off_g1 + c - ra)] : 0.f;
+    }
+    __syncthreads();
+    const int c = blockIdx.y * 256 + tid;
+    if (c >= HD + HV) return;
+    const bool dec = c < HD;
+    const int rank = dec ? ra : rg;
+    const T* w = dec ? (const T*)P.a2 + (long long)c * ra : (const T*)P.g2 + (long long)(c - HD) * rg;
+    const float* x = lds + (dec ? 0 : ra);
+    float z[RB];
+#pragma unroll
+    for (int r = 0; r < RB; ++r) z[r] = dec ? P.dt_bias[c] : 0.f;
+    int i = 0;
+    if (sizeof(T) == 2 && rank % 8 == 0 && (((uintptr_t)w) & 15) == 0) {
+      for (; i < rank; i += 8) {
+        const u32x4 a = *(const u32x4*)(w + i);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const float w0 = __uint_as_float(a[u] << 16), w1 = __uint_as_float(a[u] & 0xffff0000u);
+#pragma unroll
+          for (int r = 0; r < RB; ++r) z[r] += w0 * x[r * (ra + rg) + i + 2 * u] + w1 * x[r * (ra + rg) + i + 2 * u + 1];
+        }
+      }
+    }
+    for (; i < rank; ++i) {
+      const float w0 = ld(w + i);
+#pragma unroll
+      for (int r = 0; r < RB; ++r) z[r] += w0 * x[r * (ra + rg) + i];
+    }
+    const float ea = dec ? expf(P.a_log[c / P.D]) : 0.f;
+#pragma unroll
+    for (int r = 0; r < RB; ++r)
+      if (r < nr) {
+        if (dec)
+          P.lg[(long long)(r0 + r) * P.ld_lg + c] = -ea * delta_softplus(z[r]);
+        else
+          P.gate[(long long)(r0 + r) * P.ld_gate + c - HD] = sigmoidf(z[r]);
+      }
+    return;
+  }
+  const int unit = ((int)blockIdx.y - nlow) * 4 + wv;
+  if (unit >= 2 * P.G + P.H) return;
+  const bool isv = unit >= 2 * P.G, isq = unit < P.G;
+  const int n = isv ? P.Dv : P.D, K = P.taps;
+  const int c0 = isv ? 2 * P.G * P.D + (unit - 2 * P.G) * P.Dv : unit * P.D;  // first channel of the unit
+  const int ch = 2 * P.G * P.D + HV;
+  for (int rr = 0; rr < nr; ++rr) {
+    const int r = r0 + rr, seq = R.q_seq[r];
+    int nb = 0;  // rows of the same sequence right before r, up to taps - 1
+    while (nb < K - 1 && r - nb - 1 >= 0 && R.q_seq[r - nb - 1] == seq) ++nb;
+    const bool alone = nb == 0 && !(r + 1 < R.B && R.q_seq[r + 1] == seq);
+    float* win = P.window + (long long)seq * P.state_stride;
+    float v[DELTA_MAX / 64], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < DELTA_MAX / 64; ++u) {
+      const int d = lane + 64 * u;
+      v[u] = 0.f;
+      if (d < n) {
+        const int c = c0 + d;
+        const float cur = P.proj[(long long)r * P.ld + P.off_q + c];
+        float acc = 0.f;
+        for (int j = 0; j < K; ++j) {
+          const int back = K - 1 - j;
+          const float in = back == 0 ? cur : back <= nb ? P.proj[(long long)(r - back) * P.ld + P.off_q + c]
+                                                        : win[(long long)(K - 1 - (back - nb)) * ch + c];
+          acc += P.conv_w[(long long)c * K + j] * in;
+          if (alone && back > 0) win[(long long)(K - 1 - back) * ch + c] = back == 1 ? cur : win[(long long)(K - back) * ch + c];
+        }
+        v[u] = silu(acc);
+        ss += v[u] * v[u];
+      }
+    }
+    float f = 1.f;
+    if (!isv) f = (isq ? 1.f / sqrtf((float)P.D) : 1.f) / sqrtf(wave_sum(ss) + 1e-6f);
+#pragma unroll
+    for (int u = 0; u < DELTA_MAX / 64; ++u) {
+      const int d = lane + 64 * u;
+      if (d < n) P.x[(long long)r * P.ld_x + c0 + d] = v[u] * f;
+    }
+  }
+}
+template <typename T>
+static void launch_delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
+  const int nlow = (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + 3) / 4;
+  const int rank = P.rank_a + P.rank_g;
+  if (R.B <= 16)
+    hipLaunchKernelGGL((delta_prepare_kernel<T, 1>), dim3(R.B, nlow + nconv), dim3(256), rank * 4, s, P, R, nlow);
+  else
+    hipLaunchKernelGGL((delta_prepare_kernel<T, 8>), dim3((R.B + 7) / 8, nlow + nconv), dim3(256), 8 * rank * 4, s, P, R, nlow);
+}
+bool delta_supported(int D, int Dv, int rank_a, int rank_g) {
+  return D > 0 && Dv > 0 && D <= DELTA_MAX && Dv <= DELTA_MAX && rank_a > 0 && rank_g > 0 && rank_a + rank_g <= DELTA_MAX_RANK;
+}
+static void check_delta(const DeltaParams& P, const StepRows& R) {
+  check(R.B > 0 && P.proj && P.conv_w && P.a2 && P.g2 && P.a_log && P.dt_bias && P.norm_w && P.state && P.out && P.x && P.lg && P.gate &&
+            P.G > 0 && P.H % P.G == 0 && P.taps >= 1 && (P.taps == 1 || P.window) && delta_supported(P.D, P.Dv, P.rank_a, P.rank_g) &&
+            P.ld_x >= 2 * P.G * P.D + P.H * P.Dv && P.ld_lg >= P.H * P.D && P.ld_gate >= P.H * P.Dv && P.ld_out >= P.H * P.Dv,
+        "gated delta rule: operands or head sizes (key and value size <= 256)");
+}
+void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
+  check_delta(P, R);
+  if (P.f32)
+    launch_delta_prepare<float>(P, R, s);
+  else
+    launch_delta_prepare<bf16>(P, R, s);
+  launched("delta_prepare");
+  ConvParams C{P.proj, P.ld, P.off_q, 2 * P.G * P.D + P.H * P.Dv, P.taps, P.conv_w, nullptr, P.window, P.state_stride, nullptr, 0};
+  conv_window(C, R, s);
+}
+
+// ------------------------------------------------------------------------------------------------ token by token
+// One block per (sequence segment of the step, head), as the other recurrences: the block of the segment's first row
+// walks its rows; thread (g, j) = (tid / Dv, tid % Dv) keeps S[i][j], i = g, g + NG, ..., in registers. The head's RMS
+// norm, its weight and the gate finish the row.
+template <typename T, int MAXI, int NT>
+__global__ __launch_bounds__(NT) void delta_walk_kernel(DeltaParams P, StepRows R) {
+  __shared__ float qs[DELTA_MAX], ks[DELTA_MAX], gs[DELTA_MAX], us[DELTA_MAX], po[NT], red[4];
+  const int r0 = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  const int seq = R.q_seq[r0];
+  if (r0 > 0 && R.q_seq[r0 - 1] == seq) return;  // not the first row of its segment (uniform per block)
+  const int D = P.D, Dv = P.Dv, hg = h / (P.H / P.G);
+  const int NG = NT / Dv;
+  const int g = tid / Dv, j = tid % Dv;
+  const bool act = g < NG;
+  float* S0 = P.state + (long long)seq * P.state_stride + (long long)h * D * Dv;
+  float S[MAXI];
+#pragma unroll
+  for (int ii = 0; ii < MAXI; ++ii) {
+    const int i = g + ii * NG;
+    S[ii] = (act && i < D) ? S0[(long long)i * Dv + j] : 0.f;
+  }
+  for (int r = r0; r < R.B && R.q_seq[r] == seq; ++r) {
+    const float* x = P.x + (long long)r * P.ld_x;
+    if (tid < D) {
+      qs[tid] = x[hg * D + tid];
+      ks[tid] = x[P.G * D + hg * D + tid];
+      gs[tid] = expf(P.lg[(long long)r * P.ld_lg + h * D + tid]);
+    }
+    const float v = tid < Dv ? x[2 * P.G * D + h * Dv + tid] : 0.f;
+    const float beta = sigmoidf(P.proj[(long long)r * P.ld + P.off_b + h]);
+    const float gate = tid < Dv ? P.gate[(long long)r * P.ld_gate + h * Dv + tid] : 0.f;
+    __syncthreads();
+    float part = 0.f;
+    if (act) {
+#pragma unroll
+      for (int ii = 0; ii < MAXI; ++ii) {
+        const int i = g + ii * NG;
+        if (i < D) {
+          S[ii] *= gs[i];
+          part += S[ii] * ks[i];
+        }
+      }
+    }
+    po[tid] = part;
+    __syncthreads();
+    if (tid < Dv) {
+      float a = 0.f;
+      for (int gg = 0; gg < NG; ++gg) a += po[gg * Dv + tid];
+      us[tid] = beta * (v - a);
+    }
+    __syncthreads();
+    part = 0.f;
+    if (act) {
+      const float u = us[j];
+#pragma unroll
+      for (int ii = 0; ii < MAXI; ++ii) {
+        const int i = g + ii * NG;
+        if (i < D) {
+          S[ii] += ks[i] * u;
+          part += S[ii] * qs[i];
+        }
+      }
+    }
+    po[tid] = part;
+    __syncthreads();
+    float o = 0.f;
+    if (tid < Dv)
+      for (int gg = 0; gg < NG; ++gg) o += po[gg * Dv + tid];
+    if (tid < 256) {
+      const float w = wave_sum(o * o);
+      if ((tid & 63) == 0) red[tid >> 6] = w;
+    }
+    __syncthreads();
+    if (tid < Dv) {
+      const float ms = (red[0] + red[1] + red[2] + red[3]) / (float)Dv;
+      st((T*)P.out + (long long)r * P.ld_out + h * Dv + tid, o / sqrtf(ms + P.eps) * P.norm_w[tid] * gate * P.out_scale);
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int ii = 0; ii < MAXI; ++ii) {
+    const int i = g + ii * NG;
+    if (act && i < D) S0[(long long)i * Dv + j] = S[ii];
+  }
+}
+template <typename T>
+static void launch_delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s) {
+  const dim3 grid(R.B, P.H);
+  const int ng = 1024 / P.Dv, ni = (P.D + ng - 1) / ng;
+  if (P.D * P.Dv <= 2048 && (P.D + 256 / P.Dv - 1) / (256 / P.Dv) <= 8)
+    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 256>), grid, dim3(256), 0, s, P, R);
+  else if (ni <= 4)
+    hipLaunchKernelGGL((delta_walk_kernel<T, 4, 1024>), grid, dim3(1024), 0, s, P, R);
+  else if (ni <= 8)
+    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 1024>), grid, dim3(1024), 0, s, P, R);
+  else if (ni <= 16)
+    hipLaunchKernelGGL((delta_walk_kernel<T, 16, 1024>), grid, dim3(1024), 0, s, P, R);
+  else if (ni <= 32)
+    hipLaunchKernelGGL((delta_walk_kernel<T, 32, 1024>), grid, dim3(1024), 0, s, P, R);
+  else
+    hipLaunchKernelGGL((delta_walk_kernel<T, 64, 1024>), grid, dim3(1024), 0, s, P, R);
+}
+void delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s) {
+  check_delta(P, R);
+  if (P.f32)
+    launch_delta_walk<float>(P, R, s);
+  else
+    launch_delta_walk<bf16>(P, R, s);
+  launched("delta_walk");
+}
+
+// ------------------------------------------------------------------------------------------------ prompt portions
+// Chunks of DC tokens over the host-built chunk table {first row, rows, state slot, flags}. With l_s = ln g_s (a
+// vector over the key channels), L_t = l_0 + ... + l_t inside a chunk of n tokens that starts from state S,
+//   A[t][s] = beta_t sum_d k_t[d] k_s[d] exp(L_t[d] - L_s[d])  (s < t),   B[t][s] = the same with q_t, no beta (s <= t),
+//   u_t = beta_t v_t - beta_t S^T (k_t exp(L_t)) - sum_(s < t) A[t][s] u_s,
+// so (I + A) u = beta v - (beta k exp(L)) S: one forward substitution over the columns of both right-hand sides gives
+// u = V' - W S with V', W free of the state. Then
+//   o_t = S^T (q_t exp(L_t)) + sum_(s <= t) B[t][s] u_s,      S <- diag(exp(L_(n-1))) S + sum_s (k_s exp(L_(n-1) - L_s)) u_s^T.
+// Every exponent is <= 0. Float32 throughout; the products over the state on v_mfma_f32_16x16x4_f32 (true float32).
+//   delta_wy_kernel    (chunk, head): L (over the log decays), A, B, V' (into u), W, the keys decayed to the chunk's end
+//   delta_scan_kernel  (sequence, head, 16 value columns): walks the chunks, u = V' - W S, every chunk's incoming state
+//   delta_out_kernel   (chunk, head): the outputs, their norm and gate
+constexpr int DC = 32;
+constexpr int DELTA_CD = 128;  // largest key size of the chunked form
+int delta_chunk_rows() { return DC; }
+bool delta_chunk_supported(int D, int Dv) { return D > 0 && D <= DELTA_CD && Dv > 0 && Dv <= DELTA_MAX; }
+static inline size_t delta_wy_lds(int D) { return (size_t)(3 * DC * (D + 1) + DC * (DC + 4) + DC) * sizeof(float); }
+
+__global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunkWs W) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  const int r0 = W.chunks[4 * c], n = W.chunks[4 * c + 1];
+  const int D = P.D, Dv = P.Dv, D1 = D + 1, hg = h / (P.H / P.G);
+  constexpr int LA = DC + 4;       // rows of A 16-byte aligned
+  float* A = lds;                  // [DC][DC + 4]
+  float* qs = A + DC * LA;         // [DC][D + 1]
+  float* ks = qs + DC * D1;
+  float* Lc = ks + DC * D1;
+  float* be = Lc + DC * D1;        // [DC]
+  for (int i = tid; i < DC * D; i += 256) {
+    const int t = i / D, d = i % D;
+    const long long r = r0 + t;
+    const bool on = t < n;
+    qs[t * D1 + d] = on ? P.x[r * P.ld_x + hg * D + d] : 0.f;
+    ks[t * D1 + d] = on ? P.x[r * P.ld_x + (P.G + hg) * D + d] : 0.f;
+    Lc[t * D1 + d] = on ? P.lg[r * P.ld_lg + h * D + d] : 0.f;
+  }
+  if (tid < DC) be[tid] = tid < n ? sigmoidf(P.proj[(long long)(r0 + tid) * P.ld + P.off_b + h]) : 0.f;
+  __syncthreads();
+  for (int d = tid; d < D; d += 256) {
+    float acc = 0.f;
+    for (int t = 0; t < DC; ++t) {
+      acc += Lc[t * D1 + d];
+      Lc[t * D1 + d] = acc;
+      if (t < n) P.lg[(long long)(r0 + t) * P.ld_lg + h * D + d] = acc;  // the running log decays replace the log decays
+    }
+  }
+  __syncthreads();
+  for (int p = tid; p < DC * DC; p += 256) {
+    const int t = p / DC, sx = p % DC;
+    float a = 0.f, b = 0.f;
+    if (sx <= t && t < n) {
+      for (int d = 0; d < D; ++d) {  // exponents <= 0; exp2 on the transcendental unit (1 ulp)
+        const float e = ks[sx * D1 + d] * __builtin_amdgcn_exp2f((Lc[t * D1 + d] - Lc[sx * D1 + d]) * 1.44269504088896341f);
+        a += ks[t * D1 + d] * e;
+        b += qs[t * D1 + d] * e;
+      }
+    }
+    A[t * LA + sx] = sx < t ? be[t] * a : 0.f;
+    if (t < n) W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] = b;
+  }
+  for (int i = tid; i < n * D; i += 256) {  // keys decayed to the end of the chunk
+    const int t = i / D, d = i % D;
+    W.Kd[(long long)(r0 + t) * P.ld_lg + h * D + d] = ks[t * D1 + d] * expf(Lc[(n - 1) * D1 + d] - Lc[t * D1 + d]);
+  }
+  __syncthreads();
+  for (int col = tid; col < D + Dv; col += 256) {  // forward substitution, a column per thread
+    const bool key = col < D;
+    float x[DC];
+#pragma unroll
+    for (int t = 0; t < DC; ++t) {
+      float v = 0.f;
+      if (t < n)
+        v = be[t] * (key ? ks[t * D1 + col] * expf(Lc[t * D1 + col])
+                         : P.x[(long long)(r0 + t) * P.ld_x + 2 * P.G * D + h * Dv + col - D]);
+      x[t] = v;
+    }
+#pragma unroll
+    for (int t = 1; t < DC; ++t) {
+#pragma unroll
+      for (int s4 = 0; s4 < (t + 3) / 4; ++s4) {
+        const f32x4 a = *(const f32x4*)&A[t * LA + 4 * s4];  // zero from the diagonal on
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (4 * s4 + i < t) x[t] -= a[i] * x[4 * s4 + i];
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < DC; ++t)
+      if (t < n) {
+        if (key)
+          W.W[(long long)(r0 + t) * P.ld_lg + h * D + col] = x[t];
+        else
+          W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + col - D] = x[t];
+      }
+  }
+}
+
+// Four waves share the state's rows: wave w holds the 16-row tiles w and w + 4 of S (16 columns) in accumulator layout,
+// S[16 tile + 4 (lane / 16) + i][lane % 16]. In that layout a register is a B operand of the first product if its K
+// order is d = 4 (lane / 16) + i, so W's rows are read four consecutive channels per lane and the state never moves.
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams P, DeltaChunkWs W) {
+  __shared__ float part[4][DC][17];
+  __shared__ float us[DC][17];
+  const int c0 = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  if (!(W.chunks[4 * c0 + 3] & 1)) return;  // not the first chunk of its sequence (uniform per block)
+  const int D = P.D, Dv = P.Dv, m = lane & 15, q4 = lane >> 4;
+  const int col = blockIdx.z * 16 + m;
+  const bool cok = col < Dv;
+  const int slot = W.chunks[4 * c0 + 2];
+  float* S0 = P.state + (long long)slot * P.state_stride + (long long)h * D * Dv;
+  f32x4 S[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
+      S[j][i] = (cok && d < D) ? S0[(long long)d * Dv + col] : 0.f;
+    }
+  for (int c = c0;; ++c) {
+    const int r0 = W.chunks[4 * c], n = W.chunks[4 * c + 1], flags = W.chunks[4 * c + 3];
+    float* Sin = W.Sin + (long long)c * W.s_stride + (long long)h * D * Dv;
+    // operands of both products, requested together
+    float wa[2][2][4], kd[2][8], vp[2];
+    f32x4 el[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int dt = 16 * (wv + 4 * j);
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) {
+        const int t = 16 * mt + m;
+        const float* wr = W.W + (long long)(r0 + t) * P.ld_lg + h * D + dt + 4 * q4;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) wa[j][mt][i] = (t < n && dt + 4 * q4 + i < D) ? wr[i] : 0.f;
+      }
+#pragma unroll
+      for (int kk = 0; kk < 8; ++kk) {
+        const int t = 4 * kk + q4;
+        kd[j][kk] = (t < n && dt + m < D) ? W.Kd[(long long)(r0 + t) * P.ld_lg + h * D + dt + m] : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = dt + 4 * q4 + i;
+        el[j][i] = d < D ? P.lg[(long long)(r0 + n - 1) * P.ld_lg + h * D + d] : 0.f;
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int e = tid + 256 * k, t = e >> 4, cc = blockIdx.z * 16 + (e & 15);
+      vp[k] = (t < n && cc < Dv) ? W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + cc] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
+        if (cok && d < D) Sin[(long long)d * Dv + col] = S[j][i];
+      }
+    f32x4 acc[2];
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt) {
+      acc[mt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wa[j][mt][i], S[j][i], acc[mt], 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) part[wv][16 * mt + 4 * q4 + i][m] = acc[mt][i];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int e = tid + 256 * k, t = e >> 4, cm = e & 15, cc = blockIdx.z * 16 + cm;
+      const float u = vp[k] - (part[0][t][cm] + part[1][t][cm] + part[2][t][cm] + part[3][t][cm]);
+      us[t][cm] = u;  // rows past the chunk's end: 0 - 0
+      if (t < n && cc < Dv) W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + cc] = u;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) S[j][i] *= expf(el[j][i]);
+#pragma unroll
+      for (int kk = 0; kk < 8; ++kk) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[j][kk], us[4 * kk + q4][m], S[j], 0, 0, 0);
+    }
+    if (flags & 2) break;  // the sequence's last chunk of the step
+  }
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
+      if (cok && d < D) S0[(long long)d * Dv + col] = S[j][i];
+    }
+}
+
+static inline size_t delta_out_lds(int D, int Dv) {
+  const int Dp = (D + 15) / 16 * 16;
+  return (size_t)(DC * (Dp + 4) + DC * (DC + 4) + DC * (Dv + 1)) * sizeof(float);
+}
+template <typename T>
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams P, DeltaChunkWs W) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int r0 = W.chunks[4 * c], n = W.chunks[4 * c + 1];
+  const int D = P.D, Dv = P.Dv, hg = h / (P.H / P.G), Dp = (D + 15) / 16 * 16, LQ = Dp + 4, V1 = Dv + 1;
+  constexpr int LB = DC + 4;
+  float* qd = lds;             // [DC][Dp + 4]
+  float* Bs = qd + DC * LQ;    // [DC][DC + 4]
+  float* ob = Bs + DC * LB;    // [DC][Dv + 1]
+  for (int i = tid; i < DC * Dp; i += 256) {
+    const int t = i / Dp, d = i % Dp;
+    const long long r = r0 + t;
+    qd[t * LQ + d] = (t < n && d < D) ? P.x[r * P.ld_x + hg * D + d] * expf(P.lg[r * P.ld_lg + h * D + d]) : 0.f;
+  }
+  for (int i = tid; i < DC * DC; i += 256) {
+    const int t = i / DC, sx = i % DC;
+    Bs[t * LB + sx] = t < n ? W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] : 0.f;
+  }
+  __syncthreads();
+  const float* Sin = W.Sin + (long long)c * W.s_stride + (long long)h * D * Dv;
+  const int m = lane & 15, q4 = lane >> 4;
+  for (int ct = wv; ct * 16 < Dv; ct += 4) {
+    const int col = ct * 16 + m;
+    const bool cok = col < Dv;
+    f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+    for (int d0 = 0; d0 < Dp; d0 += 16) {
+      float b[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = d0 + 4 * q4 + i;
+        b[i] = (cok && d < D) ? Sin[(long long)d * Dv + col] : 0.f;
+      }
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) {
+        const f32x4 a = *(const f32x4*)&qd[(16 * mt + m) * LQ + d0 + 4 * q4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], acc[mt], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int s0 = 0; s0 < DC; s0 += 16) {
+      float b[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int sx = s0 + 4 * q4 + i;
+        b[i] = (cok && sx < n) ? W.u[(long long)(r0 + sx) * P.ld_gate + h * Dv + col] : 0.f;
+      }
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) {
+        const f32x4 a = *(const f32x4*)&Bs[(16 * mt + m) * LB + s0 + 4 * q4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], acc[mt], 0, 0, 0);
+      }
+    }
+    if (cok) {
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) ob[(16 * mt + 4 * q4 + i) * V1 + col] = acc[mt][i];
+    }
+  }
+  __syncthreads();
+  for (int t = wv; t < n; t += 4) {  // a wave per row: the head's RMS norm, its weight, the gate
+    float ss = 0.f;
+    for (int d = lane; d < Dv; d += 64) ss += ob[t * V1 + d] * ob[t * V1 + d];
+    const float f = P.out_scale / sqrtf(wave_sum(ss) / (float)Dv + P.eps);
+    for (int d = lane; d < Dv; d += 64)
+      st((T*)P.out + (long long)(r0 + t) * P.ld_out + h * Dv + d,
+         ob[t * V1 + d] * f * P.norm_w[d] * P.gate[(long long)(r0 + t) * P.ld_gate + h * Dv + d]);
+  }
+}
+void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& W, hipStream_t s) {
+  check_delta(P, R);
+  check(delta_chunk_supported(P.D, P.Dv) && W.chunks && W.nchunks > 0 && W.nchunks <= W.max_chunks && W.Sin && W.W && W.Kd && W.u && W.Bm &&
+            W.s_stride >= (long long)P.H * P.D * P.Dv,
+        "chunked gated delta rule: operands (key size <= 128)");
+  const dim3 grid(W.nchunks, P.H);
+  hipLaunchKernelGGL(delta_wy_kernel, grid, dim3(256), delta_wy_lds(P.D), s, P, W);
+  launched("delta_wy");
+  hipLaunchKernelGGL(delta_scan_kernel, dim3(W.nchunks, P.H, (P.Dv + 15) / 16), dim3(256), 0, s, P, W);
+  launched("delta_scan");
+  if (P.f32)
+    hipLaunchKernelGGL(delta_out_kernel<float>, grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
+  else
+    hipLaunchKernelGGL(delta_out_kernel<bf16>, grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
+  launched("delta_out");
+}
+
+}  // namespace stack
+}  // namespace omx

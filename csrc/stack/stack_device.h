@@ -64,6 +64,17 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
 __device__ __forceinline__ float silu(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
 
+// hidden unit of a routed expert from its gate and up products; w: the weight on the expert's input (1 without P.w_input)
+__device__ __forceinline__ float moe_unit(int act, float limit, float w, float gate, float up) {
+  gate *= w;
+  up *= w;
+  if (act == 1 /* MOE_ACT_CLAMPED */) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g * sigmoidf(1.702f * g) * (u + 1.f);
+  }
+  return silu(gate) * up;
+}
+
 static inline void check(bool ok, const char* what) {
   if (!ok) throw std::runtime_error(std::string("stack kernels: ") + what);
 }

@@ -10,6 +10,16 @@ static void need(bool ok, const std::string& what) {
   if (!ok) throw std::runtime_error("stack executor: " + what);
 }
 
+static void validate_mamba2(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
+  const StackWorkspace& ws = e.ws;
+  need(ws.ret.ld_o >= L.heads * L.vdim && ws.ret.obuf, "mixer output wider than its float32 buffer");
+  need(r.state && L.conv_w && L.conv_b && L.dt_bias && L.a_log && L.d_skip && L.mnorm && ws.cbuf, "Mamba-2 operands");
+  need(gated_scan_supported(SCAN_SSD, L.state, L.vdim), "Mamba-2 head sizes (state <= 256, vdim <= 256)");
+  const long long ch = (long long)L.heads * L.vdim + 2LL * L.groups * L.state;
+  need(ch <= ws.ld_cbuf && L.groups > 0 && L.heads % L.groups == 0 && L.conv >= 1, "Mamba-2 convolution sizes");
+  need(r.state_stride >= (long long)L.heads * L.state * L.vdim + (L.conv - 1) * ch, "Mamba-2 state slot too small");
+  need(L.norm_groups > 0 && (L.heads * L.vdim) % L.norm_groups == 0, "Mamba-2 norm groups");
+}
 static void validate_postnorm(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
   const StackWorkspace& ws = e.ws;
   need(L.kind >= 2 && L.kind <= 4, "a layer with output norms needs a latent attention, mLSTM or Mamba-2 mixer");
@@ -25,12 +35,7 @@ static void validate_postnorm(const StackExecutor& e, const RunDesc& r, const La
     need(gated_scan_supported(SCAN_MLSTM, L.dim, L.vdim), "mLSTM head sizes (dim <= 256, vdim <= 255, dim * (vdim + 1) <= 16384)");
     need(r.state_stride >= (long long)L.heads * (L.dim * L.vdim + L.dim + 1), "mLSTM state slot too small");
   } else {
-    need(r.state && L.conv_w && L.conv_b && L.dt_bias && L.a_log && L.d_skip && L.mnorm && ws.cbuf, "Mamba-2 operands");
-    need(gated_scan_supported(SCAN_SSD, L.state, L.vdim), "Mamba-2 head sizes (state <= 256, vdim <= 256, state * vdim <= 16384)");
-    const long long ch = (long long)L.heads * L.vdim + 2LL * L.groups * L.state;
-    need(ch <= ws.ld_cbuf && L.groups > 0 && L.heads % L.groups == 0 && L.conv >= 1, "Mamba-2 convolution sizes");
-    need(r.state_stride >= (long long)L.heads * L.state * L.vdim + (L.conv - 1) * ch, "Mamba-2 state slot too small");
-    need(L.norm_groups > 0 && (L.heads * L.vdim) % L.norm_groups == 0, "Mamba-2 norm groups");
+    validate_mamba2(e, r, L);
   }
   if (L.ff_dense) {
     need(L.w_ff && L.w_dense_down && L.norm2_w && L.norm2_b && L.ff > 0 && L.ff <= ws.ld_hmid && L.ff <= ws.ld_proj && ws.hmid,
@@ -71,12 +76,42 @@ static void validate_sandwich(const StackExecutor& e, const RunDesc& r, const La
          "gated feed-forward operands");
 }
 
+static long long prenorm_state_floats(const LayerDesc& L) {  // the mixers' part of a slot; the input windows follow
+  if (L.kind == 4)
+    return (long long)L.heads * L.state * L.vdim + (long long)(L.conv - 1) * (L.heads * L.vdim + 2 * L.groups * L.state);
+  if (L.kind == 6) return (long long)L.heads * L.dim * L.vdim;
+  if (L.r_delta)
+    return (long long)L.r_heads * L.r_dim * L.r_vdim + (long long)(L.conv - 1) * (2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim);
+  return 0;
+}
 static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
   const StackWorkspace& ws = e.ws;
   need(L.norm_w && L.w_in && L.w_o && L.n_in > 0 && L.n_in <= ws.ld_proj, "layer weights missing");
   need(L.heads * L.vdim <= ws.ld_a, "mixer output wider than its buffer");
   if (r.opens_pass) need(e.loop_in && ws.cat, "the pass-opening projection is missing");
-  if (L.kind == 2) {
+  if (e.cfg.canon_both) {
+    const long long ring = e.cfg.canon_ring, taps = e.cfg.canon_taps;
+    need(taps >= 1 && taps <= CANON_MAX_TAPS && (taps == 1 || ring >= taps) && L.canon && ws.hn && (!L.experts || L.canon2),
+         "input convolution (1..8 taps) operands");
+    need(r.state_stride >= prenorm_state_floats(L) + ring * e.cfg.E * (L.experts || L.ff_dense ? 2 : 1) && (r.state || r.state_stride == 0),
+         "state slot too small");
+  }
+  if (L.kind == 4) {
+    validate_mamba2(e, r, L);
+  } else if (L.kind == 6) {
+    need(r.state && L.decay && L.mnorm && ws.ret.obuf && ws.ret.ld_o >= L.heads * L.vdim, "constant-decay linear attention operands");
+    need(gated_scan_supported(SCAN_FIXED, L.dim, L.vdim), "constant-decay linear attention head sizes (<= 256)");
+  } else if (L.r_delta) {
+    need(r.kc && r.vc && r.state && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= 256 && L.vdim <= 256 && L.chunk >= 0,
+         "attention sizes (<= 256)");
+    need(L.heads * L.vdim + L.r_heads * L.r_vdim <= ws.ld_a, "mixer output wider than its buffer");
+    need(L.conv_w && L.a2 && L.g2 && L.a_log && L.dt_bias && L.gnorm && ws.cbuf && ws.dl_lg && ws.dl_gate &&
+             2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim <= ws.ld_cbuf && L.r_heads * L.r_dim <= ws.ld_dl_lg &&
+             L.r_heads * L.r_vdim <= ws.ld_dl_gate,
+         "gated delta rule operands or buffers");
+    need(L.r_kv_heads > 0 && L.r_heads % L.r_kv_heads == 0 && delta_supported(L.r_dim, L.r_vdim, L.r_rank, L.r_grank),
+         "gated delta rule sizes (key and value size <= 256, both low-rank maps together <= 1024)");
+  } else if (L.kind == 2) {
     need(r.kc && L.w_uk && L.w_uvT && L.dkv_norm && ws.cbuf && ws.lat && L.gate == 2, "latent attention operands");
     need(latent_supported(L.dim, L.rot_dim, L.kv_rank, L.vdim),
          "latent attention sizes (dim <= 256, kv_rank <= 256, kv_rank + rot_dim <= 1024)");
@@ -159,6 +194,117 @@ static bool chunked_scan_ok(const StackExecutor& e, const ScanParams& P, int B) 
          e.ws.ret.u_stride >= (long long)P.H * P.D * dvp && e.ws.ret.ld_o >= P.H * dvp && gated_chunk_supported(P.mode, P.D, P.Dv);
 }
 
+// Mamba-2 up to its output projection: convolution, the scan (prompt portions in chunks), the gate, the grouped norm
+void StackExecutor::mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
+  const int n_out = L.heads * L.vdim, f32 = cfg.f32;
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  const int ch = n_out + 2 * L.groups * L.state;
+  ConvParams Cv{ws.proj, ws.ld_proj, L.off_conv, ch, L.conv, L.conv_w, L.conv_b,
+                r.state + (long long)L.heads * L.state * L.vdim, r.state_stride, ws.cbuf, ws.ld_cbuf};
+  conv_silu(Cv, R, s);
+  ScanParams P{};
+  P.mode = SCAN_SSD;
+  P.proj = ws.proj;
+  P.ld = ws.ld_proj;
+  P.conv = ws.cbuf;
+  P.ld_conv = ws.ld_cbuf;
+  P.off_v = 0;                                  // x | B | C
+  P.off_k = n_out;
+  P.off_q = n_out + L.groups * L.state;
+  P.off_i = L.off_dt;
+  P.off_g = L.off_g;
+  P.H = L.heads;
+  P.G = L.groups;
+  P.D = L.state;
+  P.Dv = L.vdim;
+  P.dt_bias = L.dt_bias;
+  P.a_log = L.a_log;
+  P.d_skip = L.d_skip;
+  P.state = r.state;
+  P.state_stride = r.state_stride;
+  P.y = ws.ret.obuf;
+  P.ld_y = ws.ret.ld_o;
+  if (chunked_scan_ok(*this, P, B))
+    gated_scan_chunked(P, R, scan_ws(*this), nullptr, cfg.eps, nullptr, 0, f32, s);
+  else
+    gated_scan(P, R, s);
+  group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, L.norm_groups, L.mnorm, cfg.eps, nullptr, 0, ws.a, ws.ld_a, f32, s);
+}
+
+// linear attention with constant decays up to its output projection: the scan, one norm over all heads, the sigmoid gate
+void StackExecutor::linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
+  const int n_out = L.heads * L.vdim;
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  ScanParams P{};
+  P.mode = SCAN_FIXED;
+  P.proj = ws.proj;
+  P.ld = ws.ld_proj;
+  P.off_q = L.off_q;
+  P.off_k = L.off_k;
+  P.off_v = L.off_v;
+  P.H = P.G = L.heads;
+  P.D = L.dim;
+  P.Dv = L.vdim;
+  P.decay = L.decay;
+  P.state = r.state;
+  P.state_stride = r.state_stride;
+  P.y = ws.ret.obuf;
+  P.ld_y = ws.ret.ld_o;
+  if (chunked_scan_ok(*this, P, B))
+    gated_scan_chunked(P, R, scan_ws(*this), nullptr, cfg.eps, nullptr, 0, cfg.f32, s);
+  else
+    gated_scan(P, R, s);
+  group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, 1, L.mnorm, cfg.eps, ws.proj + L.off_g, ws.ld_proj, ws.a, ws.ld_a, cfg.f32, s);
+}
+
+// the gated delta rule beside an attention, up to the output projection; its outputs sit beside the attention's in ws.a
+void StackExecutor::delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  const long long sf = (long long)L.r_heads * L.r_dim * L.r_vdim;
+  DeltaParams P{};
+  P.proj = ws.proj;
+  P.ld = ws.ld_proj;
+  P.off_q = L.off_rq;
+  P.off_b = L.off_rb;
+  P.off_a1 = L.off_a1;
+  P.off_g1 = L.off_g1;
+  P.H = L.r_heads;
+  P.G = L.r_kv_heads;
+  P.D = L.r_dim;
+  P.Dv = L.r_vdim;
+  P.taps = L.conv;
+  P.conv_w = L.conv_w;
+  P.window = r.state + sf;
+  P.rank_a = L.r_rank;
+  P.rank_g = L.r_grank;
+  P.a2 = L.a2;
+  P.g2 = L.g2;
+  P.a_log = L.a_log;
+  P.dt_bias = L.dt_bias;
+  P.norm_w = L.gnorm;
+  P.eps = cfg.eps;
+  P.state = r.state;
+  P.state_stride = r.state_stride;
+  P.x = ws.cbuf;
+  P.ld_x = ws.ld_cbuf;
+  P.lg = ws.dl_lg;
+  P.ld_lg = ws.ld_dl_lg;
+  P.gate = ws.dl_gate;
+  P.ld_gate = ws.ld_dl_gate;
+  P.out = (char*)ws.a + (size_t)L.heads * L.vdim * (cfg.f32 ? 4 : 2);
+  P.ld_out = ws.ld_a;
+  P.out_scale = L.right_scale;
+  P.f32 = cfg.f32;
+  delta_prepare(P, R, s);
+  if (B > SMALL_B && n_chunks > 0 && ws.ret.Sin && ws.dl_W && ws.dl_Kd && ws.dl_u && ws.dl_Bm && ws.ret.u_stride >= sf &&
+      ws.dl_heads >= L.r_heads && delta_chunk_supported(L.r_dim, L.r_vdim)) {
+    DeltaChunkWs W{ws.ret.chunks, n_chunks, ws.ret.max_chunks, ws.ret.Sin, ws.ret.u_stride, ws.dl_W, ws.dl_Kd, ws.dl_u, ws.dl_Bm};
+    delta_chunked(P, R, W, s);
+  } else {
+    delta_walk(P, R, s);
+  }
+}
+
 // x <- x + LN1(mixer(x)), then x <- x + LN2(ff(x)): both sublayers read the stream itself (cast to the matrix
 // dtype), the layer norm sits on their outputs.
 void StackExecutor::layer_run_postnorm(int ri, int B, hipStream_t s) {
@@ -216,37 +362,7 @@ void StackExecutor::layer_run_postnorm(int ri, int B, hipStream_t s) {
                      f32, s);
     }
   } else {
-    const int ch = n_out + 2 * L.groups * L.state;
-    ConvParams Cv{ws.proj, ws.ld_proj, L.off_conv, ch, L.conv, L.conv_w, L.conv_b,
-                  r.state + (long long)L.heads * L.state * L.vdim, r.state_stride, ws.cbuf, ws.ld_cbuf};
-    conv_silu(Cv, R, s);
-    ScanParams P{};
-    P.mode = SCAN_SSD;
-    P.proj = ws.proj;
-    P.ld = ws.ld_proj;
-    P.conv = ws.cbuf;
-    P.ld_conv = ws.ld_cbuf;
-    P.off_v = 0;                                  // x | B | C
-    P.off_k = n_out;
-    P.off_q = n_out + L.groups * L.state;
-    P.off_i = L.off_dt;
-    P.off_g = L.off_g;
-    P.H = L.heads;
-    P.G = L.groups;
-    P.D = L.state;
-    P.Dv = L.vdim;
-    P.dt_bias = L.dt_bias;
-    P.a_log = L.a_log;
-    P.d_skip = L.d_skip;
-    P.state = r.state;
-    P.state_stride = r.state_stride;
-    P.y = ws.ret.obuf;
-    P.ld_y = ws.ret.ld_o;
-    if (chunked_scan_ok(*this, P, B))
-      gated_scan_chunked(P, R, scan_ws(*this), nullptr, cfg.eps, nullptr, 0, f32, s);
-    else
-      gated_scan(P, R, s);
-    group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, L.norm_groups, L.mnorm, cfg.eps, nullptr, 0, ws.a, ws.ld_a, f32, s);
+    mamba2_mixer(r, L, B, s);
   }
   {
     GemmParams o{ws.a, ws.ld_a, L.w_o, B, E, n_out, ws.y, E, EPI_STORE, 0.f, nullptr, 0.f, f32};
@@ -370,18 +486,31 @@ void StackExecutor::layer_run_sandwich(int ri, int B, hipStream_t s) {
 // x <- x + mixer(N1(x)), then x <- x + ff(N2(x)); N: RMS norm with a weight vector. A pass of a repeated span opens with
 // x <- W_in [x; x0]. Mixers: attention inside a sliding window with two differential maps per head and an
 // element-wise gate; attention inside a sliding window with adjacent-pair rotation and scores mixed across the heads
-// before the softmax; latent attention with one gate per head.
+// before the softmax; latent attention with one gate per head;
+// before the mixer (and, with cfg.canon_both, a convolution on the inputs of both sublayers): Mamba-2, constant-decay linear
+// attention, or attention inside blocks of positions with a gated delta rule beside it.
+void StackExecutor::norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, int B, hipStream_t s) {
+  if (!cfg.canon_both) {
+    rms_norm_cast(ws.resid, nullptr, B, cfg.E, w, cfg.eps, ws.h, cfg.f32, s);
+    return;
+  }
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  CanonParams C{ws.resid, w, cfg.eps, cfg.E, cfg.canon_taps, canon, cfg.canon_ring ? r.state + window_at : nullptr, r.state_stride,
+                ws.hn, ws.h, cfg.f32, 1, cfg.canon_ring};
+  scalar_norm_conv(C, R, s);
+}
 void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   const RunDesc& r = runs.at(ri);
   const LayerDesc& L = layers[r.layer];
-  const int E = cfg.E, f32 = cfg.f32, n_out = L.heads * L.vdim;
+  const int E = cfg.E, f32 = cfg.f32, n_out = L.heads * L.vdim + (L.r_delta ? L.r_heads * L.r_vdim : 0);
+  const long long win1 = prenorm_state_floats(L), win2 = win1 + (long long)cfg.canon_ring * E;
   if (r.opens_pass) {
     concat_cast(ws.resid, ws.x0, B, E, ws.cat, f32, s);
     GemmParams g{ws.cat, 2 * E, loop_in, B, E, 2 * E, ws.resid, E, EPI_STORE, 0.f, nullptr, 0.f, f32};
     gemm(g, s);
   }
   StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
-  const bool fused_in = gemv_ln_supported(B, E, f32);
+  const bool fused_in = !cfg.canon_both && gemv_ln_supported(B, E, f32);
   // differential attention: a K row of a key/value head holds its two maps side by side, so the K/V store sees heads
   // of 2 * dim
   AttnParams St{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, L.heads, L.kv_heads, 2 * L.dim, L.vdim, L.scale, 0.f, 0.f, 1,
@@ -390,14 +519,36 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     gemv_ln(ws.resid, E, L.norm_w, nullptr, cfg.eps, L.w_in, B, L.n_in, ws.proj, ws.ld_proj, ws.h,
             L.kind == 0 && L.maps == 2 ? &St : nullptr, &R, f32, s);
   } else {
-    rms_norm_cast(ws.resid, nullptr, B, E, L.norm_w, cfg.eps, ws.h, f32, s);
+    norm_in(r, L.norm_w, L.canon, win1, B, s);
     GemmParams g{ws.h, E, L.w_in, B, L.n_in, E, ws.proj, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
     gemm(g, s);
   }
   const bool tiled = B > SMALL_B && n_tiles > 0 && tiles;
   // a window bounds the keys of a decode step: no need to share them among blocks
-  const int splits = L.window > 0 && L.window <= 1024 ? 1 : n_splits;
-  if (L.kind == 2) {
+  const int bound = L.chunk > 0 ? L.chunk : L.window;
+  const int splits = bound > 0 && bound <= 1024 ? 1 : n_splits;
+  if (L.kind == 4) {
+    mamba2_mixer(r, L, B, s);
+  } else if (L.kind == 6) {
+    linear_mixer(r, L, B, s);
+  } else if (L.r_delta) {
+    KvStoreParams K{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, f32};
+    kv_store(K, R, s);
+    AttnParams A{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, 0.f, 0.f, 1, r.kc, r.vc,
+                 ws.a, ws.ld_a, f32, splits, ws.split_ws, ws.split_ws_floats};
+    A.window = L.window;
+    A.maps = 1;
+    A.chunk = L.chunk;
+    A.slopes = L.slopes;
+    A.hgate = L.gate == 2 ? ws.proj + L.off_g : nullptr;
+    A.ld_hgate = ws.ld_proj;
+    A.out_scale = L.left_scale;
+    if (tiled && flash_prefill_supported(A))
+      flash_prefill(A, R, tiles, n_tiles, s);
+    else
+      attention(A, R, s);
+    delta_mixer(r, L, B, s);
+  } else if (L.kind == 2) {
     const int C = L.kv_rank, W = C + L.rot_dim;
     LatentParams P{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_g, L.heads, L.dim, L.rot_dim, C, L.vdim, L.rot_dims,
                    L.inv_freq64, L.dkv_norm, cfg.eps, L.w_uk, L.w_uvT, L.w_ukT, L.w_uv, r.kc, ws.cbuf, ws.ld_cbuf, ws.lat, ws.ld_lat, ws.a,
@@ -441,7 +592,7 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   if (L.experts && fused_in) {  // decode steps: norm + router in one launch (the normed rows leave for the experts)
     gemv_ln(ws.resid, E, L.norm2_w, nullptr, cfg.eps, L.w_ff, B, L.n_ff, ws.proj, ws.ld_proj, ws.h, nullptr, nullptr, f32, s);
   } else {
-    rms_norm_cast(ws.resid, nullptr, B, E, L.norm2_w, cfg.eps, ws.h, f32, s);
+    norm_in(r, L.norm2_w, L.canon2, win2, B, s);
   }
   if (L.ff_dense) {
     if (B <= 8) {  // decode steps: gate / up projection and activation in one launch
@@ -462,7 +613,7 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   // the experts' weighted outputs are added straight into the stream (y = the stream, y_add)
   MoeParams M{ws.proj, ws.ld_proj, L.off_router, 0, 0, 0, B, E, L.experts, L.top, L.ff, 0, nullptr, ws.h, L.w_gu, L.w_down, nullptr,
               ws.eids, ws.ew, ws.ld_top, ws.sgate, ws.hmid, ws.ld_hmid, ws.resid, f32, 0, L.group_count, L.group_keep, ws.idw, 1,
-              L.route_scale};
+              L.route_scale, L.route_raw, L.expert_act, L.limit, L.scale_input};
   if (B <= SMALL_B && moe_route_sigmoid_fused_supported(M)) {  // decode steps: routing + activations in one launch
     moe_route_sigmoid_experts(M, s);
     moe_down(M, s);

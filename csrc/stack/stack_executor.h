@@ -23,10 +23,12 @@ struct StackConfig {
   float embed_scale = 1.f;
   float logit_scale = 1.f;  // block 2: logits = head x * logit_scale
   int canon_taps = 1;       // block 2: taps of the convolution added to the mixer's input (1: the current token only)
+  int canon_both = 0;       // block 3: such a convolution on the inputs of both sublayers, windows as rings of canon_ring rows
+  int canon_ring = 0;
 };
 
 struct LayerDesc {
-  int kind = 0;  // 0 attention, 1 retention, 2 latent attention, 3 mLSTM, 4 Mamba-2
+  int kind = 0;  // 0 attention, 1 retention, 2 latent attention, 3 mLSTM, 4 Mamba-2, 6 constant-decay linear attention
   int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
   float scale = 1.f, softcap = 0.f, qtemp_coef = 0.f;
   int qtemp_every = 1, rot_dims = 0;
@@ -97,6 +99,15 @@ struct LayerDesc {
   int gate = 0;                     // 1: element-wise sigmoid output gate at off_g, 2: one gate per head
   int score_talk = 0;               // the heads' scores are mixed by `talk` before the softmax
   float route_scale = 1.f;
+  int chunk = 0, v_unit = 0;        // attention inside blocks of `chunk` positions; values divided by their root mean square
+  const float* slopes = nullptr;    // [heads] distance slopes, or null
+  const float* canon2 = nullptr;    // [E][taps] convolution added to the feed-forward's input (cfg.canon_both)
+  int route_raw = 0, expert_act = 0, scale_input = 0;
+  float limit = 0.f;
+  // a gated delta rule beside the attention (r_delta != 0; sizes r_heads, r_kv_heads, r_dim, r_vdim, taps `conv`); w_o is
+  // [E][heads * vdim + r_heads * r_vdim]
+  int r_delta = 0, r_kv_heads = 0, r_grank = 0, off_rb = 0, off_g1 = 0;
+  const void* g2 = nullptr;
 };
 
 struct RunDesc {   // one execution of a layer: its own cache
@@ -137,6 +148,16 @@ struct StackWorkspace {
   float* ctot = nullptr;   // [max chunks][ld_coef / 3] the chunks' summed ln a per head
   float* hn = nullptr;     // [max_B][E] float32: normed rows before the input convolution (block 2)
   float* y2 = nullptr;     // [max_B][E] float32: the second mixer's projected output (block 2)
+  // gated delta rule: prepared q | k | v sit in cbuf
+  float* dl_lg = nullptr;   // [max_B][ld_dl_lg] log decays
+  int ld_dl_lg = 0;
+  float* dl_gate = nullptr; // [max_B][ld_dl_gate] output gates
+  int ld_dl_gate = 0;
+  float* dl_W = nullptr;    // chunked form, as DeltaChunkWs
+  float* dl_Kd = nullptr;
+  float* dl_u = nullptr;
+  float* dl_Bm = nullptr;
+  int dl_heads = 0;         // heads that dl_Bm holds per row
   float* lna = nullptr;    // chunked gated linear attention: the rows' running log decays (= coef)
   MoeGroupWs moe{};        // grouped routed feed-forward (prompt portions, bfloat16); gu == null: unused
   RetChunkWs ret{};        // chunked retention (prompt portions): chunk table, per-chunk states, o before its norm
@@ -181,6 +202,10 @@ class StackExecutor {
   void layer_run_postnorm(int ri, int B, hipStream_t s);
   void layer_run_sandwich(int ri, int B, hipStream_t s);
   void layer_run_prenorm(int ri, int B, hipStream_t s);
+  void norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, int B, hipStream_t s);
+  void mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  void linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  void delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
   void head(int n_logits, bool use_idx, hipStream_t s);
   void forward(int B, int n_logits, bool use_idx, hipStream_t s);
 };

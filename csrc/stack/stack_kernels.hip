@@ -536,6 +536,13 @@ void attn_prepare(const AttnParams& P, const StepRows& R, hipStream_t s) {
 // batch; each head keeps a running maximum and sum; every lane owns value dims lane, lane + 64, ... of every
 // head's output, and a V row is read once for all of them.
 constexpr int ATT_MAXD = 256;
+// first key that a row with n visible positions sees: the start of its block of positions, or of its sliding window
+__device__ __forceinline__ int attn_first_key(const AttnParams& P, int n) {
+  return P.chunk > 0 ? (n - 1) / P.chunk * P.chunk : P.window > 0 ? max(0, n - P.window) : 0;
+}
+__device__ __forceinline__ float attn_head_gate(const AttnParams& P, long long b, int h) {
+  return P.hgate ? P.out_scale * sigmoidf(P.hgate[b * P.ld_hgate + h]) : 1.f;
+}
 constexpr int ATT_MAXD_DECODE = 1024;  // the block-per-(row, head) kernel keeps one query in LDS: wide shared key rows fit
 template <typename T>
 __device__ __forceinline__ void load8(const T* p, float* out);
@@ -596,7 +603,7 @@ __global__ __launch_bounds__(256) void attention_kernel(AttnParams P, StepRows R
 #pragma unroll
     for (int c = 0; c < DC; ++c) acc[r][c] = 0.f;
   }
-  const int lo = P.window > 0 ? max(0, n - P.window) : 0;  // sliding window: the keys lo .. n - 1
+  const int lo = attn_first_key(P, n);  // the row sees the keys lo .. n - 1
   for (int t0 = lo + (SPLIT ? 64 * wv : 0); t0 < n; t0 += SPLIT ? 256 : 64) {
     const int t = t0 + lane;
     const bool valid = t < n;
@@ -649,6 +656,7 @@ __global__ __launch_bounds__(256) void attention_kernel(AttnParams P, StepRows R
       if (valid) {
         sc = dot[r] * P.scale;
         if (P.softcap != 0.f) sc = P.softcap * tanhf(sc / P.softcap);
+        if (P.slopes) sc -= P.slopes[min(h0 + r, P.H - 1)] * (float)(n - 1 - t);
       }
       const float mn = fmaxf(m[r], wave_max(sc));
       const float corr = expf(m[r] - mn);  // first group: exp(-inf) = 0
@@ -719,7 +727,7 @@ __global__ __launch_bounds__(256) void attention_kernel(AttnParams P, StepRows R
     if (r < nr) {
       T* out = (T*)P.out + (long long)b * P.ld_out + (h0 + r) * P.Dv;
       if (P.sink) l[r] += expf(P.sink[h0 + r] - m[r]);  // the sink: a term of the denominator without key or value
-      const float inv = 1.f / l[r];
+      const float inv = attn_head_gate(P, b, h0 + r) / l[r];
 #pragma unroll
       for (int c = 0; c < DC; ++c) {
         const int d = lane + 64 * c;
@@ -756,11 +764,12 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(AttnParams P, Ste
   const T* vc = (const T*)P.vc;
   const long long ldk = P.ldk ? P.ldk : P.D, ldv = P.ldv ? P.ldv : P.Dv;
   const int kq = lane >> 4, dq = lane & 15;
+  const float slope = P.slopes ? P.slopes[h] : 0.f;
   float m = -INFINITY, l = 0.f, acc[DPL];
 #pragma unroll
   for (int c = 0; c < DPL; ++c) acc[c] = 0.f;
   __syncthreads();
-  const int lo = P.window > 0 ? max(0, n - P.window) : 0;  // sliding window: the keys lo .. n - 1
+  const int lo = attn_first_key(P, n);  // the row sees the keys lo .. n - 1
   for (int t0 = lo + 64 * (split * 4 + wv); t0 < n; t0 += 256 * nsplit) {
     const int t = t0 + lane;
     const bool valid = t < n;
@@ -793,6 +802,7 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(AttnParams P, Ste
     if (valid) {
       sc = dot * P.scale;
       if (P.softcap != 0.f) sc = P.softcap * tanhf(sc / P.softcap);
+      sc -= slope * (float)(n - 1 - t);
     }
     const float mn = fmaxf(m, wave_max(sc));
     const float corr = expf(m - mn);
@@ -879,7 +889,7 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(AttnParams P, Ste
     return;
   }
   if (P.sink) L += expf(P.sink[h] - M);
-  const float inv = 1.f / L;
+  const float inv = attn_head_gate(P, b, h) / L;
   if (P.out32) {
     float* out = P.out32 + (long long)b * P.ld_out32 + oh * P.Dv;
 #pragma unroll
@@ -908,6 +918,7 @@ __global__ __launch_bounds__(256) void attention_merge_kernel(AttnParams P, int 
   }
   const int vh = P.vheads > 1 ? P.vheads : 1, NH = P.H * vh;  // items are (row, output head)
   if (P.sink) L += expf(P.sink[(item % NH) / vh] - M);
+  const float inv = attn_head_gate(P, item / NH, (item % NH) / vh) / L;
   T* out = (T*)P.out + (long long)(item / NH) * P.ld_out + (item % NH) * P.Dv;
   float* out32 = P.out32 ? P.out32 + (long long)(item / NH) * P.ld_out32 + (item % NH) * P.Dv : nullptr;
   for (int d = lane; d < P.Dv; d += 64) {
@@ -917,9 +928,9 @@ __global__ __launch_bounds__(256) void attention_merge_kernel(AttnParams P, int 
       if (ms != -INFINITY) o += w[(long long)sidx * (P.Dv + 2) + 2 + d] * expf(ms - M);
     }
     if (out32)
-      out32[d] = o / L;
+      out32[d] = o * inv;
     else
-      st(out + d, o / L);
+      st(out + d, o * inv);
   }
 }
 template <typename T>
@@ -1012,9 +1023,10 @@ __global__ __launch_bounds__(64) void flash_prefill_kernel(AttnParams P, StepRow
   const int* bt = R.block_table + (long long)R.q_seq[row0] * R.max_blocks;
   const int qrow = row0 + min(q, nrows - 1);
   const int qlen = q < nrows ? R.q_len[qrow] : 0;
-  const int kfirst = P.window > 0 ? qlen - P.window : 0;     // sliding window: this lane's query sees keys kfirst .. qlen - 1
+  const int kfirst = attn_first_key(P, max(qlen, 1));        // this lane's query sees keys kfirst .. qlen - 1
+  const float slope = P.slopes ? P.slopes[h] : 0.f;
   const int kmax = R.q_len[row0 + nrows - 1];
-  const int kmin = P.window > 0 ? max(0, R.q_len[row0] - P.window) & ~31 : 0;  // the first key any row of the tile sees
+  const int kmin = attn_first_key(P, R.q_len[row0]) & ~31;   // the first key any row of the tile sees
   // queries: B operand, lane (q, hf) holds dims 16 kk + 8 hf + 0..7
   bf16x8 qhi[KD], qlo[KD];
   {
@@ -1101,6 +1113,7 @@ __global__ __launch_bounds__(64) void flash_prefill_kernel(AttnParams P, StepRow
       float sc = sacc[r] * P.scale;
       if (P.softcap != 0.f) sc = P.softcap * fast_tanh(sc * inv_cap);
       const int key = t0 + 16 * (r >> 3) + 8 * hf + (r & 7);
+      sc -= slope * (float)(qlen - 1 - key);
       const bool vis = key < qlen && key >= kfirst;
       pr[r] = vis ? sc : -1e30f;
       mx = fmaxf(mx, pr[r]);
@@ -1151,7 +1164,7 @@ __global__ __launch_bounds__(64) void flash_prefill_kernel(AttnParams P, StepRow
   }
   if (q < nrows) {  // register r of tile j: value dim 32 j + (r & 3) + 8 (r >> 2) + 4 hf of this lane's query
     if (P.sink) li += expf(P.sink[h] - mi);  // the sink: a term of the denominator without key or value
-    const float inv = 1.f / li;
+    const float inv = attn_head_gate(P, qrow, h) / li;
     if (P.out32) {
       float* out = P.out32 + (long long)qrow * P.ld_out32 + oh * DV;
 #pragma unroll
@@ -1646,7 +1659,8 @@ __global__ __launch_bounds__(256) void moe_experts_kernel(MoeParams P, int vec) 
   const T* wu = wg + (long long)P.F * P.E;
   const float gate = wave_dot<T>(wg, x, P.E, lane, vec != 0);
   const float up = wave_dot<T>(wu, x, P.E, lane, vec != 0);
-  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, silu(gate) * up);
+  const float w = P.w_input ? P.ew[(long long)b * P.ld_top + jj] : 1.f;
+  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, moe_unit(P.act, P.limit, w, gate, up));
 }
 // one wave per (row, output unit): the routed experts' down rows in routing order, then the shared expert's
 template <typename T>
@@ -1660,7 +1674,8 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeParams P, int vec, int
   for (int jj = 0; jj < P.top; ++jj) {
     const int e = P.eids[(long long)b * P.ld_top + jj];
     const T* wd = (const T*)P.w_down + ((long long)e * P.E + n) * P.F;
-    y += P.ew[(long long)b * P.ld_top + jj] * wave_dot<T>(wd, hm + jj * P.F, P.F, lane, vec != 0);
+    const float w = P.w_input ? 1.f : P.ew[(long long)b * P.ld_top + jj];
+    y += w * wave_dot<T>(wd, hm + jj * P.F, P.F, lane, vec != 0);
   }
   if (P.Fs > 0)
     y += P.sgate[b] * wave_dot<T>((const T*)P.sh_down + (long long)n * P.Fs, hm + P.top * P.F, P.Fs, lane, vec_s != 0);
@@ -1701,13 +1716,21 @@ __global__ __launch_bounds__(256) void moe_sort_kernel(const int* __restrict__ e
     inv[p] = pos;
   }
 }
-// hs[pos][f] = silu(gu[pos][f]) * gu[pos][F + f], in the matrix dtype
-__global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ gu, int P, int F, bf16* __restrict__ hs) {
+// hs[pos][f] = the hidden unit of gu[pos][f], gu[pos][F + f] (moe_unit), in the matrix dtype; ew non-null: the pairs'
+// weights act on the experts' inputs
+__global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ gu, int P, int F, int act, float limit,
+                                                      const float* __restrict__ ew, int ld_top, int top,
+                                                      const int* __restrict__ srow, bf16* __restrict__ hs) {
   const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
   if (i >= (long long)P * F) return;
   const long long pos = i / F;
   const int f = (int)(i % F);
-  st(hs + i, silu(gu[pos * 2 * F + f]) * gu[pos * 2 * F + F + f]);
+  float w = 1.f;
+  if (ew) {
+    const int pair = srow[pos];
+    w = ew[(long long)(pair / top) * ld_top + pair % top];
+  }
+  st(hs + i, moe_unit(act, limit, w, gu[pos * 2 * F + f], gu[pos * 2 * F + F + f]));
 }
 // y[b][n] = (shared ? sgate[b] * y[b][n] : 0) + sum_j ew[b][j] * ds[inv[b * top + j]][n], routing order
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ y, const float* __restrict__ ds,
@@ -1719,7 +1742,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ y,
   const int b = (int)(i / E), n = (int)(i % E);
   float acc = shared ? sgate[b] * y[i] : y_add ? y[i] : 0.f;  // (y_add: y is the residual stream, no shared expert)
   float routed = 0.f;
-  for (int j = 0; j < top; ++j) routed += ew[(long long)b * ld_top + j] * ds[(long long)inv[b * top + j] * E + n];
+  for (int j = 0; j < top; ++j) routed += (ew ? ew[(long long)b * ld_top + j] : 1.f) * ds[(long long)inv[b * top + j] * E + n];
   y[i] = routed + acc;
 }
 bool moe_grouped_supported(const MoeParams& P) {
@@ -1753,7 +1776,8 @@ void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
   }
   {
     const long long n = (long long)pairs * P.F;
-    hipLaunchKernelGGL(moe_act_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, W.gu, pairs, P.F, (bf16*)W.hs);
+    hipLaunchKernelGGL(moe_act_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, W.gu, pairs, P.F, P.act, P.limit,
+                       P.w_input ? P.ew : nullptr, P.ld_top, P.top, W.srow, (bf16*)W.hs);
     launched("moe_act");
   }
   {
@@ -1777,7 +1801,7 @@ void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
   }
   {
     const long long n = (long long)P.B * P.E;
-    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, P.y, W.ds, W.inv, P.ew, P.ld_top,
+    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, P.y, W.ds, W.inv, P.w_input ? nullptr : P.ew, P.ld_top,
                        P.sgate, P.B, P.E, P.top, (int)(P.Fs > 0), P.y_add);
     launched("moe_combine");
   }

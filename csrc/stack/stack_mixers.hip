@@ -370,7 +370,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams P, StepRows R
   const bool alone = nb == 0 && !(r + 1 < R.B && R.q_seq[r + 1] == seq);
   float* win = P.state + (long long)seq * P.state_stride;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < P.ch; c += 256 * gridDim.y) {
-    float acc = P.bias[c];
+    float acc = P.bias ? P.bias[c] : 0.f;
     const float cur = P.proj[(long long)r * P.ld + P.off_in + c];
     for (int j = 0; j < K; ++j) {
       const int back = K - 1 - j;
@@ -398,15 +398,18 @@ __global__ __launch_bounds__(256) void conv_window_kernel(ConvParams P, StepRows
     }
 }
 void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s) {
-  check(R.B > 0 && P.proj && P.w && P.bias && P.out && P.ch > 0 && P.taps >= 1 && (P.taps == 1 || P.state),
+  check(R.B > 0 && P.proj && P.w && P.out && P.ch > 0 && P.taps >= 1 && (P.taps == 1 || P.state),
         "conv_silu: bad operands");
   const dim3 grid(R.B, (P.ch + 255) / 256);  // a block per (row, 256 channels)
   hipLaunchKernelGGL(conv_silu_kernel, grid, dim3(256), 0, s, P, R);
   launched("conv_silu");
-  if (P.taps > 1 && R.B > 1) {  // a single row is alone in its sequence
-    hipLaunchKernelGGL(conv_window_kernel, grid, dim3(256), 0, s, P, R);
-    launched("conv_window");
-  }
+  conv_window(P, R, s);
+}
+void conv_window(const ConvParams& P, const StepRows& R, hipStream_t s) {
+  if (P.taps <= 1 || R.B <= 1) return;  // (a single row is alone in its sequence)
+  check(P.proj && P.state && P.ch > 0, "conv_window: bad operands");
+  hipLaunchKernelGGL(conv_window_kernel, dim3(R.B, (P.ch + 255) / 256), dim3(256), 0, s, P, R);
+  launched("conv_window");
 }
 
 // ------------------------------------------------------------------------------------------------ gated state scan
@@ -415,6 +418,7 @@ void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s) {
 //               m_t = max(f + m_(t-1), i), a = exp(f + m_(t-1) - m_t), b = exp(i - m_t); q scaled by D^(-1/2); a
 //               normaliser n_t = a n_(t-1) + b k_t rides along, and
 //               y = o / (max(|n_t . q|, exp(-m_t)) + 1e-6)
+//   SCAN_FIXED: a = a constant per head, b = 1; q, k, v = silu of their projections; y = o
 //   SCAN_SSD:   dt = softplus(dt_raw + dt_bias), a = exp(-exp(A_log) dt), b = dt; q = C_t, k = B_t of the head's
 //               group, v = x_t (all three from the convolution's output); y = (o + D x_t) silu(z_t)
 // One block per (sequence segment of the step, head), as the retention kernel: the block of the segment's first
@@ -423,14 +427,14 @@ void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s) {
 // tid < D. The slot's state (S, then for the mLSTM n and m) is read once and written back once per step.
 __device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float logsigmoidf(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
-template <int MODE, int MAXI>
-__global__ __launch_bounds__(256) void gated_scan_kernel(ScanParams P, StepRows R) {
-  __shared__ float qs[256], ks[256], vs[256], po[256], os[256], nred[4];
+template <int MODE, int MAXI, int NT>
+__global__ __launch_bounds__(NT) void gated_scan_kernel(ScanParams P, StepRows R) {
+  __shared__ float qs[256], ks[256], vs[256], po[NT], nred[4];
   const int r0 = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int seq = R.q_seq[r0];
   if (r0 > 0 && R.q_seq[r0 - 1] == seq) return;  // not the first row of its segment (uniform per block)
   const int D = P.D, Dv = P.Dv;
-  const int NG = 256 / Dv;
+  const int NG = NT / Dv;
   const int g = tid / Dv, j = tid % Dv;
   const bool act = g < NG;
   const int hg = h / (P.H / P.G);
@@ -450,9 +454,12 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(ScanParams P, StepRows 
   const float qscale = MODE == SCAN_MLSTM ? 1.f / sqrtf((float)D) : 1.f;
   for (int r = r0; r < R.B && R.q_seq[r] == seq; ++r) {
     const float* row = P.proj + (long long)r * P.ld;
-    const float* src = MODE == SCAN_MLSTM ? row : P.conv + (long long)r * P.ld_conv;
+    const float* src = MODE == SCAN_SSD ? P.conv + (long long)r * P.ld_conv : row;
     float a, b;
-    if (MODE == SCAN_MLSTM) {
+    if (MODE == SCAN_FIXED) {
+      a = P.decay[h];
+      b = 1.f;
+    } else if (MODE == SCAN_MLSTM) {
       const float ig = P.cap * tanhf((row[P.off_i + h] + P.i_b[h]) / P.cap);
       const float fg = logsigmoidf(P.cap * tanhf((row[P.off_f + h] + P.f_b[h]) / P.cap));
       const float mn = fmaxf(fg + m, ig);
@@ -468,10 +475,14 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(ScanParams P, StepRows 
     if (tid < D) {
       qv = src[P.off_q + hg * D + tid] * qscale;
       kv = src[P.off_k + hg * D + tid];
+      if (MODE == SCAN_FIXED) {
+        qv = silu(qv);
+        kv = silu(kv);
+      }
       qs[tid] = qv;
       ks[tid] = kv;
     }
-    if (tid < Dv) vs[tid] = src[P.off_v + h * Dv + tid];
+    if (tid < Dv) vs[tid] = MODE == SCAN_FIXED ? silu(src[P.off_v + h * Dv + tid]) : src[P.off_v + h * Dv + tid];
     if (MODE == SCAN_MLSTM) {
       nreg = a * nreg + b * kv;
       const float pn = wave_sum(nreg * qv);
@@ -498,6 +509,8 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(ScanParams P, StepRows 
       float y;
       if (MODE == SCAN_MLSTM)
         y = o / (fmaxf(fabsf(nred[0] + nred[1] + nred[2] + nred[3]), expf(-m)) + 1e-6f);
+      else if (MODE == SCAN_FIXED)
+        y = o;
       else
         y = (o + P.d_skip[h] * vs[tid]) * silu(row[P.off_g + h * Dv + tid]);
       P.y[(long long)r * P.ld_y + h * Dv + tid] = y;
@@ -514,34 +527,46 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(ScanParams P, StepRows 
     if (tid == 0) *mptr = m;
   }
 }
-bool gated_scan_supported(int mode, int D, int Dv) {
-  (void)mode;
-  if (D <= 0 || Dv <= 0 || D > 256 || Dv > 256) return false;
-  const int ng = 256 / Dv;
-  return (D + ng - 1) / ng <= 64;
+// state elements per thread of a block of nt threads; up to 64 sit in registers
+static inline int scan_elems(int D, int Dv, int nt) {
+  const int ng = nt / Dv;
+  return (D + ng - 1) / ng;
 }
-template <int MODE>
+bool gated_scan_supported(int mode, int D, int Dv) {
+  if (D <= 0 || Dv <= 0 || D > 256 || Dv > 256) return false;
+  return scan_elems(D, Dv, mode == SCAN_MLSTM ? 256 : 1024) <= 64;
+}
+template <int MODE, int NT>
 static void launch_gated_scan(const ScanParams& P, const StepRows& R, hipStream_t s) {
-  const int ng = 256 / P.Dv, ni = (P.D + ng - 1) / ng;
+  const int ni = scan_elems(P.D, P.Dv, NT);
   const dim3 grid(R.B, P.H);
   if (ni <= 8)
-    hipLaunchKernelGGL((gated_scan_kernel<MODE, 8>), grid, dim3(256), 0, s, P, R);
+    hipLaunchKernelGGL((gated_scan_kernel<MODE, 8, NT>), grid, dim3(NT), 0, s, P, R);
   else if (ni <= 16)
-    hipLaunchKernelGGL((gated_scan_kernel<MODE, 16>), grid, dim3(256), 0, s, P, R);
+    hipLaunchKernelGGL((gated_scan_kernel<MODE, 16, NT>), grid, dim3(NT), 0, s, P, R);
   else if (ni <= 32)
-    hipLaunchKernelGGL((gated_scan_kernel<MODE, 32>), grid, dim3(256), 0, s, P, R);
+    hipLaunchKernelGGL((gated_scan_kernel<MODE, 32, NT>), grid, dim3(NT), 0, s, P, R);
   else
-    hipLaunchKernelGGL((gated_scan_kernel<MODE, 64>), grid, dim3(256), 0, s, P, R);
+    hipLaunchKernelGGL((gated_scan_kernel<MODE, 64, NT>), grid, dim3(NT), 0, s, P, R);
 }
 void gated_scan(const ScanParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.proj && P.state && P.y && P.H > 0 && P.G > 0 && P.H % P.G == 0 && gated_scan_supported(P.mode, P.D, P.Dv),
         "gated scan: operands or head sizes (key and value size <= 256, state within the registers)");
   if (P.mode == SCAN_MLSTM) {
     check(P.i_b && P.f_b && P.cap > 0.f && P.G == P.H, "gated scan: mLSTM gate operands");
-    launch_gated_scan<SCAN_MLSTM>(P, R, s);
+    launch_gated_scan<SCAN_MLSTM, 256>(P, R, s);
+  } else if (P.mode == SCAN_FIXED) {
+    check(P.decay && P.G == P.H, "gated scan: constant decays");
+    if (P.D * P.Dv <= 2048)
+      launch_gated_scan<SCAN_FIXED, 256>(P, R, s);
+    else
+      launch_gated_scan<SCAN_FIXED, 1024>(P, R, s);
   } else {
     check(P.conv && P.dt_bias && P.a_log && P.d_skip, "gated scan: state space operands");
-    launch_gated_scan<SCAN_SSD>(P, R, s);
+    if (scan_elems(P.D, P.Dv, 256) <= 64)
+      launch_gated_scan<SCAN_SSD, 256>(P, R, s);
+    else  // a large head: its state over four times the threads
+      launch_gated_scan<SCAN_SSD, 1024>(P, R, s);
   }
   launched("gated_scan");
 }
@@ -626,9 +651,13 @@ __device__ __forceinline__ void stage_qk_gated(const ScanParams& P, int row0, in
     const int c = idx / MAXD, d = idx % MAXD;
     float qv = 0.f, kv = 0.f;
     if (c < cn && d < P.D) {
-      const float* src = MODE == SCAN_MLSTM ? P.proj + (long long)(row0 + c) * P.ld : P.conv + (long long)(row0 + c) * P.ld_conv;
+      const float* src = MODE == SCAN_SSD ? P.conv + (long long)(row0 + c) * P.ld_conv : P.proj + (long long)(row0 + c) * P.ld;
       kv = src[P.off_k + hg * P.D + d];
       if (WITH_Q) qv = src[P.off_q + hg * P.D + d] * qscale;
+      if (MODE == SCAN_FIXED) {
+        kv = silu(kv);
+        if (WITH_Q) qv = silu(qv);
+      }
     }
     if (WITH_Q) Qs[c][d] = qv;
     Ks[c][d] = kv;
@@ -641,9 +670,9 @@ __device__ __forceinline__ void stage_v_gated(const ScanParams& P, int row0, int
     const int c = idx >> 6, col = jb * 64 + (idx & 63);
     float v = 0.f;
     if (c < cn) {
-      const float* src = MODE == SCAN_MLSTM ? P.proj + (long long)(row0 + c) * P.ld : P.conv + (long long)(row0 + c) * P.ld_conv;
+      const float* src = MODE == SCAN_SSD ? P.conv + (long long)(row0 + c) * P.ld_conv : P.proj + (long long)(row0 + c) * P.ld;
       if (col < P.Dv)
-        v = src[P.off_v + h * P.Dv + col];
+        v = MODE == SCAN_FIXED ? silu(src[P.off_v + h * P.Dv + col]) : src[P.off_v + h * P.Dv + col];
       else if (MODE == SCAN_MLSTM && col == P.Dv)
         v = 1.f;
     }
@@ -651,7 +680,17 @@ __device__ __forceinline__ void stage_v_gated(const ScanParams& P, int row0, int
   }
 }
 // Lc[t] = l_0 + ... + l_t and bw[t] = b_t of the chunk's rows (Lc past cn stays at its last value)
+template <int MODE>
 __device__ __forceinline__ void stage_coef(const ScanParams& P, const float* coef, int row0, int cn, int h, float* Lc, float* bw) {
+  if (MODE == SCAN_FIXED) {  // one constant per head (a decay of 0 forgets everything: its logarithm stays finite)
+    if (threadIdx.x < SC) {
+      const int t = threadIdx.x;
+      Lc[t] = fmaxf(logf(P.decay[h]), -1e30f) * (float)(min(t, cn - 1) + 1);
+      bw[t] = t < cn ? 1.f : 0.f;
+    }
+    __syncthreads();
+    return;
+  }
   if (threadIdx.x < SC) {
     const int t = threadIdx.x;
     const float* c = coef + ((long long)(row0 + min(t, cn - 1)) * P.H + h) * 3;
@@ -679,7 +718,7 @@ __global__ __launch_bounds__(256) void gated_u_kernel(ScanParams P, const int* _
   const int row0 = chunks[4 * c], cn = chunks[4 * c + 1];
   const int Dvp = P.Dv + (MODE == SCAN_MLSTM ? 1 : 0);
   const int j = tid & 63, g4 = tid >> 6, col = jb * 64 + j;
-  stage_coef(P, coef, row0, cn, h, Lc, bw);
+  stage_coef<MODE>(P, coef, row0, cn, h, Lc, bw);
   stage_qk_gated<MODE, MAXD, false>(P, row0, cn, h / (P.H / P.G), nullptr, Ks);
   stage_v_gated<MODE>(P, row0, cn, h, jb, Vs);
   __syncthreads();
@@ -741,7 +780,7 @@ __global__ __launch_bounds__(256) void gated_out_kernel(ScanParams P, const int*
   const float* sin_base = Sin + c * u_stride + (long long)h * D * Dvp;
 #pragma unroll
   for (int i = 0; i < MAXD; ++i) S[i] = (colok && i < D) ? sin_base[(long long)i * Dvp + col] : 0.f;
-  stage_coef(P, coef, row0, cn, h, Lc, bw);
+  stage_coef<MODE>(P, coef, row0, cn, h, Lc, bw);
   stage_qk_gated<MODE, MAXD, true>(P, row0, cn, h / (P.H / P.G), Qs, Ks);
   stage_v_gated<MODE>(P, row0, cn, h, jb, Vs);
   __syncthreads();
@@ -775,6 +814,8 @@ __global__ __launch_bounds__(256) void gated_out_kernel(ScanParams P, const int*
       const long long r = row0 + t;
       if (MODE == SCAN_MLSTM)
         raw[r * ld_raw + h * Dvp + col] = o;
+      else if (MODE == SCAN_FIXED)
+        P.y[r * P.ld_y + h * Dv + col] = o;
       else
         P.y[r * P.ld_y + h * Dv + col] = (o + P.d_skip[h] * Vs[t][j]) * silu(P.proj[r * P.ld + P.off_g + h * Dv + col]);
     }
@@ -837,6 +878,12 @@ void gated_scan_chunked(const ScanParams& P, const StepRows& R, const ScanChunkW
       hipLaunchKernelGGL(mlstm_finish_kernel<bf16>, g2, dim3(256), 0, s, P, R.B, W.raw, W.ld_raw, W.coef, norm_w, eps, (bf16*)out,
                          ld_out);
     launched("mlstm_finish");
+  } else if (P.mode == SCAN_FIXED) {
+    check(P.decay && P.G == P.H && P.y, "chunked constant-decay operands");
+    if (P.D <= 64)
+      launch_gated_chunked<SCAN_FIXED, 64>(P, R, W, s);
+    else
+      launch_gated_chunked<SCAN_FIXED, 128>(P, R, W, s);
   } else {
     check(P.conv && P.dt_bias && P.a_log && P.d_skip && P.y, "chunked state space operands");
     hipLaunchKernelGGL(gated_coef_ssd_kernel, dim3((R.B * P.H + 255) / 256), dim3(256), 0, s, P, R.B, W.coef);

@@ -87,6 +87,11 @@ struct AttnParams {
   // kshared: the K pool has ONE head whose row (D wide) serves every query head, while the V pool keeps its G heads
   // (query head h meets the values of head h / (H / G)): scores that are sums over all key/value heads
   int kshared;
+  int chunk;            // > 0: a row at position i sees only the keys of its own block of `chunk` positions (from 0 on)
+  const float* slopes;  // [H] or null: a score loses slopes[h] * (distance to the key)
+  const float* hgate;   // non-null: head h's output is multiplied by out_scale * sigmoid(hgate[b * ld_hgate + h])
+  int ld_hgate;
+  float out_scale;
 };
 // q *= 1 + coef * ln(floor((pos + 1) / every) + 1); k, v of every row stored at its slot
 void attn_prepare(const AttnParams& P, const StepRows& R, hipStream_t s);
@@ -141,6 +146,7 @@ void retention_chunked(const RetParams& P, const StepRows& R, const RetChunkWs& 
 int retention_chunk_rows();
 bool retention_chunk_supported(int D, int Dv);
 
+enum { MOE_ACT_SILU = 0, MOE_ACT_CLAMPED = 1 };
 struct MoeParams {
   const float* proj;    // [B][ld]: router logits at off_router, shared: scalar gate, gate rows, up rows
   int ld, off_router, off_sg, off_sgate, off_sup;
@@ -164,6 +170,10 @@ struct MoeParams {
   float* idw;
   int y_add;            // moe_down / moe_grouped: y += the feed-forward's output (y = the residual stream) instead of y =
   float route_scale;    // sigmoid router (moe_route_sigmoid): factor on the normalised weights
+  int route_raw;        // sigmoid router: the chosen scores are the weights as they are (not divided by their sum)
+  int act;              // routed experts: MOE_ACT_SILU silu(gate) up; MOE_ACT_CLAMPED g sigmoid(1.702 g) (u + 1) with
+  float limit;          // g = min(gate, limit), u = clamp(up, -limit, limit)
+  int w_input;          // a chosen expert's weight multiplies its input (its gate / up products) instead of its output
 };
 void moe_route(const MoeParams& P, hipStream_t s);   // top-k ids + softmax weights, shared gate and activation
 // softmax over all router outputs, choice by score + correction inside the best expert groups, weights = the
@@ -235,15 +245,17 @@ struct ConvParams {
   int ld, off_in;
   int ch, taps;
   const float* w;       // [ch][taps], the last tap is the current token's
-  const float* bias;    // [ch]
+  const float* bias;    // [ch] or null
   float* state;         // slot s: state + s * state_stride = [taps - 1][ch], the sequence's last inputs
   long long state_stride;
   float* out;           // [B][ld_out] float32: silu(conv)
   int ld_out;
 };
 void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s);
+// only the windows of sequences with several rows in the step (after a kernel that convolves by itself)
+void conv_window(const ConvParams& P, const StepRows& R, hipStream_t s);
 
-enum { SCAN_MLSTM = 0, SCAN_SSD = 1 };
+enum { SCAN_MLSTM = 0, SCAN_SSD = 1, SCAN_FIXED = 2 };
 struct ScanParams {
   int mode;
   const float* proj;    // [B][ld] float32
@@ -260,6 +272,7 @@ struct ScanParams {
   const float* dt_bias; // SCAN_SSD [H]
   const float* a_log;
   const float* d_skip;
+  const float* decay;   // SCAN_FIXED [H]: constant decays; q, k, v = silu of the columns in proj, y = S^T q
   float* state;         // slot s: state + s * state_stride = S [H][D][Dv] (| n [H][D] | m [H] for SCAN_MLSTM)
   long long state_stride;
   float* y;             // [B][ld_y] float32
@@ -302,7 +315,7 @@ void relu2_cast(const float* z, int ld, int rows, int F, void* out, int ld_out, 
 constexpr int CANON_MAX_TAPS = 8;
 struct CanonParams {
   const float* x;
-  const float* g;
+  const float* g;       // one number (scalar_norm_conv), or with `gvec` [E] one weight per channel
   float eps;
   int E, taps;
   const float* w;
@@ -311,6 +324,8 @@ struct CanonParams {
   float* hn;            // [B][E]
   void* out;            // [B][E] matrix dtype
   int f32;
+  int gvec;
+  int ring;             // > 0: the window is a ring of `ring` rows, the input of position p in row p % ring (0: oldest first)
 };
 void scalar_norm_conv(const CanonParams& P, const StepRows& R, hipStream_t s);
 // out[r] = x[idx ? idx[r] : r] / rms * g[0], matrix dtype
@@ -428,6 +443,65 @@ void moe_route_sigmoid(const MoeParams& P, hipStream_t s);
 // a few rows (decode steps): the same routing and the routed activations (moe_experts' work) in one launch
 void moe_route_sigmoid_experts(const MoeParams& P, hipStream_t s);
 bool moe_route_sigmoid_fused_supported(const MoeParams& P);
+// every row's keys and values into its cache slot; v_unit: each head's value divided by sqrt(mean(v^2) + eps)
+struct KvStoreParams {
+  const float* proj;    // [B][ld] float32: k [G][D] at off_k, v [G][Dv] at off_v
+  int ld, off_k, off_v;
+  int G, D, Dv;
+  int v_unit;
+  float eps;
+  void* kc;             // [blocks][G][bs][D]
+  void* vc;             // [blocks][G][bs][Dv]
+  int f32;
+};
+void kv_store(const KvStoreParams& P, const StepRows& R, hipStream_t s);
+
+// ---- gated delta rule with a decay per key channel (stack_delta.hip)
+struct DeltaParams {
+  const float* proj;    // [B][ld] float32: q [G][D] | k [G][D] | v [H][Dv] (the convolution's inputs) at off_q, write
+  int ld, off_q, off_b, off_a1, off_g1;  // strengths [H] at off_b, first factors of the low-rank maps at off_a1, off_g1
+  int H, G, D, Dv;
+  int taps;
+  const float* conv_w;  // [2 G D + H Dv][taps], the last tap is the current token's
+  float* window;        // slot s: window + s * state_stride = [taps - 1][2 G D + H Dv], oldest first
+  int rank_a, rank_g;
+  const void* a2;       // [H * D][rank_a] matrix dtype
+  const void* g2;       // [H * Dv][rank_g] matrix dtype
+  const float* a_log;   // [H]
+  const float* dt_bias; // [H * D]
+  const float* norm_w;  // [Dv]
+  float eps;
+  float* state;         // slot s: state + s * state_stride = S [H][D][Dv] float32
+  long long state_stride;
+  float* x;             // [B][ld_x] scratch: prepared q | k | v
+  int ld_x;
+  float* lg;            // [B][ld_lg] scratch: log decays [H * D] (their running sums inside a chunk, in the chunked form)
+  int ld_lg;
+  float* gate;          // [B][ld_gate] scratch: sigmoid output gate [H * Dv]
+  int ld_gate;
+  void* out;            // [B][ld_out] matrix dtype: out_scale * rms_norm(o per head) * norm_w * gate, head-major
+  int ld_out;
+  float out_scale;
+  int f32;
+};
+// convolution (its windows advanced), unit vectors, log decays and gates of the step's rows into the scratch rows
+void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s);
+void delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s);  // after delta_prepare: token by token
+bool delta_supported(int D, int Dv, int rank_a, int rank_g);
+// after delta_prepare: in chunks (prompt portions) over the host-built chunk table of the chunked retention
+struct DeltaChunkWs {
+  const int* chunks;
+  int nchunks, max_chunks;
+  float* Sin;           // [chunks][s_stride]: every chunk's incoming state
+  long long s_stride;
+  float* W;             // [B][ld_lg]
+  float* Kd;            // [B][ld_lg]
+  float* u;             // [B][ld_gate]
+  float* Bm;            // [B][H][delta_chunk_rows()]
+};
+void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& W, hipStream_t s);
+int delta_chunk_rows();
+bool delta_chunk_supported(int D, int Dv);
 
 }  // namespace stack
 }  // namespace omx

@@ -146,6 +146,37 @@ void rotate_fold(const RotFoldParams& P, const StepRows& R, hipStream_t s) {
   launched("rotate_fold");
 }
 
+// ------------------------------------------------------------------------------------------------ K/V store
+// One wave per (row, key/value head): the key as it is, the value as it is or divided by its root mean square
+template <typename T>
+__global__ __launch_bounds__(256) void kv_store_kernel(KvStoreParams P, StepRows R) {
+  const int lane = threadIdx.x & 63;
+  const long long item = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (long long)R.B * P.G) return;
+  const int b = (int)(item / P.G), g = (int)(item % P.G);
+  const float* k = P.proj + (long long)b * P.ld + P.off_k + g * P.D;
+  const float* v = P.proj + (long long)b * P.ld + P.off_v + g * P.Dv;
+  const int slot = R.slot[b];
+  const long long at = ((long long)(slot / R.bs) * P.G + g) * R.bs + slot % R.bs;
+  for (int d = lane; d < P.D; d += 64) st((T*)P.kc + at * P.D + d, k[d]);
+  float f = 1.f;
+  if (P.v_unit) {
+    float ss = 0.f;
+    for (int d = lane; d < P.Dv; d += 64) ss += v[d] * v[d];
+    f = 1.f / sqrtf(wave_sum(ss) / (float)P.Dv + P.eps);
+  }
+  for (int d = lane; d < P.Dv; d += 64) st((T*)P.vc + at * P.Dv + d, v[d] * f);
+}
+void kv_store(const KvStoreParams& P, const StepRows& R, hipStream_t s) {
+  check(R.B > 0 && P.proj && P.kc && P.vc && P.G > 0 && P.D > 0 && P.Dv > 0 && R.slot && R.bs > 0, "kv_store: bad operands");
+  const dim3 grid((unsigned)(((long long)R.B * P.G + 3) / 4));
+  if (P.f32)
+    hipLaunchKernelGGL(kv_store_kernel<float>, grid, dim3(256), 0, s, P, R);
+  else
+    hipLaunchKernelGGL(kv_store_kernel<bf16>, grid, dim3(256), 0, s, P, R);
+  launched("kv_store");
+}
+
 // ------------------------------------------------------------------------------------------------ gated dense feed-forward
 // out = relu(z[:, :F]) * z[:, F:2F], matrix dtype
 template <typename T>
@@ -198,7 +229,8 @@ void gemv_relu_glu(const void* A, int lda, const void* W, int K, int F, int M, v
 // ------------------------------------------------------------------------------------------------ sigmoid router
 // Per row: s = sigmoid of the X router logits. The experts form group_count groups of neighbours; a group ranks by
 // the sum of its two largest scores and only experts of the best group_keep groups can be chosen; the `top` largest
-// scores among them are taken (ties: the lower index), divided by their sum (+ 1e-20) and multiplied by route_scale.
+// scores among them are taken (ties: the lower index), divided by their sum (+ 1e-20; route_raw: left as they are) and
+// multiplied by route_scale.
 // One wave per row with an expert per lane (X <= 64); lane q < top ends up holding the q-th choice.
 __device__ __forceinline__ void route_sigmoid_wave(const MoeParams& P, const float* row, int lane, int& who_q, float& w_q) {
   const bool has = lane < P.X;
@@ -244,7 +276,7 @@ __device__ __forceinline__ void route_sigmoid_wave(const MoeParams& P, const flo
     if (lane == who) ch = -INFINITY;
   }
   const float sum = wave_sum(lane < P.top ? w_q : 0.f) + 1e-20f;
-  w_q = w_q / sum * P.route_scale;
+  w_q = (P.route_raw ? w_q : w_q / sum) * P.route_scale;
 }
 // the same by one thread, for up to 256 experts (sc: X floats of scratch)
 __device__ void route_sigmoid_serial(const MoeParams& P, const float* row, float* sc, int* ids, float* wts) {
@@ -293,7 +325,7 @@ __device__ void route_sigmoid_serial(const MoeParams& P, const float* row, float
     wts[jj] = bv;
     sum += bv;
   }
-  for (int jj = 0; jj < P.top; ++jj) wts[jj] = wts[jj] / sum * P.route_scale;
+  for (int jj = 0; jj < P.top; ++jj) wts[jj] = (P.route_raw ? wts[jj] : wts[jj] / sum) * P.route_scale;
 }
 constexpr int ROUTE_SIG_MAX = 256;
 __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
@@ -348,13 +380,14 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_experts_kernel(MoeParam
     P.ew[(long long)b * P.ld_top + lane] = w;
   }
   const int e = __shfl(who, jj, 64);
+  const float w_in = P.w_input ? __shfl(w, jj, 64) : 1.f;
   if (f >= P.F) return;
   const T* x = (const T*)P.h + (long long)b * P.E;
   const T* wg = (const T*)P.w_gu + ((long long)e * 2 * P.F + f) * P.E;
   const T* wu = wg + (long long)P.F * P.E;
   const float gate = wave_dot<T>(wg, x, P.E, lane, vec != 0);
   const float up = wave_dot<T>(wu, x, P.E, lane, vec != 0);
-  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, silu(gate) * up);
+  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, moe_unit(P.act, P.limit, w_in, gate, up));
 }
 bool moe_route_sigmoid_fused_supported(const MoeParams& P) { return P.X <= 64; }
 void moe_route_sigmoid_experts(const MoeParams& P, hipStream_t s) {

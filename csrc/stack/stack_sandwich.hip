@@ -17,6 +17,8 @@ namespace omx {
 namespace stack {
 
 // ------------------------------------------------------------------------------------------------ input norm + convolution
+// (the norm's weight is one number, or with P.gvec one per channel; the window sits oldest first, or with P.ring as a
+// ring over positions, where a row never overwrites an input that another row of a step of few rows still reads)
 // One block per row r. hn[r] = x[r] * g / rms(x[r]); out[r][c] = hn[r][c] + sum_j w[c][j] hn(p_r - (taps - 1) + j)[c].
 // Inputs of earlier rows of the same step are recomputed from the stream with their own row's scale (the same
 // operations in the same order as that row's block, so the value is the same bit for bit); inputs from before the
@@ -31,7 +33,8 @@ __global__ __launch_bounds__(256) void scalar_norm_conv_kernel(CanonParams P, St
   int nb = 0;  // rows of the same sequence right before r, up to taps - 1
   while (nb < K - 1 && r - nb - 1 >= 0 && R.q_seq[r - nb - 1] == seq) ++nb;
   const bool alone = nb == 0 && !(r + 1 < R.B && R.q_seq[r + 1] == seq);
-  const float g = P.g[0];
+  const float g = P.gvec ? 1.f : P.g[0];
+  const int pos = P.ring ? R.pos[r] : 0;
   float scale[CANON_MAX_TAPS];  // indexed by constants only (unrolled), so it lives in registers
 #pragma unroll
   for (int k = 0; k < CANON_MAX_TAPS; ++k) {
@@ -45,16 +48,26 @@ __global__ __launch_bounds__(256) void scalar_norm_conv_kernel(CanonParams P, St
   }
   float* win = P.window ? P.window + (long long)seq * P.stride : nullptr;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < E; c += 256 * gridDim.y) {
-    const float cur = P.x[(long long)r * E + c] * scale[0];
+    const float gc = P.gvec ? P.g[c] : 1.f;
+    const float cur = P.x[(long long)r * E + c] * scale[0] * gc;
     P.hn[(long long)r * E + c] = cur;
     float acc = cur;
 #pragma unroll
     for (int back = CANON_MAX_TAPS - 1; back >= 0; --back) {  // oldest input first, as the taps are stored
       if (back < K) {
-        const float v = back == 0 ? cur : back <= nb ? P.x[(long long)(r - back) * E + c] * scale[back]
-                                                     : win[(long long)(K - 1 - (back - nb)) * E + c];
+        float v = cur;
+        if (back > 0) {
+          if (back <= nb)
+            v = P.x[(long long)(r - back) * E + c] * scale[back] * gc;
+          else if (P.ring)
+            v = back <= pos ? win[(long long)((pos - back) % P.ring) * E + c] : 0.f;
+          else
+            v = win[(long long)(K - 1 - (back - nb)) * E + c];
+        }
         acc += P.w[(long long)c * K + (K - 1 - back)] * v;
-        if (alone && back > 0) win[(long long)(K - 1 - back) * E + c] = back == 1 ? cur : win[(long long)(K - back) * E + c];
+        if (P.ring) {
+          if (alone && back == 0 && K > 1) win[(long long)(pos % P.ring) * E + c] = cur;
+        } else if (alone && back > 0) win[(long long)(K - 1 - back) * E + c] = back == 1 ? cur : win[(long long)(K - back) * E + c];
       }
     }
     st((T*)P.out + (long long)r * E + c, acc);
@@ -68,6 +81,12 @@ __global__ __launch_bounds__(256) void canon_window_kernel(CanonParams P, StepRo
   int n = 1;  // rows of the sequence in this step, up to taps - 1
   while (n < K - 1 && r - n >= 0 && R.q_seq[r - n] == seq) ++n;
   float* win = P.window + (long long)seq * P.stride;
+  if (P.ring) {
+    const int pos = R.pos[r];
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < E; c += 256 * gridDim.y)
+      for (int back = 0; back < n; ++back) win[(long long)((pos - back) % P.ring) * E + c] = P.hn[(long long)(r - back) * E + c];
+    return;
+  }
   for (int c = blockIdx.y * 256 + threadIdx.x; c < E; c += 256 * gridDim.y)
     for (int sidx = 0; sidx < K - 1; ++sidx) {  // ascending: a thread never reads what it has overwritten
       const int back = K - 2 - sidx;
@@ -76,7 +95,7 @@ __global__ __launch_bounds__(256) void canon_window_kernel(CanonParams P, StepRo
 }
 void scalar_norm_conv(const CanonParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.x && P.g && P.hn && P.out && P.E > 0 && P.taps >= 1 && P.taps <= CANON_MAX_TAPS && P.w &&
-            (P.taps == 1 || P.window),
+            (P.taps == 1 || (P.window && (P.ring == 0 || (P.ring >= P.taps && R.pos)))),
         "scalar_norm_conv: bad operands (at most 8 taps)");
   // few rows (decode steps): the channels are shared among several blocks per row (each sums the whole row itself)
   const dim3 grid(R.B, R.B <= 64 ? std::min(8, (P.E + 255) / 256) : 1);

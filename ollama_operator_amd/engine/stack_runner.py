@@ -26,8 +26,8 @@ import time
 
 import torch
 
-from ..models.config import (BLOCK_POSTNORM, BLOCK_PRENORM, BLOCK_SANDWICH, FF_DENSE, FF_GLU, MIX_ATTENTION, MIX_LATENT,
-                             MIX_MAMBA2, MIX_MLSTM, MIX_RETENTION)
+from ..models.config import (ACT_CLAMPED_GLU, BLOCK_POSTNORM, BLOCK_PRENORM, BLOCK_SANDWICH, FF_DENSE, FF_GLU, MIX_ATTENTION,
+                             MIX_DELTA, MIX_GLA, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, MIX_MLSTM, MIX_RETENTION)
 from .runner import Runner
 from .weights import StackWeights
 
@@ -48,7 +48,8 @@ class StackExec:
         e.configure(dict(E=cfg.n_embd, V=cfg.n_vocab, eps=float(cfg.norm_eps), residual_mult=float(cfg.residual_mult),
                          logit_softcap=float(cfg.logit_softcap), f32=int(w.dtype == torch.float32),
                          max_B=r.max_batch, max_seqs=r.max_seqs, block=int(cfg.block), embed_scale=float(cfg.embed_scale),
-                         logit_scale=float(cfg.logit_scale), canon_taps=int(cfg.canon_taps)))
+                         logit_scale=float(cfg.logit_scale), canon_taps=int(cfg.canon_taps),
+                         canon_both=int(cfg.canon_both), canon_ring=int(cfg.canon_ring)))
         e.set_globals(dict(embed=p(w.embed), loop_in=p(w.loop_in), final_w=p(w.final_w), final_b=p(w.final_b),
                            head=p(w.head)))
         for i, (L, spec) in enumerate(zip(w.layers, cfg.layers)):
@@ -94,7 +95,9 @@ class StackExec:
                              ret_sin=p(r.ret_sin), ret_u_stride=r.ret_u.shape[1], cbuf=p(r.cbuf), ld_cbuf=r.cbuf.shape[1],
                              lat=p(r.latbuf), ld_lat=r.latbuf.shape[1], idw=p(r.idw), coef=p(r.scan_coef),
                              ld_coef=(r.scan_coef.shape[1] if r.scan_coef is not None else 0), ctot=p(r.scan_ctot),
-                             hn=p(r.hn), y2=p(r.ybuf2),
+                             hn=p(r.hn), y2=p(r.ybuf2), **{"dl_" + k: p(v) for k, v in r.delta_ws.items()},
+                             ld_dl_lg=r.delta_ws["lg"].shape[1], ld_dl_gate=r.delta_ws["gate"].shape[1],
+                             dl_heads=r.delta_ws["Bm"].shape[1] // 32,
                              **{"moe_" + k: (v if isinstance(v, int) else p(v)) for k, v in r.moe_ws.items()}))
         e.set_inputs(dict(tokens=p(r.d_tokens), pos=p(r.d_pos), slot=p(r.d_slot), q_len=p(r.d_qlen),
                           q_seq=p(r.d_qseq), block_table=p(r.d_block_table), max_blocks=r.max_blocks,
@@ -136,14 +139,25 @@ class StackExec:
                  window=m.window, maps=m.maps, diff=m.diff, lam=L.get("lam", 0.0), gate=int(m.gate), talk=p(L.get("talk")),
                  score_talk=int(m.score_talk), rot_dim=m.rot_dim, kv_rank=m.kv_rank, dkv_norm=p(L.get("dkv_norm")),
                  w_uk=p(L.get("w_uk")), w_uvT=p(L.get("w_uvT")), w_ukT=p(L.get("w_ukT")), w_uv=p(L.get("w_uv")),
-                 **{"off_" + k: v for k, v in L["off"].items() if k in ("q", "k", "v", "g", "router")})
+                 chunk=m.chunk, v_unit=int(m.v_unit), slopes=p(L.get("slopes")), canon=p(L.get("canon")), canon2=p(L.get("canon2")),
+                 decay=p(L.get("decay")), mnorm=p(L.get("mnorm")), state=m.state, groups=m.groups, conv=m.conv,
+                 norm_groups=m.norm_groups, conv_w=p(L.get("conv_w")), conv_b=p(L.get("conv_b")), dt_bias=p(L.get("dt_bias")),
+                 a_log=p(L.get("a_log")), d_skip=p(L.get("d_skip")), left_scale=m.left_scale, right_scale=m.right_scale,
+                 **{"off_" + k: v for k, v in L["off"].items()})
+        if m.right is not None:
+            g = m.right
+            if g.kind != MIX_DELTA:
+                raise ValueError("a pre-norm layer's second mixer is the gated delta rule")
+            d.update(r_delta=1, r_heads=g.heads, r_kv_heads=g.kv_heads, r_dim=g.dim, r_vdim=g.vdim, r_rank=g.decay_rank,
+                     r_grank=g.gate_rank, conv=g.conv, a2=p(L["a2"]), g2=p(L["g2"]), gnorm=p(L["gnorm"]))
         if f is not None:
             d.update(norm2_w=p(L["norm2_w"]), w_ff=p(L["w_ff"]), n_ff=L["n_ff"], ff=f.ff)
             if f.kind == FF_GLU:
                 d.update(ff_dense=3, w_dense_down=p(L["w_dense_down"]))
             else:
                 d.update(experts=f.experts, top=f.top, w_gu=p(L["w_gu"]), w_down=p(L["w_down"]), group_count=f.group_count,
-                         group_keep=f.group_keep, route_scale=f.route_scale)
+                         group_keep=f.group_keep, route_scale=f.route_scale, route_raw=int(not f.route_norm),
+                         expert_act=int(f.expert_act == ACT_CLAMPED_GLU), limit=f.limit, scale_input=int(f.scale_input))
         return d
 
     def bind_chunks(self, rows) -> None:
@@ -259,13 +273,15 @@ class StackRunner(Runner):
         mam = [s.mixer for s in cfg.layers if s.mixer.kind == MIX_MAMBA2]
         talk = [s.mixer for s in cfg.layers if s.mixer.talk]  # every query head against every key/value head's values
         fold = [s.mixer for s in cfg.layers if s.mixer.score_talk]  # queries folded through the score-mixing matrix
+        deltas = [s.mixer.right for s in cfg.layers if s.mixer.right is not None and s.mixer.right.kind == MIX_DELTA]
         maps = [s.mixer for s in cfg.layers if s.mixer.maps > 1]    # the maps' outputs before they are combined
         self.cbuf = torch.zeros(max_batch, (max([m.heads * m.cache_dim for m in lat] + [m.conv_channels for m in mam] +
                                                 [m.heads * m.kv_heads * m.vdim for m in talk] +
                                                 [m.heads * m.kv_heads * m.dim for m in fold] +
-                                                [m.heads * m.maps * m.vdim for m in maps], default=1) + 3) // 4 * 4, **f32)
+                                                [m.heads * m.maps * m.vdim for m in maps] +
+                                                [m.conv_channels for m in deltas], default=1) + 3) // 4 * 4, **f32)
         sandwich = cfg.block == BLOCK_SANDWICH
-        self.hn = torch.zeros(max_batch if sandwich else 1, E, **f32)      # normed rows before the input convolution
+        self.hn = torch.zeros(max_batch if sandwich or cfg.canon_both else 1, E, **f32)  # normed rows before the input convolution
         self.ybuf2 = torch.zeros(max_batch if sandwich else 1, E, **f32)   # the second mixer's projected output
         self.latbuf = torch.zeros(max_batch, (max([m.heads * m.kv_rank for m in lat], default=1) + 7) // 8 * 8, **tt)
         self.idw = torch.zeros(max_batch, **f32)
@@ -279,9 +295,10 @@ class StackRunner(Runner):
                                                    s.mixer.right.n_out if s.mixer.right is not None else 0)
                                                for s in cfg.layers), **f32)
         # chunked retention of prompt portions: the chunk table and one state per chunk (its U, its incoming state)
-        rets = [s.mixer for s in cfg.layers if s.mixer.kind in (MIX_RETENTION, MIX_MLSTM, MIX_MAMBA2)]
-        glas = [s.mixer.right for s in cfg.layers if s.mixer.right is not None]  # gated linear attention beside attention
-        rets += glas
+        rets = [s.mixer for s in cfg.layers if s.mixer.kind in (MIX_RETENTION, MIX_MLSTM, MIX_MAMBA2, MIX_LINEAR)]
+        # gated linear attention beside attention
+        glas = [s.mixer.right for s in cfg.layers if s.mixer.right is not None and s.mixer.right.kind == MIX_GLA]
+        rets += glas + deltas
         n_ch = max_batch // 32 + max_seqs + 1 if rets and max_batch > 16 else 1
         self.d_chunks = torch.zeros(n_ch, 4, **i32)
         self.d_tiles = torch.zeros(max_batch // 32 + max_seqs + 1, 2, **i32)  # attention query tiles of a step
@@ -291,6 +308,11 @@ class StackRunner(Runner):
         hmax = max([m.heads for m in rets if m.kind != MIX_RETENTION], default=0) if n_ch > 1 else 0
         # (gated linear attention: the rows' running log decays, one per head and key channel)
         self.scan_coef = torch.zeros(max_batch, max([3 * hmax] + ([m.n_q for m in glas] if n_ch > 1 else [])), **f32) if hmax else None
+        # gated delta rule: the rows' log decays and output gates; chunked form: the solved rows, decayed keys, pair weights
+        nd, nv, nh = (max([f(m) for m in deltas], default=1) for f in (lambda m: m.n_q, lambda m: m.n_out, lambda m: m.heads))
+        nb = max_batch if deltas else 1
+        self.delta_ws = dict(lg=torch.zeros(nb, nd, **f32), gate=torch.zeros(nb, nv, **f32), W=torch.zeros(nb, nd, **f32),
+                             Kd=torch.zeros(nb, nd, **f32), u=torch.zeros(nb, nv, **f32), Bm=torch.zeros(nb, nh * 32, **f32))
         self.scan_ctot = torch.zeros(n_ch, hmax, **f32) if hmax else None
         self.ret_sin = torch.zeros_like(self.ret_u)
         # decode attention over long contexts: partials {maximum, sum, output} of up to 16 splits per (row, head)
