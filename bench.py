@@ -413,6 +413,43 @@ def dekalorn_config(z: dict, vocab: int = 32000):
     return StackConfig(arch="dekalorn", n_vocab=vocab, n_embd=z["E"], layers=layers, norm_eps=1e-6, block=BLOCK_PRENORM)
 
 
+# the Rogisun design at the same widths: constant-decay linear attention, two Mamba-2 layers, a pair layer (attention in
+# blocks of positions beside a gated delta rule), twice; two-tap input convolutions; every feed-forward routes 2 of 8 experts
+ROGISUN_SIZES = {
+    "s": dict(E=1024, pattern="lmmp" * 2, lin=(8, 64, 128), mamba=(16, 64, 64, 1), H=16, G=4, D=64, chunk=1024,
+              delta=(8, 4, 64, 128), rank=32, F=512, X=8, top=2),
+    "m": dict(E=2048, pattern="lmmp" * 2, lin=(16, 64, 128), mamba=(32, 64, 128, 2), H=16, G=4, D=128, chunk=1024,
+              delta=(16, 8, 64, 128), rank=64, F=1024, X=8, top=2),
+}
+
+
+def rogisun_config(z: dict, vocab: int = 32000):
+    """A Rogisun model with the sizes of a real model's layers (random weights)."""
+    from ollama_operator_amd.models.config import (ACT_CLAMPED_GLU, BLOCK_PRENORM, FF_MOE, GATE_ELEMENT, GATE_HEAD, MIX_ATTENTION,
+                                                    MIX_DELTA, MIX_LINEAR, MIX_MAMBA2, ROUTE_SIGMOID_GROUPS, LayerSpec, MixerSpec,
+                                                    MoESpec, StackConfig)
+    layers = []
+    for c in z["pattern"]:
+        if c == "l":
+            h, d, dv = z["lin"]
+            m = MixerSpec(kind=MIX_LINEAR, heads=h, kv_heads=h, dim=d, vdim=dv, gate=GATE_ELEMENT,
+                          decay=tuple(1.0 - 2.0 ** (-2 - i % 8) for i in range(h)))
+        elif c == "m":
+            h, dv, n, g = z["mamba"]
+            m = MixerSpec(kind=MIX_MAMBA2, heads=h, kv_heads=g, dim=n, vdim=dv, state=n, groups=g, conv=4, norm_groups=g)
+        else:
+            h, g, d, dv = z["delta"]
+            m = MixerSpec(kind=MIX_ATTENTION, heads=z["H"], kv_heads=z["G"], dim=z["D"], vdim=z["D"], scale=z["D"] ** -0.5,
+                          chunk=z["chunk"], alibi=True, v_unit=True, gate=GATE_HEAD, left_scale=0.7, right_scale=1.2,
+                          right=MixerSpec(kind=MIX_DELTA, heads=h, kv_heads=g, dim=d, vdim=dv, conv=4,
+                                          decay_rank=z["rank"], gate_rank=z["rank"]))
+        f = MoESpec(kind=FF_MOE, route=ROUTE_SIGMOID_GROUPS, experts=z["X"], top=z["top"], ff=z["F"], shared_gate=False,
+                    route_norm=False, expert_act=ACT_CLAMPED_GLU, limit=4.0, scale_input=True)
+        layers.append(LayerSpec(mixer=m, mlp=f))
+    return StackConfig(arch="rogisun", n_vocab=vocab, n_embd=z["E"], layers=layers, norm_eps=1e-6, block=BLOCK_PRENORM,
+                       canon_taps=2, canon_both=True, tied_head=True)
+
+
 def suvunex_config(z: dict, vocab: int = 32000):
     """A Suvunex model with the sizes of a real model's layers (random weights)."""
     from ollama_operator_amd.models.config import (BLOCK_SANDWICH, FF_GLU, MIX_ATTENTION, MIX_GLA, QK_NORM_UNIT_LAST,
@@ -554,6 +591,15 @@ def bench_stack(a) -> None:
             out[name]["dekalorn_bf16"] = measure(r)
             out[name]["dekalorn_weights_gb"] = round(r.w.nbytes / 1e9, 3)
             r.close()
+        if a.rogisun:  # the Rogisun design at the same width and depth, through the same engine and measurement
+            d = os.path.join(a.dir, f"rogisun-{name}")
+            if not os.path.exists(os.path.join(d, "model.safetensors")):
+                write_random_stack(d, rogisun_config(ROGISUN_SIZES[name]), seed=0)
+            r = StackRunner(d, device="cuda:0", dtype="bfloat16", max_batch=a.chunk, max_seqs=2, ctx=ctx)
+            r.warmup()
+            out[name]["rogisun_bf16"] = measure(r)
+            out[name]["rogisun_weights_gb"] = round(r.w.nbytes / 1e9, 3)
+            r.close()
         if not a.stack_only:
             cfg = ModelConfig(name=f"mixtral-like-{name}", n_vocab=32000, n_embd=z["E"], n_layer=len(z["pattern"]),
                               n_head=z["H"], n_head_kv=z["G"], n_ff=z["F"], n_rot=z["D"], n_embd_head=z["D"],
@@ -581,6 +627,8 @@ def main():
     ap.add_argument("--no-bizulix", action="store_true", help="with --stack: skip the Bizulix model (profiles of one design)")
     ap.add_argument("--suvunex", action="store_true", help="with --stack: also measure the Suvunex design (attention with "
                     "sinks beside gated linear attention, mixed-heads attention, input convolutions) at the same widths")
+    ap.add_argument("--rogisun", action="store_true", help="with --stack: also measure the Rogisun design (constant-decay "
+                    "linear attention, Mamba-2, attention in blocks of positions beside a gated delta rule, clamped experts)")
     ap.add_argument("--dekalorn", action="store_true", help="with --stack: also measure the Dekalorn design (windowed "
                     "differential and mixed-score attention, latent attention, sigmoid-routed experts) at the same widths")
     ap.add_argument("--gpus", type=int, default=1)

@@ -70,6 +70,8 @@ def write_random_stack(path: str, cfg, seed: int = 0, std: float = 0.05) -> None
         return write_random_suvunex(path, cfg, seed=seed)
     if cfg.arch == "dekalorn":
         return write_random_dekalorn(path, cfg, seed=seed)
+    if cfg.arch == "rogisun":
+        return write_random_rogisun(path, cfg, seed=seed)
     g = torch.Generator().manual_seed(seed)
     E, V = cfg.n_embd, cfg.n_vocab
     T: dict = {}
@@ -342,4 +344,88 @@ def write_random_dekalorn(path: str, cfg, seed: int = 0) -> None:
     os.makedirs(path, exist_ok=True)
     with open(os.path.join(path, "config.json"), "w") as fh:
         json.dump(cfg.to_dekalorn(), fh, indent=1)
+    write_safetensors(os.path.join(path, "model.safetensors"), T)
+
+
+def write_random_rogisun(path: str, cfg, seed: int = 0) -> None:
+    """Random-init model folder of the Rogisun design (its tensor names). Projections ~ N(0, 1 / fan-in); norm weights
+    near 1; input-convolution taps of a fraction of the identity; step sizes and decays spread so that some heads and
+    key channels forget in a few tokens and others keep for hundreds; gate and up rows wide enough that the experts'
+    clamps act; router matrices wide enough that the chosen experts are not a close call. Inner sizes of low-rank maps
+    that the configuration leaves open are 8."""
+    import json
+    import os
+
+    import torch
+
+    from ..engine.safetensors_io import write_safetensors
+    from .config import MIX_LINEAR, MIX_MAMBA2
+    g = torch.Generator().manual_seed(seed)
+    E, V = cfg.n_embd, cfg.n_vocab
+    T: dict = {}
+
+    def rnd(name, shape, s, mean=0.0):
+        T[name] = (mean + s * torch.randn(*shape, generator=g)).to(torch.bfloat16)
+
+    def uni(name, shape, lo, hi):
+        T[name] = (lo + (hi - lo) * torch.rand(*shape, generator=g)).to(torch.bfloat16)
+
+    def lin(name, n_out, n_in, gain=1.0):
+        rnd(name, (n_out, n_in), gain / n_in ** 0.5)
+
+    rnd("embed", (V, E), 1.0)
+    for i, spec in enumerate(cfg.layers):
+        m, f, p = spec.mixer, spec.mlp, f"l{i}."
+        H, G, D, Dv = m.heads, m.kv_heads, m.dim, m.vdim
+        rnd(p + "norm1", (E,), 0.1, 1.0)
+        rnd(p + "canon1", (E, cfg.canon_taps), 0.3)
+        if m.kind == MIX_LINEAR:
+            lin(p + "mix.q", H * D, E)
+            lin(p + "mix.k", H * D, E)
+            lin(p + "mix.v", H * Dv, E)
+            lin(p + "mix.g", H * Dv, E, 1.5)
+            rnd(p + "mix.norm", (H * Dv,), 0.1, 1.0)
+            lin(p + "mix.o", E, H * Dv)
+        elif m.kind == MIX_MAMBA2:
+            lin(p + "mix.in", 2 * H * Dv + 2 * m.groups * m.state + H, E)
+            rnd(p + "mix.conv", (m.conv_channels, m.conv), 0.6, 0.2)
+            rnd(p + "mix.conv.b", (m.conv_channels,), 0.1)
+            uni(p + "mix.dt_bias", (H,), -4.0, -0.5)
+            uni(p + "mix.A_log", (H,), -4.0, 1.0)
+            uni(p + "mix.D", (H,), 0.5, 1.0)
+            rnd(p + "mix.norm", (H * Dv,), 0.1, 1.0)
+            lin(p + "mix.o", E, H * Dv)
+        else:
+            a, b, r = p + "mix.left.", p + "mix.right.", m.right
+            lin(a + "q", H * D, E, 1.5)
+            lin(a + "k", G * D, E, 1.5)
+            lin(a + "v", G * Dv, E)
+            lin(a + "g", H, E, 1.5)
+            lin(a + "o", E, H * Dv)
+            ra, rg = r.decay_rank or 8, r.gate_rank or 8
+            for k, n in (("q", r.kv_heads * r.dim), ("k", r.kv_heads * r.dim), ("v", r.n_out)):
+                lin(b + k, n, E, 1.5)
+                rnd(b + k + ".conv", (n, r.conv), 0.6, 0.2)
+            lin(b + "b", r.heads, E, 1.5)
+            uni(b + "A_log", (r.heads,), -3.0, 0.5)
+            lin(b + "a1", ra, E)
+            lin(b + "a2", r.n_q, ra, 1.5)
+            uni(b + "dt_bias", (r.n_q,), -5.0, 0.0)
+            lin(b + "g1", rg, E)
+            lin(b + "g2", r.n_out, rg, 1.5)
+            rnd(b + "norm", (r.vdim,), 0.1, 1.0)
+            lin(b + "o", E, r.n_out)
+        if f is None:
+            continue
+        rnd(p + "norm2", (E,), 0.1, 1.0)
+        rnd(p + "canon2", (E, cfg.canon_taps), 0.3)
+        for e in range(f.experts):
+            lin(f"{p}mlp.e{e}.gate", f.ff, E, 2.0)
+            lin(f"{p}mlp.e{e}.up", f.ff, E, 2.0)
+            lin(f"{p}mlp.e{e}.down", E, f.ff)
+        lin(p + "mlp.router", f.experts, E, 3.0)
+    rnd("final.norm", (E,), 0.1, 1.0)
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as fh:
+        json.dump(cfg.to_rogisun(), fh, indent=1)
     write_safetensors(os.path.join(path, "model.safetensors"), T)
