@@ -262,6 +262,7 @@ PYBIND11_MODULE(_stack, m) {
         w.ctot = Pp<float>(ptr(d, "ctot"));
         w.hn = Pp<float>(ptr(d, "hn"));
         w.y2 = Pp<float>(ptr(d, "y2"));
+        w.rscale = Pp<float>(ptr(d, "rscale"));
         w.lna = w.coef;
         w.dl_lg = Pp<float>(ptr(d, "dl_lg"));
         w.ld_dl_lg = geti(d, "ld_dl_lg");

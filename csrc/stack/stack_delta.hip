@@ -30,14 +30,15 @@ __device__ __forceinline__ float delta_softplus(float z) { return z > 20.f ? z :
 // (oldest first); a sequence with one row in the step advances its window here, the others in conv_window.
 template <typename T, int RB>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepRows R, int nlow) {
-  extern __shared__ float lds[];
+  extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int r0 = blockIdx.x * RB, nr = min(RB, R.B - r0);
   const int HD = P.H * P.D, HV = P.H * P.Dv, ra = P.rank_a, rg = P.rank_g;
   if ((int)blockIdx.y < nlow) {
+    const int ra4 = (ra + 3) / 4 * 4, LR = ra4 + (rg + 3) / 4 * 4;  // both maps' factors 16-byte aligned
     for (int i = tid; i < RB * (ra + rg); i += 256) {
       const int r = i / (ra + rg), c = i % (ra + rg);
-      lds[i] = r < nr ? P.proj[(long long)(r0 + r) * P.ld + (c < ra ? P.off_a1 + c : P.off_g1 + c - ra)] : 0.f;
+      lds[r * LR + (c < ra ? c : ra4 + c - ra)] = r < nr ? P.proj[(long long)(r0 + r) * P.ld + (c < ra ? P.off_a1 + c : P.off_g1 + c - ra)] : 0.f;
     }
     __syncthreads();
     const int c = blockIdx.y * 256 + tid;
@@ -45,7 +46,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
     const bool dec = c < HD;
     const int rank = dec ? ra : rg;
     const T* w = dec ? (const T*)P.a2 + (long long)c * ra : (const T*)P.g2 + (long long)(c - HD) * rg;
-    const float* x = lds + (dec ? 0 : ra);
+    const float* x = lds + (dec ? 0 : ra4);
     float z[RB];
 #pragma unroll
     for (int r = 0; r < RB; ++r) z[r] = dec ? P.dt_bias[c] : 0.f;
@@ -53,18 +54,24 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
     if (sizeof(T) == 2 && rank % 8 == 0 && (((uintptr_t)w) & 15) == 0) {
       for (; i < rank; i += 8) {
         const u32x4 a = *(const u32x4*)(w + i);
+        float w8[8];
 #pragma unroll
         for (int u = 0; u < 4; ++u) {
-          const float w0 = __uint_as_float(a[u] << 16), w1 = __uint_as_float(a[u] & 0xffff0000u);
+          w8[2 * u] = __uint_as_float(a[u] << 16);
+          w8[2 * u + 1] = __uint_as_float(a[u] & 0xffff0000u);
+        }
 #pragma unroll
-          for (int r = 0; r < RB; ++r) z[r] += w0 * x[r * (ra + rg) + i + 2 * u] + w1 * x[r * (ra + rg) + i + 2 * u + 1];
+        for (int r = 0; r < RB; ++r) {
+          const f32x4 xa = *(const f32x4*)(x + r * LR + i), xb = *(const f32x4*)(x + r * LR + i + 4);
+          z[r] += w8[0] * xa[0] + w8[1] * xa[1] + w8[2] * xa[2] + w8[3] * xa[3] + w8[4] * xb[0] + w8[5] * xb[1] + w8[6] * xb[2] +
+                  w8[7] * xb[3];
         }
       }
     }
     for (; i < rank; ++i) {
       const float w0 = ld(w + i);
 #pragma unroll
-      for (int r = 0; r < RB; ++r) z[r] += w0 * x[r * (ra + rg) + i];
+      for (int r = 0; r < RB; ++r) z[r] += w0 * x[r * LR + i];
     }
     const float ea = dec ? expf(P.a_log[c / P.D]) : 0.f;
 #pragma unroll
@@ -83,6 +90,57 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
   const int n = isv ? P.Dv : P.D, K = P.taps;
   const int c0 = isv ? 2 * P.G * P.D + (unit - 2 * P.G) * P.Dv : unit * P.D;  // first channel of the unit
   const int ch = 2 * P.G * P.D + HV;
+  if (RB > 1 && K <= 4) {  // prompt portions: a channel's inputs of all rows (and the three before) requested at once
+    float v[DELTA_MAX / 64][RB];
+#pragma unroll
+    for (int u = 0; u < DELTA_MAX / 64; ++u) {
+      const int d = lane + 64 * u;
+      if (64 * u < n) {  // uniform over the wave
+        const int c = c0 + min(d, n - 1);
+        float in[RB + 3], w[4];
+#pragma unroll
+        for (int i = 0; i < RB + 3; ++i) in[i] = P.proj[(long long)min(max(r0 - 3 + i, 0), R.B - 1) * P.ld + P.off_q + c];
+#pragma unroll
+        for (int b = 0; b < 4; ++b) w[b] = b < K ? P.conv_w[(long long)c * K + (K - 1 - b)] : 0.f;  // w[back]
+#pragma unroll
+        for (int rr = 0; rr < RB; ++rr) {
+          const int r = min(r0 + rr, R.B - 1), seq = R.q_seq[r];
+          int nb = 0;
+          while (nb < K - 1 && r - nb - 1 >= 0 && R.q_seq[r - nb - 1] == seq) ++nb;
+          const bool alone = nb == 0 && !(r + 1 < R.B && R.q_seq[r + 1] == seq);
+          float* win = P.window + (long long)seq * P.state_stride;
+          float acc = 0.f;
+#pragma unroll
+          for (int back = 3; back >= 0; --back)
+            if (back < K) acc += w[back] * (back <= nb ? in[rr + 3 - back] : win[(long long)(K - 1 - (back - nb)) * ch + c]);
+          if (alone && rr < nr && d < n)
+            for (int sx = 0; sx < K - 1; ++sx)
+              win[(long long)sx * ch + c] = sx == K - 2 ? in[rr + 3] : win[(long long)(sx + 1) * ch + c];
+          v[u][rr] = d < n ? silu(acc) : 0.f;
+        }
+      } else {
+#pragma unroll
+        for (int rr = 0; rr < RB; ++rr) v[u][rr] = 0.f;
+      }
+    }
+#pragma unroll
+    for (int rr = 0; rr < RB; ++rr) {
+      if (rr >= nr) break;  // uniform over the block
+      float f = 1.f;
+      if (!isv) {
+        float ss = 0.f;
+#pragma unroll
+        for (int u = 0; u < DELTA_MAX / 64; ++u) ss += v[u][rr] * v[u][rr];
+        f = (isq ? 1.f / sqrtf((float)P.D) : 1.f) / sqrtf(wave_sum(ss) + 1e-6f);
+      }
+#pragma unroll
+      for (int u = 0; u < DELTA_MAX / 64; ++u) {
+        const int d = lane + 64 * u;
+        if (d < n) P.x[(long long)(r0 + rr) * P.ld_x + c0 + d] = v[u][rr] * f;
+      }
+    }
+    return;
+  }
   for (int rr = 0; rr < nr; ++rr) {
     const int r = r0 + rr, seq = R.q_seq[r];
     int nb = 0;  // rows of the same sequence right before r, up to taps - 1
@@ -121,7 +179,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
 template <typename T>
 static void launch_delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
   const int nlow = (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + 3) / 4;
-  const int rank = P.rank_a + P.rank_g;
+  const int rank = (P.rank_a + 3) / 4 * 4 + (P.rank_g + 3) / 4 * 4;
   if (R.B <= 16)
     hipLaunchKernelGGL((delta_prepare_kernel<T, 1>), dim3(R.B, nlow + nconv), dim3(256), rank * 4, s, P, R, nlow);
   else
@@ -289,11 +347,11 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
   float* be = Lc + DC * D1;        // [DC]
   for (int i = tid; i < DC * D; i += 256) {
     const int t = i / D, d = i % D;
-    const long long r = r0 + t;
-    const bool on = t < n;
-    qs[t * D1 + d] = on ? P.x[r * P.ld_x + hg * D + d] : 0.f;
-    ks[t * D1 + d] = on ? P.x[r * P.ld_x + (P.G + hg) * D + d] : 0.f;
-    Lc[t * D1 + d] = on ? P.lg[r * P.ld_lg + h * D + d] : 0.f;
+    const long long r = r0 + min(t, n - 1);  // (unconditional loads: all of them in flight together)
+    const float qv = P.x[r * P.ld_x + hg * D + d], kv = P.x[r * P.ld_x + (P.G + hg) * D + d], lv = P.lg[r * P.ld_lg + h * D + d];
+    qs[t * D1 + d] = t < n ? qv : 0.f;
+    ks[t * D1 + d] = t < n ? kv : 0.f;
+    Lc[t * D1 + d] = t < n ? lv : 0.f;
   }
   if (tid < DC) be[tid] = tid < n ? sigmoidf(P.proj[(long long)(r0 + tid) * P.ld + P.off_b + h]) : 0.f;
   __syncthreads();
@@ -327,13 +385,15 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
   for (int col = tid; col < D + Dv; col += 256) {  // forward substitution, a column per thread
     const bool key = col < D;
     float x[DC];
+    if (key) {
 #pragma unroll
-    for (int t = 0; t < DC; ++t) {
-      float v = 0.f;
-      if (t < n)
-        v = be[t] * (key ? ks[t * D1 + col] * expf(Lc[t * D1 + col])
-                         : P.x[(long long)(r0 + t) * P.ld_x + 2 * P.G * D + h * Dv + col - D]);
-      x[t] = v;
+      for (int t = 0; t < DC; ++t) x[t] = be[t] * ks[t * D1 + col] * expf(Lc[t * D1 + col]);
+    } else {
+      const float* v = P.x + 2 * P.G * D + h * Dv + col - D;
+#pragma unroll
+      for (int t = 0; t < DC; ++t) x[t] = v[(long long)(r0 + min(t, n - 1)) * P.ld_x];
+#pragma unroll
+      for (int t = 0; t < DC; ++t) x[t] *= be[t];  // 0 past the chunk's end
     }
 #pragma unroll
     for (int t = 1; t < DC; ++t) {
@@ -344,6 +404,7 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
         for (int i = 0; i < 4; ++i)
           if (4 * s4 + i < t) x[t] -= a[i] * x[4 * s4 + i];
       }
+      asm volatile("" ::: "memory");  // the rows of A are read as they are needed, not all at once into registers
     }
 #pragma unroll
     for (int t = 0; t < DC; ++t)
@@ -359,94 +420,122 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
 // Four waves share the state's rows: wave w holds the 16-row tiles w and w + 4 of S (16 columns) in accumulator layout,
 // S[16 tile + 4 (lane / 16) + i][lane % 16]. In that layout a register is a B operand of the first product if its K
 // order is d = 4 (lane / 16) + i, so W's rows are read four consecutive channels per lane and the state never moves.
+// The next chunk's operands are requested before the current chunk is multiplied, always (the last chunk asks for its own
+// again: a fetch under a condition would make every later wait a wait for all of it), in two register sets that take turns.
+// Indexes past the chunk or the head are clamped: a row past the chunk's end meets u = 0, a channel past the head a key of 0.
+template <int TJ>
+struct DeltaOps {
+  float wa[TJ][2][4], kd[TJ][8], el[TJ][4], vp[2];
+};
+template <int TJ, bool VEC>
+__device__ __forceinline__ void delta_fetch(const DeltaParams& P, const DeltaChunkWs& W, int r0, int n, int h, int ct,
+                                            DeltaOps<TJ>& o) {
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, m = lane & 15, q4 = lane >> 4, D = P.D;
+#pragma unroll
+  for (int j = 0; j < TJ; ++j) {
+    const int dt = 16 * (wv + 4 * j), dq = dt + 4 * q4;
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt) {
+      const float* wr = W.W + (long long)(r0 + min(16 * mt + m, n - 1)) * P.ld_lg + h * D;
+      if constexpr (VEC) {
+        const f32x4 a = *(const f32x4*)(wr + min(dq, D - 4));
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o.wa[j][mt][i] = a[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o.wa[j][mt][i] = wr[min(dq + i, D - 1)];
+      }
+    }
+#pragma unroll
+    for (int kk = 0; kk < 8; ++kk)
+      o.kd[j][kk] = W.Kd[(long long)(r0 + min(4 * kk + q4, n - 1)) * P.ld_lg + h * D + min(dt + m, D - 1)];
+    const float* lr = P.lg + (long long)(r0 + n - 1) * P.ld_lg + h * D;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o.el[j][i] = lr[min(dq + i, D - 1)];
+  }
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int e = tid + 256 * k;
+    o.vp[k] = W.u[(long long)(r0 + min(e >> 4, n - 1)) * P.ld_gate + h * P.Dv + min(ct * 16 + (e & 15), P.Dv - 1)];
+  }
+}
+template <int TJ, bool VEC>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams P, DeltaChunkWs W) {
   __shared__ float part[4][DC][17];
   __shared__ float us[DC][17];
-  const int c0 = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int c0 = blockIdx.x, h = blockIdx.y, ct = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   if (!(W.chunks[4 * c0 + 3] & 1)) return;  // not the first chunk of its sequence (uniform per block)
   const int D = P.D, Dv = P.Dv, m = lane & 15, q4 = lane >> 4;
-  const int col = blockIdx.z * 16 + m;
+  const int col = ct * 16 + m;
   const bool cok = col < Dv;
-  const int slot = W.chunks[4 * c0 + 2];
-  float* S0 = P.state + (long long)slot * P.state_stride + (long long)h * D * Dv;
-  f32x4 S[2];
+  float* S0 = P.state + (long long)W.chunks[4 * c0 + 2] * P.state_stride + (long long)h * D * Dv;
+  f32x4 S[TJ];
 #pragma unroll
-  for (int j = 0; j < 2; ++j)
+  for (int j = 0; j < TJ; ++j)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
-      S[j][i] = (cok && d < D) ? S0[(long long)d * Dv + col] : 0.f;
+      const float v = S0[(long long)min(d, D - 1) * Dv + min(col, Dv - 1)];
+      S[j][i] = (cok && d < D) ? v : 0.f;
     }
-  for (int c = c0;; ++c) {
-    const int r0 = W.chunks[4 * c], n = W.chunks[4 * c + 1], flags = W.chunks[4 * c + 3];
+  int c = c0, r0 = W.chunks[4 * c0], n = W.chunks[4 * c0 + 1], flags = W.chunks[4 * c0 + 3];
+  int cn = min(c0 + 1, W.nchunks - 1), r0n = W.chunks[4 * cn], nn = W.chunks[4 * cn + 1], fn = W.chunks[4 * cn + 3];
+  DeltaOps<TJ> opa, opb;
+  delta_fetch<TJ, VEC>(P, W, r0, n, h, ct, opa);
+  auto step = [&](DeltaOps<TJ>& cur, DeltaOps<TJ>& nxt) {
+    const bool last = (flags & 2) != 0;  // the sequence's last chunk of the step
+    delta_fetch<TJ, VEC>(P, W, last ? r0 : r0n, last ? n : nn, h, ct, nxt);
+    cn = min(c + 2, W.nchunks - 1);      // the table's entry after the next one
+    const int r0m = W.chunks[4 * cn], nm = W.chunks[4 * cn + 1], fm = W.chunks[4 * cn + 3];
     float* Sin = W.Sin + (long long)c * W.s_stride + (long long)h * D * Dv;
-    // operands of both products, requested together
-    float wa[2][2][4], kd[2][8], vp[2];
-    f32x4 el[2];
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      const int dt = 16 * (wv + 4 * j);
-#pragma unroll
-      for (int mt = 0; mt < 2; ++mt) {
-        const int t = 16 * mt + m;
-        const float* wr = W.W + (long long)(r0 + t) * P.ld_lg + h * D + dt + 4 * q4;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) wa[j][mt][i] = (t < n && dt + 4 * q4 + i < D) ? wr[i] : 0.f;
-      }
-#pragma unroll
-      for (int kk = 0; kk < 8; ++kk) {
-        const int t = 4 * kk + q4;
-        kd[j][kk] = (t < n && dt + m < D) ? W.Kd[(long long)(r0 + t) * P.ld_lg + h * D + dt + m] : 0.f;
-      }
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = dt + 4 * q4 + i;
-        el[j][i] = d < D ? P.lg[(long long)(r0 + n - 1) * P.ld_lg + h * D + d] : 0.f;
-      }
-    }
-#pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int e = tid + 256 * k, t = e >> 4, cc = blockIdx.z * 16 + (e & 15);
-      vp[k] = (t < n && cc < Dv) ? W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + cc] : 0.f;
-    }
-#pragma unroll
-    for (int j = 0; j < 2; ++j)
+    for (int j = 0; j < TJ; ++j)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
         if (cok && d < D) Sin[(long long)d * Dv + col] = S[j][i];
       }
-    f32x4 acc[2];
 #pragma unroll
     for (int mt = 0; mt < 2; ++mt) {
-      acc[mt] = f32x4{0.f, 0.f, 0.f, 0.f};
+      f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
+      for (int j = 0; j < TJ; ++j)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(wa[j][mt][i], S[j][i], acc[mt], 0, 0, 0);
+        for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.wa[j][mt][i], S[j][i], acc, 0, 0, 0);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) part[wv][16 * mt + 4 * q4 + i][m] = acc[mt][i];
+      for (int i = 0; i < 4; ++i) part[wv][16 * mt + 4 * q4 + i][m] = acc[i];
     }
     __syncthreads();
 #pragma unroll
     for (int k = 0; k < 2; ++k) {
-      const int e = tid + 256 * k, t = e >> 4, cm = e & 15, cc = blockIdx.z * 16 + cm;
-      const float u = vp[k] - (part[0][t][cm] + part[1][t][cm] + part[2][t][cm] + part[3][t][cm]);
-      us[t][cm] = u;  // rows past the chunk's end: 0 - 0
-      if (t < n && cc < Dv) W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + cc] = u;
+      const int e = tid + 256 * k, t = e >> 4, cm = e & 15;
+      const float u = cur.vp[k] - (part[0][t][cm] + part[1][t][cm] + part[2][t][cm] + part[3][t][cm]);
+      us[t][cm] = t < n ? u : 0.f;
+      if (t < n && ct * 16 + cm < Dv) W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + ct * 16 + cm] = u;
     }
     __syncthreads();
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
+    for (int j = 0; j < TJ; ++j) {
+      const bool dok = 16 * (wv + 4 * j) + m < D;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) S[j][i] *= expf(el[j][i]);
+      for (int i = 0; i < 4; ++i) S[j][i] *= __builtin_amdgcn_exp2f(cur.el[j][i] * 1.44269504088896341f);
 #pragma unroll
-      for (int kk = 0; kk < 8; ++kk) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[j][kk], us[4 * kk + q4][m], S[j], 0, 0, 0);
+      for (int kk = 0; kk < 8; ++kk)
+        S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(dok ? cur.kd[j][kk] : 0.f, us[4 * kk + q4][m], S[j], 0, 0, 0);
     }
-    if (flags & 2) break;  // the sequence's last chunk of the step
+    ++c;
+    r0 = r0n;
+    n = nn;
+    flags = fn;
+    r0n = r0m;
+    nn = nm;
+    fn = fm;
+    return last;
+  };
+  while (!step(opa, opb) && !step(opb, opa)) {
   }
 #pragma unroll
-  for (int j = 0; j < 2; ++j)
+  for (int j = 0; j < TJ; ++j)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int d = 16 * (wv + 4 * j) + 4 * q4 + i;
@@ -538,7 +627,16 @@ void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& 
   const dim3 grid(W.nchunks, P.H);
   hipLaunchKernelGGL(delta_wy_kernel, grid, dim3(256), delta_wy_lds(P.D), s, P, W);
   launched("delta_wy");
-  hipLaunchKernelGGL(delta_scan_kernel, dim3(W.nchunks, P.H, (P.Dv + 15) / 16), dim3(256), 0, s, P, W);
+  const dim3 sg(W.nchunks, P.H, (P.Dv + 15) / 16);
+  const int vec = P.D % 4 == 0 && P.ld_lg % 4 == 0 && ((uintptr_t)W.W & 15) == 0;
+  if (P.D <= 64 && vec)
+    hipLaunchKernelGGL((delta_scan_kernel<1, true>), sg, dim3(256), 0, s, P, W);
+  else if (P.D <= 64)
+    hipLaunchKernelGGL((delta_scan_kernel<1, false>), sg, dim3(256), 0, s, P, W);
+  else if (vec)
+    hipLaunchKernelGGL((delta_scan_kernel<2, true>), sg, dim3(256), 0, s, P, W);
+  else
+    hipLaunchKernelGGL((delta_scan_kernel<2, false>), sg, dim3(256), 0, s, P, W);
   launched("delta_scan");
   if (P.f32)
     hipLaunchKernelGGL(delta_out_kernel<float>, grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);

@@ -194,6 +194,11 @@ static bool chunked_scan_ok(const StackExecutor& e, const ScanParams& P, int B) 
          e.ws.ret.u_stride >= (long long)P.H * P.D * dvp && e.ws.ret.ld_o >= P.H * dvp && gated_chunk_supported(P.mode, P.D, P.Dv);
 }
 
+// pre-norm layers, steps of a few rows: the norm of a recurrent mixer's outputs happens in the output projection's launch
+bool StackExecutor::mixer_norm_fused(const LayerDesc& L, int B) const {
+  return cfg.block == 3 && gemv_group_rms_supported(B, L.heads * L.vdim, L.kind == 6 ? 1 : L.norm_groups, cfg.f32);
+}
+
 // Mamba-2 up to its output projection: convolution, the scan (prompt portions in chunks), the gate, the grouped norm
 void StackExecutor::mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
   const int n_out = L.heads * L.vdim, f32 = cfg.f32;
@@ -228,7 +233,8 @@ void StackExecutor::mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hi
     gated_scan_chunked(P, R, scan_ws(*this), nullptr, cfg.eps, nullptr, 0, f32, s);
   else
     gated_scan(P, R, s);
-  group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, L.norm_groups, L.mnorm, cfg.eps, nullptr, 0, ws.a, ws.ld_a, f32, s);
+  if (!mixer_norm_fused(L, B))
+    group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, L.norm_groups, L.mnorm, cfg.eps, nullptr, 0, ws.a, ws.ld_a, f32, s);
 }
 
 // linear attention with constant decays up to its output projection: the scan, one norm over all heads, the sigmoid gate
@@ -254,7 +260,8 @@ void StackExecutor::linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hi
     gated_scan_chunked(P, R, scan_ws(*this), nullptr, cfg.eps, nullptr, 0, cfg.f32, s);
   else
     gated_scan(P, R, s);
-  group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, 1, L.mnorm, cfg.eps, ws.proj + L.off_g, ws.ld_proj, ws.a, ws.ld_a, cfg.f32, s);
+  if (!mixer_norm_fused(L, B))
+    group_rms_cast(ws.ret.obuf, ws.ret.ld_o, B, n_out, 1, L.mnorm, cfg.eps, ws.proj + L.off_g, ws.ld_proj, ws.a, ws.ld_a, cfg.f32, s);
 }
 
 // the gated delta rule beside an attention, up to the output projection; its outputs sit beside the attention's in ws.a
@@ -415,7 +422,7 @@ void StackExecutor::layer_run_sandwich(int ri, int B, hipStream_t s) {
   StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
   {
     CanonParams C{ws.resid, L.norm_w, cfg.eps, E, taps, L.canon, r.state ? r.state + gla_floats : nullptr, r.state_stride, ws.hn, ws.h,
-                  f32};
+                  f32, 0, ws.rscale, 0};
     scalar_norm_conv(C, R, s);
   }
   {  // every matrix that reads the mixer's input, in one product
@@ -489,15 +496,29 @@ void StackExecutor::layer_run_sandwich(int ri, int B, hipStream_t s) {
 // before the softmax; latent attention with one gate per head;
 // before the mixer (and, with cfg.canon_both, a convolution on the inputs of both sublayers): Mamba-2, constant-decay linear
 // attention, or attention inside blocks of positions with a gated delta rule beside it.
-void StackExecutor::norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, int B, hipStream_t s) {
-  if (!cfg.canon_both) {
-    rms_norm_cast(ws.resid, nullptr, B, cfg.E, w, cfg.eps, ws.h, cfg.f32, s);
-    return;
-  }
+// The sublayer's input into ws.h, and with W the product with it into ws.proj.
+void StackExecutor::norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, const void* W, int N, int B,
+                            hipStream_t s) {
+  const int E = cfg.E, f32 = cfg.f32;
   StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
-  CanonParams C{ws.resid, w, cfg.eps, cfg.E, cfg.canon_taps, canon, cfg.canon_ring ? r.state + window_at : nullptr, r.state_stride,
-                ws.hn, ws.h, cfg.f32, 1, cfg.canon_ring};
-  scalar_norm_conv(C, R, s);
+  const bool fused = W && gemv_ln_supported(B, E, f32);  // decode steps: one launch
+  if (cfg.canon_both) {
+    CanonParams C{ws.resid, w, cfg.eps, E, cfg.canon_taps, canon, cfg.canon_ring ? r.state + window_at : nullptr, r.state_stride,
+                  ws.hn, ws.h, f32, 1, ws.rscale, cfg.canon_ring};
+    if (fused && gemv_canon_supported(cfg.canon_taps)) {
+      gemv_canon(C, W, B, N, ws.proj, ws.ld_proj, R, s);
+      return;
+    }
+    scalar_norm_conv(C, R, s);
+  } else if (fused) {
+    gemv_ln(ws.resid, E, w, nullptr, cfg.eps, W, B, N, ws.proj, ws.ld_proj, ws.h, nullptr, nullptr, f32, s);
+    return;
+  } else {
+    rms_norm_cast(ws.resid, nullptr, B, E, w, cfg.eps, ws.h, f32, s);
+  }
+  if (!W) return;
+  GemmParams g{ws.h, E, W, B, N, E, ws.proj, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
+  gemm(g, s);
 }
 void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   const RunDesc& r = runs.at(ri);
@@ -515,14 +536,10 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   // of 2 * dim
   AttnParams St{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, L.heads, L.kv_heads, 2 * L.dim, L.vdim, L.scale, 0.f, 0.f, 1,
                 r.kc, r.vc, ws.a, ws.ld_a, f32};
-  if (fused_in) {  // decode steps: norm + every matrix that reads the mixer's input (+ that K/V store) in one launch
-    gemv_ln(ws.resid, E, L.norm_w, nullptr, cfg.eps, L.w_in, B, L.n_in, ws.proj, ws.ld_proj, ws.h,
-            L.kind == 0 && L.maps == 2 ? &St : nullptr, &R, f32, s);
-  } else {
-    norm_in(r, L.norm_w, L.canon, win1, B, s);
-    GemmParams g{ws.h, E, L.w_in, B, L.n_in, E, ws.proj, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
-    gemm(g, s);
-  }
+  if (fused_in && L.kind == 0 && L.maps == 2)  // decode steps: norm, input projection and that K/V store in one launch
+    gemv_ln(ws.resid, E, L.norm_w, nullptr, cfg.eps, L.w_in, B, L.n_in, ws.proj, ws.ld_proj, ws.h, &St, &R, f32, s);
+  else
+    norm_in(r, L.norm_w, L.canon, win1, L.w_in, L.n_in, B, s);
   const bool tiled = B > SMALL_B && n_tiles > 0 && tiles;
   // a window bounds the keys of a decode step: no need to share them among blocks
   const int bound = L.chunk > 0 ? L.chunk : L.window;
@@ -584,16 +601,17 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     else
       attention(A, R, s);
   }
-  {
+  if ((L.kind == 4 || L.kind == 6) && mixer_norm_fused(L, B)) {  // decode steps: the mixer's output norm with the projection
+    const bool lin = L.kind == 6;
+    gemv_group_rms(ws.ret.obuf, ws.ret.ld_o, n_out, lin ? 1 : L.norm_groups, L.mnorm, cfg.eps, lin ? ws.proj + L.off_g : nullptr,
+                   ws.ld_proj, L.w_o, B, E, ws.resid, E, f32, s);
+  } else {
     GemmParams o{ws.a, ws.ld_a, L.w_o, B, E, n_out, ws.resid, E, EPI_RESID, 1.f, nullptr, 0.f, f32};
     gemm(o, s);
   }
   if (!L.ff_dense && !L.experts) return;
-  if (L.experts && fused_in) {  // decode steps: norm + router in one launch (the normed rows leave for the experts)
-    gemv_ln(ws.resid, E, L.norm2_w, nullptr, cfg.eps, L.w_ff, B, L.n_ff, ws.proj, ws.ld_proj, ws.h, nullptr, nullptr, f32, s);
-  } else {
-    norm_in(r, L.norm2_w, L.canon2, win2, B, s);
-  }
+  // the router's product leaves with the norm where the step allows it (the normed rows leave for the experts)
+  norm_in(r, L.norm2_w, L.canon2, win2, L.experts ? L.w_ff : nullptr, L.n_ff, B, s);
   if (L.ff_dense) {
     if (B <= 8) {  // decode steps: gate / up projection and activation in one launch
       gemv_relu_glu(ws.h, E, L.w_ff, E, L.ff, B, ws.hmid, ws.ld_hmid, f32, s);
@@ -605,10 +623,6 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     GemmParams d{ws.hmid, ws.ld_hmid, L.w_dense_down, B, E, L.ff, ws.resid, E, EPI_RESID, 1.f, nullptr, 0.f, f32};
     gemm(d, s);
     return;
-  }
-  if (!fused_in) {
-    GemmParams g{ws.h, E, L.w_ff, B, L.n_ff, E, ws.proj, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
-    gemm(g, s);
   }
   // the experts' weighted outputs are added straight into the stream (y = the stream, y_add)
   MoeParams M{ws.proj, ws.ld_proj, L.off_router, 0, 0, 0, B, E, L.experts, L.top, L.ff, 0, nullptr, ws.h, L.w_gu, L.w_down, nullptr,

@@ -147,6 +147,7 @@ struct StackWorkspace {
   int ld_coef = 0;
   float* ctot = nullptr;   // [max chunks][ld_coef / 3] the chunks' summed ln a per head
   float* hn = nullptr;     // [max_B][E] float32: normed rows before the input convolution (block 2)
+  float* rscale = nullptr; // [max_B] float32: the rows' norm scales (input convolutions)
   float* y2 = nullptr;     // [max_B][E] float32: the second mixer's projected output (block 2)
   // gated delta rule: prepared q | k | v sit in cbuf
   float* dl_lg = nullptr;   // [max_B][ld_dl_lg] log decays
@@ -202,7 +203,8 @@ class StackExecutor {
   void layer_run_postnorm(int ri, int B, hipStream_t s);
   void layer_run_sandwich(int ri, int B, hipStream_t s);
   void layer_run_prenorm(int ri, int B, hipStream_t s);
-  void norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, int B, hipStream_t s);
+  void norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, const void* W, int N, int B, hipStream_t s);
+  bool mixer_norm_fused(const LayerDesc& L, int B) const;
   void mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
   void linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
   void delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);

@@ -69,16 +69,37 @@ struct QkvEpi {
   void* vc;
 };
 constexpr int LN_LDS_BYTES = 32768;
-constexpr int LN_RW = 4;  // weight rows per wave
 constexpr int LN_XR = 16;  // row elements per thread: E <= 4096
 constexpr int LN_PF = 4;  // 512-element steps of them requested before the norm (bfloat16)
-template <typename T>
+// What a block does to the rows before the product: PRE_NORM a layer or RMS norm; PRE_CANON an RMS norm and a causal
+// convolution added to its result (the window is a ring with rows to spare: block 0 may write the new inputs while the
+// other blocks still read the old ones); PRE_GROUP an RMS norm in equal parts and a sigmoid gate (a mixer's outputs).
+// add: C += the product (the residual stream).
+enum { PRE_NORM = 0, PRE_CANON = 1, PRE_GROUP = 2 };
+struct GemvPre {
+  const float* w;       // PRE_CANON: [E][taps]
+  int taps, ring;
+  float* window;
+  long long stride;
+  const int* pos;
+  const int* q_seq;
+  const float* gate;    // PRE_GROUP: [M][ld_gate] or null
+  int ld_gate, groups;
+  int ldx;              // row stride of x
+  int add;
+};
+constexpr int LN_MAX_GROUPS = 256;
+constexpr int CANON_FUSED_TAPS = 4;
+bool gemv_canon_supported(int taps) { return taps >= 1 && taps <= CANON_FUSED_TAPS; }
+// XR: row elements per thread that the prologue of PRE_CANON / PRE_GROUP holds (E <= 256 XR)
+template <typename T, int PRE, int LN_RW, int XR>
 __global__ __launch_bounds__(256) void gemv_ln_kernel(const float* __restrict__ x, int E, const float* __restrict__ nw,
                                                       const float* __restrict__ nb, float eps, const T* __restrict__ W,
                                                       int M, int N, float* __restrict__ C, int ldc, T* __restrict__ hout,
-                                                      QkvEpi q, int vec) {
+                                                      QkvEpi q, GemvPre pr, int vec) {
   __shared__ __attribute__((aligned(16))) unsigned char hs_raw[LN_LDS_BYTES];
   __shared__ float red[4];
+  __shared__ float rs[PRE == PRE_CANON ? 8 : PRE == PRE_GROUP ? LN_MAX_GROUPS : 1];
   T* hs = (T*)hs_raw;
   const int tid = threadIdx.x, lane = tid & 63;
   const int n0 = (blockIdx.x * 4 + (tid >> 6)) * LN_RW;
@@ -95,6 +116,92 @@ __global__ __launch_bounds__(256) void gemv_ln_kernel(const float* __restrict__ 
         pre[it][u] = *(const u32x4*)(W + (long long)min(n0 + u, N - 1) * E + k);
       }
   }
+  if constexpr (PRE == PRE_GROUP) {
+    for (int m = 0; m < M; ++m) {
+      const float* row = x + (long long)m * pr.ldx;
+      const float* gt = pr.gate ? pr.gate + (long long)m * pr.ld_gate : nullptr;
+      float xr[XR], gw[XR], gv[XR];
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < XR; ++j) {
+        const int i = tid + 256 * j;
+        xr[j] = i < E ? row[i] : 0.f;
+        gw[j] = i < E ? nw[i] : 0.f;
+        gv[j] = (gt && i < E) ? gt[i] : 0.f;
+        sum += xr[j] * xr[j];
+      }
+      const int per = E / pr.groups;
+      if (pr.groups == 1) {
+        const float rstd = 1.f / sqrtf(block_sum256(sum, red) / (float)E + eps);
+        if (tid == 0) rs[0] = rstd;
+      } else {
+        for (int g = tid >> 6; g < pr.groups; g += 4) {  // a wave per part
+          float ss = 0.f;
+          for (int i = lane; i < per; i += 64) ss += row[g * per + i] * row[g * per + i];
+          ss = wave_sum(ss);
+          if (lane == 0) rs[g] = 1.f / sqrtf(ss / (float)per + eps);
+        }
+      }
+      __syncthreads();
+#pragma unroll
+      for (int j = 0; j < XR; ++j) {
+        const int i = tid + 256 * j;
+        if (i < E) st(hs + (long long)m * E + i, xr[j] * rs[i / per] * gw[j] * (gt ? sigmoidf(gv[j]) : 1.f));
+      }
+      __syncthreads();  // rs is free for the next row
+    }
+  } else if constexpr (PRE == PRE_CANON) {
+    const int K = pr.taps;
+    for (int m = 0; m < M; ++m) {
+      const int seq = pr.q_seq[m], pos = pr.pos[m];
+      int same = 0;  // rows of the same sequence right before this one
+      while (same < K - 1 && m - same - 1 >= 0 && pr.q_seq[m - same - 1] == seq) ++same;
+      float* win = pr.ring ? pr.window + (long long)seq * pr.stride : nullptr;
+      // where the input `back` positions ago comes from: an earlier row of the step (still to be normed), the ring, nothing
+      const float* src[CANON_FUSED_TAPS];
+#pragma unroll
+      for (int back = 1; back < CANON_FUSED_TAPS; ++back)
+        src[back] = back >= K || back > pos ? nullptr
+                    : back <= same          ? x + (long long)(m - back) * E
+                                            : win + (long long)((pos - back) % pr.ring) * E;
+      float xr[XR], gw[XR], wt[XR][CANON_FUSED_TAPS], old[XR][CANON_FUSED_TAPS];
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < XR; ++j) {
+        const int i = min(tid + 256 * j, E - 1);
+        xr[j] = x[(long long)m * E + i];
+        gw[j] = nw[i];
+#pragma unroll
+        for (int back = 0; back < CANON_FUSED_TAPS; ++back) {
+          wt[j][back] = pr.w[(long long)i * K + max(K - 1 - back, 0)];
+          old[j][back] = 0.f;
+          if (back > 0 && src[back]) old[j][back] = src[back][i];  // (uniform)
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < XR; ++j) sum += tid + 256 * j < E ? xr[j] * xr[j] : 0.f;
+      const float rstd = 1.f / sqrtf(block_sum256(sum, red) / (float)E + eps);
+      if (tid == 0) rs[m] = rstd;
+      __syncthreads();
+#pragma unroll
+      for (int j = 0; j < XR; ++j) {
+        const int i = tid + 256 * j;
+        const float cur = xr[j] * rstd * gw[j];
+        float acc = cur;
+#pragma unroll
+        for (int back = CANON_FUSED_TAPS - 1; back > 0; --back)
+          if (back < K) acc += wt[j][back] * (back <= same ? old[j][back] * rs[max(m - back, 0)] * gw[j] : old[j][back]);
+        acc += wt[j][0] * cur;
+        if (i < E) {
+          st(hs + (long long)m * E + i, acc);
+          if (blockIdx.x == 0) {
+            if (win) win[(long long)(pos % pr.ring) * E + i] = cur;
+            hout[(long long)m * E + i] = hs[(long long)m * E + i];
+          }
+        }
+      }
+    }
+  } else
   for (int m = 0; m < M; ++m) {  // the row is read once (E <= 256 LN_XR) and normalised from registers
     const float* row = x + (long long)m * E;
     float xr[LN_XR], gw[LN_XR], gb[LN_XR];
@@ -201,13 +308,38 @@ __global__ __launch_bounds__(256) void gemv_ln_kernel(const float* __restrict__ 
           st((T*)q.vc + ((blk * q.G + i / q.Dv) * q.bs + off) * q.Dv + i % q.Dv, acc);
         }
       }
-      C[(long long)m * ldc + n] = acc;
+      if (pr.add)
+        C[(long long)m * ldc + n] += acc;
+      else
+        C[(long long)m * ldc + n] = acc;
     }
     }
   }
 }
 bool gemv_ln_supported(int M, int E, int f32) {
   return M > 0 && M <= 8 && E <= 256 * LN_XR && (long long)M * E * (f32 ? 4 : 2) <= LN_LDS_BYTES;
+}
+template <int PRE, int RW, int XR>
+static void launch_gemv_pre_x(const float* x, int E, const float* nw, const float* nb, float eps, const void* W, int M, int N, float* C,
+                              int ldc, void* hout, const QkvEpi& q, const GemvPre& pre, int f32, hipStream_t s) {
+  dim3 grid((N + 4 * RW - 1) / (4 * RW));
+  if (f32)
+    hipLaunchKernelGGL((gemv_ln_kernel<float, PRE, RW, XR>), grid, dim3(256), 0, s, x, E, nw, nb, eps, (const float*)W, M, N, C, ldc,
+                       (float*)hout, q, pre, (int)(E % 4 == 0 && ((uintptr_t)W & 15) == 0));
+  else
+    hipLaunchKernelGGL((gemv_ln_kernel<bf16, PRE, RW, XR>), grid, dim3(256), 0, s, x, E, nw, nb, eps, (const bf16*)W, M, N, C, ldc,
+                       (bf16*)hout, q, pre, (int)(E % 8 == 0 && ((uintptr_t)W & 15) == 0));
+  launched("gemv_ln");
+}
+template <int PRE, int RW>
+static void launch_gemv_pre(const float* x, int E, const float* nw, const float* nb, float eps, const void* W, int M, int N, float* C,
+                            int ldc, void* hout, const QkvEpi& q, const GemvPre& pre, int f32, hipStream_t s) {
+  if (PRE != PRE_NORM && E <= 1024)
+    launch_gemv_pre_x<PRE, RW, PRE == PRE_NORM ? LN_XR : 4>(x, E, nw, nb, eps, W, M, N, C, ldc, hout, q, pre, f32, s);
+  else if (PRE != PRE_NORM && E <= 2048)
+    launch_gemv_pre_x<PRE, RW, PRE == PRE_NORM ? LN_XR : 8>(x, E, nw, nb, eps, W, M, N, C, ldc, hout, q, pre, f32, s);
+  else
+    launch_gemv_pre_x<PRE, RW, LN_XR>(x, E, nw, nb, eps, W, M, N, C, ldc, hout, q, pre, f32, s);
 }
 void gemv_ln(const float* x, int E, const float* nw, const float* nb, float eps, const void* W, int M, int N, float* C,
              int ldc, void* hout, const AttnParams* A, const StepRows* R, int f32, hipStream_t s) {
@@ -218,14 +350,23 @@ void gemv_ln(const float* x, int E, const float* nw, const float* nb, float eps,
     q = QkvEpi{1, A->off_q, A->H * A->D, A->off_k, A->G * A->D, A->off_v, A->G * A->Dv, A->G, A->D, A->Dv, R->bs,
                A->qtemp_coef, A->qtemp_every, R->pos, R->slot, A->kc, A->vc};
   }
-  dim3 grid((N + 4 * LN_RW - 1) / (4 * LN_RW));
-  if (f32)
-    hipLaunchKernelGGL(gemv_ln_kernel<float>, grid, dim3(256), 0, s, x, E, nw, nb, eps, (const float*)W, M, N, C, ldc,
-                       (float*)hout, q, (int)(E % 4 == 0 && ((uintptr_t)W & 15) == 0));
-  else
-    hipLaunchKernelGGL(gemv_ln_kernel<bf16>, grid, dim3(256), 0, s, x, E, nw, nb, eps, (const bf16*)W, M, N, C, ldc,
-                       (bf16*)hout, q, (int)(E % 8 == 0 && ((uintptr_t)W & 15) == 0));
-  launched("gemv_ln");
+  launch_gemv_pre<PRE_NORM, 4>(x, E, nw, nb, eps, W, M, N, C, ldc, hout, q, GemvPre{}, f32, s);
+}
+void gemv_canon(const CanonParams& P, const void* W, int M, int N, float* C, int ldc, const StepRows& R, hipStream_t s) {
+  check(gemv_ln_supported(M, P.E, P.f32) && P.x && P.g && P.gvec && P.w && W && C && P.out && N > 0 && ldc >= N && R.pos && R.q_seq &&
+            gemv_canon_supported(P.taps) && (P.taps == 1 || (P.window && P.ring >= P.taps - 1 + 8)),
+        "gemv_canon: bad operands (a ring of at least taps + 7 rows)");
+  const GemvPre pre{P.w, P.taps, P.taps > 1 ? P.ring : 0, P.window, P.stride, R.pos, R.q_seq, nullptr, 0, 1, P.E, 0};
+  launch_gemv_pre<PRE_CANON, 4>(P.x, P.E, P.g, nullptr, P.eps, W, M, N, C, ldc, P.out, QkvEpi{}, pre, P.f32, s);
+}
+bool gemv_group_rms_supported(int M, int n, int groups, int f32) {
+  return gemv_ln_supported(M, n, f32) && groups >= 1 && groups <= LN_MAX_GROUPS && n % groups == 0;
+}
+void gemv_group_rms(const float* y, int ld_y, int n, int groups, const float* w, float eps, const float* gate, int ld_gate,
+                    const void* W, int M, int N, float* C, int ldc, int f32, hipStream_t s) {
+  check(gemv_group_rms_supported(M, n, groups, f32) && y && w && W && C && N > 0 && ldc >= N && ld_y >= n, "gemv_group_rms: bad operands");
+  const GemvPre pre{nullptr, 1, 0, nullptr, 0, nullptr, nullptr, gate, ld_gate, groups, ld_y, 1};
+  launch_gemv_pre<PRE_GROUP, 2>(y, n, w, nullptr, eps, W, M, N, C, ldc, nullptr, QkvEpi{}, pre, f32, s);
 }
 
 // ------------------------------------------------------------------------------------------------ FMA tile GEMM

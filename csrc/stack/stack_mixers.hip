@@ -563,9 +563,9 @@ void gated_scan(const ScanParams& P, const StepRows& R, hipStream_t s) {
       launch_gated_scan<SCAN_FIXED, 1024>(P, R, s);
   } else {
     check(P.conv && P.dt_bias && P.a_log && P.d_skip, "gated scan: state space operands");
-    if (scan_elems(P.D, P.Dv, 256) <= 64)
+    if (P.D * P.Dv <= 2048)
       launch_gated_scan<SCAN_SSD, 256>(P, R, s);
-    else  // a large head: its state over four times the threads
+    else  // its state over four times the threads
       launch_gated_scan<SCAN_SSD, 1024>(P, R, s);
   }
   launched("gated_scan");

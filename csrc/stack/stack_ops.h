@@ -325,9 +325,18 @@ struct CanonParams {
   void* out;            // [B][E] matrix dtype
   int f32;
   int gvec;
+  float* rscale;        // [B] scratch of prompt portions, or null (then they take the kernel for few rows)
   int ring;             // > 0: the window is a ring of `ring` rows, the input of position p in row p % ring (0: oldest first)
 };
 void scalar_norm_conv(const CanonParams& P, const StepRows& R, hipStream_t s);
+// decode steps (gemv_ln_supported(M, E, f32)): the vector-weight norm and its convolution (ring window) in the launch of the
+// product C = out . W^T; out is also written
+bool gemv_canon_supported(int taps);
+void gemv_canon(const CanonParams& P, const void* W, int M, int N, float* C, int ldc, const StepRows& R, hipStream_t s);
+// decode steps: group_rms_cast and the output projection added to the residual stream, C += (normed, gated y) . W^T
+void gemv_group_rms(const float* y, int ld_y, int n, int groups, const float* w, float eps, const float* gate, int ld_gate,
+                    const void* W, int M, int N, float* C, int ldc, int f32, hipStream_t s);
+bool gemv_group_rms_supported(int M, int n, int groups, int f32);
 // out[r] = x[idx ? idx[r] : r] / rms * g[0], matrix dtype
 void scalar_norm_cast(const float* x, const int* idx, int rows, int E, const float* g, float eps, void* out, int f32,
                       hipStream_t s);

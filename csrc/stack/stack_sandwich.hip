@@ -73,6 +73,87 @@ __global__ __launch_bounds__(256) void scalar_norm_conv_kernel(CanonParams P, St
     st((T*)P.out + (long long)r * E + c, acc);
   }
 }
+// Prompt portions, in two launches: every row's scale, a wave per row; then a block takes NC_ROWS consecutive rows and
+// 256 channels, and a thread runs down the rows of its channel with every input (those of the taps - 1 rows before
+// included) in registers. hn is written for the rows that canon_window_kernel reads (the last taps - 1 of a sequence) only.
+__global__ __launch_bounds__(256) void row_scale_kernel(const float* __restrict__ x, int B, int E, float eps, int vec,
+                                                        float* __restrict__ scale) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (r >= B) return;
+  const float* xr = x + (long long)r * E;
+  float ss = 0.f;
+  if (vec) {
+#pragma unroll 4
+    for (int c = lane * 4; c < E; c += 256) {
+      const f32x4 a = *(const f32x4*)(xr + c);
+      ss += a[0] * a[0] + a[1] * a[1] + a[2] * a[2] + a[3] * a[3];
+    }
+  } else {
+    for (int c = lane; c < E; c += 64) ss += xr[c] * xr[c];
+  }
+  ss = wave_sum(ss);
+  if (lane == 0) scale[r] = 1.f / sqrtf(ss / (float)E + eps);
+}
+constexpr int NC_ROWS = 8;
+template <typename T>
+__global__ __launch_bounds__(256) void norm_conv_rows_kernel(CanonParams P, StepRows R) {
+  constexpr int H = CANON_MAX_TAPS - 1, NR = NC_ROWS + H;
+  __shared__ float scale[NR];
+  __shared__ int seqs[NR + CANON_MAX_TAPS], poss[NC_ROWS];  // sequence of row r0 - H + i (-1: no such row)
+  const int r0 = blockIdx.x * NC_ROWS, K = P.taps, E = P.E;
+  const int c = threadIdx.x + 256 * blockIdx.y, cc = min(c, E - 1);
+  const float gc = P.gvec ? P.g[cc] : P.g[0];
+  float v[NR], w[CANON_MAX_TAPS];
+#pragma unroll
+  for (int i = 0; i < NR; ++i)  // rows outside are read (clamped), never used
+    v[i] = i >= H - (K - 1) ? P.x[(long long)min(max(r0 - H + i, 0), R.B - 1) * E + cc] : 0.f;
+#pragma unroll
+  for (int j = 0; j < CANON_MAX_TAPS; ++j) w[j] = j < K ? P.w[(long long)cc * K + (K - 1 - j)] : 0.f;  // w[back]
+  for (int i = threadIdx.x; i < NR + CANON_MAX_TAPS; i += 256) {
+    const int r = r0 - H + i;
+    const bool on = r >= 0 && r < R.B;
+    seqs[i] = on ? R.q_seq[r] : -1;
+    if (i < NR) scale[i] = on ? P.rscale[r] : 0.f;
+    if (i >= H && i < NR) poss[i - H] = (P.ring && on) ? R.pos[r] : 0;
+  }
+  __syncthreads();
+  if (c >= E) return;
+#pragma unroll
+  for (int i = 0; i < NR; ++i) v[i] *= scale[i] * gc;
+#pragma unroll
+  for (int i = H; i < NR; ++i) {
+    const int seq = seqs[i], r = r0 - H + i;
+    if (seq < 0) continue;  // (uniform over the block)
+    float* win = P.window ? P.window + (long long)seq * P.stride : nullptr;
+    int nb = 0;
+    while (nb < K - 1 && seqs[i - nb - 1] == seq) ++nb;
+    const int pos = poss[i - H];
+    float acc = v[i];
+#pragma unroll
+    for (int back = CANON_MAX_TAPS - 1; back >= 0; --back) {
+      if (back < K) {
+        float in = v[i - back];
+        if (back > nb) {
+          if (P.ring)
+            in = back <= pos ? win[(long long)((pos - back) % P.ring) * E + c] : 0.f;
+          else
+            in = win[(long long)(K - 1 - (back - nb)) * E + c];
+        }
+        acc += w[back] * in;
+      }
+    }
+    st((T*)P.out + (long long)r * E + c, acc);
+    if (K > 1) {
+      if (seqs[i + K - 1] != seq) P.hn[(long long)r * E + c] = v[i];
+      if (nb == 0 && seqs[i + 1] != seq) {  // alone in its sequence: advances the window here
+        if (P.ring)
+          win[(long long)(pos % P.ring) * E + c] = v[i];
+        else
+          for (int sx = 0; sx < K - 1; ++sx) win[(long long)sx * E + c] = sx == K - 2 ? v[i] : win[(long long)(sx + 1) * E + c];
+      }
+    }
+  }
+}
 __global__ __launch_bounds__(256) void canon_window_kernel(CanonParams P, StepRows R) {
   const int r = blockIdx.x, K = P.taps, E = P.E;
   const int seq = R.q_seq[r];
@@ -97,6 +178,22 @@ void scalar_norm_conv(const CanonParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.x && P.g && P.hn && P.out && P.E > 0 && P.taps >= 1 && P.taps <= CANON_MAX_TAPS && P.w &&
             (P.taps == 1 || (P.window && (P.ring == 0 || (P.ring >= P.taps && R.pos)))),
         "scalar_norm_conv: bad operands (at most 8 taps)");
+  if (R.B > 64 && P.rscale) {
+    hipLaunchKernelGGL(row_scale_kernel, dim3((R.B + 3) / 4), dim3(256), 0, s, P.x, R.B, P.E, P.eps,
+                       (int)(P.E % 4 == 0 && ((uintptr_t)P.x & 15) == 0), P.rscale);
+    launched("row_scale");
+    const dim3 grid((R.B + NC_ROWS - 1) / NC_ROWS, (P.E + 255) / 256);
+    if (P.f32)
+      hipLaunchKernelGGL(norm_conv_rows_kernel<float>, grid, dim3(256), 0, s, P, R);
+    else
+      hipLaunchKernelGGL(norm_conv_rows_kernel<bf16>, grid, dim3(256), 0, s, P, R);
+    launched("norm_conv_rows");
+    if (P.taps > 1) {
+      hipLaunchKernelGGL(canon_window_kernel, dim3(R.B, (P.E + 1023) / 1024), dim3(256), 0, s, P, R);
+      launched("canon_window");
+    }
+    return;
+  }
   // few rows (decode steps): the channels are shared among several blocks per row (each sums the whole row itself)
   const dim3 grid(R.B, R.B <= 64 ? std::min(8, (P.E + 255) / 256) : 1);
   if (P.f32)

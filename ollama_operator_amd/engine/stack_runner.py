@@ -95,7 +95,7 @@ class StackExec:
                              ret_sin=p(r.ret_sin), ret_u_stride=r.ret_u.shape[1], cbuf=p(r.cbuf), ld_cbuf=r.cbuf.shape[1],
                              lat=p(r.latbuf), ld_lat=r.latbuf.shape[1], idw=p(r.idw), coef=p(r.scan_coef),
                              ld_coef=(r.scan_coef.shape[1] if r.scan_coef is not None else 0), ctot=p(r.scan_ctot),
-                             hn=p(r.hn), y2=p(r.ybuf2), **{"dl_" + k: p(v) for k, v in r.delta_ws.items()},
+                             hn=p(r.hn), y2=p(r.ybuf2), rscale=p(r.rscale), **{"dl_" + k: p(v) for k, v in r.delta_ws.items()},
                              ld_dl_lg=r.delta_ws["lg"].shape[1], ld_dl_gate=r.delta_ws["gate"].shape[1],
                              dl_heads=r.delta_ws["Bm"].shape[1] // 32,
                              **{"moe_" + k: (v if isinstance(v, int) else p(v)) for k, v in r.moe_ws.items()}))
@@ -282,6 +282,7 @@ class StackRunner(Runner):
                                                 [m.conv_channels for m in deltas], default=1) + 3) // 4 * 4, **f32)
         sandwich = cfg.block == BLOCK_SANDWICH
         self.hn = torch.zeros(max_batch if sandwich or cfg.canon_both else 1, E, **f32)  # normed rows before the input convolution
+        self.rscale = torch.zeros(max_batch, **f32)                        # the rows' norm scales ahead of it
         self.ybuf2 = torch.zeros(max_batch if sandwich else 1, E, **f32)   # the second mixer's projected output
         self.latbuf = torch.zeros(max_batch, (max([m.heads * m.kv_rank for m in lat], default=1) + 7) // 8 * 8, **tt)
         self.idw = torch.zeros(max_batch, **f32)
