@@ -332,20 +332,24 @@ constexpr int DC = 32;
 constexpr int DELTA_CD = 128;  // largest key size of the chunked form
 int delta_chunk_rows() { return DC; }
 bool delta_chunk_supported(int D, int Dv) { return D > 0 && D <= DELTA_CD && Dv > 0 && Dv <= DELTA_MAX; }
-static inline size_t delta_wy_lds(int D) { return (size_t)(3 * DC * (D + 1) + DC * (DC + 4) + DC) * sizeof(float); }
+constexpr int DELTA_WY_MAX = DELTA_CD + DELTA_MAX;
+static inline size_t delta_wy_lds(int D, int Dv) {
+  return (size_t)(std::max(3 * DC * (D + 1), DC * (D + Dv)) + DC * (DC + 4) + DC) * sizeof(float);
+}
 
-__global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunkWs W) {
+__global__ __launch_bounds__(DELTA_WY_MAX) void delta_wy_kernel(DeltaParams P, DeltaChunkWs W) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int r0 = W.chunks[4 * c], n = W.chunks[4 * c + 1];
   const int D = P.D, Dv = P.Dv, D1 = D + 1, hg = h / (P.H / P.G);
+  const int nt = blockDim.x;         // at least D + Dv: a thread per column of the right-hand sides
   constexpr int LA = DC + 4;       // rows of A 16-byte aligned
   float* A = lds;                  // [DC][DC + 4]
-  float* qs = A + DC * LA;         // [DC][D + 1]
+  float* be = A + DC * LA;         // [DC]
+  float* qs = be + DC;             // [DC][D + 1]
   float* ks = qs + DC * D1;
   float* Lc = ks + DC * D1;
-  float* be = Lc + DC * D1;        // [DC]
-  for (int i = tid; i < DC * D; i += 256) {
+  for (int i = tid; i < DC * D; i += nt) {
     const int t = i / D, d = i % D;
     const long long r = r0 + min(t, n - 1);  // (unconditional loads: all of them in flight together)
     const float qv = P.x[r * P.ld_x + hg * D + d], kv = P.x[r * P.ld_x + (P.G + hg) * D + d], lv = P.lg[r * P.ld_lg + h * D + d];
@@ -355,16 +359,20 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
   }
   if (tid < DC) be[tid] = tid < n ? sigmoidf(P.proj[(long long)(r0 + tid) * P.ld + P.off_b + h]) : 0.f;
   __syncthreads();
-  for (int d = tid; d < D; d += 256) {
+  if (tid < D) {
     float acc = 0.f;
+#pragma unroll 8
     for (int t = 0; t < DC; ++t) {
-      acc += Lc[t * D1 + d];
-      Lc[t * D1 + d] = acc;
-      if (t < n) P.lg[(long long)(r0 + t) * P.ld_lg + h * D + d] = acc;  // the running log decays replace the log decays
+      acc += Lc[t * D1 + tid];
+      Lc[t * D1 + tid] = acc;
     }
   }
   __syncthreads();
-  for (int p = tid; p < DC * DC; p += 256) {
+  for (int i = tid; i < n * D; i += nt) {  // the running log decays replace the log decays
+    const int t = i / D, d = i % D;
+    P.lg[(long long)(r0 + t) * P.ld_lg + h * D + d] = Lc[t * D1 + d];
+  }
+  for (int p = tid; p < DC * DC; p += nt) {
     const int t = p / DC, sx = p % DC;
     float a = 0.f, b = 0.f;
     if (sx <= t && t < n) {
@@ -377,43 +385,64 @@ __global__ __launch_bounds__(256) void delta_wy_kernel(DeltaParams P, DeltaChunk
     A[t * LA + sx] = sx < t ? be[t] * a : 0.f;
     if (t < n) W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] = b;
   }
-  for (int i = tid; i < n * D; i += 256) {  // keys decayed to the end of the chunk
+  for (int i = tid; i < n * D; i += nt) {  // keys decayed to the end of the chunk
     const int t = i / D, d = i % D;
     W.Kd[(long long)(r0 + t) * P.ld_lg + h * D + d] = ks[t * D1 + d] * expf(Lc[(n - 1) * D1 + d] - Lc[t * D1 + d]);
   }
   __syncthreads();
-  for (int col = tid; col < D + Dv; col += 256) {  // forward substitution, a column per thread
-    const bool key = col < D;
-    float x[DC];
-    if (key) {
+  // forward substitution, a column of the right-hand sides per thread, in blocks of eight rows: the solved rows sit in LDS
+  // (where q, k and the log decays were), so a thread holds sixteen values at a time
+  const int col = tid, NC = D + Dv;
+  const bool key = col < D;
+  float x[DC];
+  if (key) {
 #pragma unroll
-      for (int t = 0; t < DC; ++t) x[t] = be[t] * ks[t * D1 + col] * expf(Lc[t * D1 + col]);
-    } else {
-      const float* v = P.x + 2 * P.G * D + h * Dv + col - D;
+    for (int t = 0; t < DC; ++t) x[t] = be[t] * ks[t * D1 + col] * __builtin_amdgcn_exp2f(Lc[t * D1 + col] * 1.44269504088896341f);
+  } else if (col < NC) {
+    const unsigned at = 2 * P.G * D + h * Dv + col - D;
 #pragma unroll
-      for (int t = 0; t < DC; ++t) x[t] = v[(long long)(r0 + min(t, n - 1)) * P.ld_x];
-#pragma unroll
-      for (int t = 0; t < DC; ++t) x[t] *= be[t];  // 0 past the chunk's end
+    for (int t = 0; t < DC; ++t) {
+      const float* row = P.x + (long long)(r0 + min(t, n - 1)) * P.ld_x;  // (uniform)
+      x[t] = row[at];
     }
 #pragma unroll
-    for (int t = 1; t < DC; ++t) {
+    for (int t = 0; t < DC; ++t) x[t] *= be[t];  // 0 past the chunk's end
+  }
+  __syncthreads();
+  if (col >= NC) return;
+  float* X = qs + col;  // [DC][D + Dv]
 #pragma unroll
-      for (int s4 = 0; s4 < (t + 3) / 4; ++s4) {
-        const f32x4 a = *(const f32x4*)&A[t * LA + 4 * s4];  // zero from the diagonal on
+  for (int t = 0; t < DC; ++t) X[t * NC] = x[t];
+  float* out = key ? W.W + (long long)r0 * P.ld_lg + h * D + col : W.u + (long long)r0 * P.ld_gate + h * Dv + col - D;
+  const int ldo = key ? P.ld_lg : P.ld_gate;
+#pragma unroll 1
+  for (int b0 = 0; b0 < n; b0 += 8) {
+    float y[8];
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (4 * s4 + i < t) x[t] -= a[i] * x[4 * s4 + i];
+    for (int i = 0; i < 8; ++i) y[i] = X[(b0 + i) * NC];
+#pragma unroll 1
+    for (int s0 = 0; s0 < b0; s0 += 8) {
+      float z[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) z[i] = X[(s0 + i) * NC];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const f32x4 a = *(const f32x4*)&A[(b0 + i) * LA + s0], c4 = *(const f32x4*)&A[(b0 + i) * LA + s0 + 4];
+        y[i] -= a[0] * z[0] + a[1] * z[1] + a[2] * z[2] + a[3] * z[3] + c4[0] * z[4] + c4[1] * z[5] + c4[2] * z[6] + c4[3] * z[7];
       }
-      asm volatile("" ::: "memory");  // the rows of A are read as they are needed, not all at once into registers
     }
 #pragma unroll
-    for (int t = 0; t < DC; ++t)
-      if (t < n) {
-        if (key)
-          W.W[(long long)(r0 + t) * P.ld_lg + h * D + col] = x[t];
-        else
-          W.u[(long long)(r0 + t) * P.ld_gate + h * Dv + col - D] = x[t];
-      }
+    for (int i = 1; i < 8; ++i) {
+#pragma unroll
+      for (int k = 0; k < 7; ++k)
+        if (k < i) y[i] -= A[(b0 + i) * LA + b0 + k] * y[k];
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      X[(b0 + i) * NC] = y[i];
+      if (b0 + i < n) *out = y[i];
+      out += ldo;
+    }
   }
 }
 
@@ -463,7 +492,9 @@ template <int TJ, bool VEC>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams P, DeltaChunkWs W) {
   __shared__ float part[4][DC][17];
   __shared__ float us[DC][17];
-  const int c0 = blockIdx.x, h = blockIdx.y, ct = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  // grid (head + heads * column tile, chunk): the working blocks (first chunks) are neighbours and so spread over the XCDs, a
+  // head's column tiles, which read the same W and keys, stay on one of them (8 | heads)
+  const int c0 = blockIdx.y, h = blockIdx.x % P.H, ct = blockIdx.x / P.H, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   if (!(W.chunks[4 * c0 + 3] & 1)) return;  // not the first chunk of its sequence (uniform per block)
   const int D = P.D, Dv = P.Dv, m = lane & 15, q4 = lane >> 4;
   const int col = ct * 16 + m;
@@ -625,9 +656,9 @@ void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& 
             W.s_stride >= (long long)P.H * P.D * P.Dv,
         "chunked gated delta rule: operands (key size <= 128)");
   const dim3 grid(W.nchunks, P.H);
-  hipLaunchKernelGGL(delta_wy_kernel, grid, dim3(256), delta_wy_lds(P.D), s, P, W);
+  hipLaunchKernelGGL(delta_wy_kernel, grid, dim3(std::max(256, (P.D + P.Dv + 63) / 64 * 64)), delta_wy_lds(P.D, P.Dv), s, P, W);
   launched("delta_wy");
-  const dim3 sg(W.nchunks, P.H, (P.Dv + 15) / 16);
+  const dim3 sg(P.H * ((P.Dv + 15) / 16), W.nchunks);
   const int vec = P.D % 4 == 0 && P.ld_lg % 4 == 0 && ((uintptr_t)W.W & 15) == 0;
   if (P.D <= 64 && vec)
     hipLaunchKernelGGL((delta_scan_kernel<1, true>), sg, dim3(256), 0, s, P, W);

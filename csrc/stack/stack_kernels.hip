@@ -173,8 +173,8 @@ __global__ __launch_bounds__(256) void gemv_ln_kernel(const float* __restrict__ 
         gw[j] = nw[i];
 #pragma unroll
         for (int back = 0; back < CANON_FUSED_TAPS; ++back) {
-          wt[j][back] = pr.w[(long long)i * K + max(K - 1 - back, 0)];
-          old[j][back] = 0.f;
+          wt[j][back] = old[j][back] = 0.f;
+          if (back < K) wt[j][back] = pr.w[i * K + K - 1 - back];  // (uniform)
           if (back > 0 && src[back]) old[j][back] = src[back][i];  // (uniform)
         }
       }
