@@ -382,6 +382,42 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvParams P, StepRows R
     P.out[(long long)r * P.ld_out + c] = silu(acc);
   }
 }
+// Prompt portions, up to four taps: a block takes CR_ROWS consecutive rows and 256 channels, a thread runs down the rows of its
+// channel with every input (those of the taps - 1 rows before included) in registers.
+constexpr int CR_ROWS = 8, CR_TAPS = 4;
+__global__ __launch_bounds__(256) void conv_silu_rows_kernel(ConvParams P, StepRows R) {
+  constexpr int H = CR_TAPS - 1, NR = CR_ROWS + H;
+  __shared__ int seqs[NR + 1];  // sequence of row r0 - H + i (-1: no such row)
+  const int r0 = blockIdx.x * CR_ROWS, K = P.taps;
+  const int c = blockIdx.y * 256 + threadIdx.x, cc = min(c, P.ch - 1);
+  float v[NR], w[CR_TAPS];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) v[i] = P.proj[(long long)min(max(r0 - H + i, 0), R.B - 1) * P.ld + P.off_in + cc];
+#pragma unroll
+  for (int b = 0; b < CR_TAPS; ++b) w[b] = b < K ? P.w[(long long)cc * K + K - 1 - b] : 0.f;  // w[back]
+  const float bias = P.bias ? P.bias[cc] : 0.f;
+  for (int i = threadIdx.x; i < NR + 1; i += 256) {
+    const int r = r0 - H + i;
+    seqs[i] = (r >= 0 && r < R.B) ? R.q_seq[r] : -1;
+  }
+  __syncthreads();
+  if (c >= P.ch) return;
+#pragma unroll
+  for (int i = H; i < NR; ++i) {
+    const int seq = seqs[i];
+    if (seq < 0) continue;  // (uniform over the block)
+    int nb = 0;
+    while (nb < K - 1 && seqs[i - nb - 1] == seq) ++nb;
+    float* win = P.state + (long long)seq * P.state_stride;
+    float acc = bias;
+#pragma unroll
+    for (int back = CR_TAPS - 1; back >= 0; --back)
+      if (back < K) acc += w[back] * (back <= nb ? v[i - back] : win[(long long)(K - 1 - (back - nb)) * P.ch + c]);
+    P.out[(long long)(r0 - H + i) * P.ld_out + c] = silu(acc);
+    if (nb == 0 && seqs[i + 1] != seq)  // alone in its sequence: advances the window here
+      for (int sx = 0; sx < K - 1; ++sx) win[(long long)sx * P.ch + c] = sx == K - 2 ? v[i] : win[(long long)(sx + 1) * P.ch + c];
+  }
+}
 __global__ __launch_bounds__(256) void conv_window_kernel(ConvParams P, StepRows R) {
   const int r = blockIdx.x, K = P.taps;
   const int seq = R.q_seq[r];
@@ -401,7 +437,10 @@ void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.proj && P.w && P.out && P.ch > 0 && P.taps >= 1 && (P.taps == 1 || P.state),
         "conv_silu: bad operands");
   const dim3 grid(R.B, (P.ch + 255) / 256);  // a block per (row, 256 channels)
-  hipLaunchKernelGGL(conv_silu_kernel, grid, dim3(256), 0, s, P, R);
+  if (R.B > 64 && P.taps <= CR_TAPS)
+    hipLaunchKernelGGL(conv_silu_rows_kernel, dim3((R.B + CR_ROWS - 1) / CR_ROWS, (P.ch + 255) / 256), dim3(256), 0, s, P, R);
+  else
+    hipLaunchKernelGGL(conv_silu_kernel, grid, dim3(256), 0, s, P, R);
   launched("conv_silu");
   conv_window(P, R, s);
 }
@@ -651,13 +690,9 @@ __device__ __forceinline__ void stage_qk_gated(const ScanParams& P, int row0, in
     const int c = idx / MAXD, d = idx % MAXD;
     float qv = 0.f, kv = 0.f;
     if (c < cn && d < P.D) {
-      const float* src = MODE == SCAN_SSD ? P.conv + (long long)(row0 + c) * P.ld_conv : P.proj + (long long)(row0 + c) * P.ld;
+      const float* src = P.proj + (long long)(row0 + c) * P.ld;
       kv = src[P.off_k + hg * P.D + d];
       if (WITH_Q) qv = src[P.off_q + hg * P.D + d] * qscale;
-      if (MODE == SCAN_FIXED) {
-        kv = silu(kv);
-        if (WITH_Q) qv = silu(qv);
-      }
     }
     if (WITH_Q) Qs[c][d] = qv;
     Ks[c][d] = kv;
@@ -670,9 +705,9 @@ __device__ __forceinline__ void stage_v_gated(const ScanParams& P, int row0, int
     const int c = idx >> 6, col = jb * 64 + (idx & 63);
     float v = 0.f;
     if (c < cn) {
-      const float* src = MODE == SCAN_SSD ? P.conv + (long long)(row0 + c) * P.ld_conv : P.proj + (long long)(row0 + c) * P.ld;
+      const float* src = P.proj + (long long)(row0 + c) * P.ld;
       if (col < P.Dv)
-        v = MODE == SCAN_FIXED ? silu(src[P.off_v + h * P.Dv + col]) : src[P.off_v + h * P.Dv + col];
+        v = src[P.off_v + h * P.Dv + col];
       else if (MODE == SCAN_MLSTM && col == P.Dv)
         v = 1.f;
     }
@@ -812,14 +847,167 @@ __global__ __launch_bounds__(256) void gated_out_kernel(ScanParams P, const int*
     if (colok) {
       const float o = expf(Lc[t]) * inter + intra;
       const long long r = row0 + t;
-      if (MODE == SCAN_MLSTM)
-        raw[r * ld_raw + h * Dvp + col] = o;
-      else if (MODE == SCAN_FIXED)
-        P.y[r * P.ld_y + h * Dv + col] = o;
-      else
-        P.y[r * P.ld_y + h * Dv + col] = (o + P.d_skip[h] * Vs[t][j]) * silu(P.proj[r * P.ld + P.off_g + h * Dv + col]);
+      raw[r * ld_raw + h * Dvp + col] = o;
     }
   }
+}
+// The same two steps on v_mfma_f32_16x16x4_f32 (true float32) for the modes without a normaliser, one block per (chunk,
+// head). Operand layouts: A lane (m = lane % 16, lane / 16) holds row m, K index 4 (lane / 16) + i in step i; B the same with
+// column m; the accumulator's register i is row 4 (lane / 16) + i, column m.
+template <int MODE>
+__device__ __forceinline__ const float* gated_src(const ScanParams& P, long long r) {
+  return MODE == SCAN_SSD ? P.conv + r * P.ld_conv : P.proj + r * P.ld;
+}
+template <int MODE>
+__device__ __forceinline__ float gated_act(float v) { return MODE == SCAN_FIXED ? silu(v) : v; }
+constexpr int GU_PAD = 16;
+template <int MODE, int DT>  // DT = key size / 16, rounded up
+__global__ __launch_bounds__(256) void gated_u_mfma_kernel(ScanParams P, const int* __restrict__ chunks, const float* __restrict__ coef,
+                                                           float* __restrict__ U, long long u_stride, float* __restrict__ ctot) {
+  constexpr int LD = 16 * DT + GU_PAD;
+  __shared__ float Ks[SC][LD];  // keys times their weight at the chunk's end
+  __shared__ float Lc[SC], bw[SC];
+  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int row0 = chunks[4 * c], cn = chunks[4 * c + 1];
+  const int D = P.D, Dv = P.Dv, hg = h / (P.H / P.G), m = lane & 15, q4 = lane >> 4;
+  stage_coef<MODE>(P, coef, row0, cn, h, Lc, bw);
+  if (tid == 0) ctot[(long long)c * P.H + h] = Lc[cn - 1];
+#pragma unroll
+  for (int it = 0; it < SC * DT * 16 / 256; ++it) {
+    const int idx = tid + 256 * it, t = idx / (16 * DT), d = idx % (16 * DT);
+    const float v = gated_src<MODE>(P, row0 + min(t, cn - 1))[P.off_k + hg * D + min(d, D - 1)];
+    Ks[t][d] = (t < cn && d < D) ? gated_act<MODE>(v) * expf(Lc[cn - 1] - Lc[t]) * bw[t] : 0.f;
+  }
+  __syncthreads();
+  float* out = U + c * u_stride + (long long)h * D * Dv;
+  for (int ct = wv; ct * 16 < Dv; ct += 4) {
+    const int col = ct * 16 + m;
+    float b[8];
+#pragma unroll
+    for (int kk = 0; kk < 8; ++kk)
+      b[kk] = gated_src<MODE>(P, row0 + min(4 * kk + q4, cn - 1))[P.off_v + h * Dv + min(col, Dv - 1)];
+#pragma unroll
+    for (int kk = 0; kk < 8; ++kk) b[kk] = gated_act<MODE>(b[kk]);
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < 8; ++kk) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(Ks[4 * kk + q4][16 * dt + m], b[kk], acc, 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = 16 * dt + 4 * q4 + i;
+        if (d < D && col < Dv) out[(long long)d * Dv + col] = acc[i];
+      }
+    }
+  }
+}
+template <int MODE, int DT>
+__global__ __launch_bounds__(256) void gated_out_mfma_kernel(ScanParams P, const int* __restrict__ chunks,
+                                                             const float* __restrict__ coef, const float* __restrict__ Sin,
+                                                             long long u_stride) {
+  constexpr int LD = 16 * DT + 4, LA = SC + 4;
+  __shared__ __attribute__((aligned(16))) float Qs[SC][LD], Ks[SC][LD], As[SC][LA];
+  __shared__ float Lc[SC], bw[SC];
+  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int row0 = chunks[4 * c], cn = chunks[4 * c + 1];
+  const int D = P.D, Dv = P.Dv, hg = h / (P.H / P.G), m = lane & 15, q4 = lane >> 4;
+#pragma unroll
+  for (int it = 0; it < SC * DT * 16 / 256; ++it) {
+    const int idx = tid + 256 * it, t = idx / (16 * DT), d = idx % (16 * DT);
+    const float* src = gated_src<MODE>(P, row0 + min(t, cn - 1)) + hg * D + min(d, D - 1);
+    const float qv = src[P.off_q], kv = src[P.off_k];
+    const bool on = t < cn && d < D;
+    Qs[t][d] = on ? gated_act<MODE>(qv) : 0.f;
+    Ks[t][d] = on ? gated_act<MODE>(kv) : 0.f;
+  }
+  stage_coef<MODE>(P, coef, row0, cn, h, Lc, bw);
+  __syncthreads();
+  {  // A = q k^T with its decays: a 16 x 16 tile per wave
+    const int mt = wv >> 1, nt = wv & 1;
+    f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < DT; ++j) {
+      const f32x4 a = *(const f32x4*)&Qs[16 * mt + m][16 * j + 4 * q4], b = *(const f32x4*)&Ks[16 * nt + m][16 * j + 4 * q4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], acc, 0, 0, 0);
+    }
+    const int sx = 16 * nt + m;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 16 * mt + 4 * q4 + i;
+      As[t][sx] = (sx <= t && t < cn) ? acc[i] * expf(Lc[t] - Lc[sx]) * bw[sx] : 0.f;
+    }
+  }
+  __syncthreads();
+  const float* S = Sin + c * u_stride + (long long)h * D * Dv;
+  for (int ct = wv; ct * 16 < Dv; ct += 4) {
+    const int col = ct * 16 + m, cc = min(col, Dv - 1);
+    float b[4 * DT], v[8];
+#pragma unroll
+    for (int j = 0; j < DT; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) b[4 * j + i] = S[(long long)min(16 * j + 4 * q4 + i, D - 1) * Dv + cc];  // past D: q is 0
+#pragma unroll
+    for (int s = 0; s < 8; ++s) v[s] = gated_src<MODE>(P, row0 + min(16 * (s >> 2) + 4 * q4 + (s & 3), cn - 1))[P.off_v + h * Dv + cc];
+    f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int j = 0; j < DT; ++j)
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) {
+        const f32x4 a = *(const f32x4*)&Qs[16 * mt + m][16 * j + 4 * q4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[4 * j + i], acc[mt], 0, 0, 0);
+      }
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[mt][i] *= expf(Lc[16 * mt + 4 * q4 + i]);
+#pragma unroll
+    for (int s = 0; s < 8; ++s) v[s] = gated_act<MODE>(v[s]);
+#pragma unroll
+    for (int s0 = 0; s0 < 2; ++s0)
+#pragma unroll
+      for (int mt = 0; mt < 2; ++mt) {
+        const f32x4 a = *(const f32x4*)&As[16 * mt + m][16 * s0 + 4 * q4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[mt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], v[4 * s0 + i], acc[mt], 0, 0, 0);
+      }
+    if (col >= Dv) continue;
+#pragma unroll
+    for (int mt = 0; mt < 2; ++mt)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * mt + 4 * q4 + i;
+        const long long r = row0 + t;
+        if (t < cn) {
+          float y = acc[mt][i];
+          if (MODE == SCAN_SSD)
+            y = (y + P.d_skip[h] * gated_src<MODE>(P, r)[P.off_v + h * Dv + col]) * silu(P.proj[r * P.ld + P.off_g + h * Dv + col]);
+          P.y[r * P.ld_y + h * Dv + col] = y;
+        }
+      }
+  }
+}
+template <int MODE, int DT>
+static void launch_gated_mfma(const ScanParams& P, const ScanChunkWs& W, hipStream_t s) {
+  const dim3 grid(W.nchunks, P.H);
+  hipLaunchKernelGGL((gated_u_mfma_kernel<MODE, DT>), grid, dim3(256), 0, s, P, W.chunks, W.coef, W.U, W.u_stride, W.ctot);
+  launched("gated_u_mfma");
+  const long long elems = (long long)P.H * P.D * P.Dv;
+  hipLaunchKernelGGL(gated_chunk_scan_kernel<MODE>, dim3((unsigned)((elems + 255) / 256)), dim3(256), 0, s, P, W.chunks, W.nchunks,
+                     W.U, W.Sin, W.u_stride, W.ctot);
+  launched("gated_chunk_scan");
+  hipLaunchKernelGGL((gated_out_mfma_kernel<MODE, DT>), grid, dim3(256), 0, s, P, W.chunks, W.coef, W.Sin, W.u_stride);
+  launched("gated_out_mfma");
+}
+template <int MODE>
+static void launch_gated_mfma_any(const ScanParams& P, const ScanChunkWs& W, hipStream_t s) {
+  if (P.D <= 32)
+    launch_gated_mfma<MODE, 2>(P, W, s);
+  else if (P.D <= 64)
+    launch_gated_mfma<MODE, 4>(P, W, s);
+  else
+    launch_gated_mfma<MODE, 8>(P, W, s);
 }
 // mLSTM: y = o / (max(|n . q|, exp(-m)) + 1e-6), divided by its root mean square over the head, times the norm's
 // weight and the sigmoid output gate; one wave per (row, head)
@@ -880,18 +1068,12 @@ void gated_scan_chunked(const ScanParams& P, const StepRows& R, const ScanChunkW
     launched("mlstm_finish");
   } else if (P.mode == SCAN_FIXED) {
     check(P.decay && P.G == P.H && P.y, "chunked constant-decay operands");
-    if (P.D <= 64)
-      launch_gated_chunked<SCAN_FIXED, 64>(P, R, W, s);
-    else
-      launch_gated_chunked<SCAN_FIXED, 128>(P, R, W, s);
+    launch_gated_mfma_any<SCAN_FIXED>(P, W, s);
   } else {
     check(P.conv && P.dt_bias && P.a_log && P.d_skip && P.y, "chunked state space operands");
     hipLaunchKernelGGL(gated_coef_ssd_kernel, dim3((R.B * P.H + 255) / 256), dim3(256), 0, s, P, R.B, W.coef);
     launched("gated_coef_ssd");
-    if (P.D <= 64)
-      launch_gated_chunked<SCAN_SSD, 64>(P, R, W, s);
-    else
-      launch_gated_chunked<SCAN_SSD, 128>(P, R, W, s);
+    launch_gated_mfma_any<SCAN_SSD>(P, W, s);
   }
 }
 
