@@ -3,7 +3,8 @@
 //   S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t.
 // q, k and v come through one short causal convolution with silu; q and k are unit vectors per head (q also times
 // D^(-1/2)); g = exp(-exp(A_log) softplus(z)) with z from a low-rank map, the output gate from another one.
-//   delta_prepare_kernel  convolution, silu, unit vectors, log decays and the output gate of every row
+//   delta_prepare_kernel  convolution, silu, unit vectors, log decays and the output gate of every row (and, for a layer
+//                         with an attention beside the delta rule, that attention's K/V store)
 //   delta_walk_kernel     token by token, the state in registers (decode steps, and sizes the chunks do not take)
 //   delta_wy / scan / out prompt portions in chunks (see there)
 // Everything but the matrix operands is float32. Wave = 64 lanes.
@@ -13,6 +14,7 @@
 #include <algorithm>
 
 #include "stack_device.h"
+#include "stack_kv.h"
 #include "stack_ops.h"
 
 namespace omx {
@@ -85,7 +87,12 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
     return;
   }
   const int unit = ((int)blockIdx.y - nlow) * 4 + wv;
-  if (unit >= 2 * P.G + P.H) return;
+  if (unit >= 2 * P.G + P.H) {  // past the head units: the attention's K/V store, a wave per key/value head
+    const int g = unit - 2 * P.G - P.H;
+    if (P.kv.kc && g < P.kv.G)
+      for (int rr = 0; rr < nr; ++rr) kv_store_item<T>(P.kv, R, r0 + rr, g, lane);
+    return;
+  }
   const bool isv = unit >= 2 * P.G, isq = unit < P.G;
   const int n = isv ? P.Dv : P.D, K = P.taps;
   const int c0 = isv ? 2 * P.G * P.D + (unit - 2 * P.G) * P.Dv : unit * P.D;  // first channel of the unit
@@ -178,7 +185,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
 }
 template <typename T>
 static void launch_delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
-  const int nlow = (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + 3) / 4;
+  const int nlow = (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + (P.kv.kc ? P.kv.G : 0) + 3) / 4;
   const int rank = (P.rank_a + 3) / 4 * 4 + (P.rank_g + 3) / 4 * 4;
   if (R.B <= 16)
     hipLaunchKernelGGL((delta_prepare_kernel<T, 1>), dim3(R.B, nlow + nconv), dim3(256), rank * 4, s, P, R, nlow);
@@ -196,6 +203,8 @@ static void check_delta(const DeltaParams& P, const StepRows& R) {
 }
 void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
   check_delta(P, R);
+  check(!P.kv.kc || (P.kv.proj && P.kv.vc && P.kv.G > 0 && P.kv.D > 0 && P.kv.Dv > 0 && P.kv.f32 == P.f32 && R.slot && R.bs > 0),
+        "delta_prepare: K/V store operands");
   if (P.f32)
     launch_delta_prepare<float>(P, R, s);
   else

@@ -84,6 +84,17 @@ static long long prenorm_state_floats(const LayerDesc& L) {  // the mixers' part
     return (long long)L.r_heads * L.r_dim * L.r_vdim + (long long)(L.conv - 1) * (2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim);
   return 0;
 }
+static void validate_delta(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
+  const StackWorkspace& ws = e.ws;
+  need(r.state, "gated delta rule without a state");
+  need(L.heads * L.vdim + L.r_heads * L.r_vdim <= ws.ld_a, "mixer output wider than its buffer");
+  need(L.conv_w && L.a2 && L.g2 && L.a_log && L.dt_bias && L.gnorm && ws.cbuf && ws.dl_lg && ws.dl_gate &&
+           2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim <= ws.ld_cbuf && L.r_heads * L.r_dim <= ws.ld_dl_lg &&
+           L.r_heads * L.r_vdim <= ws.ld_dl_gate,
+       "gated delta rule operands or buffers");
+  need(L.r_kv_heads > 0 && L.r_heads % L.r_kv_heads == 0 && delta_supported(L.r_dim, L.r_vdim, L.r_rank, L.r_grank),
+       "gated delta rule sizes (key and value size <= 256, both low-rank maps together <= 1024)");
+}
 static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
   const StackWorkspace& ws = e.ws;
   need(L.norm_w && L.w_in && L.w_o && L.n_in > 0 && L.n_in <= ws.ld_proj, "layer weights missing");
@@ -101,16 +112,10 @@ static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const Lay
   } else if (L.kind == 6) {
     need(r.state && L.decay && L.mnorm && ws.ret.obuf && ws.ret.ld_o >= L.heads * L.vdim, "constant-decay linear attention operands");
     need(gated_scan_supported(SCAN_FIXED, L.dim, L.vdim), "constant-decay linear attention head sizes (<= 256)");
-  } else if (L.r_delta) {
-    need(r.kc && r.vc && r.state && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= 256 && L.vdim <= 256 && L.chunk >= 0,
+  } else if (L.kind == 0 && L.maps == 1 && !L.score_talk) {
+    need(r.kc && r.vc && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= 256 && L.vdim <= 256 && L.chunk >= 0,
          "attention sizes (<= 256)");
-    need(L.heads * L.vdim + L.r_heads * L.r_vdim <= ws.ld_a, "mixer output wider than its buffer");
-    need(L.conv_w && L.a2 && L.g2 && L.a_log && L.dt_bias && L.gnorm && ws.cbuf && ws.dl_lg && ws.dl_gate &&
-             2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim <= ws.ld_cbuf && L.r_heads * L.r_dim <= ws.ld_dl_lg &&
-             L.r_heads * L.r_vdim <= ws.ld_dl_gate,
-         "gated delta rule operands or buffers");
-    need(L.r_kv_heads > 0 && L.r_heads % L.r_kv_heads == 0 && delta_supported(L.r_dim, L.r_vdim, L.r_rank, L.r_grank),
-         "gated delta rule sizes (key and value size <= 256, both low-rank maps together <= 1024)");
+    if (L.r_delta) validate_delta(e, r, L);
   } else if (L.kind == 2) {
     need(r.kc && L.w_uk && L.w_uvT && L.dkv_norm && ws.cbuf && ws.lat && L.gate == 2, "latent attention operands");
     need(latent_supported(L.dim, L.rot_dim, L.kv_rank, L.vdim),
@@ -265,8 +270,7 @@ void StackExecutor::linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hi
 }
 
 // the gated delta rule beside an attention, up to the output projection; its outputs sit beside the attention's in ws.a
-void StackExecutor::delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
-  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+DeltaParams StackExecutor::delta_params(const RunDesc& r, const LayerDesc& L) const {
   const long long sf = (long long)L.r_heads * L.r_dim * L.r_vdim;
   DeltaParams P{};
   P.proj = ws.proj;
@@ -302,9 +306,13 @@ void StackExecutor::delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hip
   P.ld_out = ws.ld_a;
   P.out_scale = L.right_scale;
   P.f32 = cfg.f32;
-  delta_prepare(P, R, s);
-  if (B > SMALL_B && n_chunks > 0 && ws.ret.Sin && ws.dl_W && ws.dl_Kd && ws.dl_u && ws.dl_Bm && ws.ret.u_stride >= sf &&
-      ws.dl_heads >= L.r_heads && delta_chunk_supported(L.r_dim, L.r_vdim)) {
+  P.kv = KvStoreParams{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, cfg.f32};
+  return P;
+}
+void StackExecutor::delta_mixer(const DeltaParams& P, int B, hipStream_t s) {  // after delta_prepare
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  if (B > SMALL_B && n_chunks > 0 && ws.ret.Sin && ws.dl_W && ws.dl_Kd && ws.dl_u && ws.dl_Bm &&
+      ws.ret.u_stride >= (long long)P.H * P.D * P.Dv && ws.dl_heads >= P.H && delta_chunk_supported(P.D, P.Dv)) {
     DeltaChunkWs W{ws.ret.chunks, n_chunks, ws.ret.max_chunks, ws.ret.Sin, ws.ret.u_stride, ws.dl_W, ws.dl_Kd, ws.dl_u, ws.dl_Bm};
     delta_chunked(P, R, W, s);
   } else {
@@ -548,9 +556,15 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     mamba2_mixer(r, L, B, s);
   } else if (L.kind == 6) {
     linear_mixer(r, L, B, s);
-  } else if (L.r_delta) {
-    KvStoreParams K{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, f32};
-    kv_store(K, R, s);
+  } else if (L.kind == 0 && L.maps == 1 && !L.score_talk) {
+    DeltaParams delta{};
+    if (L.r_delta) {
+      delta = delta_params(r, L);
+      delta_prepare(delta, R, s);  // (with the attention's K/V store)
+    } else {
+      KvStoreParams K{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, f32};
+      kv_store(K, R, s);
+    }
     AttnParams A{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, 0.f, 0.f, 1, r.kc, r.vc,
                  ws.a, ws.ld_a, f32, splits, ws.split_ws, ws.split_ws_floats};
     A.window = L.window;
@@ -564,7 +578,7 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
       flash_prefill(A, R, tiles, n_tiles, s);
     else
       attention(A, R, s);
-    delta_mixer(r, L, B, s);
+    if (L.r_delta) delta_mixer(delta, B, s);
   } else if (L.kind == 2) {
     const int C = L.kv_rank, W = C + L.rot_dim;
     LatentParams P{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_g, L.heads, L.dim, L.rot_dim, C, L.vdim, L.rot_dims,

@@ -207,7 +207,8 @@ class StackExecutor {
   bool mixer_norm_fused(const LayerDesc& L, int B) const;
   void mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
   void linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
-  void delta_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  DeltaParams delta_params(const RunDesc& r, const LayerDesc& L) const;
+  void delta_mixer(const DeltaParams& P, int B, hipStream_t s);
   void head(int n_logits, bool use_idx, hipStream_t s);
   void forward(int B, int n_logits, bool use_idx, hipStream_t s);
 };

@@ -492,6 +492,7 @@ struct DeltaParams {
   int ld_out;
   float out_scale;
   int f32;
+  KvStoreParams kv;     // kc non-null: delta_prepare also stores the keys and values of the attention beside it
 };
 // convolution (its windows advanced), unit vectors, log decays and gates of the step's rows into the scratch rows
 void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s);

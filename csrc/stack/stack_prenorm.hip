@@ -4,6 +4,7 @@
 // the mixing matrix), a gated dense feed-forward with a relu gate, and a sigmoid router with ranked groups.
 // float32 for norms, angles, gates and router; `T` is the matrix dtype (bfloat16 or float32).
 #include "stack_device.h"
+#include "stack_kv.h"
 #include "stack_ops.h"
 
 #include <algorithm>
@@ -153,19 +154,7 @@ __global__ __launch_bounds__(256) void kv_store_kernel(KvStoreParams P, StepRows
   const int lane = threadIdx.x & 63;
   const long long item = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (item >= (long long)R.B * P.G) return;
-  const int b = (int)(item / P.G), g = (int)(item % P.G);
-  const float* k = P.proj + (long long)b * P.ld + P.off_k + g * P.D;
-  const float* v = P.proj + (long long)b * P.ld + P.off_v + g * P.Dv;
-  const int slot = R.slot[b];
-  const long long at = ((long long)(slot / R.bs) * P.G + g) * R.bs + slot % R.bs;
-  for (int d = lane; d < P.D; d += 64) st((T*)P.kc + at * P.D + d, k[d]);
-  float f = 1.f;
-  if (P.v_unit) {
-    float ss = 0.f;
-    for (int d = lane; d < P.Dv; d += 64) ss += v[d] * v[d];
-    f = 1.f / sqrtf(wave_sum(ss) / (float)P.Dv + P.eps);
-  }
-  for (int d = lane; d < P.Dv; d += 64) st((T*)P.vc + at * P.Dv + d, v[d] * f);
+  kv_store_item<T>(P, R, (int)(item / P.G), (int)(item % P.G), lane);
 }
 void kv_store(const KvStoreParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.proj && P.kc && P.vc && P.G > 0 && P.D > 0 && P.Dv > 0 && R.slot && R.bs > 0, "kv_store: bad operands");
