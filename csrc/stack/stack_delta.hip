@@ -40,7 +40,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
     const int ra4 = (ra + 3) / 4 * 4, LR = ra4 + (rg + 3) / 4 * 4;  // both maps' factors 16-byte aligned
     for (int i = tid; i < RB * (ra + rg); i += 256) {
       const int r = i / (ra + rg), c = i % (ra + rg);
-      lds[r * LR + (c < ra ? c : ra4 + c - ra)] = r < nr ? P.proj[(long long)(r0 + r) * P.ld + (c < ra ? P.off_a1 + c : P.off_g1 + c - ra)] : 0.f;
+      const int col = c < ra ? P.off_a1 + c : P.off_g1 + c - ra;
+      lds[r * LR + (c < ra ? c : ra4 + c - ra)] = r < nr ? P.proj[(long long)(r0 + r) * P.ld + col] : 0.f;
     }
     __syncthreads();
     const int c = blockIdx.y * 256 + tid;

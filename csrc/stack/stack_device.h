@@ -9,6 +9,7 @@
 #include <string>
 
 #include "../kernels/wave_shuffle.h"
+#include "stack_ops.h"
 
 namespace omx {
 namespace stack {
@@ -68,7 +69,7 @@ __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z
 __device__ __forceinline__ float moe_unit(int act, float limit, float w, float gate, float up) {
   gate *= w;
   up *= w;
-  if (act == 1 /* MOE_ACT_CLAMPED */) {
+  if (act == MOE_ACT_CLAMPED) {
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g * sigmoidf(1.702f * g) * (u + 1.f);
   }

@@ -201,33 +201,34 @@ __global__ __launch_bounds__(256) void gemv_ln_kernel(const float* __restrict__ 
         }
       }
     }
-  } else
-  for (int m = 0; m < M; ++m) {  // the row is read once (E <= 256 LN_XR) and normalised from registers
-    const float* row = x + (long long)m * E;
-    float xr[LN_XR], gw[LN_XR], gb[LN_XR];
-    float sum = 0.f;
+  } else {
+    for (int m = 0; m < M; ++m) {  // the row is read once (E <= 256 LN_XR) and normalised from registers
+      const float* row = x + (long long)m * E;
+      float xr[LN_XR], gw[LN_XR], gb[LN_XR];
+      float sum = 0.f;
 #pragma unroll
-    for (int j = 0; j < LN_XR; ++j) {
-      const int i = tid + 256 * j;
-      xr[j] = i < E ? row[i] : 0.f;
-      gw[j] = i < E ? nw[i] : 0.f;
-      gb[j] = (nb && i < E) ? nb[i] : 0.f;
-      sum += xr[j];
-    }
-    const float mean = nb ? block_sum256(sum, red) / (float)E : 0.f;  // no bias vector: an RMS norm, nothing is centred
-    float sq = 0.f;
+      for (int j = 0; j < LN_XR; ++j) {
+        const int i = tid + 256 * j;
+        xr[j] = i < E ? row[i] : 0.f;
+        gw[j] = i < E ? nw[i] : 0.f;
+        gb[j] = (nb && i < E) ? nb[i] : 0.f;
+        sum += xr[j];
+      }
+      const float mean = nb ? block_sum256(sum, red) / (float)E : 0.f;  // no bias vector: an RMS norm, nothing is centred
+      float sq = 0.f;
 #pragma unroll
-    for (int j = 0; j < LN_XR; ++j) {
-      const float d = tid + 256 * j < E ? xr[j] - mean : 0.f;
-      sq += d * d;
-    }
-    const float rstd = 1.f / sqrtf(block_sum256(sq, red) / (float)E + eps);
+      for (int j = 0; j < LN_XR; ++j) {
+        const float d = tid + 256 * j < E ? xr[j] - mean : 0.f;
+        sq += d * d;
+      }
+      const float rstd = 1.f / sqrtf(block_sum256(sq, red) / (float)E + eps);
 #pragma unroll
-    for (int j = 0; j < LN_XR; ++j) {
-      const int i = tid + 256 * j;
-      if (i < E) {
-        st(hs + (long long)m * E + i, (xr[j] - mean) * rstd * gw[j] + gb[j]);
-        if (blockIdx.x == 0) hout[(long long)m * E + i] = hs[(long long)m * E + i];
+      for (int j = 0; j < LN_XR; ++j) {
+        const int i = tid + 256 * j;
+        if (i < E) {
+          st(hs + (long long)m * E + i, (xr[j] - mean) * rstd * gw[j] + gb[j]);
+          if (blockIdx.x == 0) hout[(long long)m * E + i] = hs[(long long)m * E + i];
+        }
       }
     }
   }
@@ -1942,8 +1943,8 @@ void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
   }
   {
     const long long n = (long long)P.B * P.E;
-    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, P.y, W.ds, W.inv, P.w_input ? nullptr : P.ew, P.ld_top,
-                       P.sgate, P.B, P.E, P.top, (int)(P.Fs > 0), P.y_add);
+    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, P.y, W.ds, W.inv,
+                       P.w_input ? nullptr : P.ew, P.ld_top, P.sgate, P.B, P.E, P.top, (int)(P.Fs > 0), P.y_add);
     launched("moe_combine");
   }
 }

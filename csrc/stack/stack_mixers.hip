@@ -614,7 +614,8 @@ void gated_scan(const ScanParams& P, const StepRows& R, hipStream_t s) {
 // With l_s = ln a_s and L_t = l_0 + ... + l_t inside a chunk of n tokens that starts from state S,
 //   A[t][s] = (q_t . k_s) exp(L_t - L_s) b_s for s <= t,   o_t = exp(L_t) S^T q_t + sum_s A[t][s] v_s,
 //   U = sum_s exp(L_(n-1) - L_s) b_s k_s v_s^T,              S <- exp(L_(n-1)) S + U,
-// all in float32 on the vector ALUs, over the host-built chunk table {first row, rows, state slot, flags}:
+// all in float32 (the mLSTM on the vector ALUs, the modes without a normaliser on the float32 matrix cores: the gated_*_mfma
+// kernels), over the host-built chunk table {first row, rows, state slot, flags}:
 //   0. per (row, head) coefficients {l, b, m}: gated_coef_*                       (the mLSTM's running maximum is a
 //      scan of x -> max(x + f, i), composed over a wave's 64 rows at a time)
 //   1. every chunk's U and its total log decay, chunks in parallel                (gated_u_kernel)

@@ -726,7 +726,9 @@ class StackWeights:
 
     @property
     def nbytes(self) -> int:
-        n = self.embed.numel() + (0 if self.head is self.embed else self.head.numel()) + (self.loop_in.numel() if self.loop_in is not None else 0)
+        n = self.embed.numel() + (self.loop_in.numel() if self.loop_in is not None else 0)
+        if self.head is not self.embed:
+            n += self.head.numel()
         for L in self.layers:
             n += sum(v.numel() for v in L.values() if isinstance(v, torch.Tensor) and v.dtype == self.dtype)
         return n * (2 if self.dtype == torch.bfloat16 else 4)

@@ -49,7 +49,8 @@ def standard():
     return config([(pair(), moe()),
                    (linear(), moe(experts=5, top=3, ff=16, limit=2.5)),
                    (mamba(), None),
-                   (pair(heads=4, kv_heads=4, dim=8, vdim=20, chunk=24, left=1.0, right=0.6, r=delta(heads=3, kv_heads=1, dim=18, vdim=6, conv=2)),
+                   (pair(heads=4, kv_heads=4, dim=8, vdim=20, chunk=24, left=1.0, right=0.6,
+                         r=delta(heads=3, kv_heads=1, dim=18, vdim=6, conv=2)),
                     moe(experts=4, top=1)),
                    (mamba(heads=3, vdim=10, state=12, groups=1, conv=4, norm_groups=3), moe()),
                    (linear(decay=(0.9, 0.3), dim=6, vdim=20), None)])

@@ -120,7 +120,8 @@ MECHANISMS = {
     "pair_chunk_of_one": ([(rc.pair(chunk=1, right=0.0), None)], {}),
     "pair_chunk_of_two_head_each": ([(rc.pair(heads=3, kv_heads=3, dim=6, vdim=7, chunk=2, right=0.1), None)], {}),
     "pair_one_chunk_for_all": ([(rc.pair(heads=5, kv_heads=1, dim=12, vdim=70, chunk=1000, right=0.2), None)], {}),
-    "delta_head_each_one_tap": ([(rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=2, dim=5, vdim=9, conv=1, decay_rank=3, gate_rank=11)), None)], {}),
+    "delta_head_each_one_tap": ([(rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=2, dim=5, vdim=9, conv=1, decay_rank=3,
+                                                                gate_rank=11)), None)], {}),
     "delta_wide_keys": ([(rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=1, dim=70, vdim=17, conv=3, decay_rank=16)), None)], {}),
     "delta_one_head_wide_values": ([(rc.pair(left=0.0, r=rc.delta(heads=1, kv_heads=1, dim=16, vdim=100)), None)], {}),
     "experts": ([(rc.linear(), rc.moe())], {}),
@@ -322,7 +323,9 @@ def test_attention_finds_a_far_key_in_a_wide_chunk(tmp_path, device):
 def test_state_keeps_the_first_token(tmp_path, device, kind):
     """Recurrences that do not forget: the last logits still depend on the first token, 200 positions back, and the
     engine agrees however the prompt is cut (a state that is lost or taken from a neighbour would show)."""
-    mx = {"linear": rc.linear(decay=(1.0, 0.9995)), "mamba": rc.mamba(), "delta": rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=1, dim=128, vdim=8))}[kind]   # many key directions: writes overlap little
+    mx = {"linear": rc.linear(decay=(1.0, 0.9995)), "mamba": rc.mamba(),
+          # (many key directions: writes overlap little)
+          "delta": rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=1, dim=128, vdim=8))}[kind]
     m = rc.Model(tmp_path, rc.config([(mx, None)], width=32, vocab=50), seed=12)
     if kind == "mamba":
         m.set_tensor("l0.mix.A_log", torch.full((4,), -12.0))
@@ -343,7 +346,8 @@ def test_state_keeps_the_first_token(tmp_path, device, kind):
 def test_strong_and_weak_decays_side_by_side(tmp_path, device):
     """Delta-rule channels that forget within a token (log decays of -50 and less) beside channels that keep for hundreds:
     the chunked form's exponents must not overflow, its running sums must not lose the weak ones."""
-    m = rc.Model(tmp_path, rc.config([(rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=1, dim=16, vdim=16)), None)], width=32, vocab=50), seed=14)
+    mx = rc.pair(left=0.0, r=rc.delta(heads=2, kv_heads=1, dim=16, vdim=16))
+    m = rc.Model(tmp_path, rc.config([(mx, None)], width=32, vocab=50), seed=14)
     m.set_tensor("l0.mix.right.A_log", torch.tensor([2.5, -2.0]))
     m.set_tensor("l0.mix.right.dt_bias", torch.linspace(-8.0, 6.0, 32))
     toks = rc.tokens(150, 50, seed=15)
@@ -397,7 +401,8 @@ def test_large_heads(tmp_path, device):
     layers = [(rc.mamba(heads=2, vdim=200, state=128, groups=1, norm_groups=1), None),
               (rc.linear(decay=(0.9, 0.99), dim=256, vdim=72), None),
               (rc.pair(left=0.5, r=rc.delta(heads=2, kv_heads=1, dim=160, vdim=130)), None),
-              (rc.pair(heads=2, kv_heads=1, dim=200, vdim=150, scale=0.07, left=0.5, r=rc.delta(heads=1, kv_heads=1, dim=128, vdim=256)), None)]
+              (rc.pair(heads=2, kv_heads=1, dim=200, vdim=150, scale=0.07, left=0.5,
+                       r=rc.delta(heads=1, kv_heads=1, dim=128, vdim=256)), None)]
     m = rc.Model(tmp_path, rc.config(layers, width=64, vocab=80), seed=27)
     toks = rc.tokens(70, 80, seed=28)
     want, _ = m.oracle(toks)
