@@ -200,6 +200,13 @@ PYBIND11_MODULE(_stack, m) {
         L.off_rb = geti(d, "off_rb");
         L.off_g1 = geti(d, "off_g1");
         L.g2 = Pp<const void>(ptr(d, "g2"));
+        L.route_softmax = geti(d, "route_softmax");
+        L.rot_amp = getf(d, "rot_amp", 1.f);
+        L.conv_ring = geti(d, "conv_ring");
+        L.q_rank = geti(d, "q_rank");
+        L.off_dq = geti(d, "off_dq");
+        L.dq_norm = Pp<const float>(ptr(d, "dq_norm"));
+        L.w_uq = Pp<const void>(ptr(d, "w_uq"));
         if (L.qtemp_every <= 0) throw std::runtime_error("q_temp.every must be positive");
       })
       .def("set_runs", [](StackExecutor& e, std::vector<py::dict> runs) {
@@ -256,6 +263,8 @@ PYBIND11_MODULE(_stack, m) {
         w.ld_cbuf = geti(d, "ld_cbuf");
         w.lat = Pp<void>(ptr(d, "lat"));
         w.ld_lat = geti(d, "ld_lat");
+        w.qlat = Pp<void>(ptr(d, "qlat"));
+        w.ld_qlat = geti(d, "ld_qlat");
         w.idw = Pp<float>(ptr(d, "idw"));
         w.coef = Pp<float>(ptr(d, "coef"));
         w.ld_coef = geti(d, "ld_coef");

@@ -1,8 +1,10 @@
 // Gated delta rule (interface: stack_ops.h): per head a float32 state S (D x Dv) whose rows (key channels) decay by a
-// per-token vector g; a write takes off what the state already answers to its key:
+// per-token vector g, or by one number (head_decay: template parameter HD); a write takes off what the state already
+// answers to its key:
 //   S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t.
 // q, k and v come through one short causal convolution with silu; q and k are unit vectors per head (q also times
-// D^(-1/2)); g = exp(-exp(A_log) softplus(z)) with z from a low-rank map, the output gate from another one.
+// D^(-1/2)); g = exp(-exp(A_log) softplus(z)) with z from a low-rank map, the output gate sigmoid of another one; with one
+// decay per head z comes straight from the input and the output gate is silu of a full projection.
 //   delta_prepare_kernel  convolution, silu, unit vectors, log decays and the output gate of every row (and, for a layer
 //                         with an attention beside the delta rule, that attention's K/V store)
 //   delta_walk_kernel     token by token, the state in registers (decode steps, and sizes the chunks do not take)
@@ -30,6 +32,11 @@ __device__ __forceinline__ float delta_softplus(float z) { return z > 20.f ? z :
 // for all RB rows. A convolution block takes four head units (G query heads, G key heads, H value heads), one per
 // wave, four channels per lane. Inputs from before the step's first row of the sequence come from its carried window
 // (oldest first); a sequence with one row in the step advances its window here, the others in conv_window.
+// the input `back` positions before `pos`, from before the step's rows (nb of the sequence's rows precede this one in it)
+__device__ __forceinline__ float delta_carried(const DeltaParams& P, const float* win, int back, int nb, int pos, int ch, int c) {
+  if (P.ring) return back <= pos ? win[(long long)((pos - back) % P.ring) * ch + c] : 0.f;
+  return win[(long long)(P.taps - 1 - (back - nb)) * ch + c];
+}
 template <typename T, int RB>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepRows R, int nlow) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -95,6 +102,11 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
     return;
   }
   const bool isv = unit >= 2 * P.G, isq = unit < P.G;
+  if (P.head_decay && isv && lane < nr) {  // the head's log decays, a row per lane
+    const int h = unit - 2 * P.G;
+    const long long r = r0 + lane;
+    P.lg[r * P.ld_lg + h] = -expf(P.a_log[h]) * delta_softplus(P.proj[r * P.ld + P.off_a1 + h] + P.dt_bias[h]);
+  }
   const int n = isv ? P.Dv : P.D, K = P.taps;
   const int c0 = isv ? 2 * P.G * P.D + (unit - 2 * P.G) * P.Dv : unit * P.D;  // first channel of the unit
   const int ch = 2 * P.G * P.D + HV;
@@ -120,8 +132,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
           float acc = 0.f;
 #pragma unroll
           for (int back = 3; back >= 0; --back)
-            if (back < K) acc += w[back] * (back <= nb ? in[rr + 3 - back] : win[(long long)(K - 1 - (back - nb)) * ch + c]);
-          if (alone && rr < nr && d < n)
+            if (back < K) acc += w[back] * (back <= nb ? in[rr + 3 - back] : delta_carried(P, win, back, nb, R.pos[r], ch, c));
+          if (alone && rr < nr && d < n && !P.ring)  // (rings: conv_ring_window)
             for (int sx = 0; sx < K - 1; ++sx)
               win[(long long)sx * ch + c] = sx == K - 2 ? in[rr + 3] : win[(long long)(sx + 1) * ch + c];
           v[u][rr] = d < n ? silu(acc) : 0.f;
@@ -167,9 +179,11 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
         for (int j = 0; j < K; ++j) {
           const int back = K - 1 - j;
           const float in = back == 0 ? cur : back <= nb ? P.proj[(long long)(r - back) * P.ld + P.off_q + c]
-                                                        : win[(long long)(K - 1 - (back - nb)) * ch + c];
+                                                        : delta_carried(P, win, back, nb, R.pos[r], ch, c);
           acc += P.conv_w[(long long)c * K + j] * in;
-          if (alone && back > 0) win[(long long)(K - 1 - back) * ch + c] = back == 1 ? cur : win[(long long)(K - back) * ch + c];
+          if (P.ring) {
+            if (back == 0 && R.B <= CONV_RING_ROWS) win[(long long)(R.pos[r] % P.ring) * ch + c] = cur;
+          } else if (alone && back > 0) win[(long long)(K - 1 - back) * ch + c] = back == 1 ? cur : win[(long long)(K - back) * ch + c];
         }
         v[u] = silu(acc);
         ss += v[u] * v[u];
@@ -186,8 +200,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaParams P, StepR
 }
 template <typename T>
 static void launch_delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
-  const int nlow = (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + (P.kv.kc ? P.kv.G : 0) + 3) / 4;
-  const int rank = (P.rank_a + 3) / 4 * 4 + (P.rank_g + 3) / 4 * 4;
+  const int nlow = P.head_decay ? 0 : (P.H * (P.D + P.Dv) + 255) / 256, nconv = (2 * P.G + P.H + (P.kv.kc ? P.kv.G : 0) + 3) / 4;
+  const int rank = P.head_decay ? 0 : (P.rank_a + 3) / 4 * 4 + (P.rank_g + 3) / 4 * 4;
   if (R.B <= 16)
     hipLaunchKernelGGL((delta_prepare_kernel<T, 1>), dim3(R.B, nlow + nconv), dim3(256), rank * 4, s, P, R, nlow);
   else
@@ -196,10 +210,14 @@ static void launch_delta_prepare(const DeltaParams& P, const StepRows& R, hipStr
 bool delta_supported(int D, int Dv, int rank_a, int rank_g) {
   return D > 0 && Dv > 0 && D <= DELTA_MAX && Dv <= DELTA_MAX && rank_a > 0 && rank_g > 0 && rank_a + rank_g <= DELTA_MAX_RANK;
 }
+bool delta_head_supported(int D, int Dv) { return D > 0 && Dv > 0 && D <= DELTA_MAX && Dv <= DELTA_MAX; }
 static void check_delta(const DeltaParams& P, const StepRows& R) {
-  check(R.B > 0 && P.proj && P.conv_w && P.a2 && P.g2 && P.a_log && P.dt_bias && P.norm_w && P.state && P.out && P.x && P.lg && P.gate &&
-            P.G > 0 && P.H % P.G == 0 && P.taps >= 1 && (P.taps == 1 || P.window) && delta_supported(P.D, P.Dv, P.rank_a, P.rank_g) &&
-            P.ld_x >= 2 * P.G * P.D + P.H * P.Dv && P.ld_lg >= P.H * P.D && P.ld_gate >= P.H * P.Dv && P.ld_out >= P.H * P.Dv,
+  const bool maps = P.head_decay ? delta_head_supported(P.D, P.Dv)
+                                 : P.a2 && P.g2 && P.gate && P.ld_lg >= P.H * P.D && delta_supported(P.D, P.Dv, P.rank_a, P.rank_g);
+  check(R.B > 0 && P.proj && P.conv_w && P.a_log && P.dt_bias && P.norm_w && P.state && P.out && P.x && P.lg && P.G > 0 &&
+            P.H % P.G == 0 && P.taps >= 1 && (P.taps == 1 || P.window) && maps && P.ld_x >= 2 * P.G * P.D + P.H * P.Dv &&
+            P.ld_lg >= P.H && P.ld_gate >= P.H * P.Dv && P.ld_out >= P.H * P.Dv &&
+            (P.ring == 0 || P.taps == 1 || (R.pos && P.ring >= P.taps - 1 + CONV_RING_ROWS)),
         "gated delta rule: operands or head sizes (key and value size <= 256)");
 }
 void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
@@ -211,15 +229,24 @@ void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s) {
   else
     launch_delta_prepare<bf16>(P, R, s);
   launched("delta_prepare");
-  ConvParams C{P.proj, P.ld, P.off_q, 2 * P.G * P.D + P.H * P.Dv, P.taps, P.conv_w, nullptr, P.window, P.state_stride, nullptr, 0};
+  const int ch = 2 * P.G * P.D + P.H * P.Dv;
+  if (P.ring) {
+    if (R.B > CONV_RING_ROWS) conv_ring_window(P.proj + P.off_q, P.ld, ch, P.taps, nullptr, P.window, P.state_stride, P.ring, R, s);
+    return;
+  }
+  ConvParams C{P.proj, P.ld, P.off_q, ch, P.taps, P.conv_w, nullptr, P.window, P.state_stride, nullptr, 0};
   conv_window(C, R, s);
 }
 
+template <bool HD>
+__device__ __forceinline__ float delta_gate(const DeltaParams& P, long long r, int i) {  // output gate of value channel i
+  return HD ? silu(P.proj[r * P.ld + P.off_g1 + i]) : P.gate[r * P.ld_gate + i];
+}
 // ------------------------------------------------------------------------------------------------ token by token
 // One block per (sequence segment of the step, head), as the other recurrences: the block of the segment's first row
 // walks its rows; thread (g, j) = (tid / Dv, tid % Dv) keeps S[i][j], i = g, g + NG, ..., in registers. The head's RMS
 // norm, its weight and the gate finish the row.
-template <typename T, int MAXI, int NT>
+template <typename T, int MAXI, int NT, bool HD>
 __global__ __launch_bounds__(NT) void delta_walk_kernel(DeltaParams P, StepRows R) {
   __shared__ float qs[DELTA_MAX], ks[DELTA_MAX], gs[DELTA_MAX], us[DELTA_MAX], po[NT], red[4];
   const int r0 = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -241,11 +268,11 @@ __global__ __launch_bounds__(NT) void delta_walk_kernel(DeltaParams P, StepRows 
     if (tid < D) {
       qs[tid] = x[hg * D + tid];
       ks[tid] = x[P.G * D + hg * D + tid];
-      gs[tid] = expf(P.lg[(long long)r * P.ld_lg + h * D + tid]);
+      gs[tid] = expf(P.lg[(long long)r * P.ld_lg + (HD ? h : h * D + tid)]);
     }
     const float v = tid < Dv ? x[2 * P.G * D + h * Dv + tid] : 0.f;
     const float beta = sigmoidf(P.proj[(long long)r * P.ld + P.off_b + h]);
-    const float gate = tid < Dv ? P.gate[(long long)r * P.ld_gate + h * Dv + tid] : 0.f;
+    const float gate = tid < Dv ? delta_gate<HD>(P, r, h * Dv + tid) : 0.f;
     __syncthreads();
     float part = 0.f;
     if (act) {
@@ -300,29 +327,33 @@ __global__ __launch_bounds__(NT) void delta_walk_kernel(DeltaParams P, StepRows 
     if (act && i < D) S0[(long long)i * Dv + j] = S[ii];
   }
 }
-template <typename T>
+template <typename T, bool HD>
 static void launch_delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s) {
   const dim3 grid(R.B, P.H);
   const int ng = 1024 / P.Dv, ni = (P.D + ng - 1) / ng;
   if (P.D * P.Dv <= 2048 && (P.D + 256 / P.Dv - 1) / (256 / P.Dv) <= 8)
-    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 256>), grid, dim3(256), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 256, HD>), grid, dim3(256), 0, s, P, R);
   else if (ni <= 4)
-    hipLaunchKernelGGL((delta_walk_kernel<T, 4, 1024>), grid, dim3(1024), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 4, 1024, HD>), grid, dim3(1024), 0, s, P, R);
   else if (ni <= 8)
-    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 1024>), grid, dim3(1024), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 8, 1024, HD>), grid, dim3(1024), 0, s, P, R);
   else if (ni <= 16)
-    hipLaunchKernelGGL((delta_walk_kernel<T, 16, 1024>), grid, dim3(1024), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 16, 1024, HD>), grid, dim3(1024), 0, s, P, R);
   else if (ni <= 32)
-    hipLaunchKernelGGL((delta_walk_kernel<T, 32, 1024>), grid, dim3(1024), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 32, 1024, HD>), grid, dim3(1024), 0, s, P, R);
   else
-    hipLaunchKernelGGL((delta_walk_kernel<T, 64, 1024>), grid, dim3(1024), 0, s, P, R);
+    hipLaunchKernelGGL((delta_walk_kernel<T, 64, 1024, HD>), grid, dim3(1024), 0, s, P, R);
 }
 void delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s) {
   check_delta(P, R);
-  if (P.f32)
-    launch_delta_walk<float>(P, R, s);
+  if (P.f32 && P.head_decay)
+    launch_delta_walk<float, true>(P, R, s);
+  else if (P.f32)
+    launch_delta_walk<float, false>(P, R, s);
+  else if (P.head_decay)
+    launch_delta_walk<bf16, true>(P, R, s);
   else
-    launch_delta_walk<bf16>(P, R, s);
+    launch_delta_walk<bf16, false>(P, R, s);
   launched("delta_walk");
 }
 
@@ -347,6 +378,7 @@ static inline size_t delta_wy_lds(int D, int Dv) {
   return (size_t)(std::max(3 * DC * (D + 1), DC * (D + Dv)) + DC * (DC + 4) + DC) * sizeof(float);
 }
 
+template <bool HD>
 __global__ __launch_bounds__(DELTA_WY_MAX) void delta_wy_kernel(DeltaParams P, DeltaChunkWs W) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -358,46 +390,84 @@ __global__ __launch_bounds__(DELTA_WY_MAX) void delta_wy_kernel(DeltaParams P, D
   float* be = A + DC * LA;         // [DC]
   float* qs = be + DC;             // [DC][D + 1]
   float* ks = qs + DC * D1;
-  float* Lc = ks + DC * D1;
+  float* Lc = ks + DC * D1;        // [DC][D + 1], or [DC] with one decay per head
   for (int i = tid; i < DC * D; i += nt) {
     const int t = i / D, d = i % D;
     const long long r = r0 + min(t, n - 1);  // (unconditional loads: all of them in flight together)
-    const float qv = P.x[r * P.ld_x + hg * D + d], kv = P.x[r * P.ld_x + (P.G + hg) * D + d], lv = P.lg[r * P.ld_lg + h * D + d];
+    const float qv = P.x[r * P.ld_x + hg * D + d], kv = P.x[r * P.ld_x + (P.G + hg) * D + d];
     qs[t * D1 + d] = t < n ? qv : 0.f;
     ks[t * D1 + d] = t < n ? kv : 0.f;
-    Lc[t * D1 + d] = t < n ? lv : 0.f;
+    if constexpr (!HD) {
+      const float lv = P.lg[r * P.ld_lg + h * D + d];
+      Lc[t * D1 + d] = t < n ? lv : 0.f;
+    }
+  }
+  if (HD && tid < 64) {  // the running log decays: one lane per token
+    float v = tid < n ? P.lg[(long long)(r0 + tid) * P.ld_lg + h] : 0.f;
+#pragma unroll
+    for (int o = 1; o < DC; o <<= 1) {
+      const float u = __shfl_up(v, o, 64);
+      if (tid >= o) v += u;
+    }
+    if (tid < DC) Lc[tid] = v;
+    if (tid < n) P.lg[(long long)(r0 + tid) * P.ld_lg + h] = v;
   }
   if (tid < DC) be[tid] = tid < n ? sigmoidf(P.proj[(long long)(r0 + tid) * P.ld + P.off_b + h]) : 0.f;
   __syncthreads();
-  if (tid < D) {
-    float acc = 0.f;
-#pragma unroll 8
-    for (int t = 0; t < DC; ++t) {
-      acc += Lc[t * D1 + tid];
-      Lc[t * D1 + tid] = acc;
-    }
-  }
-  __syncthreads();
-  for (int i = tid; i < n * D; i += nt) {  // the running log decays replace the log decays
-    const int t = i / D, d = i % D;
-    P.lg[(long long)(r0 + t) * P.ld_lg + h * D + d] = Lc[t * D1 + d];
-  }
-  for (int p = tid; p < DC * DC; p += nt) {
-    const int t = p / DC, sx = p % DC;
-    float a = 0.f, b = 0.f;
-    if (sx <= t && t < n) {
-      for (int d = 0; d < D; ++d) {  // exponents <= 0; exp2 on the transcendental unit (1 ulp)
-        const float e = ks[sx * D1 + d] * __builtin_amdgcn_exp2f((Lc[t * D1 + d] - Lc[sx * D1 + d]) * 1.44269504088896341f);
-        a += ks[t * D1 + d] * e;
-        b += qs[t * D1 + d] * e;
+  if constexpr (HD) {
+    // A and B are plain products with a factor per pair: a 16 x 16 tile of both per wave (the tile above the diagonal is 0)
+    if (tid < 256) {
+      const int lane = tid & 63, m = lane & 15, q4 = lane >> 4, mt = tid >> 7, nt2 = (tid >> 6) & 1;
+      f32x4 aa = f32x4{0.f, 0.f, 0.f, 0.f}, bb = aa;
+      if (nt2 <= mt) {
+        const float *kr = ks + (16 * mt + m) * D1, *qr = qs + (16 * mt + m) * D1, *kc = ks + (16 * nt2 + m) * D1;
+        for (int d0 = 0; d0 < D; d0 += 4) {
+          const int d = min(d0 + q4, D - 1);
+          const float kb = d0 + q4 < D ? kc[d] : 0.f;
+          aa = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[d], kb, aa, 0, 0, 0);
+          bb = __builtin_amdgcn_mfma_f32_16x16x4f32(qr[d], kb, bb, 0, 0, 0);
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * mt + 4 * q4 + i, sx = 16 * nt2 + m;
+        const float e = (sx <= t && t < n) ? __builtin_amdgcn_exp2f((Lc[t] - Lc[sx]) * 1.44269504088896341f) : 0.f;
+        A[t * LA + sx] = sx < t ? be[t] * aa[i] * e : 0.f;
+        if (t < n) W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] = bb[i] * e;
       }
     }
-    A[t * LA + sx] = sx < t ? be[t] * a : 0.f;
-    if (t < n) W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] = b;
+  } else {
+    if (tid < D) {
+      float acc = 0.f;
+#pragma unroll 8
+      for (int t = 0; t < DC; ++t) {
+        acc += Lc[t * D1 + tid];
+        Lc[t * D1 + tid] = acc;
+      }
+    }
+    __syncthreads();
+    for (int i = tid; i < n * D; i += nt) {  // the running log decays replace the log decays
+      const int t = i / D, d = i % D;
+      P.lg[(long long)(r0 + t) * P.ld_lg + h * D + d] = Lc[t * D1 + d];
+    }
+    for (int p = tid; p < DC * DC; p += nt) {
+      const int t = p / DC, sx = p % DC;
+      float a = 0.f, b = 0.f;
+      if (sx <= t && t < n) {
+        for (int d = 0; d < D; ++d) {  // exponents <= 0; exp2 on the transcendental unit (1 ulp)
+          const float e = ks[sx * D1 + d] * __builtin_amdgcn_exp2f((Lc[t * D1 + d] - Lc[sx * D1 + d]) * 1.44269504088896341f);
+          a += ks[t * D1 + d] * e;
+          b += qs[t * D1 + d] * e;
+        }
+      }
+      A[t * LA + sx] = sx < t ? be[t] * a : 0.f;
+      if (t < n) W.Bm[((long long)(r0 + t) * P.H + h) * DC + sx] = b;
+    }
   }
   for (int i = tid; i < n * D; i += nt) {  // keys decayed to the end of the chunk
     const int t = i / D, d = i % D;
-    W.Kd[(long long)(r0 + t) * P.ld_lg + h * D + d] = ks[t * D1 + d] * expf(Lc[(n - 1) * D1 + d] - Lc[t * D1 + d]);
+    const float e = HD ? Lc[n - 1] - Lc[t] : Lc[(n - 1) * D1 + d] - Lc[t * D1 + d];
+    W.Kd[(long long)(r0 + t) * W.ld_w + h * D + d] = ks[t * D1 + d] * expf(e);
   }
   __syncthreads();
   // forward substitution, a column of the right-hand sides per thread, in blocks of eight rows: the solved rows sit in LDS
@@ -407,7 +477,8 @@ __global__ __launch_bounds__(DELTA_WY_MAX) void delta_wy_kernel(DeltaParams P, D
   float x[DC];
   if (key) {
 #pragma unroll
-    for (int t = 0; t < DC; ++t) x[t] = be[t] * ks[t * D1 + col] * __builtin_amdgcn_exp2f(Lc[t * D1 + col] * 1.44269504088896341f);
+    for (int t = 0; t < DC; ++t)
+      x[t] = be[t] * ks[t * D1 + col] * __builtin_amdgcn_exp2f((HD ? Lc[t] : Lc[t * D1 + col]) * 1.44269504088896341f);
   } else if (col < NC) {
     const unsigned at = 2 * P.G * D + h * Dv + col - D;
 #pragma unroll
@@ -423,8 +494,8 @@ __global__ __launch_bounds__(DELTA_WY_MAX) void delta_wy_kernel(DeltaParams P, D
   float* X = qs + col;  // [DC][D + Dv]
 #pragma unroll
   for (int t = 0; t < DC; ++t) X[t * NC] = x[t];
-  float* out = key ? W.W + (long long)r0 * P.ld_lg + h * D + col : W.u + (long long)r0 * P.ld_gate + h * Dv + col - D;
-  const int ldo = key ? P.ld_lg : P.ld_gate;
+  float* out = key ? W.W + (long long)r0 * W.ld_w + h * D + col : W.u + (long long)r0 * P.ld_gate + h * Dv + col - D;
+  const int ldo = key ? W.ld_w : P.ld_gate;
 #pragma unroll 1
   for (int b0 = 0; b0 < n; b0 += 8) {
     float y[8];
@@ -466,7 +537,7 @@ template <int TJ>
 struct DeltaOps {
   float wa[TJ][2][4], kd[TJ][8], el[TJ][4], vp[2];
 };
-template <int TJ, bool VEC>
+template <int TJ, bool VEC, bool HD>
 __device__ __forceinline__ void delta_fetch(const DeltaParams& P, const DeltaChunkWs& W, int r0, int n, int h, int ct,
                                             DeltaOps<TJ>& o) {
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, m = lane & 15, q4 = lane >> 4, D = P.D;
@@ -475,7 +546,7 @@ __device__ __forceinline__ void delta_fetch(const DeltaParams& P, const DeltaChu
     const int dt = 16 * (wv + 4 * j), dq = dt + 4 * q4;
 #pragma unroll
     for (int mt = 0; mt < 2; ++mt) {
-      const float* wr = W.W + (long long)(r0 + min(16 * mt + m, n - 1)) * P.ld_lg + h * D;
+      const float* wr = W.W + (long long)(r0 + min(16 * mt + m, n - 1)) * W.ld_w + h * D;
       if constexpr (VEC) {
         const f32x4 a = *(const f32x4*)(wr + min(dq, D - 4));
 #pragma unroll
@@ -487,10 +558,10 @@ __device__ __forceinline__ void delta_fetch(const DeltaParams& P, const DeltaChu
     }
 #pragma unroll
     for (int kk = 0; kk < 8; ++kk)
-      o.kd[j][kk] = W.Kd[(long long)(r0 + min(4 * kk + q4, n - 1)) * P.ld_lg + h * D + min(dt + m, D - 1)];
-    const float* lr = P.lg + (long long)(r0 + n - 1) * P.ld_lg + h * D;
+      o.kd[j][kk] = W.Kd[(long long)(r0 + min(4 * kk + q4, n - 1)) * W.ld_w + h * D + min(dt + m, D - 1)];
+    const float* lr = P.lg + (long long)(r0 + n - 1) * P.ld_lg + (HD ? h : h * D);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) o.el[j][i] = lr[min(dq + i, D - 1)];
+    for (int i = 0; i < 4; ++i) o.el[j][i] = lr[HD ? 0 : min(dq + i, D - 1)];
   }
 #pragma unroll
   for (int k = 0; k < 2; ++k) {
@@ -498,7 +569,7 @@ __device__ __forceinline__ void delta_fetch(const DeltaParams& P, const DeltaChu
     o.vp[k] = W.u[(long long)(r0 + min(e >> 4, n - 1)) * P.ld_gate + h * P.Dv + min(ct * 16 + (e & 15), P.Dv - 1)];
   }
 }
-template <int TJ, bool VEC>
+template <int TJ, bool VEC, bool HD>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams P, DeltaChunkWs W) {
   __shared__ float part[4][DC][17];
   __shared__ float us[DC][17];
@@ -522,10 +593,10 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaParams P, DeltaChu
   int c = c0, r0 = W.chunks[4 * c0], n = W.chunks[4 * c0 + 1], flags = W.chunks[4 * c0 + 3];
   int cn = min(c0 + 1, W.nchunks - 1), r0n = W.chunks[4 * cn], nn = W.chunks[4 * cn + 1], fn = W.chunks[4 * cn + 3];
   DeltaOps<TJ> opa, opb;
-  delta_fetch<TJ, VEC>(P, W, r0, n, h, ct, opa);
+  delta_fetch<TJ, VEC, HD>(P, W, r0, n, h, ct, opa);
   auto step = [&](DeltaOps<TJ>& cur, DeltaOps<TJ>& nxt) {
     const bool last = (flags & 2) != 0;  // the sequence's last chunk of the step
-    delta_fetch<TJ, VEC>(P, W, last ? r0 : r0n, last ? n : nn, h, ct, nxt);
+    delta_fetch<TJ, VEC, HD>(P, W, last ? r0 : r0n, last ? n : nn, h, ct, nxt);
     cn = min(c + 2, W.nchunks - 1);      // the table's entry after the next one
     const int r0m = W.chunks[4 * cn], nm = W.chunks[4 * cn + 1], fm = W.chunks[4 * cn + 3];
     float* Sin = W.Sin + (long long)c * W.s_stride + (long long)h * D * Dv;
@@ -588,7 +659,7 @@ static inline size_t delta_out_lds(int D, int Dv) {
   const int Dp = (D + 15) / 16 * 16;
   return (size_t)(DC * (Dp + 4) + DC * (DC + 4) + DC * (Dv + 1)) * sizeof(float);
 }
-template <typename T>
+template <typename T, bool HD>
 __global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams P, DeltaChunkWs W) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
@@ -601,7 +672,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams P, DeltaChun
   for (int i = tid; i < DC * Dp; i += 256) {
     const int t = i / Dp, d = i % Dp;
     const long long r = r0 + t;
-    qd[t * LQ + d] = (t < n && d < D) ? P.x[r * P.ld_x + hg * D + d] * expf(P.lg[r * P.ld_lg + h * D + d]) : 0.f;
+    qd[t * LQ + d] = (t < n && d < D) ? P.x[r * P.ld_x + hg * D + d] * expf(P.lg[r * P.ld_lg + (HD ? h : h * D + d)]) : 0.f;
   }
   for (int i = tid; i < DC * DC; i += 256) {
     const int t = i / DC, sx = i % DC;
@@ -657,33 +728,40 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaParams P, DeltaChun
     const float f = P.out_scale / sqrtf(wave_sum(ss) / (float)Dv + P.eps);
     for (int d = lane; d < Dv; d += 64)
       st((T*)P.out + (long long)(r0 + t) * P.ld_out + h * Dv + d,
-         ob[t * V1 + d] * f * P.norm_w[d] * P.gate[(long long)(r0 + t) * P.ld_gate + h * Dv + d]);
+         ob[t * V1 + d] * f * P.norm_w[d] * delta_gate<HD>(P, r0 + t, h * Dv + d));
   }
+}
+template <bool HD>
+static void launch_delta_chunked(const DeltaParams& P, const DeltaChunkWs& W, hipStream_t s) {
+  const dim3 grid(W.nchunks, P.H);
+  hipLaunchKernelGGL(delta_wy_kernel<HD>, grid, dim3(std::max(256, (P.D + P.Dv + 63) / 64 * 64)), delta_wy_lds(P.D, P.Dv), s, P, W);
+  launched("delta_wy");
+  const dim3 sg(P.H * ((P.Dv + 15) / 16), W.nchunks);
+  const int vec = P.D % 4 == 0 && W.ld_w % 4 == 0 && ((uintptr_t)W.W & 15) == 0;
+  if (P.D <= 64 && vec)
+    hipLaunchKernelGGL((delta_scan_kernel<1, true, HD>), sg, dim3(256), 0, s, P, W);
+  else if (P.D <= 64)
+    hipLaunchKernelGGL((delta_scan_kernel<1, false, HD>), sg, dim3(256), 0, s, P, W);
+  else if (vec)
+    hipLaunchKernelGGL((delta_scan_kernel<2, true, HD>), sg, dim3(256), 0, s, P, W);
+  else
+    hipLaunchKernelGGL((delta_scan_kernel<2, false, HD>), sg, dim3(256), 0, s, P, W);
+  launched("delta_scan");
+  if (P.f32)
+    hipLaunchKernelGGL((delta_out_kernel<float, HD>), grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
+  else
+    hipLaunchKernelGGL((delta_out_kernel<bf16, HD>), grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
+  launched("delta_out");
 }
 void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& W, hipStream_t s) {
   check_delta(P, R);
   check(delta_chunk_supported(P.D, P.Dv) && W.chunks && W.nchunks > 0 && W.nchunks <= W.max_chunks && W.Sin && W.W && W.Kd && W.u && W.Bm &&
-            W.s_stride >= (long long)P.H * P.D * P.Dv,
+            W.s_stride >= (long long)P.H * P.D * P.Dv && W.ld_w >= P.H * P.D,
         "chunked gated delta rule: operands (key size <= 128)");
-  const dim3 grid(W.nchunks, P.H);
-  hipLaunchKernelGGL(delta_wy_kernel, grid, dim3(std::max(256, (P.D + P.Dv + 63) / 64 * 64)), delta_wy_lds(P.D, P.Dv), s, P, W);
-  launched("delta_wy");
-  const dim3 sg(P.H * ((P.Dv + 15) / 16), W.nchunks);
-  const int vec = P.D % 4 == 0 && P.ld_lg % 4 == 0 && ((uintptr_t)W.W & 15) == 0;
-  if (P.D <= 64 && vec)
-    hipLaunchKernelGGL((delta_scan_kernel<1, true>), sg, dim3(256), 0, s, P, W);
-  else if (P.D <= 64)
-    hipLaunchKernelGGL((delta_scan_kernel<1, false>), sg, dim3(256), 0, s, P, W);
-  else if (vec)
-    hipLaunchKernelGGL((delta_scan_kernel<2, true>), sg, dim3(256), 0, s, P, W);
+  if (P.head_decay)
+    launch_delta_chunked<true>(P, W, s);
   else
-    hipLaunchKernelGGL((delta_scan_kernel<2, false>), sg, dim3(256), 0, s, P, W);
-  launched("delta_scan");
-  if (P.f32)
-    hipLaunchKernelGGL(delta_out_kernel<float>, grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
-  else
-    hipLaunchKernelGGL(delta_out_kernel<bf16>, grid, dim3(256), delta_out_lds(P.D, P.Dv), s, P, W);
-  launched("delta_out");
+    launch_delta_chunked<false>(P, W, s);
 }
 
 }  // namespace stack

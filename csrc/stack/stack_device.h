@@ -65,6 +65,16 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
 __device__ __forceinline__ float silu(float z) { return z / (1.f + expf(-z)); }
 __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
 
+__device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
+// rotation by pos * f: the angle and its reduction to [-pi, pi] in float64 (a float32 angle at position 10^3 is off by 10^-4),
+// sine and cosine of the reduced angle in float32
+__device__ __forceinline__ void rotary_cs(int pos, double f, float amp, float& c, float& s) {
+  const double ang = (double)pos * f;
+  const float red = (float)(ang - 6.283185307179586 * rint(ang * 0.15915494309189535));
+  c = amp * cosf(red);
+  s = amp * sinf(red);
+}
+
 // hidden unit of a routed expert from its gate and up products; w: the weight on the expert's input (1 without P.w_input)
 __device__ __forceinline__ float moe_unit(int act, float limit, float w, float gate, float up) {
   gate *= w;
@@ -73,8 +83,11 @@ __device__ __forceinline__ float moe_unit(int act, float limit, float w, float g
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g * sigmoidf(1.702f * g) * (u + 1.f);
   }
+  if (act == MOE_ACT_GELU_UP) return gelu_erf(up);
   return silu(gate) * up;
 }
+// rows of an expert's first matrix per hidden unit: gate and up, or up alone
+__host__ __device__ __forceinline__ int moe_rows(int act) { return act == MOE_ACT_GELU_UP ? 1 : 2; }
 
 static inline void check(bool ok, const char* what) {
   if (!ok) throw std::runtime_error(std::string("stack kernels: ") + what);
@@ -119,6 +132,14 @@ __device__ __forceinline__ float wave_dot<float>(const float* __restrict__ w, co
     for (int k = lane; k < K; k += 64) acc += w[k] * x[k];
   }
   return wave_sum(acc);
+}
+// hidden unit f of routed expert e for the activations x, by one wave
+template <typename T>
+__device__ __forceinline__ float moe_hidden(const MoeParams& P, int e, int f, const T* x, float w, int lane, bool vec) {
+  const T* w0 = (const T*)P.w_gu + ((long long)e * moe_rows(P.act) * P.F + f) * P.E;
+  if (P.act == MOE_ACT_GELU_UP) return moe_unit(P.act, P.limit, w, 0.f, wave_dot<T>(w0, x, P.E, lane, vec));
+  const float gate = wave_dot<T>(w0, x, P.E, lane, vec), up = wave_dot<T>(w0 + (long long)P.F * P.E, x, P.E, lane, vec);
+  return moe_unit(P.act, P.limit, w, gate, up);
 }
 template <typename T>
 static inline bool vec_ok(const void* p, long long ld_elems, int K) {

@@ -80,6 +80,8 @@ static long long prenorm_state_floats(const LayerDesc& L) {  // the mixers' part
   if (L.kind == 4)
     return (long long)L.heads * L.state * L.vdim + (long long)(L.conv - 1) * (L.heads * L.vdim + 2 * L.groups * L.state);
   if (L.kind == 6) return (long long)L.heads * L.dim * L.vdim;
+  if (L.kind == 7) return (long long)L.heads * L.dim * L.vdim + (long long)L.conv_ring * (2 * L.kv_heads * L.dim + L.heads * L.vdim);
+  if (L.qk_norm == QK_NORM_WHOLE_FIRST) return (long long)L.conv_ring * ((L.heads + L.kv_heads) * L.dim + L.kv_heads * L.vdim);
   if (L.r_delta)
     return (long long)L.r_heads * L.r_dim * L.r_vdim + (long long)(L.conv - 1) * (2 * L.r_kv_heads * L.r_dim + L.r_heads * L.r_vdim);
   return 0;
@@ -94,6 +96,25 @@ static void validate_delta(const StackExecutor& e, const RunDesc& r, const Layer
        "gated delta rule operands or buffers");
   need(L.r_kv_heads > 0 && L.r_heads % L.r_kv_heads == 0 && delta_supported(L.r_dim, L.r_vdim, L.r_rank, L.r_grank),
        "gated delta rule sizes (key and value size <= 256, both low-rank maps together <= 1024)");
+}
+static void validate_head_delta(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
+  const StackWorkspace& ws = e.ws;
+  need(r.state && r.state_stride >= prenorm_state_floats(L), "gated delta rule without a state, or its slot too small");
+  need(L.conv_w && L.a_log && L.dt_bias && L.gnorm && ws.cbuf && ws.dl_lg && ws.dl_gate && L.conv >= 1 &&
+           (L.conv == 1 || L.conv_ring >= L.conv - 1 + CONV_RING_ROWS) && 2 * L.kv_heads * L.dim + L.heads * L.vdim <= ws.ld_cbuf &&
+           L.heads * L.dim <= ws.ld_dl_lg && L.heads * L.vdim <= ws.ld_dl_gate,
+       "gated delta rule operands or buffers");
+  need(L.kv_heads > 0 && L.heads % L.kv_heads == 0 && delta_head_supported(L.dim, L.vdim),
+       "gated delta rule sizes (key and value size <= 256)");
+}
+static void validate_conv_attention(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
+  need(r.kc && r.vc && L.conv_w && L.q_norm && L.k_norm && L.chunk >= 0 && L.window >= 0 && e.ws.cbuf && L.heads * L.dim <= e.ws.ld_cbuf &&
+           (L.rot_dims == 0 || L.inv_freq64) && L.rot_dims % 2 == 0 && L.rot_dims <= L.dim,
+       "attention with convolutions: operands or buffers");
+  need(L.conv == 1 || (L.conv_ring >= L.conv - 1 + CONV_RING_ROWS && r.state && r.state_stride >= prenorm_state_floats(L)),
+       "attention with convolutions: its state slot is too small");
+  need(L.dim <= 256 && L.vdim <= 256 && qkv_conv_supported(L.heads, L.kv_heads, L.dim, L.vdim),
+       "attention sizes (<= 256, up to 14336 query, key or value rows)");
 }
 static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const LayerDesc& L) {
   const StackWorkspace& ws = e.ws;
@@ -112,12 +133,20 @@ static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const Lay
   } else if (L.kind == 6) {
     need(r.state && L.decay && L.mnorm && ws.ret.obuf && ws.ret.ld_o >= L.heads * L.vdim, "constant-decay linear attention operands");
     need(gated_scan_supported(SCAN_FIXED, L.dim, L.vdim), "constant-decay linear attention head sizes (<= 256)");
+  } else if (L.kind == 7) {
+    validate_head_delta(e, r, L);
+  } else if (L.kind == 0 && L.qk_norm == QK_NORM_WHOLE_FIRST) {
+    validate_conv_attention(e, r, L);
   } else if (L.kind == 0 && L.maps == 1 && !L.score_talk) {
     need(r.kc && r.vc && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= 256 && L.vdim <= 256 && L.chunk >= 0,
          "attention sizes (<= 256)");
     if (L.r_delta) validate_delta(e, r, L);
   } else if (L.kind == 2) {
-    need(r.kc && L.w_uk && L.w_uvT && L.dkv_norm && ws.cbuf && ws.lat && L.gate == 2, "latent attention operands");
+    need(r.kc && L.w_uk && L.w_uvT && L.dkv_norm && ws.cbuf && ws.lat && (L.gate == 2 || L.gate == 0) && L.window >= 0,
+         "latent attention operands");
+    need(L.q_rank == 0 || (L.dq_norm && L.w_uq && ws.qlat && L.q_rank <= ws.ld_qlat && L.off_q >= L.n_in &&
+                           L.off_q + L.heads * (L.dim + L.rot_dim) <= ws.ld_proj),
+         "latent attention: the queries' latent");
     need(latent_supported(L.dim, L.rot_dim, L.kv_rank, L.vdim),
          "latent attention sizes (dim <= 256, kv_rank <= 256, kv_rank + rot_dim <= 1024)");
     need(L.heads * (L.kv_rank + L.rot_dim) <= ws.ld_cbuf && L.heads * L.kv_rank <= ws.ld_lat, "latent attention buffers");
@@ -135,11 +164,13 @@ static void validate_prenorm(const StackExecutor& e, const RunDesc& r, const Lay
     }
   }
   if (L.ff_dense) {
-    need(L.ff_dense == 3 && L.w_ff && L.w_dense_down && L.norm2_w && L.ff > 0 && L.ff <= ws.ld_hmid && 2 * L.ff <= ws.ld_proj && ws.hmid,
+    need((L.ff_dense == 3 || L.ff_dense == 4) && L.w_ff && L.w_dense_down && L.norm2_w && L.ff > 0 && L.ff <= ws.ld_hmid &&
+             2 * L.ff <= ws.ld_proj && ws.hmid,
          "gated feed-forward operands");
   } else if (L.experts) {
     need(L.w_ff && L.norm2_w && L.n_ff <= ws.ld_proj && L.top > 0 && L.top <= MOE_MAX_TOP && L.top <= ws.ld_top &&
-             L.top * L.ff <= ws.ld_hmid && ws.hmid && ws.eids && ws.ew && L.w_gu && L.w_down && L.experts <= 256,
+             L.top * L.ff + L.shared_ff <= ws.ld_hmid && (!L.shared_ff || L.sh_down) && ws.hmid && ws.eids && ws.ew && L.w_gu &&
+             L.w_down && L.experts <= 256,
          "routed feed-forward operands (up to 256 experts)");
   }
 }
@@ -271,21 +302,23 @@ void StackExecutor::linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hi
 
 // the gated delta rule beside an attention, up to the output projection; its outputs sit beside the attention's in ws.a
 DeltaParams StackExecutor::delta_params(const RunDesc& r, const LayerDesc& L) const {
-  const long long sf = (long long)L.r_heads * L.r_dim * L.r_vdim;
+  const bool alone = L.kind == 7;  // no attention beside it: one decay per head
   DeltaParams P{};
   P.proj = ws.proj;
   P.ld = ws.ld_proj;
-  P.off_q = L.off_rq;
+  P.off_q = alone ? L.off_q : L.off_rq;
   P.off_b = L.off_rb;
   P.off_a1 = L.off_a1;
-  P.off_g1 = L.off_g1;
-  P.H = L.r_heads;
-  P.G = L.r_kv_heads;
-  P.D = L.r_dim;
-  P.Dv = L.r_vdim;
+  P.off_g1 = alone ? L.off_g : L.off_g1;
+  P.H = alone ? L.heads : L.r_heads;
+  P.G = alone ? L.kv_heads : L.r_kv_heads;
+  P.D = alone ? L.dim : L.r_dim;
+  P.Dv = alone ? L.vdim : L.r_vdim;
   P.taps = L.conv;
   P.conv_w = L.conv_w;
-  P.window = r.state + sf;
+  P.window = r.state + (long long)P.H * P.D * P.Dv;
+  P.head_decay = alone;
+  P.ring = L.conv_ring;
   P.rank_a = L.r_rank;
   P.rank_g = L.r_grank;
   P.a2 = L.a2;
@@ -302,22 +335,74 @@ DeltaParams StackExecutor::delta_params(const RunDesc& r, const LayerDesc& L) co
   P.ld_lg = ws.ld_dl_lg;
   P.gate = ws.dl_gate;
   P.ld_gate = ws.ld_dl_gate;
-  P.out = (char*)ws.a + (size_t)L.heads * L.vdim * (cfg.f32 ? 4 : 2);
+  P.out = (char*)ws.a + (alone ? 0 : (size_t)L.heads * L.vdim * (cfg.f32 ? 4 : 2));
   P.ld_out = ws.ld_a;
-  P.out_scale = L.right_scale;
+  P.out_scale = alone ? 1.f : L.right_scale;
   P.f32 = cfg.f32;
-  P.kv = KvStoreParams{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, cfg.f32};
+  if (!alone)
+    P.kv = KvStoreParams{ws.proj, ws.ld_proj, L.off_k, L.off_v, L.kv_heads, L.dim, L.vdim, L.v_unit, cfg.eps, r.kc, r.vc, cfg.f32};
   return P;
 }
 void StackExecutor::delta_mixer(const DeltaParams& P, int B, hipStream_t s) {  // after delta_prepare
   StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
   if (B > SMALL_B && n_chunks > 0 && ws.ret.Sin && ws.dl_W && ws.dl_Kd && ws.dl_u && ws.dl_Bm &&
       ws.ret.u_stride >= (long long)P.H * P.D * P.Dv && ws.dl_heads >= P.H && delta_chunk_supported(P.D, P.Dv)) {
-    DeltaChunkWs W{ws.ret.chunks, n_chunks, ws.ret.max_chunks, ws.ret.Sin, ws.ret.u_stride, ws.dl_W, ws.dl_Kd, ws.dl_u, ws.dl_Bm};
+    DeltaChunkWs W{ws.ret.chunks, n_chunks, ws.ret.max_chunks, ws.ret.Sin, ws.ret.u_stride, ws.dl_W, ws.dl_Kd, ws.dl_u, ws.dl_Bm,
+                   ws.ld_dl_lg};
     delta_chunked(P, R, W, s);
   } else {
     delta_walk(P, R, s);
   }
+}
+
+// softmax attention of one mixer: query tiles on the matrix cores for prompt portions, else the per-row kernels
+void StackExecutor::softmax_mixer(const AttnParams& A, int B, hipStream_t s) {
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  if (B > SMALL_B && n_tiles > 0 && tiles && flash_prefill_supported(A))
+    flash_prefill(A, R, tiles, n_tiles, s);
+  else
+    attention(A, R, s);
+}
+// a window or block of positions bounds the keys of a decode step: up to 1024 of them are not shared among blocks
+int StackExecutor::bounded_splits(int bound) const { return bound > 0 && bound <= 1024 ? 1 : n_splits; }
+
+// pre-norm layers: latent attention up to its output projection; its input columns are in ws.proj
+void StackExecutor::latent_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
+  const int C = L.kv_rank, W = C + L.rot_dim, f32 = cfg.f32;
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  if (L.q_rank) {  // the queries from a normed latent of their own, into columns behind the input stack's
+    const int nq = L.heads * (L.dim + L.rot_dim);
+    float* q = ws.proj + L.off_q;
+    if (gemv_group_rms_supported(B, L.q_rank, 1, f32)) {  // decode steps: the norm in the product's launch
+      gemv_group_rms(ws.proj + L.off_dq, ws.ld_proj, L.q_rank, 1, L.dq_norm, cfg.eps, nullptr, 0, L.w_uq, B, nq, q, ws.ld_proj, 0, f32, s);
+    } else {
+      group_rms_cast(ws.proj + L.off_dq, ws.ld_proj, B, L.q_rank, 1, L.dq_norm, cfg.eps, nullptr, 0, ws.qlat, ws.ld_qlat, f32, s);
+      GemmParams g{ws.qlat, ws.ld_qlat, L.w_uq, B, nq, L.q_rank, q, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
+      gemm(g, s);
+    }
+  }
+  LatentParams P{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_g, L.heads, L.dim, L.rot_dim, C, L.vdim, L.rot_dims,
+                 L.inv_freq64, L.dkv_norm, cfg.eps, L.w_uk, L.w_uvT, L.w_ukT, L.w_uv, r.kc, ws.cbuf, ws.ld_cbuf, ws.lat, ws.ld_lat, ws.a,
+                 ws.ld_a, f32, L.gate == 2 ? 1 : 2, L.rot_amp};
+  latent_prepare(P, R, s);
+  AttnParams A{ws.cbuf, ws.ld_cbuf, 0, 0, 0, L.heads, 1, W, C, L.scale, 0.f, 0.f, 1, r.kc, r.kc, ws.lat, ws.ld_lat, f32,
+               bounded_splits(L.window), ws.split_ws, ws.split_ws_floats, W, W, nullptr};
+  A.window = L.window;
+  softmax_mixer(A, B, s);
+  latent_expand(P, B, s);
+}
+// pre-norm layers: attention whose q, k and v pass a convolution each, up to its output projection
+void StackExecutor::conv_attention_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s) {
+  StepRows R{B, in.pos, in.slot, in.q_len, in.q_seq, in.block_table, in.max_blocks, in.bs};
+  QkvConvParams Q{ws.proj, ws.ld_proj, L.in_b, L.heads, L.kv_heads, L.dim, L.vdim, L.conv, L.conv_w, r.state, r.state_stride, L.conv_ring,
+                  L.q_norm, L.k_norm, cfg.eps, L.rot_dims, L.inv_freq64, L.rot_amp, ws.cbuf, ws.ld_cbuf, r.kc, r.vc, cfg.f32};
+  qkv_conv_prepare(Q, R, s);
+  AttnParams A{ws.cbuf, ws.ld_cbuf, 0, 0, 0, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, 0.f, 0.f, 1, r.kc, r.vc, ws.a, ws.ld_a, cfg.f32,
+               bounded_splits(L.chunk > 0 ? L.chunk : L.window), ws.split_ws, ws.split_ws_floats};
+  A.window = L.window;
+  A.chunk = L.chunk;
+  A.maps = 1;
+  softmax_mixer(A, B, s);
 }
 
 // x <- x + LN1(mixer(x)), then x <- x + LN2(ff(x)): both sublayers read the stream itself (cast to the matrix
@@ -501,8 +586,8 @@ void StackExecutor::layer_run_sandwich(int ri, int B, hipStream_t s) {
 // x <- x + mixer(N1(x)), then x <- x + ff(N2(x)); N: RMS norm with a weight vector. A pass of a repeated span opens with
 // x <- W_in [x; x0]. Mixers: attention inside a sliding window with two differential maps per head and an
 // element-wise gate; attention inside a sliding window with adjacent-pair rotation and scores mixed across the heads
-// before the softmax; latent attention with one gate per head;
-// before the mixer (and, with cfg.canon_both, a convolution on the inputs of both sublayers): Mamba-2, constant-decay linear
+// before the softmax; latent attention; attention whose q, k and v pass convolutions; a gated delta rule with one decay per
+// head; and (with cfg.canon_both a convolution sits on the inputs of both sublayers) Mamba-2, constant-decay linear
 // attention, or attention inside blocks of positions with a gated delta rule beside it.
 // The sublayer's input into ws.h, and with W the product with it into ws.proj.
 void StackExecutor::norm_in(const RunDesc& r, const float* w, const float* canon, long long window_at, const void* W, int N, int B,
@@ -548,14 +633,17 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     gemv_ln(ws.resid, E, L.norm_w, nullptr, cfg.eps, L.w_in, B, L.n_in, ws.proj, ws.ld_proj, ws.h, &St, &R, f32, s);
   else
     norm_in(r, L.norm_w, L.canon, win1, L.w_in, L.n_in, B, s);
-  const bool tiled = B > SMALL_B && n_tiles > 0 && tiles;
-  // a window bounds the keys of a decode step: no need to share them among blocks
-  const int bound = L.chunk > 0 ? L.chunk : L.window;
-  const int splits = bound > 0 && bound <= 1024 ? 1 : n_splits;
+  const int splits = bounded_splits(L.chunk > 0 ? L.chunk : L.window);
   if (L.kind == 4) {
     mamba2_mixer(r, L, B, s);
   } else if (L.kind == 6) {
     linear_mixer(r, L, B, s);
+  } else if (L.kind == 7) {
+    const DeltaParams delta = delta_params(r, L);
+    delta_prepare(delta, R, s);
+    delta_mixer(delta, B, s);
+  } else if (L.kind == 0 && L.qk_norm == QK_NORM_WHOLE_FIRST) {
+    conv_attention_mixer(r, L, B, s);
   } else if (L.kind == 0 && L.maps == 1 && !L.score_talk) {
     DeltaParams delta{};
     if (L.r_delta) {
@@ -574,34 +662,17 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     A.hgate = L.gate == 2 ? ws.proj + L.off_g : nullptr;
     A.ld_hgate = ws.ld_proj;
     A.out_scale = L.left_scale;
-    if (tiled && flash_prefill_supported(A))
-      flash_prefill(A, R, tiles, n_tiles, s);
-    else
-      attention(A, R, s);
+    softmax_mixer(A, B, s);
     if (L.r_delta) delta_mixer(delta, B, s);
   } else if (L.kind == 2) {
-    const int C = L.kv_rank, W = C + L.rot_dim;
-    LatentParams P{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_g, L.heads, L.dim, L.rot_dim, C, L.vdim, L.rot_dims,
-                   L.inv_freq64, L.dkv_norm, cfg.eps, L.w_uk, L.w_uvT, L.w_ukT, L.w_uv, r.kc, ws.cbuf, ws.ld_cbuf, ws.lat, ws.ld_lat, ws.a,
-                   ws.ld_a, f32, 1};
-    latent_prepare(P, R, s);
-    AttnParams A{ws.cbuf, ws.ld_cbuf, 0, 0, 0, L.heads, 1, W, C, L.scale, 0.f, 0.f, 1, r.kc, r.kc, ws.lat, ws.ld_lat, f32,
-                 n_splits, ws.split_ws, ws.split_ws_floats, W, W, nullptr};
-    if (tiled && flash_prefill_supported(A))
-      flash_prefill(A, R, tiles, n_tiles, s);
-    else
-      attention(A, R, s);
-    latent_expand(P, B, s);
+    latent_mixer(r, L, B, s);
   } else if (L.maps == 2) {
     // the 2 * heads query maps are heads of their own
     if (!fused_in) attn_prepare(St, R, s);
     AttnParams A{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, 2 * L.heads, L.kv_heads, L.dim, L.vdim, L.scale, 0.f, 0.f, 1, r.kc,
                  r.vc, ws.a, ws.ld_a, f32, splits, ws.split_ws, ws.split_ws_floats, 2 * L.dim, 0, nullptr, 0, ws.cbuf, ws.ld_cbuf,
                  L.window, 2, 0};
-    if (tiled && flash_prefill_supported(A))
-      flash_prefill(A, R, tiles, n_tiles, s);
-    else
-      attention(A, R, s);
+    softmax_mixer(A, B, s);
     diff_combine(ws.cbuf, ws.ld_cbuf, B, L.heads, L.vdim, L.lam, L.diff, cfg.eps, ws.proj + L.off_g, ws.ld_proj, ws.a, ws.ld_a, f32, s);
   } else {
     RotFoldParams F{ws.proj, ws.ld_proj, L.off_q, L.off_k, L.off_v, L.heads, L.kv_heads, L.dim, L.vdim, L.rot_dims, L.inv_freq64,
@@ -610,15 +681,12 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
     // one key row per token serves every head: its width is all key/value heads' keys, the folded queries match it
     AttnParams A{ws.cbuf, ws.ld_cbuf, 0, 0, 0, L.heads, L.kv_heads, L.kv_heads * L.dim, L.vdim, L.scale, 0.f, 0.f, 1, r.kc, r.vc, ws.a,
                  ws.ld_a, f32, splits, ws.split_ws, ws.split_ws_floats, 0, 0, nullptr, 0, nullptr, 0, L.window, 1, 1};
-    if (tiled && flash_prefill_supported(A))
-      flash_prefill(A, R, tiles, n_tiles, s);
-    else
-      attention(A, R, s);
+    softmax_mixer(A, B, s);
   }
   if ((L.kind == 4 || L.kind == 6) && mixer_norm_fused(L, B)) {  // decode steps: the mixer's output norm with the projection
     const bool lin = L.kind == 6;
     gemv_group_rms(ws.ret.obuf, ws.ret.ld_o, n_out, lin ? 1 : L.norm_groups, L.mnorm, cfg.eps, lin ? ws.proj + L.off_g : nullptr,
-                   ws.ld_proj, L.w_o, B, E, ws.resid, E, f32, s);
+                   ws.ld_proj, L.w_o, B, E, ws.resid, E, 1, f32, s);
   } else {
     GemmParams o{ws.a, ws.ld_a, L.w_o, B, E, n_out, ws.resid, E, EPI_RESID, 1.f, nullptr, 0.f, f32};
     gemm(o, s);
@@ -627,21 +695,22 @@ void StackExecutor::layer_run_prenorm(int ri, int B, hipStream_t s) {
   // the router's product leaves with the norm where the step allows it (the normed rows leave for the experts)
   norm_in(r, L.norm2_w, L.canon2, win2, L.experts ? L.w_ff : nullptr, L.n_ff, B, s);
   if (L.ff_dense) {
+    const int glu = L.ff_dense == 4 ? GLU_SILU : GLU_RELU;
     if (B <= 8) {  // decode steps: gate / up projection and activation in one launch
-      gemv_relu_glu(ws.h, E, L.w_ff, E, L.ff, B, ws.hmid, ws.ld_hmid, f32, s);
+      gemv_act_glu(glu, ws.h, E, L.w_ff, E, L.ff, B, ws.hmid, ws.ld_hmid, f32, s);
     } else {
       GemmParams g{ws.h, E, L.w_ff, B, L.n_ff, E, ws.proj, ws.ld_proj, EPI_STORE, 0.f, nullptr, 0.f, f32};
       gemm(g, s);
-      relu_glu_cast(ws.proj, ws.ld_proj, B, L.ff, ws.hmid, ws.ld_hmid, f32, s);
+      act_glu_cast(glu, ws.proj, ws.ld_proj, B, L.ff, ws.hmid, ws.ld_hmid, f32, s);
     }
     GemmParams d{ws.hmid, ws.ld_hmid, L.w_dense_down, B, E, L.ff, ws.resid, E, EPI_RESID, 1.f, nullptr, 0.f, f32};
     gemm(d, s);
     return;
   }
   // the experts' weighted outputs are added straight into the stream (y = the stream, y_add)
-  MoeParams M{ws.proj, ws.ld_proj, L.off_router, 0, 0, 0, B, E, L.experts, L.top, L.ff, 0, nullptr, ws.h, L.w_gu, L.w_down, nullptr,
-              ws.eids, ws.ew, ws.ld_top, ws.sgate, ws.hmid, ws.ld_hmid, ws.resid, f32, 0, L.group_count, L.group_keep, ws.idw, 1,
-              L.route_scale, L.route_raw, L.expert_act, L.limit, L.scale_input};
+  MoeParams M{ws.proj, ws.ld_proj, L.off_router, 0, 0, L.off_sup, B, E, L.experts, L.top, L.ff, L.shared_ff, nullptr, ws.h, L.w_gu,
+              L.w_down, L.sh_down, ws.eids, ws.ew, ws.ld_top, nullptr, ws.hmid, ws.ld_hmid, ws.resid, f32, 0, L.group_count,
+              L.group_keep, ws.idw, 1, L.route_scale, L.route_raw, L.expert_act, L.limit, L.scale_input, L.route_softmax};
   if (B <= SMALL_B && moe_route_sigmoid_fused_supported(M)) {  // decode steps: routing + activations in one launch
     moe_route_sigmoid_experts(M, s);
     moe_down(M, s);

@@ -28,7 +28,8 @@ struct StackConfig {
 };
 
 struct LayerDesc {
-  int kind = 0;  // 0 attention, 1 retention, 2 latent attention, 3 mLSTM, 4 Mamba-2, 6 constant-decay linear attention
+  int kind = 0;  // 0 attention, 1 retention, 2 latent attention, 3 mLSTM, 4 Mamba-2, 6 constant-decay linear attention,
+                 // 7 gated delta rule with one decay per head
   int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
   float scale = 1.f, softcap = 0.f, qtemp_coef = 0.f;
   int qtemp_every = 1, rot_dims = 0;
@@ -91,8 +92,8 @@ struct LayerDesc {
   const float* a2_b = nullptr;
   const float* gnorm = nullptr;
   const void* w_o2 = nullptr;       // [E][r_heads * r_vdim]
-  // layers with RMS norms on the sublayers' inputs: norm_w / norm2_w are the weight vectors; ff_dense == 3 is the gated
-  // dense feed-forward with a relu gate; experts use the sigmoid router
+  // layers with RMS norms on the sublayers' inputs: norm_w / norm2_w are the weight vectors; ff_dense == 3 / 4 is the gated
+  // dense feed-forward with a relu / silu gate; experts use the sigmoid (route_softmax: softmax) router
   int window = 0;                   // sliding window of the attention (0: none)
   int maps = 1;                     // 2: differential attention (two query / key maps per head)
   float diff = 0.f, lam = 0.f;      // o = (a1 - lam a2) / rms * (1 - diff)
@@ -106,8 +107,17 @@ struct LayerDesc {
   float limit = 0.f;
   // a gated delta rule beside the attention (r_delta != 0; sizes r_heads, r_kv_heads, r_dim, r_vdim, taps `conv`); w_o is
   // [E][heads * vdim + r_heads * r_vdim]
+  // (kind 7: the delta rule alone, with heads, kv_heads, dim, vdim, conv; the columns q | k | v at off_q, write strengths at
+  // off_rb, decays' inputs at off_a1, output gate at off_g)
   int r_delta = 0, r_kv_heads = 0, r_grank = 0, off_rb = 0, off_g1 = 0;
   const void* g2 = nullptr;
+  int route_softmax = 0;
+  float rot_amp = 1.f;              // factor on the rotation's sine and cosine
+  int conv_ring = 0;                // rows of the convolution's carried inputs, if they are a ring over positions
+  // latent attention with queries from a latent of their own: its columns at off_dq; the queries' product lands at off_q
+  int q_rank = 0, off_dq = 0;
+  const float* dq_norm = nullptr;   // [q_rank]
+  const void* w_uq = nullptr;       // [heads * (dim + rot_dim)][q_rank]
 };
 
 struct RunDesc {   // one execution of a layer: its own cache
@@ -142,6 +152,8 @@ struct StackWorkspace {
   int ld_cbuf = 0;
   void* lat = nullptr;     // [max_B][ld_lat] matrix dtype: attention outputs in latent space
   int ld_lat = 0;
+  void* qlat = nullptr;    // [max_B][ld_qlat] matrix dtype: the normed latent of the queries
+  int ld_qlat = 0;
   float* idw = nullptr;    // [max_B] weight of the chosen identity experts
   float* coef = nullptr;   // [max_B][ld_coef] chunked gated scan: per (row, head) {ln a, b, m}
   int ld_coef = 0;
@@ -207,6 +219,10 @@ class StackExecutor {
   bool mixer_norm_fused(const LayerDesc& L, int B) const;
   void mamba2_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
   void linear_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  void latent_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  void conv_attention_mixer(const RunDesc& r, const LayerDesc& L, int B, hipStream_t s);
+  void softmax_mixer(const AttnParams& A, int B, hipStream_t s);
+  int bounded_splits(int bound) const;
   DeltaParams delta_params(const RunDesc& r, const LayerDesc& L) const;
   void delta_mixer(const DeltaParams& P, int B, hipStream_t s);
   void head(int n_logits, bool use_idx, hipStream_t s);

@@ -364,9 +364,9 @@ bool gemv_group_rms_supported(int M, int n, int groups, int f32) {
   return gemv_ln_supported(M, n, f32) && groups >= 1 && groups <= LN_MAX_GROUPS && n % groups == 0;
 }
 void gemv_group_rms(const float* y, int ld_y, int n, int groups, const float* w, float eps, const float* gate, int ld_gate,
-                    const void* W, int M, int N, float* C, int ldc, int f32, hipStream_t s) {
+                    const void* W, int M, int N, float* C, int ldc, int add, int f32, hipStream_t s) {
   check(gemv_group_rms_supported(M, n, groups, f32) && y && w && W && C && N > 0 && ldc >= N && ld_y >= n, "gemv_group_rms: bad operands");
-  const GemvPre pre{nullptr, 1, 0, nullptr, 0, nullptr, nullptr, gate, ld_gate, groups, ld_y, 1};
+  const GemvPre pre{nullptr, 1, 0, nullptr, 0, nullptr, nullptr, gate, ld_gate, groups, ld_y, add};
   launch_gemv_pre<PRE_GROUP, 2>(y, n, w, nullptr, eps, W, M, N, C, ldc, nullptr, QkvEpi{}, pre, f32, s);
 }
 
@@ -1796,13 +1796,9 @@ __global__ __launch_bounds__(256) void moe_experts_kernel(MoeParams P, int vec) 
   const int b = blockIdx.y / P.top, jj = blockIdx.y % P.top;
   if (f >= P.F) return;
   const int e = P.eids[(long long)b * P.ld_top + jj];
-  const T* x = (const T*)P.h + (long long)b * P.E;
-  const T* wg = (const T*)P.w_gu + ((long long)e * 2 * P.F + f) * P.E;
-  const T* wu = wg + (long long)P.F * P.E;
-  const float gate = wave_dot<T>(wg, x, P.E, lane, vec != 0);
-  const float up = wave_dot<T>(wu, x, P.E, lane, vec != 0);
   const float w = P.w_input ? P.ew[(long long)b * P.ld_top + jj] : 1.f;
-  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, moe_unit(P.act, P.limit, w, gate, up));
+  const float u = moe_hidden<T>(P, e, f, (const T*)P.h + (long long)b * P.E, w, lane, vec != 0);
+  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, u);
 }
 // one wave per (row, output unit): the routed experts' down rows in routing order, then the shared expert's
 template <typename T>
@@ -1820,7 +1816,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeParams P, int vec, int
     y += w * wave_dot<T>(wd, hm + jj * P.F, P.F, lane, vec != 0);
   }
   if (P.Fs > 0)
-    y += P.sgate[b] * wave_dot<T>((const T*)P.sh_down + (long long)n * P.Fs, hm + P.top * P.F, P.Fs, lane, vec_s != 0);
+    y += (P.sgate ? P.sgate[b] : 1.f) * wave_dot<T>((const T*)P.sh_down + (long long)n * P.Fs, hm + P.top * P.F, P.Fs, lane, vec_s != 0);
   if (lane == 0) P.y[(long long)b * P.E + n] = P.y_add ? P.y[(long long)b * P.E + n] + y : y;
 }
 // ---- prompt portions: pairs (row, routed expert) sorted by expert, one matrix-core product per expert tile
@@ -1858,8 +1854,8 @@ __global__ __launch_bounds__(256) void moe_sort_kernel(const int* __restrict__ e
     inv[p] = pos;
   }
 }
-// hs[pos][f] = the hidden unit of gu[pos][f], gu[pos][F + f] (moe_unit), in the matrix dtype; ew non-null: the pairs'
-// weights act on the experts' inputs
+// hs[pos][f] = the hidden unit of gu[pos][f], gu[pos][F + f] (moe_unit; without a gate: of gu[pos][f]), in the matrix dtype;
+// ew non-null: the pairs' weights act on the experts' inputs
 __global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ gu, int P, int F, int act, float limit,
                                                       const float* __restrict__ ew, int ld_top, int top,
                                                       const int* __restrict__ srow, bf16* __restrict__ hs) {
@@ -1872,7 +1868,8 @@ __global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ 
     const int pair = srow[pos];
     w = ew[(long long)(pair / top) * ld_top + pair % top];
   }
-  st(hs + i, moe_unit(act, limit, w, gu[pos * 2 * F + f], gu[pos * 2 * F + F + f]));
+  const int nu = moe_rows(act);
+  st(hs + i, moe_unit(act, limit, w, gu[pos * nu * F + f], gu[pos * nu * F + (nu - 1) * F + f]));
 }
 // y[b][n] = (shared ? sgate[b] * y[b][n] : 0) + sum_j ew[b][j] * ds[inv[b * top + j]][n], routing order
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ y, const float* __restrict__ ds,
@@ -1882,7 +1879,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ y,
   const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
   if (i >= (long long)B * E) return;
   const int b = (int)(i / E), n = (int)(i % E);
-  float acc = shared ? sgate[b] * y[i] : y_add ? y[i] : 0.f;  // (y_add: y is the residual stream, no shared expert)
+  float acc = shared ? sgate[b] * y[i] : y_add ? y[i] : 0.f;  // (y_add: y is the residual stream)
   float routed = 0.f;
   for (int j = 0; j < top; ++j) routed += (ew ? ew[(long long)b * ld_top + j] : 1.f) * ds[(long long)inv[b * top + j] * E + n];
   y[i] = routed + acc;
@@ -1892,9 +1889,10 @@ bool moe_grouped_supported(const MoeParams& P) {
          P.ld_hmid % 8 == 0));
 }
 void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
-  check(moe_grouped_supported(P) && W.rank && W.srow && W.inv && W.tiles && W.ntiles && W.gu && W.hs && W.ds && !(P.y_add && P.Fs > 0),
+  check(moe_grouped_supported(P) && W.rank && W.srow && W.inv && W.tiles && W.ntiles && W.gu && W.hs && W.ds &&
+            (P.Fs == 0 || P.sgate || P.y_add),
         "grouped routed feed-forward: workspace or sizes");
-  const int pairs = P.B * P.top;
+  const int pairs = P.B * P.top, n1 = moe_rows(P.act) * P.F;
   const int tile_m = pairs / P.X >= 192 ? 128 : 64;
   const int max_tiles = (pairs + tile_m - 1) / tile_m + P.X;
   check(pairs <= W.max_pairs && max_tiles <= W.max_tiles, "grouped routed feed-forward: workspace too small");
@@ -1903,16 +1901,16 @@ void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
   launched("moe_sort");
   // gate | up of every pair with its expert's matrix
   {
-    Epi e{EPI_STORE, W.gu, 2 * P.F, 0.f, nullptr, 0.f};
-    Group G{W.tiles, W.ntiles, W.srow, P.top, (long long)2 * P.F * P.E};
+    Epi e{EPI_STORE, W.gu, n1, 0.f, nullptr, 0.f};
+    Group G{W.tiles, W.ntiles, W.srow, P.top, (long long)n1 * P.E};
     if (tile_m == 128) {
-      dim3 grid((2 * P.F + 127) / 128, max_tiles);
+      dim3 grid((n1 + 127) / 128, max_tiles);
       hipLaunchKernelGGL((gemm_mfma_kernel<2, 2>), grid, dim3(256), 0, s, (const bf16*)P.h, P.E, (const bf16*)P.w_gu, pairs,
-                         2 * P.F, P.E, e, G);
+                         n1, P.E, e, G);
     } else {
-      dim3 grid((2 * P.F + 63) / 64, max_tiles);
+      dim3 grid((n1 + 63) / 64, max_tiles);
       hipLaunchKernelGGL((gemm_mfma_kernel<1, 1>), grid, dim3(256), 0, s, (const bf16*)P.h, P.E, (const bf16*)P.w_gu, pairs,
-                         2 * P.F, P.E, e, G);
+                         n1, P.E, e, G);
     }
     launched("moe_gemm gate/up");
   }
@@ -1936,15 +1934,15 @@ void moe_grouped(const MoeParams& P, const MoeGroupWs& W, hipStream_t s) {
     }
     launched("moe_gemm down");
   }
-  if (P.Fs > 0) {  // the shared expert's down projection over every row, into y
-    GemmParams g{(const bf16*)P.hmid + P.top * P.F, P.ld_hmid, P.sh_down, P.B, P.E, P.Fs, P.y, P.E, EPI_STORE, 0.f, nullptr,
-                 0.f, 0};
+  if (P.Fs > 0) {  // the shared expert's down projection over every row, into y (the stream: added to it)
+    GemmParams g{(const bf16*)P.hmid + P.top * P.F, P.ld_hmid, P.sh_down, P.B, P.E, P.Fs, P.y, P.E, P.y_add ? EPI_RESID : EPI_STORE,
+                 1.f, nullptr, 0.f, 0};
     gemm(g, s);
   }
   {
     const long long n = (long long)P.B * P.E;
     hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, P.y, W.ds, W.inv,
-                       P.w_input ? nullptr : P.ew, P.ld_top, P.sgate, P.B, P.E, P.top, (int)(P.Fs > 0), P.y_add);
+                       P.w_input ? nullptr : P.ew, P.ld_top, P.sgate, P.B, P.E, P.top, (int)(P.Fs > 0 && !P.y_add), P.y_add);
     launched("moe_combine");
   }
 }
@@ -2084,7 +2082,7 @@ void moe_fused_small(const MoeParams& P, const void* a, int lda, const void* w_o
 static void check_moe(const MoeParams& P, bool bias) {  // bias: the caller reads router_b
   check(P.B > 0 && P.X > 0 && P.top > 0 && P.top <= P.X + P.identity && P.top <= MOE_MAX_TOP && P.F > 0 && P.proj && P.h && P.w_gu &&
             P.w_down && P.eids && P.ew && P.hmid && P.y && (P.router_b || !bias) && P.ld_top >= P.top &&
-            P.ld_hmid >= P.top * P.F + P.Fs && (P.Fs == 0 || (P.sh_down && P.sgate)),
+            P.ld_hmid >= P.top * P.F + P.Fs && (P.Fs == 0 || (P.sh_down && (P.sgate || P.y_add))),
         "routed feed-forward: bad operands (top <= 16)");
 }
 void moe_route(const MoeParams& P, hipStream_t s) {

@@ -126,10 +126,10 @@ void post_norm_add(float* x, const float* y, int rows, int E, const float* w, co
 // computed in float64 (a float32 angle at position 10^3 is already off by 10^-4).
 constexpr int LAT_RB = 8;
 constexpr int LAT_MAXD = 256, LAT_MAXC = 512;
-__device__ __forceinline__ float rotate_pair_elem(const float* v, int j, int rot_dims, int pos, const double* inv_freq) {
+__device__ __forceinline__ float rotate_pair_elem(const float* v, int j, int rot_dims, int pos, const double* inv_freq, float amp) {
   if (j >= rot_dims) return v[j];
   const double ang = (double)pos * inv_freq[j >> 1];
-  const float c = (float)cos(ang), sn = (float)sin(ang);
+  const float c = amp * (float)cos(ang), sn = amp * (float)sin(ang);
   const float a = v[j & ~1], b = v[j | 1];
   return (j & 1) ? b * c + a * sn : a * c - b * sn;
 }
@@ -150,7 +150,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentParams P, Ste
       const float inv = 1.f / sqrtf(block_sum256(sq, red) / (float)C + P.eps);
       T* dst = cache + (long long)R.slot[b] * W;
       for (int c = tid; c < C; c += 256) st(dst + c, dkv[c] * inv * P.norm_w[c]);
-      for (int j = tid; j < Rr; j += 256) st(dst + C + j, rotate_pair_elem(dkv + C, j, P.rot_dims, R.pos[b], P.inv_freq));
+      for (int j = tid; j < Rr; j += 256) st(dst + C + j, rotate_pair_elem(dkv + C, j, P.rot_dims, R.pos[b], P.inv_freq, P.rot_amp));
     }
     return;
   }
@@ -176,7 +176,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentParams P, Ste
   for (int idx = tid; idx < nr * Rr; idx += 256) {
     const int i = idx / Rr, j = idx % Rr, b = r0 + i;
     const float* qr = P.proj + (long long)b * P.ld + P.off_q + h * (D + Rr) + D;
-    P.qa[(long long)b * P.ld_qa + h * W + C + j] = rotate_pair_elem(qr, j, P.rot_dims, R.pos[b], P.inv_freq);
+    P.qa[(long long)b * P.ld_qa + h * W + C + j] = rotate_pair_elem(qr, j, P.rot_dims, R.pos[b], P.inv_freq, P.rot_amp);
   }
 }
 // out[b][h * Dv + j] = (sum_c W_uvT[h][c][j] lat[b][h * C + c]) * sigmoid(g[b][h * Dv + j]); grid (row groups, H,
@@ -216,8 +216,8 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(LatentParams P, int 
     const int i = idx >> 6, col = blockIdx.z * 64 + (idx & 63);
     if (col < Dv) {
       const float o = part[0][i][idx & 63] + part[1][i][idx & 63] + part[2][i][idx & 63] + part[3][i][idx & 63];
-      const float g = P.proj[(long long)(r0 + i) * P.ld + P.off_g + (P.gate_heads ? h : h * Dv + col)];
-      st((T*)P.out + (long long)(r0 + i) * P.ld_out + h * Dv + col, o * sigmoidf(g));
+      const float f = P.gate_heads == 2 ? 1.f : sigmoidf(P.proj[(long long)(r0 + i) * P.ld + P.off_g + (P.gate_heads ? h : h * Dv + col)]);
+      st((T*)P.out + (long long)(r0 + i) * P.ld_out + h * Dv + col, o * f);
     }
   }
 }
@@ -280,11 +280,11 @@ __global__ __launch_bounds__(256) void latent_prepare_small_kernel(LatentParams 
   const float inv = 1.f / sqrtf(block_sum256(sq, red) / (float)C + P.eps);
   T* dst = (T*)P.cache + (long long)R.slot[b] * W;
   for (int c = tid; c < C; c += 256) st(dst + c, dkv[c] * inv * P.norm_w[c]);
-  for (int j = tid; j < Rr; j += 256) st(dst + C + j, rotate_pair_elem(dkv + C, j, P.rot_dims, R.pos[b], P.inv_freq));
+  for (int j = tid; j < Rr; j += 256) st(dst + C + j, rotate_pair_elem(dkv + C, j, P.rot_dims, R.pos[b], P.inv_freq, P.rot_amp));
   for (int idx = tid; idx < P.H * Rr; idx += 256) {
     const int h = idx / Rr, j = idx % Rr;
     const float* qr = P.proj + (long long)b * P.ld + P.off_q + h * (D + Rr) + D;
-    P.qa[(long long)b * P.ld_qa + h * W + C + j] = rotate_pair_elem(qr, j, P.rot_dims, R.pos[b], P.inv_freq);
+    P.qa[(long long)b * P.ld_qa + h * W + C + j] = rotate_pair_elem(qr, j, P.rot_dims, R.pos[b], P.inv_freq, P.rot_amp);
   }
 }
 // wave (h, j) -> out[b][h * Dv + j] = (W_uv[h * Dv + j][:] . lat[b][h * C :]) * sigmoid(g[b][h * Dv + j]) for every row b
@@ -297,8 +297,10 @@ __global__ __launch_bounds__(256) void latent_expand_small_kernel(LatentParams P
   const T* w = (const T*)P.w_uv + (long long)item * P.C;
   for (int b = 0; b < B; ++b) {
     const float v = wave_dot<T>(w, (const T*)P.lat + (long long)b * P.ld_lat + h * P.C, P.C, lane, vec != 0);
-    if (lane == 0)
-      st((T*)P.out + (long long)b * P.ld_out + item, v * sigmoidf(P.proj[(long long)b * P.ld + P.off_g + (P.gate_heads ? h : item)]));
+    if (lane == 0) {
+      const float f = P.gate_heads == 2 ? 1.f : sigmoidf(P.proj[(long long)b * P.ld + P.off_g + (P.gate_heads ? h : item)]);
+      st((T*)P.out + (long long)b * P.ld_out + item, v * f);
+    }
   }
 }
 bool latent_supported(int D, int R, int C, int Dv) {
@@ -432,6 +434,24 @@ __global__ __launch_bounds__(256) void conv_window_kernel(ConvParams P, StepRows
       win[(long long)sidx * P.ch + c] = back < n ? P.proj[(long long)(r - back) * P.ld + P.off_in + c]
                                                  : win[(long long)(sidx + n) * P.ch + c];
     }
+}
+// a block per (row, 256 channels); the last taps - 1 rows of every sequence have something to leave behind
+__global__ __launch_bounds__(256) void conv_ring_kernel(const float* __restrict__ proj, int ld, int ch, int taps,
+                                                        const float* __restrict__ bias, float* __restrict__ window, long long stride,
+                                                        int ring, StepRows R) {
+  const int r = blockIdx.x, seq = R.q_seq[r];
+  if (r + taps - 1 < R.B && R.q_seq[r + taps - 1] == seq) return;  // (a sequence's rows are neighbours)
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c < ch)
+    window[(long long)seq * stride + (long long)(R.pos[r] % ring) * ch + c] = proj[(long long)r * ld + c] + (bias ? bias[c] : 0.f);
+}
+void conv_ring_window(const float* proj, int ld, int ch, int taps, const float* bias, float* window, long long stride, int ring,
+                      const StepRows& R, hipStream_t s) {
+  if (taps <= 1) return;
+  check(R.B > 0 && proj && window && ch > 0 && ring >= taps - 1 && R.pos && R.q_seq && stride >= (long long)ring * ch,
+        "conv_ring_window: bad operands");
+  hipLaunchKernelGGL(conv_ring_kernel, dim3(R.B, (ch + 255) / 256), dim3(256), 0, s, proj, ld, ch, taps, bias, window, stride, ring, R);
+  launched("conv_ring_window");
 }
 void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s) {
   check(R.B > 0 && P.proj && P.w && P.out && P.ch > 0 && P.taps >= 1 && (P.taps == 1 || P.state),

@@ -146,20 +146,20 @@ void retention_chunked(const RetParams& P, const StepRows& R, const RetChunkWs& 
 int retention_chunk_rows();
 bool retention_chunk_supported(int D, int Dv);
 
-enum { MOE_ACT_SILU = 0, MOE_ACT_CLAMPED = 1 };
+enum { MOE_ACT_SILU = 0, MOE_ACT_CLAMPED = 1, MOE_ACT_GELU_UP = 2 };
 struct MoeParams {
   const float* proj;    // [B][ld]: router logits at off_router, shared: scalar gate, gate rows, up rows
   int ld, off_router, off_sg, off_sgate, off_sup;
   int B, E, X, top, F, Fs;
   const float* router_b;
   const void* h;        // [B][E] matrix dtype (the normed activations)
-  const void* w_gu;     // [X][2F][E]
+  const void* w_gu;     // [X][2F][E] (MOE_ACT_GELU_UP: [X][F][E])
   const void* w_down;   // [X][E][F]
   const void* sh_down;  // [E][Fs]
   int* eids;            // [B][ld_top]
   float* ew;
   int ld_top;
-  float* sgate;         // [B]
+  float* sgate;         // [B], or null: the shared expert has no gate
   void* hmid;           // [B][ld_hmid] matrix dtype: top x F expert activations, then Fs shared
   int ld_hmid;
   float* y;             // [B][E] float32 feed-forward output
@@ -172,8 +172,9 @@ struct MoeParams {
   float route_scale;    // sigmoid router (moe_route_sigmoid): factor on the normalised weights
   int route_raw;        // sigmoid router: the chosen scores are the weights as they are (not divided by their sum)
   int act;              // routed experts: MOE_ACT_SILU silu(gate) up; MOE_ACT_CLAMPED g sigmoid(1.702 g) (u + 1) with
-  float limit;          // g = min(gate, limit), u = clamp(up, -limit, limit)
+  float limit;          // g = min(gate, limit), u = clamp(up, -limit, limit); MOE_ACT_GELU_UP gelu(up), no gate
   int w_input;          // a chosen expert's weight multiplies its input (its gate / up products) instead of its output
+  int route_softmax;    // sigmoid router: the scores are a softmax over all experts
 };
 void moe_route(const MoeParams& P, hipStream_t s);   // top-k ids + softmax weights, shared gate and activation
 // softmax over all router outputs, choice by score + correction inside the best expert groups, weights = the
@@ -234,7 +235,8 @@ struct LatentParams {
   void* out;            // [B][ld_out] matrix dtype: (W_uv_h lat_h) * sigmoid(g), head-major
   int ld_out;
   int f32;
-  int gate_heads;       // 1: the gate is one number per head ([H] at off_g) instead of one per output element
+  int gate_heads;       // 1: the gate is one number per head ([H] at off_g) instead of one per output element; 2: no gate
+  float rot_amp = 1.f;  // factor on sine and cosine
 };
 void latent_prepare(const LatentParams& P, const StepRows& R, hipStream_t s);
 void latent_expand(const LatentParams& P, int B, hipStream_t s);
@@ -254,6 +256,12 @@ struct ConvParams {
 void conv_silu(const ConvParams& P, const StepRows& R, hipStream_t s);
 // only the windows of sequences with several rows in the step (after a kernel that convolves by itself)
 void conv_window(const ConvParams& P, const StepRows& R, hipStream_t s);
+// carried inputs as a ring: the input of position p (+ bias, if any) sits in row p % ring of a slot's [ring][ch]. A kernel that
+// convolves by itself writes the inputs of a step of at most CONV_RING_ROWS rows, which the ring (taps - 1 + CONV_RING_ROWS
+// rows) keeps apart from those still to be read; after larger steps this writes each sequence's last taps - 1 inputs.
+constexpr int CONV_RING_ROWS = 8;
+void conv_ring_window(const float* proj, int ld, int ch, int taps, const float* bias, float* window, long long stride, int ring,
+                      const StepRows& R, hipStream_t s);
 
 enum { SCAN_MLSTM = 0, SCAN_SSD = 1, SCAN_FIXED = 2 };
 struct ScanParams {
@@ -333,15 +341,16 @@ void scalar_norm_conv(const CanonParams& P, const StepRows& R, hipStream_t s);
 // product C = out . W^T; out is also written
 bool gemv_canon_supported(int taps);
 void gemv_canon(const CanonParams& P, const void* W, int M, int N, float* C, int ldc, const StepRows& R, hipStream_t s);
-// decode steps: group_rms_cast and the output projection added to the residual stream, C += (normed, gated y) . W^T
+// decode steps: group_rms_cast and the product with its result in one launch, C = (normed, gated y) . W^T, or with `add`
+// (an output projection added to the residual stream) C +=
 void gemv_group_rms(const float* y, int ld_y, int n, int groups, const float* w, float eps, const float* gate, int ld_gate,
-                    const void* W, int M, int N, float* C, int ldc, int f32, hipStream_t s);
+                    const void* W, int M, int N, float* C, int ldc, int add, int f32, hipStream_t s);
 bool gemv_group_rms_supported(int M, int n, int groups, int f32);
 // out[r] = x[idx ? idx[r] : r] / rms * g[0], matrix dtype
 void scalar_norm_cast(const float* x, const int* idx, int rows, int E, const float* g, float eps, void* out, int f32,
                       hipStream_t s);
 
-enum { QK_NORM_NONE = 0, QK_NORM_WEIGHT_FIRST = 1, QK_NORM_UNIT_LAST = 2 };
+enum { QK_NORM_NONE = 0, QK_NORM_WEIGHT_FIRST = 1, QK_NORM_UNIT_LAST = 2, QK_NORM_WHOLE_FIRST = 3 };
 struct QkPrepParams {
   float* proj;          // [B][ld] float32: q at off_q (finished in place), k at off_k, v at off_v
   int ld, off_q, off_k, off_v;
@@ -441,13 +450,15 @@ struct RotFoldParams {
 };
 void rotate_fold(const RotFoldParams& P, const StepRows& R, hipStream_t s);
 bool rotate_fold_supported(int H, int G, int D);
-// out = relu(z[:, :F]) * z[:, F:2F], matrix dtype
-void relu_glu_cast(const float* z, int ld, int rows, int F, void* out, int ld_out, int f32, hipStream_t s);
-// out[m][k] = relu(A[m] . W[k]) * (A[m] . W[F + k]), matrix dtype: gate / up projection of a few rows (M <= 16) + activation
-void gemv_relu_glu(const void* A, int lda, const void* W, int K, int F, int M, void* out, int ld_out, int f32, hipStream_t s);
-// sigmoid scores; a group of neighbours ranks by the sum of its two largest scores, only the best group_keep groups
-// stay; the `top` largest scores, divided by their sum, times route_scale -> eids / ew, as moe_route leaves them, so
-// moe_experts, moe_down and moe_grouped follow unchanged (no shared expert, no router bias)
+enum { GLU_RELU = 0, GLU_SILU = 1 };
+// out = act(z[:, :F]) * z[:, F:2F], matrix dtype
+void act_glu_cast(int act, const float* z, int ld, int rows, int F, void* out, int ld_out, int f32, hipStream_t s);
+// out[m][k] = act(A[m] . W[k]) * (A[m] . W[F + k]), matrix dtype: gate / up projection of a few rows (M <= 16) + activation
+void gemv_act_glu(int act, const void* A, int lda, const void* W, int K, int F, int M, void* out, int ld_out, int f32, hipStream_t s);
+// sigmoid (route_softmax: softmax) scores; a group of neighbours ranks by the sum of its two largest scores, only the best
+// group_keep groups stay; the `top` largest scores, divided by their sum, times route_scale -> eids / ew, as moe_route
+// leaves them, so moe_experts, moe_down and moe_grouped follow unchanged (no router bias); with Fs the shared expert's
+// activation gelu(up) is written behind the routed ones (up rows at off_sup; MOE_ACT_GELU_UP only)
 void moe_route_sigmoid(const MoeParams& P, hipStream_t s);
 // a few rows (decode steps): the same routing and the routed activations (moe_experts' work) in one launch
 void moe_route_sigmoid_experts(const MoeParams& P, hipStream_t s);
@@ -465,7 +476,33 @@ struct KvStoreParams {
 };
 void kv_store(const KvStoreParams& P, const StepRows& R, hipStream_t s);
 
-// ---- gated delta rule with a decay per key channel (stack_delta.hip)
+// ---- attention whose q, k and v carry biases and pass a short convolution each, q and k then RMS-normed over all their
+// heads at once and rotated in halves (stack_qkv.hip): the finished queries, the keys and values in the row's cache slot
+struct QkvConvParams {
+  const float* proj;    // [B][ld] float32: q [H * D] | k [G * D] | v [G * Dv], side by side
+  int ld;
+  const float* bias;    // [n] like those columns, or null
+  int H, G, D, Dv, taps;
+  const float* w;       // [n][taps], the last tap is the current token's
+  float* window;        // slot s: window + s * stride = [ring][n] (taps > 1), see conv_ring_window
+  long long stride;
+  int ring;
+  const float* q_norm;  // [H * D]
+  const float* k_norm;  // [G * D]
+  float eps;
+  int rot_dims;         // pairs (i, i + rot_dims / 2) of every head turn by pos * inv_freq[i]
+  const double* inv_freq;
+  float rot_amp;        // factor on sine and cosine
+  float* q;             // [B][ld_q] float32
+  int ld_q;
+  void* kc;             // [blocks][G][bs][D]
+  void* vc;             // [blocks][G][bs][Dv]
+  int f32;
+};
+void qkv_conv_prepare(const QkvConvParams& P, const StepRows& R, hipStream_t s);
+bool qkv_conv_supported(int H, int G, int D, int Dv);
+
+// ---- gated delta rule with a decay per key channel, or one per head (stack_delta.hip)
 struct DeltaParams {
   const float* proj;    // [B][ld] float32: q [G][D] | k [G][D] | v [H][Dv] (the convolution's inputs) at off_q, write
   int ld, off_q, off_b, off_a1, off_g1;  // strengths [H] at off_b, first factors of the low-rank maps at off_a1, off_g1
@@ -493,21 +530,27 @@ struct DeltaParams {
   float out_scale;
   int f32;
   KvStoreParams kv;     // kc non-null: delta_prepare also stores the keys and values of the attention beside it
+  // head_decay: one decay per head, softplus(z + dt_bias) with z [H] at off_a1 and dt_bias [H] (no low-rank maps: rank_a,
+  // rank_g, a2, g2 and gate unused); lg holds [H] per row; the output gate is silu of the columns [H * Dv] at off_g1
+  int head_decay;
+  int ring;             // > 0: the window is a ring of `ring` rows (conv_ring_window), else oldest first
 };
 // convolution (its windows advanced), unit vectors, log decays and gates of the step's rows into the scratch rows
 void delta_prepare(const DeltaParams& P, const StepRows& R, hipStream_t s);
 void delta_walk(const DeltaParams& P, const StepRows& R, hipStream_t s);  // after delta_prepare: token by token
 bool delta_supported(int D, int Dv, int rank_a, int rank_g);
+bool delta_head_supported(int D, int Dv);  // with head_decay
 // after delta_prepare: in chunks (prompt portions) over the host-built chunk table of the chunked retention
 struct DeltaChunkWs {
   const int* chunks;
   int nchunks, max_chunks;
   float* Sin;           // [chunks][s_stride]: every chunk's incoming state
   long long s_stride;
-  float* W;             // [B][ld_lg]
-  float* Kd;            // [B][ld_lg]
+  float* W;             // [B][ld_w] (at least H * D)
+  float* Kd;            // [B][ld_w]
   float* u;             // [B][ld_gate]
   float* Bm;            // [B][H][delta_chunk_rows()]
+  int ld_w;
 };
 void delta_chunked(const DeltaParams& P, const StepRows& R, const DeltaChunkWs& W, hipStream_t s);
 int delta_chunk_rows();

@@ -1,7 +1,7 @@
 // Kernels of layers with RMS norms (weight vectors) on the inputs of both sublayers: the norm itself, the
 // finishing of differential attention (two softmax maps per head over the same values), the preparation of
 // attention whose scores are mixed across the heads before the softmax (rotation + the queries folded through
-// the mixing matrix), a gated dense feed-forward with a relu gate, and a sigmoid router with ranked groups.
+// the mixing matrix), a gated dense feed-forward with a relu or silu gate, and a sigmoid or softmax router with ranked groups.
 // float32 for norms, angles, gates and router; `T` is the matrix dtype (bfloat16 or float32).
 #include "stack_device.h"
 #include "stack_kv.h"
@@ -167,31 +167,32 @@ void kv_store(const KvStoreParams& P, const StepRows& R, hipStream_t s) {
 }
 
 // ------------------------------------------------------------------------------------------------ gated dense feed-forward
-// out = relu(z[:, :F]) * z[:, F:2F], matrix dtype
+__device__ __forceinline__ float glu_act(int act, float g) { return act == GLU_SILU ? silu(g) : fmaxf(g, 0.f); }
+// out = act(z[:, :F]) * z[:, F:2F], matrix dtype
 template <typename T>
-__global__ __launch_bounds__(256) void relu_glu_kernel(const float* __restrict__ z, int ld, int rows, int F, T* __restrict__ out,
+__global__ __launch_bounds__(256) void act_glu_kernel(int act, const float* __restrict__ z, int ld, int rows, int F, T* __restrict__ out,
                                                        int ld_out) {
   const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
   if (i >= (long long)rows * F) return;
   const long long r = i / F;
   const int f = (int)(i % F);
-  st(out + r * ld_out + f, fmaxf(z[r * ld + f], 0.f) * z[r * ld + F + f]);
+  st(out + r * ld_out + f, glu_act(act, z[r * ld + f]) * z[r * ld + F + f]);
 }
-void relu_glu_cast(const float* z, int ld, int rows, int F, void* out, int ld_out, int f32, hipStream_t s) {
-  check(rows > 0 && F > 0 && z && out && ld >= 2 * F && ld_out >= F, "relu_glu_cast: bad operands");
+void act_glu_cast(int act, const float* z, int ld, int rows, int F, void* out, int ld_out, int f32, hipStream_t s) {
+  check(rows > 0 && F > 0 && z && out && ld >= 2 * F && ld_out >= F, "act_glu_cast: bad operands");
   const long long n = (long long)rows * F;
   const dim3 grid((unsigned)((n + 255) / 256));
   if (f32)
-    hipLaunchKernelGGL(relu_glu_kernel<float>, grid, dim3(256), 0, s, z, ld, rows, F, (float*)out, ld_out);
+    hipLaunchKernelGGL(act_glu_kernel<float>, grid, dim3(256), 0, s, act, z, ld, rows, F, (float*)out, ld_out);
   else
-    hipLaunchKernelGGL(relu_glu_kernel<bf16>, grid, dim3(256), 0, s, z, ld, rows, F, (bf16*)out, ld_out);
-  launched("relu_glu_cast");
+    hipLaunchKernelGGL(act_glu_kernel<bf16>, grid, dim3(256), 0, s, act, z, ld, rows, F, (bf16*)out, ld_out);
+  launched("act_glu_cast");
 }
-// out[m][k] = relu(A[m] . W[k]) * (A[m] . W[F + k]), matrix dtype: the gate / up projection of a few rows with its
+// out[m][k] = act(A[m] . W[k]) * (A[m] . W[F + k]), matrix dtype: the gate / up projection of a few rows with its
 // activation in one launch (W [2F][K]: gate rows, then up rows); one wave per hidden unit takes both rows
 template <typename T>
-__global__ __launch_bounds__(256) void gemv_relu_glu_kernel(const T* __restrict__ A, int lda, const T* __restrict__ W, int K, int F,
-                                                            int M, T* __restrict__ out, int ld_out, int vec) {
+__global__ __launch_bounds__(256) void gemv_act_glu_kernel(int act, const T* __restrict__ A, int lda, const T* __restrict__ W, int K,
+                                                           int F, int M, T* __restrict__ out, int ld_out, int vec) {
   const int lane = threadIdx.x & 63;
   const int f = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (f >= F) return;
@@ -200,30 +201,36 @@ __global__ __launch_bounds__(256) void gemv_relu_glu_kernel(const T* __restrict_
   for (int m = 0; m < M; ++m) {
     const T* x = A + (long long)m * lda;
     const float g = wave_dot<T>(wg, x, K, lane, vec != 0), u = wave_dot<T>(wu, x, K, lane, vec != 0);
-    if (lane == 0) st(out + (long long)m * ld_out + f, fmaxf(g, 0.f) * u);
+    if (lane == 0) st(out + (long long)m * ld_out + f, glu_act(act, g) * u);
   }
 }
-void gemv_relu_glu(const void* A, int lda, const void* W, int K, int F, int M, void* out, int ld_out, int f32, hipStream_t s) {
-  check(M > 0 && M <= 16 && A && W && out && K > 0 && F > 0 && ld_out >= F, "gemv_relu_glu: bad operands (up to 16 rows)");
+void gemv_act_glu(int act, const void* A, int lda, const void* W, int K, int F, int M, void* out, int ld_out, int f32, hipStream_t s) {
+  check(M > 0 && M <= 16 && A && W && out && K > 0 && F > 0 && ld_out >= F, "gemv_act_glu: bad operands (up to 16 rows)");
   const dim3 grid((F + 3) / 4);
   if (f32)
-    hipLaunchKernelGGL(gemv_relu_glu_kernel<float>, grid, dim3(256), 0, s, (const float*)A, lda, (const float*)W, K, F, M, (float*)out,
+    hipLaunchKernelGGL(gemv_act_glu_kernel<float>, grid, dim3(256), 0, s, act, (const float*)A, lda, (const float*)W, K, F, M, (float*)out,
                        ld_out, (int)(vec_ok<float>(A, lda, K) && vec_ok<float>(W, K, K)));
   else
-    hipLaunchKernelGGL(gemv_relu_glu_kernel<bf16>, grid, dim3(256), 0, s, (const bf16*)A, lda, (const bf16*)W, K, F, M, (bf16*)out,
+    hipLaunchKernelGGL(gemv_act_glu_kernel<bf16>, grid, dim3(256), 0, s, act, (const bf16*)A, lda, (const bf16*)W, K, F, M, (bf16*)out,
                        ld_out, (int)(vec_ok<bf16>(A, lda, K) && vec_ok<bf16>(W, K, K)));
-  launched("gemv_relu_glu");
+  launched("gemv_act_glu");
 }
 
 // ------------------------------------------------------------------------------------------------ sigmoid router
-// Per row: s = sigmoid of the X router logits. The experts form group_count groups of neighbours; a group ranks by
-// the sum of its two largest scores and only experts of the best group_keep groups can be chosen; the `top` largest
-// scores among them are taken (ties: the lower index), divided by their sum (+ 1e-20; route_raw: left as they are) and
-// multiplied by route_scale.
+// Per row: s = sigmoid of the X router logits, or their softmax (route_softmax). The experts form group_count groups of
+// neighbours; a group ranks by the sum of its two largest scores and only experts of the best group_keep groups can be
+// chosen; the `top` largest scores among them are taken (ties: the lower index), divided by their sum (+ 1e-20; route_raw:
+// left as they are) and multiplied by route_scale.
 // One wave per row with an expert per lane (X <= 64); lane q < top ends up holding the q-th choice.
 __device__ __forceinline__ void route_sigmoid_wave(const MoeParams& P, const float* row, int lane, int& who_q, float& w_q) {
   const bool has = lane < P.X;
-  const float sc = has ? sigmoidf(row[P.off_router + lane]) : -INFINITY;
+  float sc = has ? row[P.off_router + lane] : -INFINITY;
+  if (P.route_softmax) {
+    const float ex = expf(sc - wave_max(sc)), sum = wave_sum(ex);  // (a lane without an expert: exp(-inf) = 0)
+    sc = has ? ex / sum : -INFINITY;
+  } else {
+    sc = has ? sigmoidf(sc) : -INFINITY;
+  }
   float ch = sc;
   if (P.group_count > 1) {
     const int per = P.X / P.group_count, mine = has ? lane / per : -1;
@@ -269,7 +276,14 @@ __device__ __forceinline__ void route_sigmoid_wave(const MoeParams& P, const flo
 }
 // the same by one thread, for up to 256 experts (sc: X floats of scratch)
 __device__ void route_sigmoid_serial(const MoeParams& P, const float* row, float* sc, int* ids, float* wts) {
-  for (int e = 0; e < P.X; ++e) sc[e] = sigmoidf(row[P.off_router + e]);
+  if (P.route_softmax) {
+    float mx = -INFINITY, total = 0.f;
+    for (int e = 0; e < P.X; ++e) mx = fmaxf(mx, row[P.off_router + e]);
+    for (int e = 0; e < P.X; ++e) total += sc[e] = expf(row[P.off_router + e] - mx);
+    for (int e = 0; e < P.X; ++e) sc[e] /= total;
+  } else {
+    for (int e = 0; e < P.X; ++e) sc[e] = sigmoidf(row[P.off_router + e]);
+  }
   if (P.group_count > 1) {
     const int per = P.X / P.group_count;
     unsigned long long kept = 0ull;
@@ -317,6 +331,7 @@ __device__ void route_sigmoid_serial(const MoeParams& P, const float* row, float
   for (int jj = 0; jj < P.top; ++jj) wts[jj] = (P.route_raw ? wts[jj] : wts[jj] / sum) * P.route_scale;
 }
 constexpr int ROUTE_SIG_MAX = 256;
+template <typename T>
 __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
   __shared__ float sc[4][ROUTE_SIG_MAX];
   __shared__ int ids[4][MOE_MAX_TOP];
@@ -325,6 +340,8 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
   const int b = blockIdx.x * 4 + wv;
   if (b >= P.B) return;
   const float* row = P.proj + (long long)b * P.ld;
+  T* hs = (T*)P.hmid + (long long)b * P.ld_hmid + P.top * P.F;  // the shared expert's activation
+  for (int f = lane; f < P.Fs; f += 64) st(hs + f, gelu_erf(row[P.off_sup + f]));
   if (P.X <= 64) {
     int who;
     float w;
@@ -344,23 +361,32 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
 static void check_route_sigmoid(const MoeParams& P) {
   check(P.B > 0 && P.proj && P.eids && P.ew && P.X > 0 && P.X <= ROUTE_SIG_MAX && P.top > 0 && P.top <= MOE_MAX_TOP && P.top <= P.X &&
             P.ld_top >= P.top && P.group_count >= 1 && P.group_count <= 64 && P.X % P.group_count == 0 && P.group_keep >= 1 &&
-            P.group_keep <= P.group_count && P.group_keep * (P.X / P.group_count) >= P.top && P.Fs == 0 && P.identity == 0,
+            P.group_keep <= P.group_count && P.group_keep * (P.X / P.group_count) >= P.top && P.identity == 0 &&
+            (P.Fs == 0 || (P.act == MOE_ACT_GELU_UP && P.hmid && P.ld_hmid >= P.top * P.F + P.Fs)),
         "sigmoid router: operands or sizes (up to 256 experts in up to 64 groups, top <= 16)");
 }
 void moe_route_sigmoid(const MoeParams& P, hipStream_t s) {
   check_route_sigmoid(P);
-  hipLaunchKernelGGL(moe_route_sigmoid_kernel, dim3((P.B + 3) / 4), dim3(256), 0, s, P);
+  if (P.f32)
+    hipLaunchKernelGGL(moe_route_sigmoid_kernel<float>, dim3((P.B + 3) / 4), dim3(256), 0, s, P);
+  else
+    hipLaunchKernelGGL(moe_route_sigmoid_kernel<bf16>, dim3((P.B + 3) / 4), dim3(256), 0, s, P);
   launched("moe_route_sigmoid");
 }
-// ---- a few rows (decode steps): routing and the routed activations in one launch. Grid (ff units / 4, row x top);
-// every wave routes its row itself (a few dozen operations) and takes hidden unit f of routed expert jj; block
-// (0, row, 0) records ids and weights for the down projection.
+// ---- a few rows (decode steps): routing and the routed (and shared) activations in one launch. Grid (ff units / 4, row x
+// (top, and one more with a shared expert)); every wave routes its row itself (a few dozen operations) and takes hidden unit
+// f of routed expert jj; block (0, row, 0) records ids and weights for the down projection.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_sigmoid_experts_kernel(MoeParams P, int vec) {
   const int lane = threadIdx.x & 63;
   const int f = blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int b = blockIdx.y / P.top, jj = blockIdx.y % P.top;
+  const int places = P.top + (P.Fs > 0 ? 1 : 0), b = blockIdx.y / places, jj = blockIdx.y % places;
   const float* row = P.proj + (long long)b * P.ld;
+  if (jj == P.top) {  // shared expert: a unit per thread
+    const int fs = blockIdx.x * 256 + threadIdx.x;
+    if (fs < P.Fs) st((T*)P.hmid + (long long)b * P.ld_hmid + P.top * P.F + fs, gelu_erf(row[P.off_sup + fs]));
+    return;
+  }
   int who;
   float w;
   route_sigmoid_wave(P, row, lane, who, w);
@@ -371,19 +397,15 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_experts_kernel(MoeParam
   const int e = __shfl(who, jj, 64);
   const float w_in = P.w_input ? __shfl(w, jj, 64) : 1.f;
   if (f >= P.F) return;
-  const T* x = (const T*)P.h + (long long)b * P.E;
-  const T* wg = (const T*)P.w_gu + ((long long)e * 2 * P.F + f) * P.E;
-  const T* wu = wg + (long long)P.F * P.E;
-  const float gate = wave_dot<T>(wg, x, P.E, lane, vec != 0);
-  const float up = wave_dot<T>(wu, x, P.E, lane, vec != 0);
-  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, moe_unit(P.act, P.limit, w_in, gate, up));
+  const float u = moe_hidden<T>(P, e, f, (const T*)P.h + (long long)b * P.E, w_in, lane, vec != 0);
+  if (lane == 0) st((T*)P.hmid + (long long)b * P.ld_hmid + jj * P.F + f, u);
 }
 bool moe_route_sigmoid_fused_supported(const MoeParams& P) { return P.X <= 64; }
 void moe_route_sigmoid_experts(const MoeParams& P, hipStream_t s) {
   check_route_sigmoid(P);
   check(moe_route_sigmoid_fused_supported(P) && P.h && P.w_gu && P.hmid && P.F > 0 && P.ld_hmid >= P.top * P.F,
         "fused sigmoid router: operands or sizes (up to 64 experts)");
-  const dim3 grid((P.F + 3) / 4, P.B * P.top);
+  const dim3 grid(std::max((P.F + 3) / 4, (P.Fs + 255) / 256), P.B * (P.top + (P.Fs > 0 ? 1 : 0)));
   if (P.f32)
     hipLaunchKernelGGL(moe_route_sigmoid_experts_kernel<float>, grid, dim3(256), 0, s, P,
                        (int)(vec_ok<float>(P.h, P.E, P.E) && vec_ok<float>(P.w_gu, P.E, P.E)));

@@ -26,8 +26,9 @@ import time
 
 import torch
 
-from ..models.config import (ACT_CLAMPED_GLU, BLOCK_POSTNORM, BLOCK_PRENORM, BLOCK_SANDWICH, FF_DENSE, FF_GLU, MIX_ATTENTION,
-                             MIX_DELTA, MIX_GLA, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, MIX_MLSTM, MIX_RETENTION)
+from ..models.config import (ACT_CLAMPED_GLU, ACT_GELU_UP, ACT_SILU, BLOCK_POSTNORM, BLOCK_PRENORM, BLOCK_SANDWICH, FF_DENSE,
+                             FF_GLU, MIX_ATTENTION, MIX_DELTA, MIX_GLA, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, MIX_MLSTM, MIX_RETENTION,
+                             QK_NORM_WHOLE_FIRST, ROUTE_SOFTMAX_SCORES)
 from .runner import Runner
 from .weights import StackWeights
 
@@ -93,7 +94,8 @@ class StackExec:
                              split_ws=p(r.split_ws), split_ws_floats=r.split_ws.numel(),
                              ret_chunks=p(r.d_chunks), ret_max_chunks=r.d_chunks.shape[0], ret_u=p(r.ret_u),
                              ret_sin=p(r.ret_sin), ret_u_stride=r.ret_u.shape[1], cbuf=p(r.cbuf), ld_cbuf=r.cbuf.shape[1],
-                             lat=p(r.latbuf), ld_lat=r.latbuf.shape[1], idw=p(r.idw), coef=p(r.scan_coef),
+                             lat=p(r.latbuf), ld_lat=r.latbuf.shape[1], qlat=p(r.qlat), ld_qlat=r.qlat.shape[1],
+                             idw=p(r.idw), coef=p(r.scan_coef),
                              ld_coef=(r.scan_coef.shape[1] if r.scan_coef is not None else 0), ctot=p(r.scan_ctot),
                              hn=p(r.hn), y2=p(r.ybuf2), rscale=p(r.rscale), **{"dl_" + k: p(v) for k, v in r.delta_ws.items()},
                              ld_dl_lg=r.delta_ws["lg"].shape[1], ld_dl_gate=r.delta_ws["gate"].shape[1],
@@ -143,6 +145,9 @@ class StackExec:
                  decay=p(L.get("decay")), mnorm=p(L.get("mnorm")), state=m.state, groups=m.groups, conv=m.conv,
                  norm_groups=m.norm_groups, conv_w=p(L.get("conv_w")), conv_b=p(L.get("conv_b")), dt_bias=p(L.get("dt_bias")),
                  a_log=p(L.get("a_log")), d_skip=p(L.get("d_skip")), left_scale=m.left_scale, right_scale=m.right_scale,
+                 rot_amp=L["rot_amp"], in_b=p(L.get("in_b")), qk_norm=int(m.qk_norm), q_norm=p(L.get("q_norm")),
+                 k_norm=p(L.get("k_norm")), q_rank=m.q_rank, dq_norm=p(L.get("dq_norm")), w_uq=p(L.get("w_uq")), gnorm=p(L.get("gnorm")),
+                 conv_ring=m.conv_rows if m.conv_ring else 0,
                  **{"off_" + k: v for k, v in L["off"].items()})
         if m.right is not None:
             g = m.right
@@ -153,11 +158,13 @@ class StackExec:
         if f is not None:
             d.update(norm2_w=p(L["norm2_w"]), w_ff=p(L["w_ff"]), n_ff=L["n_ff"], ff=f.ff)
             if f.kind == FF_GLU:
-                d.update(ff_dense=3, w_dense_down=p(L["w_dense_down"]))
+                d.update(ff_dense=4 if f.act == ACT_SILU else 3, w_dense_down=p(L["w_dense_down"]))
             else:
                 d.update(experts=f.experts, top=f.top, w_gu=p(L["w_gu"]), w_down=p(L["w_down"]), group_count=f.group_count,
                          group_keep=f.group_keep, route_scale=f.route_scale, route_raw=int(not f.route_norm),
-                         expert_act=int(f.expert_act == ACT_CLAMPED_GLU), limit=f.limit, scale_input=int(f.scale_input))
+                         expert_act={ACT_CLAMPED_GLU: 1, ACT_GELU_UP: 2}.get(f.expert_act, 0), limit=f.limit,
+                         scale_input=int(f.scale_input), route_softmax=int(f.route == ROUTE_SOFTMAX_SCORES),
+                         shared_ff=f.shared_ff, sh_down=p(L.get("sh_down")))
         return d
 
     def bind_chunks(self, rows) -> None:
@@ -230,18 +237,20 @@ class StackRunner(Runner):
         self.kc, self.vc, self.states = [], [], []
         for li, _ps, _first in self.runs:
             m = cfg.layers[li].mixer
-            if cfg.block == BLOCK_SANDWICH or cfg.canon_both:  # K/V pools of attention, and one state row per slot: [the mixers'
-                attn = m.kind == MIX_ATTENTION                 # state | input windows]
-                self.kc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.dim, **tt) if attn else None)
-                self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt) if attn else None)
+            if cfg.block in (BLOCK_SANDWICH, BLOCK_PRENORM):  # pools of the softmax mixers, and one state row per slot: [the
+                kv = m.kind == MIX_ATTENTION                  # mixers' state | input windows]
+                if kv and m.score_talk:      # one K row per token: every key/value head's key side by side
+                    kshape = (1, m.kv_heads * m.dim)
+                elif kv:                     # (with two maps per head a K row holds [map 1 | map 2])
+                    kshape = (m.kv_heads, m.dim * m.maps)
+                else:                        # latent attention: one row per token, latent | shared rotated key part
+                    kshape = (1, m.cache_dim)
+                self.kc.append(torch.zeros(n_blocks, kshape[0], block_size, kshape[1], **tt) if kv or m.kind == MIX_LATENT else None)
+                self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt) if kv else None)
                 ns = cfg.run_state_floats(li)
                 self.states.append(torch.zeros(max_seqs, ns, **f32) if ns else None)
-            elif m.kind == MIX_ATTENTION and m.score_talk:  # one K row per token: every key/value head's key side by side
-                self.kc.append(torch.zeros(n_blocks, 1, block_size, m.kv_heads * m.dim, **tt))
-                self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt))
-                self.states.append(None)
-            elif m.kind == MIX_ATTENTION:                   # (with two maps per head a K row holds [map 1 | map 2])
-                self.kc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.dim * m.maps, **tt))
+            elif m.kind == MIX_ATTENTION:
+                self.kc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.dim, **tt))
                 self.vc.append(torch.zeros(n_blocks, m.kv_heads, block_size, m.vdim, **tt))
                 self.states.append(None)
             elif m.kind == MIX_LATENT:  # one row per token: latent | shared rotated key part (the latent is the value too)
@@ -262,23 +271,26 @@ class StackRunner(Runner):
         self.x0 = torch.zeros(max_batch, E, **f32)          # the embedding output (re-enters at every pass)
         self.hbuf = torch.zeros(max_batch, E, **tt)         # normed activations, the input projection's operand
         self.catbuf = torch.zeros(max_batch, 2 * E, **tt)   # [x; x0], the pass-opening projection's operand
-        n_proj = max(max(L["n_in"], L.get("n_ff", 0)) for L in self.w.layers)
+        n_proj = max(max(L["n_in"], L.get("n_ff", 0), L.get("n_proj", 0)) for L in self.w.layers)
         self.proj = torch.zeros(max_batch, (n_proj + 3) // 4 * 4, **f32)  # rows 16-byte aligned
         self.abuf = torch.zeros(max_batch, (max(s.mixer.n_out_all for s in cfg.layers) + 7) // 8 * 8, **tt)
         self.hmid = torch.zeros(max_batch, (max([f.ff if f.kind in (FF_DENSE, FF_GLU) else f.top * f.ff + f.shared_ff for f in mlps],
                                                 default=1) + 7) // 8 * 8, **tt)
+        # the normed latent that queries come from (matrix dtype)
+        self.qlat = torch.zeros(max_batch, (max([s.mixer.q_rank for s in cfg.layers] + [1]) + 7) // 8 * 8, **tt)
         # latent attention: queries folded onto the latent (float32), outputs in latent space (matrix dtype);
         # Mamba-2: the convolution's output (float32). idw: per-row weight of the chosen identity experts
         lat = [s.mixer for s in cfg.layers if s.mixer.kind == MIX_LATENT]
         mam = [s.mixer for s in cfg.layers if s.mixer.kind == MIX_MAMBA2]
         talk = [s.mixer for s in cfg.layers if s.mixer.talk]  # every query head against every key/value head's values
         fold = [s.mixer for s in cfg.layers if s.mixer.score_talk]  # queries folded through the score-mixing matrix
-        deltas = [s.mixer.right for s in cfg.layers if s.mixer.right is not None and s.mixer.right.kind == MIX_DELTA]
+        deltas = [x for s in cfg.layers for x in (s.mixer, s.mixer.right) if x is not None and x.kind == MIX_DELTA]
+        convs = [s.mixer for s in cfg.layers if s.mixer.kind == MIX_ATTENTION and s.mixer.qk_norm == QK_NORM_WHOLE_FIRST]
         maps = [s.mixer for s in cfg.layers if s.mixer.maps > 1]    # the maps' outputs before they are combined
         self.cbuf = torch.zeros(max_batch, (max([m.heads * m.cache_dim for m in lat] + [m.conv_channels for m in mam] +
                                                 [m.heads * m.kv_heads * m.vdim for m in talk] +
                                                 [m.heads * m.kv_heads * m.dim for m in fold] +
-                                                [m.heads * m.maps * m.vdim for m in maps] +
+                                                [m.heads * m.maps * m.vdim for m in maps] + [m.n_q for m in convs] +
                                                 [m.conv_channels for m in deltas], default=1) + 3) // 4 * 4, **f32)
         sandwich = cfg.block == BLOCK_SANDWICH
         self.hn = torch.zeros(max_batch if sandwich or cfg.canon_both else 1, E, **f32)  # normed rows before the input convolution

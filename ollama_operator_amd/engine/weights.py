@@ -432,7 +432,7 @@ class StackWeights:
         mat = lambda *ts: torch.cat([t.to(torch.float32) for t in ts], 0).to(dtype).contiguous().to(device)  # noqa: E731
         vec = lambda t: t.to(torch.float32).reshape(-1).contiguous().to(device)  # noqa: E731
         self.embed = mat(get("embed", (V, E)))
-        self.loop_in = mat(get("loop.in", (E, 2 * E))) if cfg.loop_times else None
+        self.loop_in = mat(get("loop.in", (E, 2 * E))) if cfg.loop_times and cfg.loop_mix else None
         self.layers = []
         self._get, self._mat, self._vec = get, mat, vec
         for i, spec in enumerate(cfg.layers):
@@ -485,12 +485,17 @@ class StackWeights:
         if cfg.block == BLOCK_SANDWICH:   # an RMS norm with one number as its weight
             self.final_w, self.final_b = vec(get("final.norm", ())), None
         elif cfg.block == BLOCK_PRENORM:  # an RMS norm with a weight vector
-            self.final_w, self.final_b = vec(get("final.norm", (E,))), None
+            self.final_w, self.final_b = self._norm_weight("final.norm"), None
         else:
             self.final_w, self.final_b = vec(get("final.norm", (E,))), vec(get("final.norm.b", (E,)))
         # (a design without a head of its own reads the logits off the embedding table)
         self.head = self.embed if cfg.tied_head else mat(get("head", (V, E)))
         self.local = dict(E=E, V=V)
+
+    def _norm_weight(self, name: str) -> torch.Tensor:
+        """Weight vector of a layer's RMS norm; a design that stores its distance from one gets it added here."""
+        w = self._vec(self._get(name, (self.cfg.n_embd,)))
+        return w + 1.0 if self.cfg.norm_plus_one else w
 
     def _load_postnorm_layer(self, L: dict, p: str, spec) -> None:
         """A layer whose sublayers read the stream itself and whose norms sit on their outputs. The mixer's
@@ -580,6 +585,20 @@ class StackWeights:
         L["a_log"], L["dt_bias"] = vec(get(b + "A_log", (r.heads,))), vec(get(b + "dt_bias", (r.n_q,)))
         L["gnorm"] = vec(get(b + "norm", (r.vdim,)))
 
+    def _load_head_delta(self, L: dict, p: str, m) -> tuple[list, dict]:
+        """A gated delta rule with one decay per head: its tensors into L; its input matrices (q | k | v, which pass one
+        convolution and sit side by side, the write strengths, the decays' inputs, the output gate) and their columns."""
+        get, vec, E = self._get, self._vec, self.cfg.n_embd
+        rows = dict(q=m.kv_heads * m.dim, k=m.kv_heads * m.dim, v=m.n_out, b=m.heads, a=m.heads, g=m.n_out)
+        L["conv_w"] = vec(torch.cat([get(f"{p}mix.{k}.conv", (rows[k], m.conv)).to(torch.float32) for k in "qkv"], 0))
+        L["a_log"], L["dt_bias"] = vec(get(p + "mix.A_log", (m.heads,))), vec(get(p + "mix.dt_bias", (m.heads,)))
+        L["gnorm"] = vec(get(p + "mix.norm", (m.vdim,)))
+        off, n = {}, 0
+        for key, k in (("q", "q"), ("k", "k"), ("v", "v"), ("rb", "b"), ("a1", "a"), ("g", "g")):
+            off[key] = n
+            n += rows[k]
+        return [get(f"{p}mix.{k}", (rows[k], E)) for k in "qkvbag"], off
+
     def _load_sandwich_layer(self, st, p: str, spec) -> dict:
         """A layer with scalar-weight RMS norms around both sublayers. The matrices that read the mixer's input are
         one stack `w_in` (attention q | k | [v], then a second mixer's q | k | v | gate | first decay factor) with
@@ -645,24 +664,36 @@ class StackWeights:
 
     def _load_prenorm_layer(self, st, p: str, spec) -> dict:
         """A layer with RMS norms (weight vectors) on the inputs of both sublayers. The mixer's matrices that read its
-        normed input are one stack `w_in` (attention q | k | v | [gate]; latent attention q | dkv | gate), the
-        feed-forward's are a second stack `w_ff` (gate | up of the dense one, or the router) because it reads the
-        updated stream. Constants that are functions of the weights alone are worked out here in float32: the
-        differential attention's lambda, and the score-mixing matrix with the heads' factors folded in
-        (M[h][g] = talk[h][g] * temp[g]), the heads' distance slopes. Rotary frequencies are float64. A second mixer
-        beside the attention adds its matrices to the stack `w_in`, and its output projection sits beside the
-        attention's in `w_o` (the layer's result is one product over both mixers' outputs, whose scales are applied
-        to the outputs); the inner sizes of its low-rank maps come from the tensors' shapes."""
-        from ..models.config import FF_GLU, GATE_HEAD, GATE_NONE, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, rotary_inv_freq
+        normed input are one stack `w_in` (attention q | k | v | [gate]; latent attention q | dkv | gate, or with queries
+        from a latent of their own dq | dkv, then `w_uq` reads that latent), the feed-forward's are a second stack `w_ff`
+        (gate | up of the dense one, or router | shared up) because it reads the updated stream.
+        Constants that are functions of the weights alone are worked out here in float32: the differential attention's
+        lambda, and the score-mixing matrix with the heads' factors folded in (M[h][g] = talk[h][g] * temp[g]), the
+        heads' distance slopes. Rotary frequencies are float64. A second mixer beside the attention adds its matrices
+        to the stack `w_in`, and its output projection sits beside the attention's in `w_o` (the layer's result is one
+        product over both mixers' outputs, whose scales are applied to the outputs); the inner sizes of its low-rank
+        maps come from the tensors' shapes."""
+        from ..models.config import (ACT_GELU_UP, FF_GLU, GATE_HEAD, GATE_NONE, MIX_DELTA, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2,
+                                     QK_NORM_WHOLE_FIRST, rotary_amplitude, rotary_inv_freq)
         get, mat, vec = self._get, self._mat, self._vec
         cfg, dev = self.cfg, self.device
         E, m, f = cfg.n_embd, spec.mixer, spec.mlp
         H, G, D, Dv = m.heads, m.kv_heads, m.dim, m.vdim
-        L: dict = dict(norm_w=vec(get(p + "norm1", (E,))))
+        L: dict = dict(norm_w=self._norm_weight(p + "norm1"))
         if m.kind == MIX_LATENT:
             C, R = m.kv_rank, m.rot_dim
-            parts = [get(p + "mix.q", (H * (D + R), E)), get(p + "mix.dkv", (C + R, E)), get(p + "mix.g", (H, E))]
-            off = dict(q=0, k=H * (D + R), g=H * (D + R) + C + R)
+            if m.q_rank:  # the queries' product lands behind the stack's own columns, 16-byte aligned
+                parts = [get(p + "mix.dq", (m.q_rank, E)), get(p + "mix.dkv", (C + R, E))]
+                off = dict(dq=0, k=m.q_rank, q=(m.q_rank + C + R + 3) // 4 * 4)
+                L["dq_norm"] = vec(get(p + "mix.dq.norm", (m.q_rank,)))
+                L["w_uq"] = mat(get(p + "mix.uq", (H * (D + R), m.q_rank)))
+                L["n_proj"] = off["q"] + H * (D + R)
+            else:
+                parts = [get(p + "mix.q", (H * (D + R), E)), get(p + "mix.dkv", (C + R, E))]
+                off = dict(q=0, k=H * (D + R))
+            if m.gate == GATE_HEAD:
+                off["g"] = sum(t.shape[0] for t in parts)
+                parts.append(get(p + "mix.g", (H, E)))
             L["dkv_norm"] = vec(get(p + "mix.dkv.norm", (C,)))
             L["w_uk"] = mat(get(p + "mix.uk", (H * D, C)))
             L["w_uvT"] = mat(get(p + "mix.uv", (H * Dv, C)).view(H, Dv, C).transpose(1, 2).reshape(H * C, Dv))
@@ -670,6 +701,8 @@ class StackWeights:
             L["w_uv"] = mat(get(p + "mix.uv", (H * Dv, C)))
         elif m.kind == MIX_MAMBA2:
             parts, off = self._load_mamba2(L, p, m)
+        elif m.kind == MIX_DELTA:
+            parts, off = self._load_head_delta(L, p, m)
         elif m.kind == MIX_LINEAR:
             parts = [get(p + "mix.q", (H * D, E)), get(p + "mix.k", (H * D, E)), get(p + "mix.v", (H * Dv, E)),
                      get(p + "mix.g", (H * Dv, E))]
@@ -680,6 +713,11 @@ class StackWeights:
             a = p + ("mix.left." if m.right is not None else "mix.")
             parts = [get(a + "q", (m.n_q, E)), get(a + "k", (m.n_k, E)), get(a + "v", (m.n_v, E))]
             off = dict(q=0, k=m.n_q, v=m.n_q + m.n_k)
+            if m.bias:
+                L["in_b"] = vec(torch.cat([get(a + k + ".b", (n,)) for k, n in (("q", m.n_q), ("k", m.n_k), ("v", m.n_v))]))
+            if m.qk_norm == QK_NORM_WHOLE_FIRST:  # q, k and v pass a convolution each
+                L["conv_w"] = vec(torch.cat([get(a + k + ".conv", (n, m.conv)) for k, n in (("q", m.n_q), ("k", m.n_k), ("v", m.n_v))]))
+                L["q_norm"], L["k_norm"] = vec(get(a + "q.norm", (m.n_q,))), vec(get(a + "k.norm", (m.n_k,)))
             if m.gate != GATE_NONE:
                 parts.append(get(a + "g", (H if m.gate == GATE_HEAD else m.n_out, E)))
                 off["g"] = m.n_q + m.n_k + m.n_v
@@ -694,6 +732,7 @@ class StackWeights:
                 L["talk"] = (talk * temp[None, :]).reshape(-1).contiguous().to(dev)
         L["inv_freq64"] = (torch.tensor(rotary_inv_freq(m.rot_dims, m.rot_base, m.rot_scaling), dtype=torch.float64, device=dev)
                            if m.rot_dims else None)
+        L["rot_amp"] = rotary_amplitude(m.rot_scaling)
         if m.right is not None:
             self._load_delta(L, st, p + "mix.right.", m.right, parts, off)
             L["w_o"] = mat(torch.cat([get(p + "mix.left.o", (E, m.n_out)), get(p + "mix.right.o", (E, m.right.n_out))], 1))
@@ -705,22 +744,29 @@ class StackWeights:
             L["canon"] = vec(get(p + "canon1", (E, cfg.canon_taps)))
         if f is None:
             return L
-        L["norm2_w"] = vec(get(p + "norm2", (E,)))
+        L["norm2_w"] = self._norm_weight(p + "norm2")
         if cfg.canon_both:
             L["canon2"] = vec(get(p + "canon2", (E, cfg.canon_taps)))
         if f.kind == FF_GLU:
             L["w_ff"], L["n_ff"] = mat(get(p + "mlp.gate", (f.ff, E)), get(p + "mlp.up", (f.ff, E))), 2 * f.ff
             L["w_dense_down"] = mat(get(p + "mlp.down", (E, f.ff)))
             return L
-        X, F = f.experts, f.ff
-        L["w_ff"], L["n_ff"] = mat(get(p + "mlp.router", (X, E))), X
+        X, F, Fs = f.experts, f.ff, f.shared_ff
+        ff_parts = [get(p + "mlp.router", (X, E))]
         off["router"] = 0
+        if Fs:
+            if f.expert_act != ACT_GELU_UP:
+                raise ValueError("a pre-norm layer's shared expert has no gate")
+            ff_parts.append(get(p + "mlp.shared.up", (Fs, E)))
+            off["sup"] = X
+            L["sh_down"] = mat(get(p + "mlp.shared.down", (E, Fs)))
+        L["w_ff"], L["n_ff"] = mat(*ff_parts), X + Fs
         gu, dn = [], []
         for e in range(X):
             q = f"{p}mlp.e{e}."
-            gu += [get(q + "gate", (F, E)), get(q + "up", (F, E))]
+            gu += [get(q + k, (F, E)) for k in (("gate", "up") if f.unit_rows == 2 else ("up",))]
             dn.append(get(q + "down", (E, F)))
-        L["w_gu"] = mat(*gu).view(X, 2 * F, E)
+        L["w_gu"] = mat(*gu).view(X, f.unit_rows * F, E)
         L["w_down"] = mat(*dn).view(X, E, F)
         return L
 

@@ -252,8 +252,8 @@ MIX_MAMBA2 = 4      # selective state space layer (scalar decay per head) behind
 MIX_GLA = 5         # gated linear attention: a state matrix whose rows (key channels) decay by a per-token vector
 MIX_LINEAR = 6      # linear attention with one constant decay per head, activated queries, keys and values and one norm
                     # over all heads
-MIX_DELTA = 7       # gated delta rule: rows of the state decay by a per-token vector, a write takes off what the state
-                    # already answers to its key
+MIX_DELTA = 7       # gated delta rule: rows of the state decay by a per-token vector (or the whole state by one number per
+                    # head), a write takes off what the state already answers to its key
 STATE_MIXERS = (MIX_RETENTION, MIX_MLSTM, MIX_MAMBA2, MIX_GLA, MIX_LINEAR, MIX_DELTA)   # mixers that own a per-sequence state slot
 
 BLOCK_PARALLEL = 0  # x <- x + m (mixer(LN(x)) + ff(LN(x))): one norm, both sublayers read it
@@ -263,21 +263,23 @@ BLOCK_SANDWICH = 2  # x <- x + s1 N1b(mixer(conv_in(N1(x)))), then x <- x + s2 N
                     # added to the mixer's input
 BLOCK_PRENORM = 3   # x <- x + mixer(N1(x)), then x <- x + ff(N2(x)): RMS norms with a weight vector on the sublayers' inputs,
                     # optionally with a short causal convolution added to what each sublayer reads
-CANON_FUSED_ROWS = 8  # a carried input window is a ring over positions with this many rows to spare, so that one launch
-                      # may read the old inputs and write the new ones of up to this many rows
+CANON_FUSED_ROWS = 8  # a convolution's carried inputs as a ring over positions have this many rows to spare, so that one
+                      # launch may read the old inputs and write the new ones of up to this many rows
 
 FF_MOE = 0          # routed experts (+ shared expert)
 FF_DENSE = 1        # W_down act(W_up h), act = relu(z)^2
 FF_GLU = 2          # W_down (act(W_gate h) * (W_up h)), act = the tanh form of gelu
 ACT_GELU_TANH = 0   # activation of a gated dense feed-forward (FF_GLU)
 ACT_RELU = 1
-ACT_SILU = 2             # (experts) silu(gate) * up
+ACT_SILU = 2             # silu(gate) * up (experts, and FF_GLU)
 ACT_CLAMPED_GLU = 3      # (experts) g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(1.702 g) (u + 1)
+ACT_GELU_UP = 4          # (experts, the shared one too) no gate: gelu(up), the erf form
 ROUTE_TOPK_SOFTMAX = 0   # top-k of (logits + bias), softmax over the chosen logits
 ROUTE_SCORE_GROUPS = 1   # softmax over all outputs; choice by score + correction inside the best expert groups;
                          # weights = the chosen scores; trailing outputs may be identity experts
 ROUTE_SIGMOID_GROUPS = 2  # sigmoid scores; a group ranks by the sum of its two largest scores; the chosen scores are
                           # divided by their sum and multiplied by a constant
+ROUTE_SOFTMAX_SCORES = 3  # the same with scores that are a softmax over all experts
 GATE_NONE = 0
 GATE_ELEMENT = 1            # the mixer's output is multiplied element by element with sigmoid(W_g h)
 GATE_HEAD = 2               # one sigmoid gate per head
@@ -286,6 +288,7 @@ GATE_HEAD = 2               # one sigmoid gate per head
 QK_NORM_NONE = 0
 QK_NORM_WEIGHT_FIRST = 1    # RMS norm with a [dim] weight shared by the heads, before the rotation
 QK_NORM_UNIT_LAST = 2       # division by the root mean square (no weight), after the rotation
+QK_NORM_WHOLE_FIRST = 3     # one RMS norm over all heads' rows of the projection with a weight of that size, before the rotation
 SINK_NONE = 0
 SINK_LEARNED = 1            # exp(sink_h), a learned number per head, joins the softmax denominator
 SINK_ONE = 2                # a sink of score 0: the denominator holds one extra 1
@@ -299,6 +302,14 @@ def rotary_inv_freq(dims: int, base: float, scaling: tuple = ()) -> list:
         return f
     if scaling[0] == "linear":
         return [x / float(scaling[1]) for x in f]
+    if scaling[0] == "yarn":
+        _, factor, fast, slow, original = scaling
+
+        def index(turns):  # the dimension that turns this often over `original` positions
+            return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+        lo, hi = max(math.floor(index(fast)), 0), min(math.ceil(index(slow)), dims - 1)
+        ramp = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(dims // 2)]
+        return [x / factor * r + x * (1.0 - r) for x, r in zip(f, ramp)]
     if scaling[0] != "bands":
         raise UnsupportedArchitecture(f"unknown rotary scaling {scaling[0]!r}")
     _, factor, low, high, original = scaling
@@ -313,6 +324,12 @@ def rotary_inv_freq(dims: int, base: float, scaling: tuple = ()) -> list:
             t = (original / wave - low) / (high - low)
             out.append((1.0 - t) * x / factor + t * x)
     return out
+
+
+def rotary_amplitude(scaling: tuple = ()) -> float:
+    """Factor on sine and cosine that comes with the frequencies' scaling."""
+    import math
+    return 0.1 * math.log(scaling[1]) + 1.0 if scaling and scaling[0] == "yarn" else 1.0
 
 
 @dataclass
@@ -336,18 +353,21 @@ class MixerSpec:
     # sink in the softmax denominator; sigmoid output gate
     rot_dim: int = 0
     kv_rank: int = 0
+    q_rank: int = 0             # > 0: the queries come from an RMS-normed latent of their own
     # mlstm
     gate_cap: float = 0.0       # gate pre-activations pass cap * tanh(z / cap)
     # mamba2: heads x vdim channels, `state` rows per head, `groups` shared B / C groups
     state: int = 0
     groups: int = 1
-    conv: int = 1               # taps of the causal convolution (the last one is the current token's)
+    conv: int = 1               # taps of the causal convolution (the last one is the current token's); on attention: of q, k, v
+    conv_ring: bool = False     # its carried inputs are a ring over positions (CANON_FUSED_ROWS rows to spare), else oldest first
     norm_groups: int = 1        # the gated output is RMS-normed in this many equal parts
     # attention options of the sandwich block's mixers
     bias: bool = False          # q, k, v (and with o_bias the output) projections carry biases
     o_bias: bool = False
     rot_scaling: tuple = ()     # () none; ("linear", factor); ("bands", factor, low, high, original): long waves
-                                # divided by factor, short ones kept, a linear blend between
+                                # divided by factor, short ones kept, a linear blend between; ("yarn", factor, fast,
+                                # slow, original): a linear blend over the dimension's index, sine and cosine scaled too
     qk_norm: int = QK_NORM_NONE
     sink: int = SINK_NONE
     talk: bool = False          # the heads' softmax weights are mixed by a [heads, heads] matrix before the values
@@ -356,6 +376,8 @@ class MixerSpec:
     tau: float = 1.0            # decay = sigmoid(z)^(1 / tau)
     decay_rank: int = 0         # inner size of the low-rank map that gives z (read from the tensor's shape)
     gate_rank: int = 0          # delta rule: inner size of the low-rank map behind the output gate (from the tensor's shape)
+    head_decay: bool = False    # delta rule: one decay per head straight from the input (no low-rank map), output gate
+                                # silu of a full projection
     # a second mixer that reads the same input; the layer's result is left_scale * this + right_scale * right
     right: "MixerSpec | None" = None
     left_scale: float = 1.0
@@ -394,10 +416,16 @@ class MixerSpec:
         return self.n_out + (self.right.n_out if self.right is not None else 0)
 
     @property
-    def conv_channels(self) -> int:   # mamba2: x | B | C pass the convolution; delta rule: q | k | v
+    def conv_channels(self) -> int:   # mamba2: x | B | C pass the convolution; delta rule and attention: q | k | v
         if self.kind == MIX_DELTA:
             return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+        if self.kind == MIX_ATTENTION:
+            return self.n_q + self.n_k + self.n_v
         return self.heads * self.vdim + 2 * self.groups * self.state
+
+    @property
+    def conv_rows(self) -> int:       # carried inputs of the convolution
+        return self.conv - 1 + (CANON_FUSED_ROWS if self.conv_ring else 0) if self.conv > 1 else 0
 
     @property
     def cache_dim(self) -> int:       # latent attention: cached row = latent | shared rotated key part
@@ -407,13 +435,15 @@ class MixerSpec:
     def state_floats(self) -> int:
         """float32 words of the per-sequence state of one run of this mixer."""
         if self.kind == MIX_DELTA:      # S [H][dim][vdim] | the convolution's last inputs (q | k | v)
-            return self.heads * self.dim * self.vdim + (self.conv - 1) * self.conv_channels
+            return self.heads * self.dim * self.vdim + self.conv_rows * self.conv_channels
+        if self.kind == MIX_ATTENTION:  # the convolution's last inputs (q | k | v)
+            return self.conv_rows * self.conv_channels
         if self.kind in (MIX_RETENTION, MIX_GLA, MIX_LINEAR):
             return self.heads * self.dim * self.vdim
         if self.kind == MIX_MLSTM:      # S [H][dim][vdim] | n [H][dim] | m [H]
             return self.heads * (self.dim * self.vdim + self.dim + 1)
         if self.kind == MIX_MAMBA2:     # S [H][state][vdim] | the convolution's last taps - 1 inputs
-            return self.heads * self.state * self.vdim + (self.conv - 1) * self.conv_channels
+            return self.heads * self.state * self.vdim + self.conv_rows * self.conv_channels
         return 0
 
 
@@ -430,8 +460,8 @@ class MoESpec:
     group_keep: int = 1         # only experts of the best group_keep groups can be chosen
     shared_gate: bool = True    # the shared expert sits behind a scalar sigmoid gate
     act: int = ACT_GELU_TANH    # FF_GLU: the gate's activation
-    route_scale: float = 1.0    # ROUTE_SIGMOID_GROUPS: factor on the weights
-    route_norm: bool = True     # ROUTE_SIGMOID_GROUPS: the chosen scores are divided by their sum
+    route_scale: float = 1.0    # ROUTE_SIGMOID_GROUPS, ROUTE_SOFTMAX_SCORES: factor on the weights
+    route_norm: bool = True     # the same: the chosen scores are divided by their sum
     expert_act: int = ACT_SILU
     limit: float = 0.0          # ACT_CLAMPED_GLU
     scale_input: bool = False   # a chosen expert's weight multiplies its input instead of its output
@@ -439,6 +469,11 @@ class MoESpec:
     @property
     def n_router(self) -> int:
         return self.experts + self.identity
+
+    @property
+    def unit_rows(self) -> int:
+        """Rows of an expert's first matrix per hidden unit: gate and up, or up alone."""
+        return 1 if self.expert_act == ACT_GELU_UP else 2
 
 
 @dataclass
@@ -456,6 +491,7 @@ class StackConfig:
     loop_start: int = 0
     loop_stop: int = 0
     loop_times: int = 0         # 0 = no repeated span
+    loop_mix: bool = True       # a pass opens with a projection of [x; embedding output]; else passes follow one another
     norm_eps: float = 1e-5
     residual_mult: float = 1.0
     logit_softcap: float = 0.0
@@ -464,6 +500,7 @@ class StackConfig:
     logit_scale: float = 1.0    # logits = head x * logit_scale
     canon_taps: int = 1         # taps of the convolution added to the mixer's input (sandwich block, and pre-norm block with
                                 # canon_both; the last one is the current token's, with 1 nothing is carried)
+    norm_plus_one: bool = False  # pre-norm block: the layers' and the final norm's weights are stored as distance from one
     tied_head: bool = False     # logits = embedding table x (no head matrix)
     canon_both: bool = False    # pre-norm block: the inputs of both sublayers pass such a convolution
     ctx_len: int = 1 << 20      # the design has no positional table: bounded by the cache pool only
@@ -486,13 +523,14 @@ class StackConfig:
         a, b = self.loop_start, self.loop_stop
         out = [(i, 0, False) for i in range(a)]
         for p in range(self.loop_times):
-            out += [(i, p, i == a) for i in range(a, b)]
+            out += [(i, p, self.loop_mix and i == a) for i in range(a, b)]
         return out + [(i, 0, False) for i in range(b, L)]
 
     @property
     def has_state(self) -> bool:
         """Some layer carries a recurrent state: a cached prefix cannot be cut back to an earlier length."""
-        return self.canon_taps > 1 or any(s.mixer.kind in STATE_MIXERS or s.mixer.right is not None for s in self.layers)
+        return self.canon_taps > 1 or any(s.mixer.kind in STATE_MIXERS or s.mixer.state_floats or s.mixer.right is not None
+                                          for s in self.layers)
 
     def run_state_floats(self, li: int) -> int:
         """float32 words of the per-sequence state of one run of layer li: the mixer's (and its second mixer's) state
@@ -971,7 +1009,130 @@ class StackConfig:
         return dict(architecture="Rogisun", vocab=self.n_vocab, width=self.n_embd, layers=out, norm=dict(eps=self.norm_eps),
                     canon=dict(taps=self.canon_taps))
 
+    # -- config.json of the Gavasun design
+    @classmethod
+    def from_gavasun(cls, c: dict) -> "StackConfig":
+        def bad(msg):
+            raise UnsupportedArchitecture("Gavasun: " + msg)
+
+        def rotary(m: dict, dim: int) -> dict:
+            rot = m.get("rot") or {}
+            sc = rot.get("scaling") or {}
+            scaling = ()
+            if sc:
+                scaling = ("yarn", float(sc["factor"]), float(sc["fast"]), float(sc["slow"]), float(sc["original"]))
+                if min(scaling[1:]) <= 0:
+                    bad("rot.scaling: its numbers must be positive")
+            dims = int(rot.get("dims", dim if rot else 0))
+            if dims % 2 or not 0 <= dims <= dim:
+                bad("rot.dims must be even and at most the rotated size")
+            base = float(rot.get("base", 10000.0))
+            if base <= 0 or (scaling and base == 1.0):
+                bad("rot.base must be positive (and not 1 with scaled frequencies)")
+            return dict(rot_dims=dims, rot_base=base, rot_scaling=scaling)
+
+        def mask_size(m: dict) -> int:
+            size = int((m.get("mask") or {}).get("size", 0))
+            if size < 0 or (m.get("mask") and size == 0):
+                bad("mask.size must be positive")
+            return size
+
+        layers = []
+        for ent in c["layers"]:
+            m, t = ent["mixer"], ent["type"]
+            H = int(m["heads"])
+            if t == "delta":
+                mx = MixerSpec(kind=MIX_DELTA, heads=H, kv_heads=int(m.get("kv_heads", H)), dim=int(m["dim"]),
+                               vdim=int(m.get("vdim", m["dim"])), conv=int(m["conv"]), conv_ring=True, head_decay=True,
+                               gate=GATE_ELEMENT)
+            elif t == "latent_attention":
+                mx = MixerSpec(kind=MIX_LATENT, heads=H, kv_heads=1, dim=int(m["dim"]), vdim=int(m["vdim"]), scale=float(m["scale"]),
+                               rot_dim=int(m["rot_dim"]), kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), rot_pairs=True,
+                               window=mask_size(m), **rotary(m, int(m["rot_dim"])))
+                if min(mx.kv_rank, mx.q_rank) <= 0 or mx.rot_dim < 0:
+                    bad("latent attention sizes must be positive")
+            elif t == "attention":
+                mx = MixerSpec(kind=MIX_ATTENTION, heads=H, kv_heads=int(m.get("kv_heads", H)), dim=int(m["dim"]),
+                               vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]), bias=True, conv=int(m.get("conv", 1)),
+                               conv_ring=True, qk_norm=QK_NORM_WHOLE_FIRST, chunk=mask_size(m), **rotary(m, int(m["dim"])))
+            else:
+                raise UnsupportedArchitecture(f"unknown mixer type {t!r}")
+            if min(mx.heads, mx.kv_heads, mx.dim, mx.vdim) <= 0 or mx.heads % mx.kv_heads or mx.conv < 1:
+                bad("heads must be a positive multiple of kv_heads, sizes and taps positive")
+            mlp = None
+            f = ent.get("mlp")
+            if f:
+                kind = f.get("kind")
+                if kind == "dense":
+                    mlp = MoESpec(kind=FF_GLU, ff=int(f["ff"]), act=ACT_SILU)
+                elif kind == "moe":
+                    r, sh = f["router"], f.get("shared") or {}
+                    mlp = MoESpec(kind=FF_MOE, route=ROUTE_SOFTMAX_SCORES, experts=int(r["experts"]), top=int(r["top"]),
+                                  ff=int(f["expert"]["ff"]), shared_ff=int(sh.get("ff", 0)), shared_gate=False,
+                                  expert_act=ACT_GELU_UP)
+                    if not 0 < mlp.top <= mlp.experts or mlp.shared_ff < 0:
+                        bad("router: top must be in 1..experts")
+                else:
+                    raise UnsupportedArchitecture(f"unknown feed-forward kind {kind!r}")
+                if mlp.ff <= 0:
+                    bad("hidden sizes must be positive")
+            layers.append(LayerSpec(mixer=mx, mlp=mlp))
+        loop = c.get("loop") or {}
+        cfg = cls(arch="gavasun", n_vocab=int(c["vocab"]), n_embd=int(c["width"]), layers=layers,
+                  loop_start=int(loop.get("start", 0)), loop_stop=int(loop.get("stop", 0)),
+                  loop_times=int(loop.get("times", 0)) if loop else 0, loop_mix=False, norm_eps=float(c["norm"]["eps"]),
+                  norm_plus_one=True, block=BLOCK_PRENORM,
+                  embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)), name=str(c.get("name", "")))
+        if cfg.loop_times and not 0 <= cfg.loop_start < cfg.loop_stop <= len(layers):
+            bad("loop: need 0 <= start < stop <= number of layers")
+        return cfg
+
+    def to_gavasun(self) -> dict:
+        """The config.json this configuration is read from (random-init fixtures, tests)."""
+        def rotary(m: MixerSpec) -> dict:
+            if not m.rot_dims:
+                return {}
+            d = dict(base=m.rot_base, dims=m.rot_dims)
+            if m.rot_scaling:
+                _, factor, fast, slow, original = m.rot_scaling
+                d["scaling"] = dict(factor=factor, fast=fast, slow=slow, original=original)
+            return dict(rot=d)
+
+        def mask(size: int) -> dict:
+            return dict(mask=dict(size=size)) if size else {}
+
+        out = []
+        for s in self.layers:
+            m = s.mixer
+            if m.kind == MIX_DELTA and m.head_decay:
+                ent = dict(type="delta", mixer=dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, conv=m.conv))
+            elif m.kind == MIX_LATENT and m.q_rank:
+                ent = dict(type="latent_attention", mixer=dict(heads=m.heads, dim=m.dim, rot_dim=m.rot_dim, vdim=m.vdim,
+                                                               kv_rank=m.kv_rank, q_rank=m.q_rank, scale=m.scale, **mask(m.window),
+                                                               **rotary(m)))
+            elif m.kind == MIX_ATTENTION and m.qk_norm == QK_NORM_WHOLE_FIRST:
+                ent = dict(type="attention", mixer=dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, scale=m.scale,
+                                                        conv=m.conv, **mask(m.chunk), **rotary(m)))
+            else:
+                raise UnsupportedArchitecture("Gavasun has no mixer of this kind")
+            f = s.mlp
+            if f is None:
+                ent["mlp"] = None
+            elif f.kind == FF_GLU:
+                ent["mlp"] = dict(kind="dense", ff=f.ff)
+            else:
+                ent["mlp"] = dict(kind="moe", expert=dict(ff=f.ff), router=dict(experts=f.experts, top=f.top),
+                                  **({"shared": dict(ff=f.shared_ff)} if f.shared_ff else {}))
+            out.append(ent)
+        c = dict(architecture="Gavasun", vocab=self.n_vocab, width=self.n_embd, layers=out, norm=dict(eps=self.norm_eps),
+                 embedding=dict(scale=self.embed_scale))
+        if self.loop_times:
+            c["loop"] = dict(start=self.loop_start, stop=self.loop_stop, times=self.loop_times)
+        return c
+
     def to_config_json(self) -> dict:
+        if self.arch == "gavasun":
+            return self.to_gavasun()
         if self.arch == "rogisun":
             return self.to_rogisun()
         if self.arch == "dekalorn":
@@ -982,7 +1143,8 @@ class StackConfig:
 
 
 STACK_ARCHS = {"Bizulix": StackConfig.from_bizulix, "Norevik": StackConfig.from_norevik, "Suvunex": StackConfig.from_suvunex,
-               "Dekalorn": StackConfig.from_dekalorn, "Rogisun": StackConfig.from_rogisun}
+               "Dekalorn": StackConfig.from_dekalorn, "Rogisun": StackConfig.from_rogisun,
+               "Gavasun": StackConfig.from_gavasun}
 
 
 def is_stack_model(path: str) -> bool:

@@ -266,13 +266,14 @@ def stack_post_norm_add(x, y, w, b, eps, idw=None):
     x += F.layer_norm(y, (y.shape[-1],), w, b, eps)
 
 
-def stack_rotate_pairs(x, pos, inv_freq):
-    """x [B, ..., R] float32: dims (2i, 2i + 1), i < len(inv_freq), turn by pos * inv_freq[i] (float64 angles)."""
+def stack_rotate_pairs(x, pos, inv_freq, amp=1.0):
+    """x [B, ..., R] float32: dims (2i, 2i + 1), i < len(inv_freq), turn by pos * inv_freq[i] (float64 angles) and grow by
+    amp."""
     n = inv_freq.numel()
     ang = pos.double()[:, None] * inv_freq.double()[None, :]
     while ang.dim() < x.dim():
         ang = ang.unsqueeze(1)
-    c, s = torch.cos(ang).float(), torch.sin(ang).float()
+    c, s = amp * torch.cos(ang).float(), amp * torch.sin(ang).float()
     u, v = x[..., 0:2 * n:2], x[..., 1:2 * n:2]
     out = x.clone()
     out[..., 0:2 * n:2] = u * c - v * s
@@ -280,30 +281,32 @@ def stack_rotate_pairs(x, pos, inv_freq):
     return out
 
 
-def stack_latent_prepare(proj, off, m, L, pos, slot, cache, bs, eps):
+def stack_latent_prepare(proj, off, m, L, pos, slot, cache, bs, eps, q=None):
     """The cached row of every token, [rms_norm(latent) * w | rotated shared key part], stored at its slot; returns
-    the queries folded onto the latent: per head [W_uk_h^T q_plain | rotated q part], float32 [B, H, C + R]."""
+    the queries (q, or columns of proj) folded onto the latent: per head [W_uk_h^T q_plain | rotated q part], float32
+    [B, H, C + R]."""
     B, H, D, R, C = proj.shape[0], m.heads, m.dim, m.rot_dim, m.kv_rank
-    q = proj[:, off["q"]:off["q"] + H * (D + R)].view(B, H, D + R)
+    q = (proj[:, off["q"]:off["q"] + H * (D + R)] if q is None else q).view(B, H, D + R)
     dkv = proj[:, off["k"]:off["k"] + C + R]
     c = dkv[:, :C] * torch.rsqrt(dkv[:, :C].pow(2).mean(-1, keepdim=True) + eps) * L["dkv_norm"]
     kr, qr = dkv[:, C:], q[..., D:]
     if L["inv_freq"] is not None:
-        kr, qr = stack_rotate_pairs(kr, pos, L["inv_freq"]), stack_rotate_pairs(qr, pos, L["inv_freq"])
+        amp = L.get("rot_amp", 1.0)
+        kr, qr = stack_rotate_pairs(kr, pos, L["inv_freq"], amp), stack_rotate_pairs(qr, pos, L["inv_freq"], amp)
     blk, o = slot.long() // bs, slot.long() % bs
     cache[blk, 0, o] = torch.cat([c, kr], 1).to(cache.dtype)
     qa = torch.einsum("bhd,hdc->bhc", q[..., :D], L["w_uk"].float().view(H, D, C))
     return torch.cat([qa, qr], -1)
 
 
-def stack_latent_attention(qa, cache, C, block_table, q_seq, q_len, bs, scale, sink):
-    """qa [B, H, C + R]; cache [blocks, 1, bs, C + R]; the first C dims of a cached row are also its value.
-    softmax with exp(sink_h) added to the denominator. Returns float32 [B, H, C]."""
+def stack_latent_attention(qa, cache, C, block_table, q_seq, q_len, bs, scale, sink, window=0):
+    """qa [B, H, C + R]; cache [blocks, 1, bs, C + R]; the first C dims of a cached row are also its value. window > 0: a row
+    sees its last `window` keys. softmax with exp(sink_h) added to the denominator. Returns float32 [B, H, C]."""
     B, H, _ = qa.shape
     out = torch.empty(B, H, C, dtype=torch.float32, device=qa.device)
     for b in range(B):
         n = int(q_len[b])
-        t = torch.arange(n, device=qa.device)
+        t = torch.arange(max(0, n - window) if window else 0, n, device=qa.device)
         bt = block_table[int(q_seq[b])].long()
         kk = cache[bt[t // bs], 0, t % bs].float()            # [n, C + R]
         s = (qa[b] @ kk.T) * scale                            # [H, n]
@@ -408,11 +411,11 @@ def stack_canon_conv(hn, w, window, q_seq):
     return out
 
 
-def stack_rotate_half64(x, pos, inv_freq):
-    """x [B, H, D] float32: dims i and i + n (n = len(inv_freq)) turn by pos * inv_freq[i]; float64 angles."""
+def stack_rotate_half64(x, pos, inv_freq, amp=1.0):
+    """x [B, H, D] float32: dims i and i + n (n = len(inv_freq)) turn by pos * inv_freq[i] and grow by amp; float64 angles."""
     n = inv_freq.numel()
     ang = pos.double()[:, None] * inv_freq.double()[None, :]
-    c, s = torch.cos(ang).float()[:, None, :], torch.sin(ang).float()[:, None, :]
+    c, s = amp * torch.cos(ang).float()[:, None, :], amp * torch.sin(ang).float()[:, None, :]
     u, v = x[..., :n], x[..., n:2 * n]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * n:]], -1)
 
@@ -503,9 +506,37 @@ def stack_canon_ring(hn, w, ring, pos, q_seq):
     return out
 
 
+def stack_conv_ring(u, w, ring, pos, q_seq):
+    """Causal per-channel convolution of u [B, ch] over each sequence's rows (w [ch, taps], the last tap is the current
+    token's), continued from `ring` [slots, R, ch], where the input of position p sits in row p % R; the rows' inputs are
+    written there in place. Nothing precedes position 0."""
+    K, R = w.shape[1], ring.shape[1]
+    out = torch.zeros_like(u)
+    for b in range(u.shape[0]):
+        st, p = ring[int(q_seq[b])], int(pos[b])
+        if K > 1:
+            st[p % R] = u[b]
+        for back in range(min(K, p + 1)):
+            out[b] += w[:, K - 1 - back] * (st[(p - back) % R] if back else u[b])
+    return out
+
+
+def stack_qkv_conv_prepare(proj, off, m, L, ring, pos, q_seq, eps):
+    """Attention whose q, k and v carry biases and pass a short convolution each: q and k are then RMS-normed over all their
+    heads at once and rotated. Returns q [B, H, D], k [B, G, D], v [B, G, Dv]."""
+    B, H, G, D, Dv = proj.shape[0], m.heads, m.kv_heads, m.dim, m.vdim
+    n = m.n_q + m.n_k + m.n_v
+    x = stack_conv_ring(proj[:, :n] + L["in_b"], L["conv_w"].view(n, m.conv), ring, pos, q_seq)
+    q = stack_rms_norm(x[:, :m.n_q], L["q_norm"], eps).view(B, H, D)
+    k = stack_rms_norm(x[:, m.n_q:m.n_q + m.n_k], L["k_norm"], eps).view(B, G, D)
+    if m.rot_dims:
+        q, k = (stack_rotate_half64(t, pos, L["inv_freq64"], L["rot_amp"]) for t in (q, k))
+    return q, k, x[:, m.n_q + m.n_k:].view(B, G, Dv)
+
+
 def stack_delta_rule(q, k, v, decay, beta, S, q_seq):
     """Per row: S [slots, H, D, Dv] <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q. q, k [B, G, D]
-    with head h using head h // (H / G), v [B, H, Dv], decay [B, H, D], beta [B, H]. Returns float32 [B, H, Dv]."""
+    with head h using head h // (H / G), v [B, H, Dv], decay [B, H, D] (or [B, H, 1]), beta [B, H]. Returns float32 [B, H, Dv]."""
     B, H, _ = v.shape
     out = torch.empty_like(v)
     hg = torch.arange(H, device=v.device) // (H // k.shape[1])
@@ -522,6 +553,8 @@ def stack_expert_mid(gu, ff, act, limit, w=None):
     """A routed expert's hidden activation from its gate | up products; w: the routing weight on the expert's input."""
     if w is not None:
         gu = gu * w
+    if act == 4:  # ACT_GELU_UP
+        return F.gelu(gu)
     if act == 3:  # ACT_CLAMPED_GLU
         g, u = torch.clamp(gu[:ff], max=limit), torch.clamp(gu[ff:], min=-limit, max=limit)
         return g * torch.sigmoid(1.702 * g) * (u + 1.0)
@@ -569,11 +602,12 @@ def stack_rotate_fold(q, k, pos, inv_freq, mix, groups):
     return qf.reshape(B, H, G * D), k
 
 
-def stack_route_sigmoid(z, top, group_count, group_keep, scale, norm=True):
-    """Router logits [B, X] -> sigmoid scores; a group of neighbours ranks by the sum of its two largest scores and
-    only the best `group_keep` groups stay; the `top` largest scores among them (ties: the lower index), with `norm`
-    divided by their sum (+ 1e-20), times `scale`. Returns expert ids [B, top] int32 and weights [B, top]."""
-    s = torch.sigmoid(z)
+def stack_route_sigmoid(z, top, group_count, group_keep, scale, norm=True, softmax=False):
+    """Router logits [B, X] -> sigmoid scores (or their softmax over all experts); a group of neighbours ranks by the
+    sum of its two largest scores and only the best `group_keep` groups stay; the `top` largest scores among them
+    (ties: the lower index), with `norm` divided by their sum (+ 1e-20), times `scale`. Returns expert ids [B, top]
+    int32 and weights [B, top]."""
+    s = torch.softmax(z, -1) if softmax else torch.sigmoid(z)
     choice = s
     if group_count > 1:
         per = z.shape[1] // group_count
@@ -772,10 +806,26 @@ class TorchStackExecutor:
         o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * L["gnorm"]).reshape(B, H * Dv)
         return o * torch.sigmoid(proj[:, off["g1"]:off["g1"] + m.gate_rank] @ L["g2"].float().T)
 
+    def _head_delta(self, L, m, proj, st, pos, qseq):
+        """The gated delta rule with one decay per head, up to its output projection; st [slots, state | convolution ring]."""
+        B, H, G, D, Dv, ch, off = proj.shape[0], m.heads, m.kv_heads, m.dim, m.vdim, m.conv_channels, L["off"]
+        nS, nq = H * D * Dv, G * D
+        ring = (st[:, nS:nS + m.conv_rows * ch].view(st.shape[0], m.conv_rows, ch) if m.conv_rows
+                else torch.zeros(st.shape[0], 1, ch))
+        x = F.silu(stack_conv_ring(proj[:, off["q"]:off["q"] + ch], L["conv_w"].view(ch, m.conv), ring, pos, qseq))
+        unit = lambda t: t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)  # noqa: E731
+        q, k = unit(x[:, :nq].view(B, G, D)) * float(D) ** -0.5, unit(x[:, nq:2 * nq].view(B, G, D))
+        decay = torch.exp(-torch.exp(L["a_log"]) * F.softplus(proj[:, off["a1"]:off["a1"] + H] + L["dt_bias"]))
+        o = stack_delta_rule(q, k, x[:, 2 * nq:].view(B, H, Dv), decay[:, :, None], torch.sigmoid(proj[:, off["rb"]:off["rb"] + H]),
+                             st[:, :nS].view(-1, H, D, Dv), qseq)
+        o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + self.r.cfg.norm_eps) * L["gnorm"]).reshape(B, H * Dv)
+        return o * F.silu(proj[:, off["g"]:off["g"] + H * Dv])
+
     def layer_run_prenorm(self, ri: int, B: int):
         """x <- x + mixer(N1(x)), then x <- x + ff(N2(x)), N an RMS norm with a weight vector, optionally with a causal
         convolution added to its result; a pass of a repeated span opens with x <- W_in [x; x0]."""
-        from ..models.config import FF_GLU, GATE_HEAD, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2
+        from ..models.config import (ACT_SILU, FF_GLU, GATE_HEAD, MIX_DELTA, MIX_LATENT, MIX_LINEAR, MIX_MAMBA2, QK_NORM_WHOLE_FIRST,
+                                     ROUTE_SOFTMAX_SCORES)
         r = self.r
         w, cfg, T = r.w, r.cfg, r.w.dtype
         li, _ps, opens = r.runs[ri]
@@ -806,14 +856,26 @@ class TorchStackExecutor:
             a = self._mamba2(L, m, proj, st, qseq)
         elif m.kind == MIX_LINEAR:
             a = self._linear(L, m, proj, st, qseq)
+        elif m.kind == MIX_DELTA:
+            a = self._head_delta(L, m, proj, st, pos, qseq)
         elif m.kind == MIX_LATENT:
-            C = m.kv_rank
-            qa = stack_latent_prepare(proj, off, m, dict(L, inv_freq=L["inv_freq64"]), pos, r.d_slot[:B], r.kc[ri], bs, eps)
+            C, q = m.kv_rank, None
+            if m.q_rank:  # queries from a normed latent of their own
+                r.qlat[:B, :m.q_rank] = stack_rms_norm(proj[:, off["dq"]:off["dq"] + m.q_rank], L["dq_norm"], eps).to(T)
+                q = stack_matmul(r.qlat[:B, :m.q_rank], L["w_uq"])
+            qa = stack_latent_prepare(proj, off, m, dict(L, inv_freq=L["inv_freq64"]), pos, r.d_slot[:B], r.kc[ri], bs, eps, q)
             lat = stack_latent_attention(qa, r.kc[ri], C, r.d_block_table, qseq, qlen, bs, m.scale,
-                                         torch.full((H,), -float("inf"), device=qa.device))
+                                         torch.full((H,), -float("inf"), device=qa.device), m.window)
             r.latbuf[:B, :H * C] = lat.reshape(B, H * C).to(T)
             ov = torch.einsum("bhc,hcv->bhv", r.latbuf[:B, :H * C].float().view(B, H, C), L["w_uvT"].float().view(H, C, Dv))
-            a = (ov * torch.sigmoid(proj[:, off["g"]:off["g"] + H])[:, :, None]).reshape(B, n_out)
+            a = (ov * torch.sigmoid(proj[:, off["g"]:off["g"] + H])[:, :, None] if m.gate == GATE_HEAD else ov).reshape(B, n_out)
+        elif m.qk_norm == QK_NORM_WHOLE_FIRST:
+            ch = m.conv_channels
+            ring = st[:, :m.conv_rows * ch].view(-1, m.conv_rows, ch) if m.conv_rows else torch.zeros(r.max_seqs, 1, ch)
+            q, k, v = stack_qkv_conv_prepare(proj, off, m, L, ring, pos, qseq, eps)
+            r.kc[ri][blk, :, o], r.vc[ri][blk, :, o] = k.to(T), v.to(T)
+            a = stack_attention_window(q, r.kc[ri], r.vc[ri], r.d_block_table, qseq, qlen, bs, m.scale, m.window,
+                                       [0] * H, [h // (H // G) for h in range(H)], m.chunk).reshape(B, n_out)
         else:
             q = proj[:, off["q"]:off["q"] + m.n_q]
             k = proj[:, off["k"]:off["k"] + m.n_k]
@@ -852,10 +914,12 @@ class TorchStackExecutor:
         proj = stack_matmul(h, L["w_ff"])
         r.proj[:B, :proj.shape[1]] = proj
         if f.kind == FF_GLU:
-            r.hmid[:B, :f.ff] = (torch.relu(proj[:, :f.ff]) * proj[:, f.ff:2 * f.ff]).to(T)
+            act = F.silu if f.act == ACT_SILU else torch.relu
+            r.hmid[:B, :f.ff] = (act(proj[:, :f.ff]) * proj[:, f.ff:2 * f.ff]).to(T)
             x += stack_matmul(r.hmid[:B, :f.ff], L["w_dense_down"])
             return
-        ids, wt = stack_route_sigmoid(proj[:, :f.experts], f.top, f.group_count, f.group_keep, f.route_scale, f.route_norm)
+        ids, wt = stack_route_sigmoid(proj[:, :f.experts], f.top, f.group_count, f.group_keep, f.route_scale, f.route_norm,
+                                      f.route == ROUTE_SOFTMAX_SCORES)
         r.eids[:B, :f.top], r.ew[:B, :f.top] = ids, wt
         y = torch.zeros_like(x)
         for b in range(B):
@@ -864,6 +928,9 @@ class TorchStackExecutor:
                 gu = stack_matmul(h[b:b + 1], L["w_gu"][e])[0]
                 mid = stack_expert_mid(gu, f.ff, f.expert_act, f.limit, wt[b, j] if f.scale_input else None).to(T)
                 y[b] += (1.0 if f.scale_input else wt[b, j]) * stack_matmul(mid[None], L["w_down"][e])[0]
+        if f.shared_ff:
+            mid = stack_expert_mid(proj[:, off["sup"]:off["sup"] + f.shared_ff], f.shared_ff, f.expert_act, f.limit).to(T)
+            y += stack_matmul(mid, L["sh_down"])
         x += y
 
     def layer_run_sandwich(self, ri: int, B: int):
