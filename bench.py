@@ -450,6 +450,46 @@ def rogisun_config(z: dict, vocab: int = 32000):
                        canon_taps=2, canon_both=True, tied_head=True)
 
 
+# the Gavasun design at the same widths: a delta rule with one decay per head, windowed latent attention with a query latent,
+# attention behind short convolutions in blocks of positions, another delta rule, twice; a dense first feed-forward, then 2 of 8
+# ungated experts and a shared one
+GAVASUN_SIZES = {
+    "s": dict(E=1024, pattern="dlad" * 2, delta=(8, 4, 64, 128), lat=(16, 64, 32, 64, 192, 512, 1024), attn=(16, 4, 64, 1024),
+              F=512, Fs=512, X=8, top=2, dense=2048),
+    "m": dict(E=2048, pattern="dlad" * 2, delta=(16, 8, 64, 128), lat=(16, 128, 64, 128, 192, 1024, 1024), attn=(16, 4, 128, 1024),
+              F=1024, Fs=1024, X=8, top=2, dense=4096),
+}
+
+
+def gavasun_config(z: dict, vocab: int = 32000):
+    """A Gavasun model with the sizes of a real model's layers (random weights)."""
+    from ollama_operator_amd.models.config import (ACT_GELU_UP, ACT_SILU, BLOCK_PRENORM, FF_GLU, FF_MOE, GATE_ELEMENT, MIX_ATTENTION,
+                                                    MIX_DELTA, MIX_LATENT, QK_NORM_WHOLE_FIRST, ROUTE_SOFTMAX_SCORES, LayerSpec,
+                                                    MixerSpec, MoESpec, StackConfig)
+    layers = []
+    for i, c in enumerate(z["pattern"]):
+        if c == "d":
+            h, g, d, dv = z["delta"]
+            m = MixerSpec(kind=MIX_DELTA, heads=h, kv_heads=g, dim=d, vdim=dv, conv=4, conv_ring=True, head_decay=True,
+                          gate=GATE_ELEMENT)
+        elif c == "l":
+            h, d, r, dv, rank, q_rank, window = z["lat"]
+            m = MixerSpec(kind=MIX_LATENT, heads=h, kv_heads=1, dim=d, vdim=dv, rot_dim=r, kv_rank=rank, q_rank=q_rank,
+                          scale=(d + r) ** -0.5, rot_dims=r, rot_base=5e4, rot_scaling=("yarn", 4.0, 32.0, 1.0, 4096.0),
+                          rot_pairs=True, window=window)
+        else:
+            h, g, d, chunk = z["attn"]
+            m = MixerSpec(kind=MIX_ATTENTION, heads=h, kv_heads=g, dim=d, vdim=d, scale=d ** -0.5, bias=True, conv=4, conv_ring=True,
+                          qk_norm=QK_NORM_WHOLE_FIRST, chunk=chunk, rot_dims=d // 2, rot_base=1e6,
+                          rot_scaling=("yarn", 2.0, 32.0, 1.0, 4096.0))
+        f = (MoESpec(kind=FF_GLU, ff=z["dense"], act=ACT_SILU) if i == 0 else
+             MoESpec(kind=FF_MOE, route=ROUTE_SOFTMAX_SCORES, experts=z["X"], top=z["top"], ff=z["F"], shared_ff=z["Fs"],
+                     shared_gate=False, expert_act=ACT_GELU_UP))
+        layers.append(LayerSpec(mixer=m, mlp=f))
+    return StackConfig(arch="gavasun", n_vocab=vocab, n_embd=z["E"], layers=layers, norm_eps=1e-6, block=BLOCK_PRENORM,
+                       loop_mix=False, norm_plus_one=True, embed_scale=4.0)
+
+
 def suvunex_config(z: dict, vocab: int = 32000):
     """A Suvunex model with the sizes of a real model's layers (random weights)."""
     from ollama_operator_amd.models.config import (BLOCK_SANDWICH, FF_GLU, MIX_ATTENTION, MIX_GLA, QK_NORM_UNIT_LAST,
@@ -564,41 +604,21 @@ def bench_stack(a) -> None:
             r.warmup()
             out[name] = {"bizulix_bf16": measure(r), "weights_gb": round(r.w.nbytes / 1e9, 3)}
             r.close()
-        if a.norevik:  # the Norevik design at the same width and depth, through the same engine and measurement
-            d = os.path.join(a.dir, f"norevik-{name}")
+        # the other designs at the same width and depth, through the same engine and measurement
+        for design, on, sizes, make in (("norevik", a.norevik, NOREVIK_SIZES, norevik_config),
+                                        ("suvunex", a.suvunex, SUVUNEX_SIZES, suvunex_config),
+                                        ("dekalorn", a.dekalorn, DEKALORN_SIZES, dekalorn_config),
+                                        ("rogisun", a.rogisun, ROGISUN_SIZES, rogisun_config),
+                                        ("gavasun", a.gavasun, GAVASUN_SIZES, gavasun_config)):
+            if not on:
+                continue
+            d = os.path.join(a.dir, f"{design}-{name}")
             if not os.path.exists(os.path.join(d, "model.safetensors")):
-                write_random_stack(d, norevik_config(NOREVIK_SIZES[name]), seed=0)
+                write_random_stack(d, make(sizes[name]), seed=0)
             r = StackRunner(d, device="cuda:0", dtype="bfloat16", max_batch=a.chunk, max_seqs=2, ctx=ctx)
             r.warmup()
-            out[name]["norevik_bf16"] = measure(r)
-            out[name]["norevik_weights_gb"] = round(r.w.nbytes / 1e9, 3)
-            r.close()
-        if a.suvunex:  # the Suvunex design at the same width and depth, through the same engine and measurement
-            d = os.path.join(a.dir, f"suvunex-{name}")
-            if not os.path.exists(os.path.join(d, "model.safetensors")):
-                write_random_stack(d, suvunex_config(SUVUNEX_SIZES[name]), seed=0)
-            r = StackRunner(d, device="cuda:0", dtype="bfloat16", max_batch=a.chunk, max_seqs=2, ctx=ctx)
-            r.warmup()
-            out[name]["suvunex_bf16"] = measure(r)
-            out[name]["suvunex_weights_gb"] = round(r.w.nbytes / 1e9, 3)
-            r.close()
-        if a.dekalorn:  # the Dekalorn design at the same width and depth, through the same engine and measurement
-            d = os.path.join(a.dir, f"dekalorn-{name}")
-            if not os.path.exists(os.path.join(d, "model.safetensors")):
-                write_random_stack(d, dekalorn_config(DEKALORN_SIZES[name]), seed=0)
-            r = StackRunner(d, device="cuda:0", dtype="bfloat16", max_batch=a.chunk, max_seqs=2, ctx=ctx)
-            r.warmup()
-            out[name]["dekalorn_bf16"] = measure(r)
-            out[name]["dekalorn_weights_gb"] = round(r.w.nbytes / 1e9, 3)
-            r.close()
-        if a.rogisun:  # the Rogisun design at the same width and depth, through the same engine and measurement
-            d = os.path.join(a.dir, f"rogisun-{name}")
-            if not os.path.exists(os.path.join(d, "model.safetensors")):
-                write_random_stack(d, rogisun_config(ROGISUN_SIZES[name]), seed=0)
-            r = StackRunner(d, device="cuda:0", dtype="bfloat16", max_batch=a.chunk, max_seqs=2, ctx=ctx)
-            r.warmup()
-            out[name]["rogisun_bf16"] = measure(r)
-            out[name]["rogisun_weights_gb"] = round(r.w.nbytes / 1e9, 3)
+            out[name][design + "_bf16"] = measure(r)
+            out[name][design + "_weights_gb"] = round(r.w.nbytes / 1e9, 3)
             r.close()
         if not a.stack_only:
             cfg = ModelConfig(name=f"mixtral-like-{name}", n_vocab=32000, n_embd=z["E"], n_layer=len(z["pattern"]),
@@ -629,6 +649,8 @@ def main():
                     "sinks beside gated linear attention, mixed-heads attention, input convolutions) at the same widths")
     ap.add_argument("--rogisun", action="store_true", help="with --stack: also measure the Rogisun design (constant-decay "
                     "linear attention, Mamba-2, attention in blocks of positions beside a gated delta rule, clamped experts)")
+    ap.add_argument("--gavasun", action="store_true", help="with --stack: also measure the Gavasun design (delta rule, latent "
+                    "attention and attention behind short convolutions in turn, ungated experts) at the same widths")
     ap.add_argument("--dekalorn", action="store_true", help="with --stack: also measure the Dekalorn design (windowed "
                     "differential and mixed-score attention, latent attention, sigmoid-routed experts) at the same widths")
     ap.add_argument("--gpus", type=int, default=1)

@@ -72,6 +72,8 @@ def write_random_stack(path: str, cfg, seed: int = 0, std: float = 0.05) -> None
         return write_random_dekalorn(path, cfg, seed=seed)
     if cfg.arch == "rogisun":
         return write_random_rogisun(path, cfg, seed=seed)
+    if cfg.arch == "gavasun":
+        return write_random_gavasun(path, cfg, seed=seed)
     g = torch.Generator().manual_seed(seed)
     E, V = cfg.n_embd, cfg.n_vocab
     T: dict = {}
@@ -428,4 +430,82 @@ def write_random_rogisun(path: str, cfg, seed: int = 0) -> None:
     os.makedirs(path, exist_ok=True)
     with open(os.path.join(path, "config.json"), "w") as fh:
         json.dump(cfg.to_rogisun(), fh, indent=1)
+    write_safetensors(os.path.join(path, "model.safetensors"), T)
+
+
+def write_random_gavasun(path: str, cfg, seed: int = 0) -> None:
+    """Random-init model folder of the Gavasun design (its tensor names). Projections ~ N(0, 1 / fan-in), queries and keys
+    with a gain so that the softmax is not flat; the layers' norm weights near 0 (they are distances from one); decays
+    spread so that some heads forget in a few tokens and others keep for hundreds; router matrices wide enough that the
+    chosen experts are not a close call."""
+    import json
+    import os
+
+    import torch
+
+    from ..engine.safetensors_io import write_safetensors
+    from .config import FF_GLU, MIX_DELTA, MIX_LATENT
+    g = torch.Generator().manual_seed(seed)
+    E, V = cfg.n_embd, cfg.n_vocab
+    T: dict = {}
+
+    def rnd(name, shape, s, mean=0.0):
+        T[name] = (mean + s * torch.randn(*shape, generator=g)).to(torch.bfloat16)
+
+    def uni(name, shape, lo, hi):
+        T[name] = (lo + (hi - lo) * torch.rand(*shape, generator=g)).to(torch.bfloat16)
+
+    def lin(name, n_out, n_in, gain=1.0):
+        rnd(name, (n_out, n_in), gain / n_in ** 0.5)
+
+    rnd("embed", (V, E), 1.0 / max(cfg.embed_scale, 1e-6))
+    for i, spec in enumerate(cfg.layers):
+        m, f, p = spec.mixer, spec.mlp, f"l{i}."
+        H, G, D, Dv = m.heads, m.kv_heads, m.dim, m.vdim
+        rnd(p + "norm1", (E,), 0.1)
+        if m.kind == MIX_DELTA:
+            for k, n in (("q", G * D), ("k", G * D), ("v", H * Dv)):
+                lin(p + "mix." + k, n, E, 1.5)
+                rnd(f"{p}mix.{k}.conv", (n, m.conv), 0.6, 0.2)
+            lin(p + "mix.b", H, E, 1.5)
+            lin(p + "mix.a", H, E)
+            uni(p + "mix.A_log", (H,), -3.0, 0.5)
+            uni(p + "mix.dt_bias", (H,), -5.0, 0.0)
+            lin(p + "mix.g", H * Dv, E, 1.5)
+            rnd(p + "mix.norm", (Dv,), 0.1, 1.0)
+        elif m.kind == MIX_LATENT:
+            lin(p + "mix.dq", m.q_rank, E)
+            rnd(p + "mix.dq.norm", (m.q_rank,), 0.1, 1.0)
+            lin(p + "mix.uq", H * (D + m.rot_dim), m.q_rank, 2.0)
+            lin(p + "mix.dkv", m.kv_rank + m.rot_dim, E, 2.0)
+            rnd(p + "mix.dkv.norm", (m.kv_rank,), 0.1, 1.0)
+            lin(p + "mix.uk", H * D, m.kv_rank, 1.5)
+            lin(p + "mix.uv", H * Dv, m.kv_rank)
+        else:
+            for k, n in (("q", m.n_q), ("k", m.n_k), ("v", m.n_v)):
+                lin(p + "mix." + k, n, E)
+                rnd(f"{p}mix.{k}.b", (n,), 0.3)
+                rnd(f"{p}mix.{k}.conv", (n, m.conv), 0.5, 0.2)
+            rnd(p + "mix.q.norm", (m.n_q,), 0.2, 1.4)
+            rnd(p + "mix.k.norm", (m.n_k,), 0.2, 1.4)
+        lin(p + "mix.o", E, H * Dv)
+        if f is None:
+            continue
+        rnd(p + "norm2", (E,), 0.1)
+        if f.kind == FF_GLU:
+            for k, (a, b) in (("gate", (f.ff, E)), ("up", (f.ff, E)), ("down", (E, f.ff))):
+                lin(p + "mlp." + k, a, b)
+            continue
+        for e in range(f.experts):
+            lin(f"{p}mlp.e{e}.up", f.ff, E)
+            lin(f"{p}mlp.e{e}.down", E, f.ff)
+        lin(p + "mlp.router", f.experts, E, 3.0)
+        if f.shared_ff:
+            lin(p + "mlp.shared.up", f.shared_ff, E)
+            lin(p + "mlp.shared.down", E, f.shared_ff)
+    rnd("final.norm", (E,), 0.1)
+    lin("head", V, E)
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as fh:
+        json.dump(cfg.to_gavasun(), fh, indent=1)
     write_safetensors(os.path.join(path, "model.safetensors"), T)

@@ -100,6 +100,12 @@ def in_chunk(n, size):
     return (i[None, :] <= i[:, None]) & (i[None, :] // size == i[:, None] // size)
 
 
+def visible(n, rule, m):
+    """Mask of one layer; without a size every earlier position is seen."""
+    size = (m.get("mask") or {}).get("size")
+    return rule(n, size) if size else in_window(n, n)
+
+
 # --------------------------------------------------------------------------------------------- mixers
 def gated_delta(h, W, m, eps):
     """Delta rule with one decay per head: the state forgets, then what it would answer to the new key is taken off the
@@ -136,7 +142,7 @@ def latent_attention(h, W, m, eps):
     q_rot = rotate(q[:, :, D:], m.get("rot"), True)
     k = (c @ W["uk"].T).view(n, H, D)
     v = (c @ W["uv"].T).view(n, H, Dv)
-    see = in_window(n, m["mask"]["size"])
+    see = visible(n, in_window, m)
     out = torch.zeros(n, H, Dv, dtype=F64)
     for hd in range(H):
         s = (q[:, hd, :D] @ k[:, hd].T + q_rot[:, hd] @ k_rot.T) * m["scale"]
@@ -152,7 +158,7 @@ def chunk_attention(h, W, m, eps):
     q = rotate((unit_rms(q, eps) * W["q.norm"]).view(n, H, D), m.get("rot"), False)
     k = rotate((unit_rms(k, eps) * W["k.norm"]).view(n, G, D), m.get("rot"), False)
     v = v.view(n, G, Dv)
-    see = in_chunk(n, m["mask"]["size"])
+    see = visible(n, in_chunk, m)
     out = torch.zeros(n, H, Dv, dtype=F64)
     for hd in range(H):
         g = hd // (H // G)
