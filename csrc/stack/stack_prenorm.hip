@@ -331,6 +331,7 @@ __device__ void route_sigmoid_serial(const MoeParams& P, const float* row, float
   for (int jj = 0; jj < P.top; ++jj) wts[jj] = (P.route_raw ? wts[jj] : wts[jj] / sum) * P.route_scale;
 }
 constexpr int ROUTE_SIG_MAX = 256;
+// a wave per row: blocks (x, 0) route, blocks (x, 1 ...) take 256 units each of the shared expert's activation
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
   __shared__ float sc[4][ROUTE_SIG_MAX];
@@ -340,8 +341,16 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(MoeParams P) {
   const int b = blockIdx.x * 4 + wv;
   if (b >= P.B) return;
   const float* row = P.proj + (long long)b * P.ld;
-  T* hs = (T*)P.hmid + (long long)b * P.ld_hmid + P.top * P.F;  // the shared expert's activation
-  for (int f = lane; f < P.Fs; f += 64) st(hs + f, gelu_erf(row[P.off_sup + f]));
+  if (blockIdx.y > 0) {
+    T* hs = (T*)P.hmid + (long long)b * P.ld_hmid + P.top * P.F;
+    const int f0 = (blockIdx.y - 1) * 256;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int f = f0 + 64 * k + lane;
+      if (f < P.Fs) st(hs + f, gelu_erf(row[P.off_sup + f]));
+    }
+    return;
+  }
   if (P.X <= 64) {
     int who;
     float w;
@@ -367,10 +376,11 @@ static void check_route_sigmoid(const MoeParams& P) {
 }
 void moe_route_sigmoid(const MoeParams& P, hipStream_t s) {
   check_route_sigmoid(P);
+  const dim3 grid((P.B + 3) / 4, 1 + (P.Fs + 255) / 256);
   if (P.f32)
-    hipLaunchKernelGGL(moe_route_sigmoid_kernel<float>, dim3((P.B + 3) / 4), dim3(256), 0, s, P);
+    hipLaunchKernelGGL(moe_route_sigmoid_kernel<float>, grid, dim3(256), 0, s, P);
   else
-    hipLaunchKernelGGL(moe_route_sigmoid_kernel<bf16>, dim3((P.B + 3) / 4), dim3(256), 0, s, P);
+    hipLaunchKernelGGL(moe_route_sigmoid_kernel<bf16>, grid, dim3(256), 0, s, P);
   launched("moe_route_sigmoid");
 }
 // ---- a few rows (decode steps): routing and the routed (and shared) activations in one launch. Grid (ff units / 4, row x

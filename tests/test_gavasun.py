@@ -159,6 +159,9 @@ MECHANISMS = {
     "attention_one_chunk_for_all": ([(gc.attn(heads=5, kv_heads=1, dim=12, vdim=70, chunk=1000), None)], {}),
     "attention_no_mask_no_rotation": ([(gc.attn(chunk=0, rot_dims=0), None)], {}),
     "attention_one_tap": ([(gc.attn(conv=1), None)], {}),
+    "attention_two_taps": ([(gc.attn(conv=2), None)], {}),
+    "attention_four_taps": ([(gc.attn(heads=4, dim=24, vdim=20, rot_dims=16, conv=4), None)], {}),
+    "attention_four_taps_wide_row": ([(gc.attn(heads=33, kv_heads=3, dim=64, vdim=8, rot_dims=64, conv=4), None)], {}),
     "attention_seven_taps": ([(gc.attn(conv=7, chunk=20), None)], {}),
     "attention_one_head": ([(gc.attn(heads=1, kv_heads=1, dim=8, vdim=8, rot_dims=8), None)], {}),
     "dense": ([(gc.delta(), gc.dense())], {}),
